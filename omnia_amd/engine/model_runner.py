@@ -116,7 +116,7 @@ class ModelRunner:
         self.vocab = model.cfg.vocab_size
         self.stateful = getattr(model, "stateful", False)  # recurrent layers: state slots
         # layer-list models: visible key ranges of prefill portions, query tile height
-        self.key_ranges = getattr(model, "has_pages", False)
+        self.key_ranges = getattr(model, "key_ranges", False)
         self.q_tile = getattr(model, "q_tile", None)
         self.use_graphs = use_graphs and (self.is_gpu or self.sim)
         self.buckets = [b for b in BATCH_BUCKETS if b < max_batch] + [max_batch]

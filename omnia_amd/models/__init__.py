@@ -1,5 +1,5 @@
-"""Model families served by the in-node engine (Llama-3 dense, Mixtral MoE, Sivadra
-layer lists)."""
+"""Model families served by the in-node engine (Llama-3 dense, Mixtral MoE, and the
+layer lists Sivadra and Sekazen)."""
 from .config import REGISTRY, ModelConfig, resolve  # noqa: F401
 
 
@@ -18,11 +18,11 @@ def build_model(cfg: ModelConfig, device="cpu", dtype=None, seed: int = 0, **kw)
         from .mixtral import MixtralModel
 
         return MixtralModel(cfg, device=device, dtype=dtype, seed=seed, **kw)
-    if cfg.arch == "sivadra":
+    if cfg.layers:
         from .hybrid import HybridModel
 
         if kw.pop("ep_mode", "tp") != "tp":
-            raise ValueError(f"{cfg.arch} has no experts to distribute")
+            raise ValueError(f"{cfg.arch}: layer-list models do not distribute experts")
         return HybridModel(cfg, device=device, dtype=dtype, seed=seed, **kw)
     raise ValueError(f"unsupported arch {cfg.arch}")
 

@@ -11,14 +11,15 @@ import dataclasses
 import math
 from dataclasses import dataclass, field
 
-from .layers import (DeltaSpec, DenseMLPSpec, LatentAttentionSpec, LayerSpec, RotarySpec,
-                     YarnSpec, tensor_shapes)
+from .layers import (DESIGNS, AttentionSpec, BandSpec, DeltaSpec, DenseMLPSpec, DesignSpec,
+                     ExpertsSpec, LatentAttentionSpec, LayerSpec, RotarySpec, YarnSpec,
+                     tensor_shapes)
 
 
 @dataclass(frozen=True)
 class ModelConfig:
     name: str
-    arch: str = "llama"  # llama | mixtral | sivadra
+    arch: str = "llama"  # llama | mixtral | a layer-list family (layers.DESIGNS)
     vocab_size: int = 128256
     hidden_size: int = 4096
     intermediate_size: int = 14336
@@ -37,6 +38,7 @@ class ModelConfig:
     # layer-list models (models/hybrid.py): one LayerSpec per layer; the uniform
     # head / intermediate sizes above do not apply to them
     layers: tuple = ()
+    logit_softcap: float = 0.0  # > 0: logits <- cap tanh(logits / cap)
     # tokenizer special ids (llama-3 layout)
     bos_token_id: int = 128000
     eos_token_ids: tuple = (128001, 128009)
@@ -55,8 +57,7 @@ class ModelConfig:
 
     def kv_bytes_per_token(self, dtype_bytes: int = 2) -> int:
         if self.layers:
-            return dtype_bytes * sum(l.mixer.padded_cache_width for l in self.layers
-                                     if l.mixer.kind == "latent_attention")
+            return dtype_bytes * sum(l.mixer.padded_cache_width for l in self.layers)
         return 2 * self.num_layers * self.kv_size * dtype_bytes
 
     @property
@@ -71,16 +72,20 @@ class ModelConfig:
                    for m in (l.mixer for l in self.layers) if m.kind == "delta")
 
     @property
+    def design(self) -> DesignSpec:
+        return DESIGNS[self.arch]
+
+    @property
     def key_window(self) -> int:
-        """Longest window of any attention layer (0: some layer sees the whole past,
-        or no layer attends)."""
+        """Longest window of any latent-attention layer (0: some layer sees the whole
+        past, or no layer gathers keys)."""
         w = [l.mixer.window for l in self.layers if l.mixer.kind == "latent_attention"]
         return 0 if not w or min(w) == 0 else max(w)
 
     def num_params(self) -> int:
         if self.layers:
-            return sum(math.prod(s) for s in tensor_shapes(self.layers, self.hidden_size,
-                                                           self.vocab_size).values())
+            return sum(math.prod(s) for s in tensor_shapes(
+                self.layers, self.hidden_size, self.vocab_size, self.design).values())
         d, i, L = self.hidden_size, self.intermediate_size, self.num_layers
         attn = d * (self.q_size + 2 * self.kv_size) + self.q_size * d
         mlp = 3 * d * i * max(1, self.num_experts) + (d * self.num_experts if self.is_moe else 0)
@@ -180,10 +185,59 @@ LLAMA_1B = ModelConfig(name="llama-1b-shape", vocab_size=32768, hidden_size=2048
                        intermediate_size=8192, num_layers=16, num_heads=16, num_kv_heads=8,
                        bos_token_id=256, eos_token_ids=(257,))
 
+
+
+def _paired(pairs: int, attn: AttentionSpec, window: int, mlp: ExpertsSpec) -> tuple:
+    """``pairs`` x (an attention layer with keys of its own, then one with ``window``
+    that attends to the same keys), each with a mixture of experts."""
+    out: list = []
+    for _ in range(pairs):
+        out.append(LayerSpec(attn, mlp))
+        out.append(LayerSpec(dataclasses.replace(attn, window=window, kv_from=len(out) - 1),
+                             mlp))
+    return tuple(out)
+
+
+# Sekazen: post-normed layer list of windowed grouped-query attention with sinks, key /
+# value borrowing and sparse experts
+TINY_SEKAZEN = ModelConfig(
+    name="tiny-sekazen", arch="sekazen", vocab_size=512, hidden_size=160, num_layers=4,
+    intermediate_size=96, max_position=4096, logit_softcap=20.0, bos_token_id=256,
+    eos_token_ids=(257,), tie_embeddings=True,
+    layers=_paired(
+        2, AttentionSpec(heads=6, kv_heads=2, dim=40, vdim=48, scale=0.15, window=56,
+                         rotary=RotarySpec(16, 10000.0, bands=BandSpec(8.0, 1.0, 4.0, 256))),
+        24, ExpertsSpec(ff=96, experts=6, top=2, limit=4.0)))
+# serving-sized shapes (random-init): width, depth, heads and experts of the Mixtral config
+# of the same size
+SEKAZEN_3B = ModelConfig(
+    name="sekazen-3b", arch="sekazen", vocab_size=32768, hidden_size=2048, num_layers=16,
+    intermediate_size=4096, max_position=131072, logit_softcap=30.0, bos_token_id=256,
+    eos_token_ids=(257,), tie_embeddings=True,
+    layers=_paired(
+        8, AttentionSpec(heads=16, kv_heads=8, dim=128, vdim=128, scale=128 ** -0.5, window=4096,
+                         rotary=RotarySpec(64, 500000.0, bands=BandSpec(8.0, 1.0, 4.0, 8192))),
+        1024, ExpertsSpec(ff=4096, experts=8, top=2, limit=7.0)))
+SEKAZEN_8X7B = ModelConfig(
+    name="sekazen-8x7b", arch="sekazen", vocab_size=32000, hidden_size=4096, num_layers=32,
+    intermediate_size=14336, max_position=131072, logit_softcap=30.0, bos_token_id=1,
+    eos_token_ids=(2,), tie_embeddings=True,
+    layers=_paired(
+        16, AttentionSpec(heads=32, kv_heads=8, dim=128, vdim=128, scale=128 ** -0.5,
+                          window=4096,
+                          rotary=RotarySpec(64, 1e6, bands=BandSpec(8.0, 1.0, 4.0, 8192))),
+        1024, ExpertsSpec(ff=14336, experts=8, top=2, limit=7.0)))
+# the Mixtral of sekazen-3b's width, depth and experts (design comparison)
+MIXTRAL_3B = ModelConfig(name="mixtral-3b-shape", arch="mixtral", vocab_size=32768,
+                         hidden_size=2048, intermediate_size=4096, num_layers=16, num_heads=16,
+                         num_kv_heads=8, num_experts=8, experts_per_token=2, bos_token_id=256,
+                         eos_token_ids=(257,))
+
 REGISTRY: dict[str, ModelConfig] = {
     c.name: c for c in [LLAMA3_8B, LLAMA31_8B, LLAMA3_70B, MIXTRAL_8X7B, TINY_LLAMA, TINY_MIXTRAL,
                    TINY_MIXTRAL_E8, EMBED_1B, TINY_EMBED, TINY_LLAMA_H8, TINY_SIVADRA,
-                   SIVADRA_1B, SIVADRA_8B, LLAMA_1B]
+                   SIVADRA_1B, SIVADRA_8B, LLAMA_1B, TINY_SEKAZEN, SEKAZEN_3B, SEKAZEN_8X7B,
+                   MIXTRAL_3B]
 }
 ALIASES = {
     "meta-llama/Meta-Llama-3-8B": "llama-3-8b",

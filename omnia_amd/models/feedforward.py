@@ -1,0 +1,90 @@
+"""Feed-forwards of layer-list models: how each one packs its checkpoint tensors and runs
+a step.
+
+``forward(w, h, is_decode)`` returns the operands of the residual kernel that follows:
+``{"m": projection, slabs or per-slot parts, "bias": ..., "slots": ...}``.  Padding
+happens in ``pack``, as in the mixers.
+"""
+from __future__ import annotations
+
+import torch
+import torch.nn.functional as F
+
+from .. import ops
+from ..ops import mixers as mops
+
+
+def _up8(n: int) -> int:
+    return (n + 7) // 8 * 8
+
+
+class BiasedSwiGLU:
+    """``W_down(silu(W_gate h + b) * (W_up h + b)) + b``."""
+
+    def __init__(self, spec, model):
+        self.spec, self.model = spec, model
+
+    def pack(self, get, d: int) -> dict:
+        ff = _up8(self.spec.ff)
+
+        def rows(n):
+            t = get(n)
+            return F.pad(t, (0, d - t.shape[1], 0, ff - t.shape[0]))
+
+        def vec(n, width):
+            t = get(n).float()
+            return F.pad(t, (0, width - t.numel())).contiguous()
+
+        down = get("down")
+        return {"gate_up": torch.cat([rows("gate"), rows("up")]).contiguous(),
+                "gate_up_b": torch.cat([vec("gate.b", ff), vec("up.b", ff)]),
+                "down": F.pad(down, (0, ff - down.shape[1], 0, d - down.shape[0])).contiguous(),
+                "down_b": vec("down.b", d)}
+
+    def _act(self, h, w: dict, is_decode) -> torch.Tensor:
+        """One fused prefill GEMM, or a GEMM whose bias / activation kernel also reduces
+        split-K slabs."""
+        m, W, b = self.model, w["gate_up"], w["gate_up_b"]
+        M, K = h.shape
+        N = W.shape[0]
+        if m._pgemm_ok(M, K, N // 2, is_decode, 128):
+            return ops.pgemm(1, h, W, bias=b)
+        cfg = m._wcfg(M, N // 2, K, 1, is_decode)
+        if cfg is not None:  # a tuned SwiGLU shape, as slabs (bias and activation follow)
+            nw, nwaves, S = cfg
+            p = m._wgemm(2, h, W, S, nw, nwaves,
+                         out=m._parts("gu", S, M, N, m._slab_dtype(nwaves)))
+        else:
+            p = m._slabs("gate_up", h, W, is_decode)
+        return mops.bias_swiglu(p, b, m.dtype)
+
+    def forward(self, w: dict, h: torch.Tensor, is_decode: bool) -> dict:
+        a = self._act(h, w, is_decode)
+        return {"m": self.model._slabs("down", a, w["down"], is_decode), "bias": w["down_b"]}
+
+
+class Experts:
+    """Sparse mixture of clamped GLUs (grouped MFMA kernels, no host sync)."""
+
+    def __init__(self, spec, model):
+        self.spec, self.model = spec, model
+
+    def pack(self, get, d: int) -> dict:
+        s, m = self.spec, self.model
+        E, ff, fp = s.experts, s.ff, s.ff_pad
+        r = get("router")
+        gu = torch.zeros(E, 2 * fp, d, dtype=m.dtype, device=m.device)
+        down = torch.zeros(E, d, fp, dtype=m.dtype, device=m.device)
+        for e in range(E):
+            t = get(f"e{e}.gate")
+            gu[e, :ff, :t.shape[1]] = t
+            gu[e, fp:fp + ff, :t.shape[1]] = get(f"e{e}.up")
+            t = get(f"e{e}.down")
+            down[e, :t.shape[0], :ff] = t
+        return {"router": F.pad(r, (0, d - r.shape[1])).contiguous(), "gate_up": gu, "down": down}
+
+    def forward(self, w: dict, h: torch.Tensor, is_decode: bool) -> dict:
+        return {"m": mops.experts(h, w, self.spec), "slots": True}
+
+
+MLPS = {"dense": BiasedSwiGLU, "moe": Experts}

@@ -1,18 +1,20 @@
-"""Layer-list models (``ModelConfig.layers``) on the engine's paged cache: Sivadra.
+"""Layer-list models (``ModelConfig.layers``) on the engine's paged cache: Sivadra, Sekazen.
 
-Every layer is ``x += norm1b(mixer(norm1(x)))`` and, with a feed-forward,
-``x += norm2b(ff(norm2(x)))`` around an fp32 residual stream; the mixers
-(:mod:`omnia_amd.models.mixers`) are chosen per layer.  The Dynamic-Tanh norm has
-no row statistics, so the post-norm, the residual update and the next sublayer's
-pre-norm are one elementwise kernel behind each output projection:
+Every layer is ``x += post(mixer(pre(x)))`` and, with a feed-forward,
+``x += post(ff(pre(x)))`` around an fp32 residual stream; mixers
+(:mod:`omnia_amd.models.mixers`) and feed-forwards (:mod:`omnia_amd.models.feedforward`)
+are chosen per layer, norms and head per family (``layers.DesignSpec``).  The
+post-norm, the residual update and the next sublayer's pre-norm (if the family has
+one) are one kernel behind each sublayer, which also reduces split-K slabs or sums a
+token's experts:
 
-    tanh_norm_embed -> [ in GEMM -> mixer kernels -> o GEMM -> tanh_norm_residual
-                         (-> gate_up GEMM -> bias_swiglu -> down GEMM ->
-                          tanh_norm_residual) ] * layers -> head GEMM
+    norm_embed -> [ in GEMM -> mixer kernels -> o GEMM -> norm_residual
+                    (-> feed-forward -> norm_residual) ] * layers -> head GEMM
+                    (-> softcap)
 
-A layer may use another layer's tensors; its pages / state are its own.  bf16
-models keep what feeds a softmax or a recurrence in fp32; fp32 models run every
-kernel and GEMM in fp32.
+A layer may use another layer's tensors (its pages / state are its own), or attend to
+another layer's pages.  bf16 models keep what feeds a softmax, a router or a recurrence
+in fp32; fp32 models run every kernel and GEMM in fp32.
 """
 from __future__ import annotations
 
@@ -26,39 +28,40 @@ from .. import ops
 from ..ops import mixers as mops
 from ..parallel import state as pstate
 from .config import ModelConfig
+from .feedforward import MLPS
 from .layers import tensor_shapes
 from .mixers import MIXERS, rotary_table
 from .projection import Parts, Projections
 
 
-def _up8(n: int) -> int:
-    return (n + 7) // 8 * 8
-
-
 @dataclass
 class HybridCache:
-    """Per layer: pages [num_blocks, block_size, width] of an attention layer, or the
+    """Per layer: the page tensors [num_blocks, ...] of an attention layer, or the
     (recurrent state, convolution inputs) pools of a recurrent one, indexed by the
-    sequence's state slot.  Block 0 is the null page of padded rows; slot 0 is unused
-    (padded rows carry slot -1)."""
+    sequence's state slot.  A layer that borrows another one's keys and values has that
+    layer's entry.  Block 0 is the null page of padded rows; slot 0 is unused (padded
+    rows carry slot -1)."""
 
-    layers: list  # (pages | None, (state, conv) | None)
+    layers: list  # (page tensors | None, (state, conv) | None)
     block_size: int
     num_blocks: int
     n_slots: int
 
     def page_tensors(self) -> list:
-        return [p for p, _ in self.layers if p is not None]
+        seen = {id(t): t for pages, _ in self.layers if pages is not None for t in pages}
+        return list(seen.values())
 
     def state_tensors(self) -> list:
         return [t for _, st in self.layers if st is not None for t in st]
 
 
-def random_tensor(name: str, shape: tuple, num_layers: int, gen, device) -> torch.Tensor:
+def random_tensor(name: str, shape: tuple, cfg: ModelConfig, gen, device) -> torch.Tensor:
     """Random-init checkpoint tensor (no checkpoint at hand), fp32."""
     leaf = name.split(".", 1)[1] if "." in name else name
     if leaf.endswith("alpha"):
         return torch.full(shape, 0.5, device=device)
+    if leaf == "mix.sink" or (cfg.design.norm == "rms" and leaf.startswith("norm")):
+        return torch.zeros(shape, device=device)  # norm weights stored around zero
     if leaf.startswith("norm") or name.startswith("final.") or leaf.endswith(".norm"):
         return torch.zeros(shape, device=device) if leaf.endswith(".b") else \
             torch.ones(shape, device=device)
@@ -75,13 +78,13 @@ def random_tensor(name: str, shape: tuple, num_layers: int, gen, device) -> torc
     if leaf.endswith(".conv"):
         return t.normal_(0.0, shape[1] ** -0.5, generator=gen)
     std = 0.02
-    if leaf in ("mix.o", "mlp.down"):
-        std /= math.sqrt(2 * num_layers)
+    if leaf == "mix.o" or leaf.endswith("down"):
+        std /= math.sqrt(2 * cfg.num_layers)
     return t.normal_(0.0, std, generator=gen)
 
 
 class HybridModel(Projections):
-    q_tile = 128  # query rows of one prefill attention workgroup (latent.hip)
+    q_tile = 128  # query rows of one prefill attention tile (latent.hip, gqa_prefill.hip)
 
     def __init__(self, cfg: ModelConfig, device="cpu", dtype=torch.bfloat16, seed: int = 0,
                  weights=None, decode_part_size: int = 512):
@@ -93,12 +96,17 @@ class HybridModel(Projections):
         self.tp, self.tpr = 1, 0
         self.cfg, self.device, self.dtype, self.seed = cfg, torch.device(device), dtype, seed
         self.stateful = cfg.stateful
-        self.has_pages = any(l.mixer.kind == "latent_attention" for l in cfg.layers)
+        # prefill works on a dense copy of each portion's visible keys
+        self.key_ranges = any(l.mixer.kind == "latent_attention" for l in cfg.layers)
         self.vocab_local, self.vocab_start = cfg.vocab_size, 0
-        self.d = _up8(cfg.hidden_size)  # padded width: zero columns stay zero
+        # padded width (zero columns stay zero): whole k-tiles of the grouped expert GEMMs
+        m = 64 if any(l.mlp is not None and l.mlp.kind == "moe" for l in cfg.layers) else 8
+        self.d = -(-cfg.hidden_size // m) * m
         self._ws: dict = {}
         self._tables: dict = {}
         self.mixers = [MIXERS[l.mixer.kind](l.mixer, self) for l in cfg.layers]
+        self.mlps = [None if l.mlp is None else MLPS[l.mlp.kind](l.mlp, self)
+                     for l in cfg.layers]
         self.w = self._pack(weights if weights is not None else self._random())
         ops.dgemm_prepare(self.device)
 
@@ -109,69 +117,74 @@ class HybridModel(Projections):
         return self._tables[rot]
 
     def _random(self):
-        shapes = tensor_shapes(self.cfg.layers, self.cfg.hidden_size, self.cfg.vocab_size)
+        cfg = self.cfg
+        shapes = tensor_shapes(cfg.layers, cfg.hidden_size, cfg.vocab_size, cfg.design)
         g = torch.Generator(device=self.device).manual_seed(self.seed)
 
         def get(name):
-            return random_tensor(name, shapes[name], self.cfg.num_layers, g, self.device)
+            return random_tensor(name, shapes[name], cfg, g, self.device)
 
         return get
 
     def _pack(self, get) -> dict:
         """``get(name)`` -> checkpoint tensor; kernel-ready weights."""
-        d, dev = self.d, self.device
+        cfg, d, dev, design = self.cfg, self.d, self.device, self.cfg.design
         seen: dict = {}
 
         def raw(name):
             return get(name).to(device=dev, dtype=self.dtype)
 
-        def vec(name, n):
-            t = get(name).to(device=dev, dtype=self.dtype).float()
-            return F.pad(t, (0, n - t.numel())).contiguous()
+        def part(prefix):
+            made: dict = {}
+
+            def one(n):
+                if n not in made:
+                    made[n] = raw(prefix + n)
+                return made[n]
+
+            return one
+
+        def vec(t):
+            t = t.float()
+            return F.pad(t, (0, d - t.numel())).contiguous()
 
         def norm(name):
-            return mops.TanhNorm(float(raw(name + ".alpha")), vec(name, d), vec(name + ".b", d))
+            if name is None:
+                return None
+            if design.norm == "tanh":
+                return mops.TanhNorm(float(raw(name + ".alpha")), vec(raw(name)),
+                                     vec(raw(name + ".b")))
+            return mops.RMSNorm(vec(1.0 + raw(name).float()), cfg.hidden_size, cfg.rms_eps)
+
+        def norms(p, k):
+            return [norm(p + n if n else None) for n in design.sublayer_norms(k)]
 
         def cols(t):
             return F.pad(t, (0, d - t.shape[1])).contiguous()
 
-        w = {"embed": cols(raw("embed")), "head": cols(raw("head")), "layers": [],
-             "final_norm": norm("final.norm")}
-        for i, l in enumerate(self.cfg.layers):
+        w = {"embed": cols(raw("embed")), "layers": [], "final_norm": norm("final.norm"),
+             "embed_norm": norm("embed.norm") if design.embed_norm else None}
+        w["head"] = w["embed"] if design.tied else cols(raw("head"))
+        for i, l in enumerate(cfg.layers):
             own = i if l.weights_of is None else l.weights_of
             if own not in seen:
                 p = f"l{own}."
-                cache: dict = {}
-
-                def mix(n, p=p, cache=cache):
-                    if n not in cache:
-                        cache[n] = raw(p + "mix." + n)
-                    return cache[n]
-
-                layer = {"norm1": norm(p + "norm1"), "norm1b": norm(p + "norm1b"),
-                         "mix": self.mixers[i].pack(mix, d)}
+                layer = {"mix": self.mixers[i].pack(part(p + "mix."), d), "mlp": None}
+                layer["pre1"], layer["post1"] = norms(p, 1)
                 if l.mlp is not None:
-                    ff = _up8(l.mlp.ff)
-
-                    def rows(n, p=p, ff=ff):
-                        t = raw(p + "mlp." + n)
-                        return F.pad(t, (0, d - t.shape[1], 0, ff - t.shape[0]))
-
-                    down = raw(p + "mlp.down")
-                    layer.update(
-                        norm2=norm(p + "norm2"), norm2b=norm(p + "norm2b"),
-                        gate_up=torch.cat([rows("gate"), rows("up")]).contiguous(),
-                        gate_up_b=torch.cat([vec(p + "mlp.gate.b", ff), vec(p + "mlp.up.b", ff)]),
-                        down=F.pad(down, (0, ff - down.shape[1], 0, d - down.shape[0])).contiguous(),
-                        down_b=vec(p + "mlp.down.b", d))
+                    layer["mlp"] = self.mlps[i].pack(part(p + "mlp."), d)
+                    layer["pre2"], layer["post2"] = norms(p, 2)
                 seen[own] = layer
             w["layers"].append(seen[own])
         return w
 
     # ------------------------------------------------------------ cache
     def allocate_cache(self, num_blocks: int, block_size: int, n_slots: int) -> HybridCache:
-        return HybridCache([m.alloc(num_blocks, block_size, n_slots) for m in self.mixers],
-                           block_size, num_blocks, n_slots)
+        layers: list = []
+        for m in self.mixers:
+            j = m.spec.kv_from
+            layers.append(m.alloc(num_blocks, block_size, n_slots) if j is None else layers[j])
+        return HybridCache(layers, block_size, num_blocks, n_slots)
 
     # ------------------------------------------------------------ forward
     def project(self, x: torch.Tensor, w: torch.Tensor, is_decode: bool) -> torch.Tensor:
@@ -185,40 +198,21 @@ class HybridModel(Projections):
         m = self._proj(tag, x, w, is_decode)
         return m.t if isinstance(m, Parts) else m
 
-    def _act(self, h, w: dict, is_decode) -> torch.Tensor:
-        """``silu(W_gate h + b) * (W_up h + b)``: one fused prefill GEMM, or a GEMM whose
-        bias / activation kernel also reduces split-K slabs."""
-        W, b = w["gate_up"], w["gate_up_b"]
-        M, K = h.shape
-        N = W.shape[0]
-        if self._pgemm_ok(M, K, N // 2, is_decode, 128):
-            return ops.pgemm(1, h, W, bias=b)
-        cfg = self._wcfg(M, N // 2, K, 1, is_decode)
-        if cfg is not None:  # a tuned SwiGLU shape, as slabs (bias and activation follow)
-            nw, nwaves, S = cfg
-            m = self._wgemm(2, h, W, S, nw, nwaves,
-                            out=self._parts("gu", S, M, N, self._slab_dtype(nwaves)))
-        else:
-            m = self._slabs("gate_up", h, W, is_decode)
-        return mops.bias_swiglu(m, b, self.dtype)
-
     def run_layers(self, fb, kv: HybridCache, trace: list | None = None) -> torch.Tensor:
         """Final-normed rows of the step; ``trace`` receives the residual stream after
         every layer (tests)."""
         self._min_rows = self.PGEMM_MIXED_MIN_ROWS if fb.num_decode else self.PGEMM_MIN_ROWS
         ws, dt, dec = self.w["layers"], self.dtype, fb.is_decode
-        x, h = mops.tanh_norm_embed(fb.input_ids, self.w["embed"], self.cfg.vocab_size,
-                                    ws[0]["norm1"], fb.ids_src, fb.tok_slots)
-        for i, (w, mixer) in enumerate(zip(ws, self.mixers)):
-            after = ws[i + 1]["norm1"] if i + 1 < len(ws) else self.w["final_norm"]
-            mlp = "gate_up" in w
+        x, h = mops.norm_embed(fb.input_ids, self.w["embed"], self.cfg.vocab_size,
+                               self.w["embed_norm"], ws[0]["pre1"], fb.ids_src, fb.tok_slots)
+        for i, (w, mixer, mlp) in enumerate(zip(ws, self.mixers, self.mlps)):
+            after = ws[i + 1]["pre1"] if i + 1 < len(ws) else self.w["final_norm"]
             o = mixer.forward(w["mix"], h, fb, kv.layers[i])
-            h = mops.tanh_norm_residual(x, self._slabs("o", o, w["mix"]["o"], dec), w["norm1b"],
-                                        w["norm2"] if mlp else after, dt)
+            h = mops.norm_residual(x, self._slabs("o", o, w["mix"]["o"], dec), w["post1"],
+                                   w["pre2"] if mlp else after, dt)
             if mlp:
-                a = self._act(h, w, dec)
-                h = mops.tanh_norm_residual(x, self._slabs("down", a, w["down"], dec),
-                                            w["norm2b"], after, dt, w["down_b"])
+                h = mops.norm_residual(x, post=w["post2"], pre=after, dtype=dt,
+                                       **mlp.forward(w["mlp"], h, dec))
             if trace is not None:
                 trace.append(x[:, :self.cfg.hidden_size].clone())
         return h
@@ -227,8 +221,11 @@ class HybridModel(Projections):
         W = self.w["head"]
         cfg = self._wcfg(h.shape[0], W.shape[0], h.shape[1], 0, is_decode)
         if cfg is not None and cfg[2] == 1:
-            return ops.wgemm(0, h, W, 1, cfg[0], cfg[1])
-        return ops.linear(h, W)
+            z = ops.wgemm(0, h, W, 1, cfg[0], cfg[1])
+        else:
+            z = ops.linear(h, W)
+        cap = self.cfg.logit_softcap
+        return mops.softcap_(z, cap) if cap else z
 
     def forward(self, fb, kv: HybridCache, gather: bool = True) -> torch.Tensor:
         h = self.run_layers(fb, kv)

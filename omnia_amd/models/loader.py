@@ -178,7 +178,7 @@ def load_layer_list_checkpoint(path: str | Path, cfg: ModelConfig):
     from .layers import tensor_shapes
 
     rd = _Reader(path)
-    shapes = tensor_shapes(cfg.layers, cfg.hidden_size, cfg.vocab_size)
+    shapes = tensor_shapes(cfg.layers, cfg.hidden_size, cfg.vocab_size, cfg.design)
     for name, shape in shapes.items():
         if not rd.has(name):
             raise ValueError(f"{path}: tensor {name} is missing")
@@ -198,21 +198,20 @@ def load_checkpoint(path: str | Path, cfg: ModelConfig, tp: int = 1, rank: int =
 
 
 def _layer_list_config(c: dict, name: str) -> ModelConfig:
-    from .layers import parse_layers
+    from .layers import DESIGNS, parse_layers
 
     layers = parse_layers(c["layers"])
     vocab = int(c["vocab"])
+    arch = c["architecture"].lower()
     return ModelConfig(
-        name=name, arch=c["architecture"].lower(), vocab_size=vocab,
+        name=name, arch=arch, vocab_size=vocab,
         hidden_size=int(c["width"]), num_layers=len(layers), layers=layers,
         intermediate_size=max([l.mlp.ff for l in layers if l.mlp is not None], default=0),
-        rms_eps=float(c["norm"]["eps"]),
+        rms_eps=float(c["norm"]["eps"]), logit_softcap=float(c.get("logit_softcap") or 0.0),
+        tie_embeddings=DESIGNS[arch].tied,
         max_position=int(c.get("max_position", 131072)),
         bos_token_id=int(c.get("bos", min(256, vocab - 1))),
         eos_token_ids=tuple(c.get("eos", (min(257, vocab - 1),))))
-
-
-LAYER_LIST_ARCHS = {"sivadra"}
 
 
 def config_from_hf(path: str | Path, name: str | None = None) -> ModelConfig:
@@ -220,7 +219,9 @@ def config_from_hf(path: str | Path, name: str | None = None) -> ModelConfig:
     a layer-list architecture (``architecture`` + ``layers``)."""
     c = json.loads((Path(path) / "config.json").read_text())
     if "architecture" in c and "layers" in c:
-        if c["architecture"].lower() not in LAYER_LIST_ARCHS:
+        from .layers import DESIGNS
+
+        if c["architecture"].lower() not in DESIGNS:
             raise ValueError(f"unsupported architecture {c['architecture']!r}")
         return _layer_list_config(c, name or Path(path).name)
     arch = "mixtral" if "mixtral" in c.get("model_type", "") else "llama"

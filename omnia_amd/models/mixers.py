@@ -13,6 +13,7 @@ import torch.nn.functional as F
 
 from .. import ops
 from ..ops import mixers as mops
+from .layers import GQA_WIDTHS
 
 
 def _pad2(w: torch.Tensor, rows: int, cols: int) -> torch.Tensor:
@@ -83,8 +84,8 @@ class LatentAttention:
     def alloc(self, num_blocks: int, block_size: int, n_slots: int):
         # zeros: the padding columns of a row are never written, and a page's unwritten
         # rows stay finite under the masked tail of a tile
-        return torch.zeros(num_blocks, block_size, self.spec.padded_cache_width,
-                           dtype=self.model.dtype, device=self.model.device), None
+        return (torch.zeros(num_blocks, block_size, self.spec.padded_cache_width,
+                            dtype=self.model.dtype, device=self.model.device),), None
 
     def splits(self, rows: int, max_keys: int) -> int:
         """Parts each row's keys are cut into: enough workgroups to fill the chip."""
@@ -119,7 +120,7 @@ class LatentAttention:
 
     def forward(self, w: dict, h: torch.Tensor, fb, cache) -> torch.Tensor:
         s, m = self.spec, self.model
-        pages, _ = cache
+        (pages,), _ = cache
         x = m.project(h, w["in"], fb.is_decode)
         cq = mops.latent_prep(pages, x, w["q_norm"], w["kv_norm"], fb.positions, fb.slots,
                               self.table, s.q_rank_pad, s.latent_pad, m.cfg.rms_eps)
@@ -182,4 +183,86 @@ class GatedDelta:
         return y
 
 
-MIXERS = {"latent_attention": LatentAttention, "delta": GatedDelta}
+class GroupedQueryAttention:
+    """Windowed attention with sinks over pages of keys and values -- its own, or (spec
+    ``kv_from``) those of an earlier layer, whose cache entry it is handed."""
+
+    def __init__(self, spec, model):
+        self.spec, self.model = spec, model
+        self.table = model.rotary(spec.rotary)
+        self.mfma = (model.device.type == "cuda" and model.dtype == torch.bfloat16
+                     and spec.dim_pad in GQA_WIDTHS and spec.v_pad in GQA_WIDTHS)
+
+    def pack(self, get, d: int) -> dict:
+        s = self.spec
+        own = s.kv_from is None
+
+        def heads(n, count, dim, pad):
+            t = get(n).view(count, dim, -1)
+            return F.pad(t, (0, d - t.shape[2], 0, pad - dim)).reshape(count * pad, d)
+
+        def norm(n):
+            return F.pad(get(n).float(), (0, s.dim_pad - s.dim)).contiguous()
+
+        rows = [heads("q", s.heads, s.dim, s.dim_pad)]
+        if own:
+            rows += [heads("k", s.kv_heads, s.dim, s.dim_pad),
+                     heads("v", s.kv_heads, s.vdim, s.v_pad)]
+        w = {"in": _rows_to(rows, d), "q_norm": norm("q.norm"),
+             "o": _head_cols(get("o"), s.heads, s.v_pad, d),
+             "sink": get("sink").float().contiguous() if s.sink else None}
+        if own:
+            w["k_norm"] = norm("k.norm")
+        return w
+
+    def alloc(self, num_blocks: int, block_size: int, n_slots: int):
+        s, m = self.spec, self.model
+        # zeros: the null page that padded rows read stays finite
+        return tuple(torch.zeros(num_blocks, s.kv_heads, block_size, w, dtype=m.dtype,
+                                 device=m.device) for w in (s.dim_pad, s.v_pad)), None
+
+    # decode workgroups wanted before a row's keys are cut no further, and the fewest
+    # keys of a part
+    DECODE_GROUPS, MIN_PART, MAX_PART = 1024, 128, 1024
+
+    def splits(self, rows: int, max_keys: int) -> int:
+        s = self.spec
+        keys = min(max_keys, s.window) if s.window else max_keys
+        groups = rows * s.kv_heads * -(-(s.heads // s.kv_heads) // 8)
+        return max(1, -(-keys // self.MAX_PART),
+                   min(-(-self.DECODE_GROUPS // groups), -(-keys // self.MIN_PART)))
+
+    def _decode(self, w, q, pages, bt, positions, out):
+        page = pages[0].shape[2]
+        if self.mfma and page & (page - 1) == 0:
+            return mops.gqa_decode(q, pages, bt, positions, self.spec, w["sink"],
+                                   self.splits(q.shape[0], bt.shape[1] * page), out)
+        return mops.gqa_attend(q, pages, bt, None, positions, self.spec, w["sink"], out)
+
+    def _prefill(self, w, q, pages, fb, positions, out):
+        page = pages[0].shape[2]
+        if self.mfma and page & (page - 1) == 0:
+            return mops.gqa_prefill(q, pages, fb, self.spec, w["sink"], out)
+        return mops.gqa_attend(q, pages, fb.block_tables, fb.q_start_loc, positions, self.spec,
+                               w["sink"], out)
+
+    def forward(self, w: dict, h: torch.Tensor, fb, cache) -> torch.Tensor:
+        s, m = self.spec, self.model
+        pages, _ = cache
+        q = mops.gqa_prep(m._slabs("in", h, w["in"], fb.is_decode), w, s,
+                          pages if s.kv_from is None else None, fb.positions, fb.slots,
+                          self.table, m.dtype, m.cfg.rms_eps)
+        if fb.is_decode:
+            return self._decode(w, q, pages, fb.block_tables, fb.positions, None)
+        nd, T = fb.num_decode, h.shape[0]
+        if not nd:
+            return self._prefill(w, q, pages, fb, fb.positions, None)
+        out = torch.empty(T, s.heads * s.v_pad, dtype=h.dtype, device=h.device)
+        self._decode(w, q[:nd], pages, fb.dec_block_tables, fb.positions[:nd], out[:nd])
+        if T > nd:
+            self._prefill(w, q[nd:], pages, fb, fb.positions[nd:], out[nd:])
+        return out
+
+
+MIXERS = {"latent_attention": LatentAttention, "delta": GatedDelta,
+          "attention": GroupedQueryAttention}

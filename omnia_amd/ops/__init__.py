@@ -735,10 +735,11 @@ MOE_LIBRARY_ROWS = 1024  # mean rows/expert above which eager calls use hipBLASL
 MOE_TILE256_ROWS = int(os.environ.get("OMNIA_MOE_TILE256_ROWS", "512"))
 
 
-def _moe_grouped(x, w_gu, w_down, ids, wts, k, n_experts, e_lo, e_hi, bm):
+def _moe_grouped(x, w_gu, w_down, ids, wts, k, n_experts, e_lo, e_hi, bm, glu=None):
     """Grouped expert FFN over device-sorted assignments, no host sync: Y [T*k, d]
     (row t*k + j = slot j of token t, routing weight applied; other experts' rows
-    unwritten).  ``bm`` 256: the 256x256 MFMA prefill tile; 64: moe.hip."""
+    unwritten).  ``bm`` 256: the 256x256 MFMA prefill tile; 64: moe.hip.  ``glu`` =
+    (alpha, limit): clamped GLU experts whose INPUT takes the routing weight."""
     kk = kernels()
     n = ids.numel()
     mb = kk.moe_max_blocks(n, e_hi - e_lo, bm)
@@ -749,6 +750,10 @@ def _moe_grouped(x, w_gu, w_down, ids, wts, k, n_experts, e_lo, e_hi, bm):
     act = torch.empty(mb * bm, w_down.shape[2], dtype=x.dtype, device=x.device)
     Y = torch.empty(n, x.shape[1], dtype=x.dtype, device=x.device)
     gemm = kk.pgemm_moe if bm == 256 else kk.moe_gemm
+    if glu is not None:
+        gemm(2, act, x, w_gu, sorted_ids, blk, nblk, wts.view(-1), k, n, e_lo, *glu)
+        gemm(1, Y, act, w_down, sorted_ids, blk, nblk, None, k, n, e_lo)
+        return Y
     gemm(0, act, x, w_gu, sorted_ids, blk, nblk, None, k, n, e_lo)
     gemm(1, Y, act, w_down, sorted_ids, blk, nblk, wts.view(-1), k, n, e_lo)
     return Y

@@ -24,7 +24,8 @@ int omnia_pgemm_splitk(void* parts, const void* X, const void* W, int M, int N, 
                        int sched, hipStream_t s);
 int omnia_pgemm_moe(int mode, void* out, const void* A, const void* W, const int* sorted,
                     const int* blk_expert, const int* n_blocks, const float* route_w, int K,
-                    int N, int topk, int n_assign, int e_lo, int max_blocks, hipStream_t s);
+                    int N, int topk, int n_assign, int e_lo, int max_blocks, float alpha,
+                    float limit, hipStream_t s);
 int omnia_pgemm_variant(int variant, void* out, const void* X, const void* W, int M, int N,
                         int K, hipStream_t s);
 int omnia_rmsnorm(void* out, const void* x, void* residual, const void* w, int rows, int d,
@@ -80,9 +81,12 @@ int omnia_moe_router_topk(int* ids, float* wts, const void* x, const void* route
                           int d, int E, int k, int renorm, hipStream_t s);
 int omnia_moe_align(int* sorted, int* blk_expert, int* n_blocks, const int* ids, int n, int E,
                     int e_lo, int e_hi, int max_blocks, int bm, hipStream_t s);
-int omnia_moe_gemm(int mode, void* out, const void* A, const void* W, const int* sorted,
-                   const int* blk_expert, const int* n_blocks, const float* route_w, int K,
-                   int N, int topk, int n_assign, int e_lo, int max_blocks, hipStream_t s);
+int omnia_moe_route(int* ids, float* wts, const void* x, const void* router, int f32, int n_tok,
+                    int d, int E, int k, int sigmoid, int renorm, hipStream_t s);
+int omnia_moe_gemm(int mode, void* out, const void* A, const void* W, int f32, const int* sorted,
+                   const int* blk_expert, const int* n_blocks, const float* route_w, int K, int N,
+                   int topk, int n_assign, int e_lo, int max_blocks, float alpha, float limit,
+                   hipStream_t s);
 int omnia_moe_combine(void* out, const void* Y, const int* ids, int n_tok, int d, int topk,
                       int e_lo, int e_hi, hipStream_t s);
 int omnia_ipc_handle_size();
@@ -144,6 +148,31 @@ int omnia_delta_scan(float* o, float* state, void* conv_state, float* rec, const
 int omnia_delta_norm(void* y, const float* o, const void* x, int f32, int64_t ldx, int zoff,
                      const float* norm_w, int T, int H, int V, int Vs, int Vp, float eps,
                      hipStream_t s);
+int omnia_rms_embed(void* h, float* x, const int* ids, const void* table, int f32, int T, int d,
+                    int vocab, const float* we, const float* wp, float inv_n, float eps,
+                    const int64_t* src, const int* tok_slots, hipStream_t s);
+int omnia_rms_residual(void* h, int f32, float* x, const void* m, int ptype, int S,
+                       int64_t row_stride, int64_t part_stride, int rows, int d,
+                       const float* w_post, const float* w_pre, float inv_n, float eps,
+                       hipStream_t s);
+int omnia_softcap(void* z, int f32, int64_t n, float cap, hipStream_t s);
+int omnia_gqa_prep(void* q, void* kc, void* vc, int f32, const void* x, int ptype, int S,
+                   int64_t slab, int64_t ldx, const float* wq, const float* wk,
+                   const int* positions, const int64_t* slots, const float* cos_sin, int T, int H,
+                   int G, int D, int Dp, int Vp, int R, int page, float eps, hipStream_t s);
+int omnia_gqa_attend(void* out, int f32, const void* q, const void* kc, const void* vc,
+                     const int* block_tables, int bt_stride, const int* q_start, int nseq,
+                     const int* positions, int T, int page, int H, int G, int Dp, int Vp,
+                     int window, float scale, const float* sinks, hipStream_t s);
+int omnia_gqa_decode(void* out, float* part_o, float* part_ml, const void* q, const void* kc,
+                     const void* vc, const int* block_tables, int bt_stride, const int* positions,
+                     int T, int page, int H, int G, int Dp, int Vp, int window, float scale,
+                     const float* sinks, int splits, int max_keys, hipStream_t s);
+int omnia_gqa_prefill(void* out, const void* q, const void* kc, const void* vc,
+                      const int* block_tables, int bt_stride, const int* q_start,
+                      const int* seq_lens, const int* tile_seq, const int* tile_q0, int n_tiles,
+                      int page, int H, int G, int Dp, int Vp, int window, float scale,
+                      const float* sinks, hipStream_t s);
 int omnia_latent_prep(void* cq, void* cache, const void* x, int f32, int64_t ldx, const float* wq,
                       const float* wc, const int* positions, const int64_t* slots,
                       const float* cos_sin, int T, int Q, int Qp, int C, int Cp, int R, int Lp,
@@ -586,9 +615,12 @@ void moe_align(at::Tensor sorted, at::Tensor blk_expert, at::Tensor n_blocks, at
 // the 256x256-tile grouped MoE GEMMs (pgemm.hip EPI 5 / 6) over 256-row segments
 void pgemm_moe(int64_t mode, at::Tensor out, at::Tensor A, at::Tensor W, at::Tensor sorted,
                at::Tensor blk_expert, at::Tensor n_blocks, c10::optional<at::Tensor> route_w,
-               int64_t topk, int64_t n_assign, int64_t e_lo) {
+               int64_t topk, int64_t n_assign, int64_t e_lo, double alpha, double limit) {
   CHECK_GPU(A); CHECK_BF16(A); CHECK_BF16(W); CHECK_BF16(out);
   CHECK_I32(sorted); CHECK_I32(blk_expert); CHECK_I32(n_blocks);
+  if (route_w.has_value())
+    TORCH_CHECK(route_w->is_cuda() && route_w->is_contiguous() && route_w->numel() == n_assign &&
+                route_w->scalar_type() == at::kFloat, "route weights fp32 [T*k]");
   TORCH_CHECK(A.is_contiguous() && W.is_contiguous() && out.is_contiguous(), "contiguous");
   TORCH_CHECK(W.dim() == 3, "W [E_local, rows, K]");
   const int K = W.size(2);
@@ -596,7 +628,7 @@ void pgemm_moe(int64_t mode, at::Tensor out, at::Tensor A, at::Tensor W, at::Ten
   TORCH_CHECK(sorted.numel() == (int64_t)mb * 256, "sorted must hold max_blocks*256 rows");
   TORCH_CHECK(A.size(-1) == K && K % 128 == 0, "K mismatch / K % 128");
   int N;
-  if (mode == 0) {
+  if (mode != 1) {
     N = W.size(1) / 2;
     TORCH_CHECK(N % 128 == 0 && out.size(0) == (int64_t)mb * 256 && out.size(1) == N,
                 "act [max_blocks*256, I]");
@@ -605,26 +637,53 @@ void pgemm_moe(int64_t mode, at::Tensor out, at::Tensor A, at::Tensor W, at::Ten
     N = W.size(1);
     TORCH_CHECK(N % 256 == 0 && out.size(0) == n_assign && out.size(1) == N, "Y [T*k, d]");
     TORCH_CHECK(A.size(0) == (int64_t)mb * 256, "act rows");
-    TORCH_CHECK(route_w.has_value() && route_w->numel() == n_assign &&
-                route_w->scalar_type() == at::kFloat, "route weights");
   }
   CHECK_RC(omnia_pgemm_moe((int)mode, out.data_ptr(), A.data_ptr(), W.data_ptr(),
                            sorted.data_ptr<int>(), blk_expert.data_ptr<int>(),
                            n_blocks.data_ptr<int>(), opt_ptr<float>(route_w), K, N, topk,
-                           n_assign, e_lo, mb, cur_stream()), "pgemm_moe");
+                           n_assign, e_lo, mb, (float)alpha, (float)limit, cur_stream()),
+           "pgemm_moe");
 }
 
+// router: fp32 logits, sigmoid / softmax scores; x [T, d] and router [E, d] bf16 or fp32
+void moe_route(at::Tensor ids, at::Tensor wts, at::Tensor x, at::Tensor router, int64_t k,
+               bool sigmoid, bool renorm) {
+  CHECK_GPU(x); CHECK_I32(ids);
+  const bool f32 = x.scalar_type() == at::kFloat;
+  TORCH_CHECK((f32 || x.scalar_type() == at::kBFloat16) && router.scalar_type() == x.scalar_type(),
+              "x and router: bf16 or fp32");
+  TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && router.is_cuda() && router.dim() == 2 &&
+              router.is_contiguous() && router.size(1) == x.size(1) && x.size(1) % 8 == 0,
+              "x [T, d], router [E, d]");
+  const int T = x.size(0), E = router.size(0);
+  TORCH_CHECK(ids.numel() == (int64_t)T * k && wts.numel() == (int64_t)T * k && wts.is_cuda() &&
+              wts.scalar_type() == at::kFloat && ids.is_contiguous() && wts.is_contiguous(),
+              "ids/wts [T, k]");
+  CHECK_RC(omnia_moe_route(ids.data_ptr<int>(), wts.data_ptr<float>(), x.data_ptr(),
+                           router.data_ptr(), f32, T, x.size(1), E, k, sigmoid, renorm,
+                           cur_stream()), "moe_route");
+}
+
+// modes in moe.hip; A, W and out all bf16 or all fp32
 void moe_gemm(int64_t mode, at::Tensor out, at::Tensor A, at::Tensor W, at::Tensor sorted,
               at::Tensor blk_expert, at::Tensor n_blocks, c10::optional<at::Tensor> route_w,
-              int64_t topk, int64_t n_assign, int64_t e_lo) {
-  CHECK_GPU(A); CHECK_BF16(A); CHECK_BF16(W); CHECK_BF16(out);
+              int64_t topk, int64_t n_assign, int64_t e_lo, double alpha, double limit) {
+  CHECK_GPU(A); CHECK_GPU(W); CHECK_GPU(out);
+  const bool f32 = A.scalar_type() == at::kFloat;
+  TORCH_CHECK((f32 || A.scalar_type() == at::kBFloat16) && W.scalar_type() == A.scalar_type() &&
+              out.scalar_type() == A.scalar_type(), "A, W, out: bf16 or fp32");
+  CHECK_I32(sorted); CHECK_I32(blk_expert); CHECK_I32(n_blocks);
   TORCH_CHECK(A.is_contiguous() && W.is_contiguous() && out.is_contiguous(), "contiguous");
   TORCH_CHECK(W.dim() == 3, "W [E_local, rows, K]");
   const int K = W.size(2);
   const int mb = blk_expert.numel();
+  TORCH_CHECK(sorted.numel() == (int64_t)mb * 64, "sorted must hold max_blocks*64 rows");
   TORCH_CHECK(A.size(-1) == K && K % 64 == 0, "K mismatch / K % 64");
+  if (route_w.has_value())
+    TORCH_CHECK(route_w->is_cuda() && route_w->is_contiguous() && route_w->numel() == n_assign &&
+                route_w->scalar_type() == at::kFloat, "route weights fp32 [T*k]");
   int N;
-  if (mode == 0) {
+  if (mode != 1) {
     N = W.size(1) / 2;
     TORCH_CHECK(N % 32 == 0 && out.size(0) == (int64_t)mb * 64 && out.size(1) == N,
                 "act [max_blocks*64, I]");
@@ -633,12 +692,12 @@ void moe_gemm(int64_t mode, at::Tensor out, at::Tensor A, at::Tensor W, at::Tens
     N = W.size(1);
     TORCH_CHECK(N % 64 == 0 && out.size(0) == n_assign && out.size(1) == N, "Y [T*k, d]");
     TORCH_CHECK(A.size(0) == (int64_t)mb * 64, "act rows");
-    TORCH_CHECK(route_w.has_value() && route_w->numel() == n_assign, "route weights");
   }
-  CHECK_RC(omnia_moe_gemm((int)mode, out.data_ptr(), A.data_ptr(), W.data_ptr(),
+  CHECK_RC(omnia_moe_gemm((int)mode, out.data_ptr(), A.data_ptr(), W.data_ptr(), f32,
                           sorted.data_ptr<int>(), blk_expert.data_ptr<int>(),
                           n_blocks.data_ptr<int>(), opt_ptr<float>(route_w), K, N, topk,
-                          n_assign, e_lo, mb, cur_stream()), "moe_gemm");
+                          n_assign, e_lo, mb, (float)alpha, (float)limit, cur_stream()),
+           "moe_gemm");
 }
 
 void moe_combine(at::Tensor out, at::Tensor Y, at::Tensor ids, int64_t topk, int64_t e_lo,
@@ -1467,12 +1526,165 @@ void latent_prefill(at::Tensor out, at::Tensor q, at::Tensor kx, at::Tensor kr, 
                Tk, window, (float)scale, gate.data_ptr(), ldg, cur_stream()), "latent_prefill");
 }
 
+// ------------------------------------------- RMS norms around an fp32 residual stream
+const float* opt_vecf(const OptT& t, int64_t n, const char* what) {
+  return t.has_value() && t->defined() ? vecf(*t, n, what) : nullptr;
+}
+
+void rms_embed(at::Tensor h, at::Tensor x, at::Tensor ids, at::Tensor table, int64_t vocab,
+               OptT w_embed, OptT w_pre, double inv_n, double eps, OptT src, OptT tok_slots) {
+  const int f32 = is_f32(table, "table");
+  TORCH_CHECK(table.dim() == 2 && table.is_contiguous() && table.size(0) >= vocab, "table [V, d]");
+  const int64_t T = ids.numel(), d = table.size(1);
+  like(h, table, T * d, "h");
+  const int64_t* sp = nullptr;
+  if (src.has_value() && src->defined()) {
+    TORCH_CHECK(src->is_cuda() && src->scalar_type() == at::kLong && src->is_contiguous() &&
+                src->numel() == T && tok_slots.has_value(), "src int64 [T] with tok_slots");
+    CHECK_I32(*tok_slots);
+    sp = src->data_ptr<int64_t>();
+  }
+  CHECK_RC(omnia_rms_embed(h.data_ptr(), outf(x, T * d, "x"), veci(ids, T, "ids"),
+                           table.data_ptr(), f32, T, d, vocab, opt_vecf(w_embed, d, "w_embed"),
+                           opt_vecf(w_pre, d, "w_pre"), (float)inv_n, (float)eps, sp,
+                           opt_ptr<int>(tok_slots), cur_stream()), "rms_embed");
+}
+
+// m: projection [M, d], split-K slabs [S, M, d], or (slots) per-token parts [M, S, d]
+void rms_residual(at::Tensor h, at::Tensor x, at::Tensor m, bool slots, at::Tensor w_post,
+                  OptT w_pre, double inv_n, double eps) {
+  const int f32 = is_f32(h, "h");
+  const Proj p = proj(m);
+  const int64_t d = p.N, S = slots ? p.M : p.S, M = slots ? m.size(0) : p.M;
+  TORCH_CHECK(!slots || m.dim() == 3, "slots [M, S, d]");
+  like(h, h, M * d, "h");
+  CHECK_RC(omnia_rms_residual(h.data_ptr(), f32, outf(x, M * d, "x"), m.data_ptr(), p.type, S,
+                              slots ? S * d : d, slots ? d : M * d, M, d,
+                              vecf(w_post, d, "w_post"), opt_vecf(w_pre, d, "w_pre"),
+                              (float)inv_n, (float)eps, cur_stream()), "rms_residual");
+}
+
+void softcap(at::Tensor z, double cap) {
+  const int f32 = is_f32(z, "logits");
+  TORCH_CHECK(z.is_contiguous() && cap > 0, "contiguous logits, cap > 0");
+  CHECK_RC(omnia_softcap(z.data_ptr(), f32, z.numel(), (float)cap, cur_stream()), "softcap");
+}
+
+// ------------------------------------------------------------ grouped-query attention
+// k pages [NB, G, page, Dp], v pages [NB, G, page, Vp]
+void check_kv(const at::Tensor& k, const at::Tensor& v, const at::Tensor& ref) {
+  TORCH_CHECK(k.is_cuda() && k.dim() == 4 && k.is_contiguous() && v.is_cuda() && v.dim() == 4 &&
+              v.is_contiguous() && k.scalar_type() == ref.scalar_type() &&
+              v.scalar_type() == ref.scalar_type() && k.size(0) == v.size(0) &&
+              k.size(1) == v.size(1) && k.size(2) == v.size(2), "k / v pages [NB, G, page, width]");
+}
+
+// x: [T, (H*Dp | G*Dp | G*Vp) + padding] or its slabs; k / v pages absent: q only
+void gqa_prep(at::Tensor q, OptT k, OptT v, at::Tensor x, at::Tensor wq, OptT wk,
+              at::Tensor positions, at::Tensor slots, at::Tensor cos_sin, int64_t H, int64_t D,
+              double eps) {
+  const int f32 = is_f32(q, "q");
+  const Proj p = proj(x);
+  const int64_t T = positions.numel(), R = cos_sin.size(1), Dp = wq.numel();
+  const bool own = k.has_value() && k->defined();
+  int64_t G = 0, Vp = 0, page = 1;
+  if (own) {
+    TORCH_CHECK(v.has_value() && wk.has_value(), "k pages come with v pages and a k norm");
+    check_kv(*k, *v, q);
+    G = k->size(1);
+    page = k->size(2);
+    Vp = v->size(3);
+    TORCH_CHECK(k->size(3) == Dp, "k page width");
+  }
+  TORCH_CHECK(p.M == T && p.N >= H * Dp + G * (Dp + Vp), "projection row width");
+  like(q, q, T * H * Dp, "q");
+  TORCH_CHECK(slots.is_cuda() && slots.scalar_type() == at::kLong && slots.is_contiguous() &&
+              slots.numel() == T, "slots int64 [T]");
+  CHECK_RC(omnia_gqa_prep(q.data_ptr(), own ? k->data_ptr() : nullptr,
+                          own ? v->data_ptr() : nullptr, f32, x.data_ptr(), p.type, p.S,
+                          p.M * p.N, p.N, vecf(wq, Dp, "wq"),
+                          own ? vecf(*wk, Dp, "wk") : nullptr, veci(positions, T, "positions"),
+                          slots.data_ptr<int64_t>(), rot_table(cos_sin, R), T, H, G, D, Dp, Vp, R,
+                          page, (float)eps, cur_stream()), "gqa_prep");
+}
+
+struct KV { int64_t G, page, Dp, Vp; };
+KV kv_sizes(const at::Tensor& out, const at::Tensor& q, const at::Tensor& k, const at::Tensor& v,
+            int64_t T, int64_t H, const OptT& sinks) {
+  check_kv(k, v, q);
+  const KV s{k.size(1), k.size(2), k.size(3), v.size(3)};
+  TORCH_CHECK(H % s.G == 0, "query heads over key/value heads");
+  like(q, q, T * H * s.Dp, "q");
+  like(out, q, T * H * s.Vp, "out");
+  opt_vecf(sinks, H, "sinks");
+  return s;
+}
+
+void gqa_attend(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor block_tables,
+                OptT q_start, at::Tensor positions, int64_t H, int64_t window, double scale,
+                OptT sinks) {
+  const int f32 = is_f32(q, "q");
+  const int64_t T = positions.numel();
+  const KV s = kv_sizes(out, q, k, v, T, H, sinks);
+  const bool pre = q_start.has_value() && q_start->defined();
+  const int64_t nseq = pre ? q_start->numel() - 1 : T;
+  CHECK_RC(omnia_gqa_attend(out.data_ptr(), f32, q.data_ptr(), k.data_ptr(), v.data_ptr(),
+                            tables(block_tables, nseq), block_tables.stride(0),
+                            pre ? veci(*q_start, nseq + 1, "q_start") : nullptr, nseq,
+                            veci(positions, T, "positions"), T, s.page, H, s.G, s.Dp, s.Vp, window,
+                            (float)scale, opt_ptr<float>(sinks), cur_stream()), "gqa_attend");
+}
+
+void gqa_decode(at::Tensor out, OptT part_o, OptT part_ml, at::Tensor q, at::Tensor k,
+                at::Tensor v, at::Tensor block_tables, at::Tensor positions, int64_t H,
+                int64_t window, double scale, OptT sinks, int64_t splits) {
+  CHECK_GPU(q); CHECK_BF16(q);
+  const int64_t T = positions.numel();
+  const KV s = kv_sizes(out, q, k, v, T, H, sinks);
+  float *po = nullptr, *pm = nullptr;
+  if (splits > 1) {
+    TORCH_CHECK(part_o.has_value() && part_ml.has_value(), "partials for splits > 1");
+    po = outf(*part_o, T * H * splits * s.Vp, "part_o");
+    pm = outf(*part_ml, T * H * splits * 2, "part_ml");
+  }
+  // a row's context fits its block-table row, so no row sees more keys than this
+  int64_t keys = block_tables.size(1) * s.page;
+  if (window > 0 && window < keys) keys = window;
+  CHECK_RC(omnia_gqa_decode(out.data_ptr(), po, pm, q.data_ptr(), k.data_ptr(), v.data_ptr(),
+                            tables(block_tables, T), block_tables.stride(0),
+                            veci(positions, T, "positions"), T, s.page, H, s.G, s.Dp, s.Vp, window,
+                            (float)scale, opt_ptr<float>(sinks), splits, keys, cur_stream()),
+           "gqa_decode");
+}
+
+void gqa_prefill(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor block_tables,
+                 at::Tensor q_start, at::Tensor seq_lens, at::Tensor tile_seq, at::Tensor tile_q0,
+                 int64_t H, int64_t window, double scale, OptT sinks) {
+  CHECK_GPU(q); CHECK_BF16(q);
+  TORCH_CHECK(q.dim() == 2, "q [T, H*Dp]");
+  const KV s = kv_sizes(out, q, k, v, q.size(0), H, sinks);
+  const int64_t nseq = seq_lens.numel(), nt = tile_seq.numel();
+  CHECK_RC(omnia_gqa_prefill(out.data_ptr(), q.data_ptr(), k.data_ptr(), v.data_ptr(),
+                             tables(block_tables, nseq), block_tables.stride(0),
+                             veci(q_start, nseq + 1, "q_start"), veci(seq_lens, nseq, "seq_lens"),
+                             veci(tile_seq, nt, "tile_seq"), veci(tile_q0, nt, "tile_q0"), nt,
+                             s.page, H, s.G, s.Dp, s.Vp, window, (float)scale,
+                             opt_ptr<float>(sinks), cur_stream()), "gqa_prefill");
+}
+
 }  // namespace
 
 PYBIND11_MODULE(_omnia_kernels, m) {
   m.doc() = "omnia_amd hand-written CDNA4 (gfx950) HIP kernels";
   m.def("rmsnorm", &rmsnorm);
   m.def("tanh_norm_embed", &tanh_norm_embed);
+  m.def("rms_embed", &rms_embed);
+  m.def("rms_residual", &rms_residual);
+  m.def("softcap", &softcap);
+  m.def("gqa_prep", &gqa_prep);
+  m.def("gqa_attend", &gqa_attend);
+  m.def("gqa_decode", &gqa_decode);
+  m.def("gqa_prefill", &gqa_prefill);
   m.def("tanh_norm_residual", &tanh_norm_residual);
   m.def("bias_swiglu", &bias_swiglu);
   m.def("delta_prep", &delta_prep);
@@ -1510,9 +1722,16 @@ PYBIND11_MODULE(_omnia_kernels, m) {
   m.def("moe_router_topk", &moe_router_topk);
   m.def("moe_max_blocks", &moe_max_blocks, py::arg("n_assign"), py::arg("n_experts"),
         py::arg("bm") = 64);
-  m.def("pgemm_moe", &pgemm_moe);
+  m.def("pgemm_moe", &pgemm_moe, py::arg("mode"), py::arg("out"), py::arg("A"), py::arg("W"),
+        py::arg("sorted"), py::arg("blk_expert"), py::arg("n_blocks"), py::arg("route_w"),
+        py::arg("topk"), py::arg("n_assign"), py::arg("e_lo"), py::arg("alpha") = 0.0,
+        py::arg("limit") = 0.0);
+  m.def("moe_route", &moe_route);
   m.def("moe_align", &moe_align);
-  m.def("moe_gemm", &moe_gemm);
+  m.def("moe_gemm", &moe_gemm, py::arg("mode"), py::arg("out"), py::arg("A"), py::arg("W"),
+        py::arg("sorted"), py::arg("blk_expert"), py::arg("n_blocks"), py::arg("route_w"),
+        py::arg("topk"), py::arg("n_assign"), py::arg("e_lo"), py::arg("alpha") = 0.0,
+        py::arg("limit") = 0.0);
   m.def("moe_combine", &moe_combine);
   m.def("dgemm", &dgemm);
   m.def("wgemm", &wgemm);

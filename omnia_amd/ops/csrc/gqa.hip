@@ -1,0 +1,538 @@
+// Grouped-query attention with a sliding window, query/key norms and attention sinks
+// for gfx950: the paged form for any head widths (attention.hip is the 128-wide,
+// unlimited one).
+//
+//   k pages [num_pages][G][page][Dp], v pages [num_pages][G][page][Vp]
+//
+// Query head h reads key/value head h / (H / G).  A query at position i sees keys j with
+// 0 <= i - j < window (window 0: all); the softmax denominator of head h also holds
+// exp(sink[h]) (sinks null: none).  Scores, softmax and norms are fp32.
+//
+//   gqa_prep     one fused projection row [q (H*Dp) | k (G*Dp) | v (G*Vp)] (or its split-K
+//                slabs) -> per-head RMS norm of q and k, rotate-half rotary on the first R
+//                dimensions, q rows out, k / v rows into the pages.  G = 0: q only (a layer
+//                that attends to another layer's pages)
+//   gqa_attend   generic attention (any size, bf16 or fp32), decode and prefill
+//   gqa_decode   bf16 decode: Q K^T on MFMA, P V on the VALU, the visible keys cut into
+//                equal parts on the device, + gqa_merge
+//   gqa_prefill  bf16 prefill (gqa_prefill.hip)
+#include "common.h"
+
+using namespace omnia;
+
+namespace {
+
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef _Float16 half4v __attribute__((ext_vector_type(4)));
+
+constexpr float kLog2e = 1.4426950408889634f;
+
+__device__ __forceinline__ float4v mfma16(short8 a, short8 b, float4v c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a),
+                                                 __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
+}
+
+template <typename P>
+__device__ __forceinline__ float4v load4(const P* p) {
+  if constexpr (sizeof(P) == 4) {
+    return *reinterpret_cast<const float4v*>(p);
+  } else if constexpr (__is_same(P, _Float16)) {
+    const half4v h = *reinterpret_cast<const half4v*>(p);
+    return float4v{(float)h[0], (float)h[1], (float)h[2], (float)h[3]};
+  } else {
+    const short4v h = *reinterpret_cast<const short4v*>(p);
+    return float4v{bf2f((uint16_t)h[0]), bf2f((uint16_t)h[1]), bf2f((uint16_t)h[2]),
+                   bf2f((uint16_t)h[3])};
+  }
+}
+__device__ __forceinline__ void store4(float* p, float4v v) { *reinterpret_cast<float4v*>(p) = v; }
+__device__ __forceinline__ void store4(bf16_t* p, float4v v) {
+  uint2v k;
+  k[0] = pack_bf2(v[0], v[1]);
+  k[1] = pack_bf2(v[2], v[3]);
+  *reinterpret_cast<uint2v*>(p) = k;
+}
+
+__device__ __forceinline__ int find_seq(const int* q_start, int nseq, int t) {
+  int lo = 0, hi = nseq - 1;
+  while (lo < hi) {
+    const int mid = (lo + hi + 1) >> 1;
+    if (q_start[mid] <= t) lo = mid; else hi = mid - 1;
+  }
+  return lo;
+}
+
+// ------------------------------------------------------------------- gqa_prep
+// 1 << lg lanes own one head row of one token, 4 columns a lane and step (NC steps).
+struct PrepArgs {
+  const float* wq;
+  const float* wk;       // per-dimension norm weights [Dp]
+  const int* positions;
+  const int64_t* slots;  // < 0: no write (padded row)
+  const float* cos_sin;  // [positions][R] = (cos[R/2] | sin[R/2])
+  int64_t ldx, slab;
+  int S, T, H, G, D, Dp, Vp, R, page, lg;
+  float eps;
+};
+
+template <typename T, typename P, int NC>
+__global__ __launch_bounds__(256) void prep_kernel(T* __restrict__ q, T* __restrict__ kc,
+                                                   T* __restrict__ vc, const P* __restrict__ x,
+                                                   PrepArgs a) {
+  __shared__ __attribute__((aligned(16))) float rows[256 * NC * 4];
+  const int lph = 1 << a.lg, l = threadIdx.x & (lph - 1);
+  const int NH = a.H + 2 * a.G;
+  const int64_t job = ((int64_t)blockIdx.x * 256 + threadIdx.x) >> a.lg;
+  const bool live = job < (int64_t)a.T * NH;
+  const int t = live ? (int)(job / NH) : 0, hs = live ? (int)(job % NH) : 0;
+  const bool isq = hs < a.H, isv = hs >= a.H + a.G;
+  const int width = isv ? a.Vp : a.Dp;
+  const int col = isv ? (a.H + a.G) * a.Dp + (hs - a.H - a.G) * a.Vp : hs * a.Dp;
+  const P* xr = x + (int64_t)t * a.ldx + col;
+  float4v v[NC];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NC; ++i) {
+    const int c = (l + (i << a.lg)) * 4;
+    v[i] = float4v{0.f, 0.f, 0.f, 0.f};
+    if (c < width) {
+      v[i] = load4(xr + c);
+      for (int s = 1; s < a.S; ++s) v[i] += load4(xr + s * a.slab + c);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) ss += v[i][j] * v[i][j];
+    }
+  }
+  float* row = rows + (threadIdx.x >> a.lg << a.lg) * NC * 4;
+  if (!isv) {
+    for (int o = lph >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+    const float r = 1.f / sqrtf(ss / (float)a.D + a.eps);
+    const float* w = isq ? a.wq : a.wk;
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+      const int c = (l + (i << a.lg)) * 4;
+      if (c < width) {
+        v[i] = v[i] * r * *reinterpret_cast<const float4v*>(w + c);
+        store4(row + c, v[i]);
+      }
+    }
+  }
+  __syncthreads();
+  if (!live) return;
+  T* dst;
+  if (isq) {
+    dst = q + ((int64_t)t * a.H + hs) * a.Dp;
+  } else {
+    const int64_t slot = a.slots[t];
+    if (slot < 0) return;
+    const int64_t blk = slot / a.page, off = slot - blk * a.page;
+    const int g = isv ? hs - a.H - a.G : hs - a.H;
+    dst = (isv ? vc : kc) + ((blk * a.G + g) * a.page + off) * width;
+  }
+  const float* cs = a.cos_sin + (int64_t)a.positions[t] * a.R;
+  const int half = a.R >> 1, turned = isv ? 0 : a.R;
+#pragma unroll
+  for (int i = 0; i < NC; ++i) {
+    const int c = (l + (i << a.lg)) * 4;
+    if (c >= width) continue;
+    float4v y = v[i];
+    if (c < turned) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int e = c + j;
+        if (e < turned) {
+          const bool first = e < half;
+          const int p = first ? e : e - half;
+          const float other = row[first ? e + half : p];
+          y[j] = v[i][j] * cs[p] + (first ? -other : other) * cs[half + p];
+        }
+      }
+    }
+    store4(dst + c, y);
+  }
+}
+
+// ----------------------------------------------------------------- gqa_attend
+// grid (T, H), 256 threads.  Tiles of 256 keys: a thread scores one key, then owns value
+// columns.  The sink is the first term of the online softmax.
+template <typename T>
+__global__ __launch_bounds__(256) void attend_kernel(
+    T* __restrict__ out, const T* __restrict__ q, const T* __restrict__ kc,
+    const T* __restrict__ vc, const int* __restrict__ block_tables, int bt_stride,
+    const int* __restrict__ q_start, int nseq, const int* __restrict__ positions, int page, int H,
+    int G, int Dp, int Vp, int window, float scale, const float* __restrict__ sinks) {
+  extern __shared__ float sm[];
+  float* qs = sm;        // [Dp]
+  float* acc = qs + Dp;  // [Vp]
+  float* p = acc + Vp;   // [256]
+  float* scratch = p + 256;  // [8]
+  const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, g = h / (H / G);
+  const int s = q_start ? find_seq(q_start, nseq, t) : t;
+  const int* bt = block_tables + (int64_t)s * bt_stride;
+  const int pos = positions[t];
+  const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+  const T* qr = q + ((int64_t)t * H + h) * Dp;
+  for (int i = tid; i < Dp; i += 256) qs[i] = ldf(qr + i);
+  for (int i = tid; i < Vp; i += 256) acc[i] = 0.f;
+  auto at = [&](int key) {  // row index of a key in the pages
+    return ((int64_t)bt[key / page] * G + g) * page + key % page;
+  };
+  float m = sinks ? sinks[h] : -INFINITY, l = sinks ? 1.f : 0.f;
+  for (int k0 = lo; k0 <= pos; k0 += 256) {
+    const int n = min(256, pos + 1 - k0);
+    __syncthreads();
+    float sc = -INFINITY;
+    if (tid < n) {
+      const T* row = kc + at(k0 + tid) * Dp;
+      float a = 0.f;
+      for (int i = 0; i < Dp; ++i) a += qs[i] * ldf(row + i);
+      sc = a * scale;
+    }
+    const float mn = fmaxf(m, block_max(sc, scratch));
+    const float e = tid < n ? expf(sc - mn) : 0.f;
+    p[tid] = e;
+    const float alpha = expf(m - mn);
+    l = l * alpha + block_sum(e, scratch);
+    m = mn;
+    __syncthreads();
+    for (int c = tid; c < Vp; c += 256) {
+      float a = acc[c] * alpha;
+      for (int j = 0; j < n; ++j) a += p[j] * ldf(vc + at(k0 + j) * Vp + c);
+      acc[c] = a;
+    }
+  }
+  for (int c = tid; c < Vp; c += 256) stf(out + ((int64_t)t * H + h) * Vp + c, acc[c] / l);
+}
+
+// ----------------------------------------------------------------- gqa_decode
+// The visible keys of a row, [lo, pos], in parts of part_len keys: decided on the device
+// from the live length, so one captured graph splits every context evenly.
+constexpr int MIN_PART = 64;
+
+__device__ __forceinline__ int part_len(int n, int splits) {
+  return max(((n + splits - 1) / splits + 15) / 16 * 16, MIN_PART);
+}
+
+// grid (rows, G * head chunks, splits), NW waves.  KK = Dp / 32; LPR lanes own a value
+// row (8 columns each); GH query heads of one key/value head per workgroup (a head past
+// the group's end recomputes the last one and is not written).
+//   1 scores   each wave takes groups of 16 keys: K rows as the MFMA A operand, Q^T
+//              (16 columns, GH real) as B; UG groups of loads in flight
+//   2 softmax  per head over the part, in LDS
+//   3 P V      64 / LPR value rows a wave and step, U steps of loads in flight
+template <int KK, int LPR, int GH, int NW>
+__global__ __launch_bounds__(64 * NW) void decode_kernel(
+    bf16_t* __restrict__ out, float* __restrict__ part_o, float* __restrict__ part_ml,
+    const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
+    const int* __restrict__ block_tables, int bt_stride, const int* __restrict__ positions, int H,
+    int G, int nch, int page_lg, int Vp, int window, float scale_log2,
+    const float* __restrict__ sinks, int cap) {
+  constexpr int Dp = 32 * KK, UG = KK > 4 ? 2 : 4, U = 4, TG = 64 / LPR;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  float* stat = reinterpret_cast<float*>(smem);  // [2 * GH], padded to 16
+  float* scores = stat + 16;                     // [GH][cap]
+  float* red = scores;                           // [NW][GH][Vp]: after the last scores read
+  int* pages = reinterpret_cast<int*>(scores + max(GH * cap, NW * GH * Vp));
+  const int b = blockIdx.x, g = blockIdx.y / nch, ch0 = blockIdx.y % nch, part = blockIdx.z;
+  const int group = H / G, h0 = g * group + ch0 * GH, hn = min(GH, group - ch0 * GH);
+  const int pos = positions[b];
+  const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+  const int vis = pos + 1 - lo, splits = gridDim.z;
+  const int pl = part_len(vis, splits);
+  const int p0 = lo + part * pl;
+  if (p0 > pos) return;
+  const int n = min(pl, pos + 1 - p0), nparts = (vis + pl - 1) / pl;
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, pmask = (1 << page_lg) - 1;
+  const int pg0 = p0 >> page_lg, npg = ((p0 + n - 1) >> page_lg) - pg0 + 1;
+  for (int i = tid; i < npg; i += 64 * NW)
+    pages[i] = block_tables[(int64_t)b * bt_stride + pg0 + i];
+
+  short8 qf[KK];
+  {
+    const int c = lane & 15;
+    const bf16_t* qrow = q + ((int64_t)b * H + h0 + min(c, hn - 1)) * Dp + 8 * (lane >> 4);
+#pragma unroll
+    for (int kk = 0; kk < KK; ++kk) qf[kk] = *reinterpret_cast<const short8*>(qrow + 32 * kk);
+  }
+  __syncthreads();
+  auto at = [&](int i) {  // row of the part's i-th key
+    const int key = p0 + i;
+    return (((int64_t)pages[(key >> page_lg) - pg0] * G + g) << page_lg) + (key & pmask);
+  };
+  const int ngroups = (n + 15) / 16;
+  for (int grp0 = w; grp0 < ngroups; grp0 += NW * UG) {
+    short8 a[UG][KK];
+#pragma unroll
+    for (int u = 0; u < UG; ++u) {  // groups past the end re-read the last key
+      const bf16_t* row = kc + at(min((grp0 + NW * u) * 16 + (lane & 15), n - 1)) * Dp +
+                          8 * (lane >> 4);
+#pragma unroll
+      for (int kk = 0; kk < KK; ++kk) a[u][kk] = *reinterpret_cast<const short8*>(row + 32 * kk);
+    }
+#pragma unroll
+    for (int u = 0; u < UG; ++u) {
+      const int grp = grp0 + NW * u;
+      if (grp >= ngroups) break;
+      float4v acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kk = 0; kk < KK; ++kk) acc = mfma16(a[u][kk], qf[kk], acc);
+      const int c = lane & 15;  // acc[r]: key grp*16 + 4*(lane>>4) + r, head c
+      if (c < GH) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int i = grp * 16 + 4 * (lane >> 4) + r;
+          if (i < n) scores[c * cap + i] = acc[r] * scale_log2;
+        }
+      }
+    }
+  }
+  // first value rows in flight across the softmax
+  const int tg = lane / LPR, vch = lane % LPR;
+  const bool vlive = vch * 8 < Vp;
+  short8 vv[U];
+  auto vload = [&](int base) {
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (vlive)
+        vv[u] = *reinterpret_cast<const short8*>(
+            vc + at(min(base + u * TG * NW + tg, n - 1)) * Vp + vch * 8);
+  };
+#pragma unroll
+  for (int u = 0; u < U; ++u) vv[u] = short8{0, 0, 0, 0, 0, 0, 0, 0};
+  vload(w * TG);
+  __syncthreads();
+  for (int c = w; c < GH; c += NW) {
+    float m = -INFINITY;
+    for (int i = lane; i < n; i += 64) m = fmaxf(m, scores[c * cap + i]);
+    m = wave_max(m);
+    float s = 0.f;
+    for (int i = lane; i < n; i += 64) {
+      const float p = exp2f(scores[c * cap + i] - m);
+      scores[c * cap + i] = p;
+      s += p;
+    }
+    s = wave_sum(s);
+    if (lane == 0) {
+      stat[2 * c] = m;
+      stat[2 * c + 1] = s;
+    }
+  }
+  __syncthreads();
+  float acc[GH][8];
+#pragma unroll
+  for (int c = 0; c < GH; ++c)
+#pragma unroll
+    for (int j = 0; j < 8; ++j) acc[c][j] = 0.f;
+  for (int base = w * TG; base < n; base += TG * NW * U) {
+    short8 cur[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) cur[u] = vv[u];
+    vload(base + TG * NW * U);
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int i = base + u * TG * NW + tg;
+      if (i < n) {
+#pragma unroll
+        for (int c = 0; c < GH; ++c) {
+          const float p = scores[c * cap + i];
+#pragma unroll
+          for (int j = 0; j < 8; ++j) acc[c][j] += p * bf2f((uint16_t)cur[u][j]);
+        }
+      }
+    }
+  }
+#pragma unroll
+  for (int c = 0; c < GH; ++c)
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      float v = acc[c][j];
+#pragma unroll
+      for (int o = LPR; o < 64; o <<= 1) v += __shfl_xor(v, o, 64);
+      acc[c][j] = v;
+    }
+  __syncthreads();  // every wave is done with `scores`, which `red` overlays
+  if (tg == 0 && vlive) {
+#pragma unroll
+    for (int c = 0; c < GH; ++c)
+#pragma unroll
+      for (int j = 0; j < 8; ++j) red[(w * GH + c) * Vp + vch * 8 + j] = acc[c][j];
+  }
+  __syncthreads();
+  for (int i = tid; i < hn * Vp; i += 64 * NW) {
+    const int c = i / Vp, d = i - c * Vp, h = h0 + c;
+    float v = 0.f;
+#pragma unroll
+    for (int k = 0; k < NW; ++k) v += red[(k * GH + c) * Vp + d];
+    const float m = stat[2 * c], s = stat[2 * c + 1];
+    if (nparts == 1) {
+      if (sinks) {
+        const float sk = sinks[h] * kLog2e, mm = fmaxf(m, sk), e = exp2f(m - mm);
+        v = v * e / (s * e + exp2f(sk - mm));
+      } else {
+        v = v / s;
+      }
+      out[((int64_t)b * H + h) * Vp + d] = f2bf(v);
+    } else {
+      const int64_t slot = ((int64_t)b * H + h) * splits + part;
+      part_o[slot * Vp + d] = v;
+      if (d == 0) {
+        part_ml[slot * 2] = m;
+        part_ml[slot * 2 + 1] = s;
+      }
+    }
+  }
+}
+
+// grid (rows * H), 128 threads
+__global__ __launch_bounds__(128) void merge_kernel(bf16_t* __restrict__ out,
+                                                    const float* __restrict__ part_o,
+                                                    const float* __restrict__ part_ml,
+                                                    const int* __restrict__ positions, int H,
+                                                    int Vp, int window, int splits,
+                                                    const float* __restrict__ sinks) {
+  const int bh = blockIdx.x, b = bh / H, h = bh - b * H;
+  const int pos = positions[b];
+  const int vis = pos + 1 - (window > 0 ? max(0, pos - window + 1) : 0);
+  const int pl = part_len(vis, splits), nparts = (vis + pl - 1) / pl;
+  if (nparts <= 1) return;
+  const float* ml = part_ml + (int64_t)bh * splits * 2;
+  const float* po = part_o + (int64_t)bh * splits * Vp;
+  const float sk = sinks ? sinks[h] * kLog2e : -INFINITY;
+  float m = sk;
+  for (int p = 0; p < nparts; ++p) m = fmaxf(m, ml[2 * p]);
+  float tot = sinks ? exp2f(sk - m) : 0.f;
+  for (int p = 0; p < nparts; ++p) tot += exp2f(ml[2 * p] - m) * ml[2 * p + 1];
+  const float inv = 1.f / tot;
+  for (int d = threadIdx.x; d < Vp; d += 128) {
+    float v = 0.f;
+    for (int p = 0; p < nparts; ++p) v += exp2f(ml[2 * p] - m) * po[(int64_t)p * Vp + d];
+    out[(int64_t)bh * Vp + d] = f2bf(v * inv);
+  }
+}
+
+int log2i(int n) {
+  for (int i = 0; i < 31; ++i)
+    if (n == (1 << i)) return i;
+  return -1;
+}
+
+}  // namespace
+
+extern "C" {
+
+// ptype: storage of x -- 0 bf16, 1 fp32, 2 fp16 (slabs)
+int omnia_gqa_prep(void* q, void* kc, void* vc, int f32, const void* x, int ptype, int S,
+                   int64_t slab, int64_t ldx, const float* wq, const float* wk,
+                   const int* positions, const int64_t* slots, const float* cos_sin, int T, int H,
+                   int G, int D, int Dp, int Vp, int R, int page, float eps, hipStream_t s) {
+  if (Dp % 4 || Vp % 4 || ldx % 4 || slab % 4 || S < 1 || R % 2 || R > D || D > Dp || page < 1)
+    return -1;
+  const int w = Dp > Vp || G == 0 ? Dp : Vp;
+  if (w > 1024) return -2;
+  if (T == 0) return 0;
+  int lg = 1;
+  while (lg < 6 && (4 << lg) < w) ++lg;
+  const int64_t threads = ((int64_t)T * (H + 2 * G)) << lg;
+  PrepArgs a{wq, wk, positions, slots, cos_sin, ldx, slab, S,  T,  H,  G,
+             D,  Dp, Vp,        R,     page,    lg,  eps};
+  const dim3 grid((unsigned)((threads + 255) / 256));
+#define OMNIA_GP(TT, PP)                                                                       \
+  do {                                                                                         \
+    if (w <= 256)                                                                              \
+      prep_kernel<TT, PP, 1><<<grid, 256, 0, s>>>((TT*)q, (TT*)kc, (TT*)vc, (const PP*)x, a);  \
+    else                                                                                       \
+      prep_kernel<TT, PP, 4><<<grid, 256, 0, s>>>((TT*)q, (TT*)kc, (TT*)vc, (const PP*)x, a);  \
+  } while (0)
+  if (f32) {
+    if (ptype != 1) return -3;
+    OMNIA_GP(float, float);
+  } else if (ptype == 0) {
+    OMNIA_GP(bf16_t, bf16_t);
+  } else if (ptype == 1) {
+    OMNIA_GP(bf16_t, float);
+  } else {
+    OMNIA_GP(bf16_t, _Float16);
+  }
+#undef OMNIA_GP
+  return (int)hipGetLastError();
+}
+
+int omnia_gqa_attend(void* out, int f32, const void* q, const void* kc, const void* vc,
+                     const int* block_tables, int bt_stride, const int* q_start, int nseq,
+                     const int* positions, int T, int page, int H, int G, int Dp, int Vp,
+                     int window, float scale, const float* sinks, hipStream_t s) {
+  if (G < 1 || H % G || page < 1 || window < 0) return -1;
+  if (T == 0) return 0;
+  const size_t lds = (size_t)(Dp + Vp + 256 + 8) * 4;
+  if (lds > 64 * 1024 || H > 65535) return -2;
+  const dim3 grid(T, H);
+  if (f32)
+    attend_kernel<float><<<grid, 256, lds, s>>>((float*)out, (const float*)q, (const float*)kc,
+                                                (const float*)vc, block_tables, bt_stride, q_start,
+                                                nseq, positions, page, H, G, Dp, Vp, window, scale,
+                                                sinks);
+  else
+    attend_kernel<bf16_t><<<grid, 256, lds, s>>>(
+        (bf16_t*)out, (const bf16_t*)q, (const bf16_t*)kc, (const bf16_t*)vc, block_tables,
+        bt_stride, q_start, nseq, positions, page, H, G, Dp, Vp, window, scale, sinks);
+  return (int)hipGetLastError();
+}
+
+// max_keys: no row sees more keys than this (sizes the score tile)
+int omnia_gqa_decode(void* out, float* part_o, float* part_ml, const void* q, const void* kc,
+                     const void* vc, const int* block_tables, int bt_stride, const int* positions,
+                     int T, int page, int H, int G, int Dp, int Vp, int window, float scale,
+                     const float* sinks, int splits, int max_keys, hipStream_t s) {
+  const int lg = log2i(page);
+  if (lg < 0 || G < 1 || H % G || Dp % 32 || Dp > 256 || Vp % 8 || Vp > 256 || splits < 1 ||
+      max_keys < 1 || window < 0 || H > 65535 || splits > 65535)
+    return -1;
+  if (T == 0) return 0;
+  const int group = H / G, gh = group >= 5 ? 8 : group >= 3 ? 4 : group;
+  const int nch = (group + gh - 1) / gh;
+  int cap = ((max_keys + splits - 1) / splits + 15) / 16 * 16;
+  cap = cap < MIN_PART ? MIN_PART : cap;
+  // two-wave workgroups once there are enough of them to keep the chip's loads in flight
+  const int nw = (int64_t)T * G * nch * splits >= 1024 ? 2 : 4;
+  const int tile = gh * cap > nw * gh * Vp ? gh * cap : nw * gh * Vp;
+  const size_t lds = 64 + (size_t)tile * 4 + (size_t)(cap / page + 2) * 4;
+  if (lds > 96 * 1024) return -2;
+  const dim3 grid(T, G * nch, splits);
+#define OMNIA_GD(KK, LP, GH, NN)                                                               \
+  decode_kernel<KK, LP, GH, NN><<<grid, 64 * NN, lds, s>>>(                                    \
+      (bf16_t*)out, part_o, part_ml, (const bf16_t*)q, (const bf16_t*)kc, (const bf16_t*)vc,   \
+      block_tables, bt_stride, positions, H, G, nch, lg, Vp, window, scale * kLog2e, sinks, cap)
+#define OMNIA_GD_N(KK, LP, GH) \
+  do { if (nw == 2) OMNIA_GD(KK, LP, GH, 2); else OMNIA_GD(KK, LP, GH, 4); } while (0)
+#define OMNIA_GD_G(KK, LP)                      \
+  do {                                          \
+    if (gh == 1) OMNIA_GD_N(KK, LP, 1);         \
+    else if (gh == 2) OMNIA_GD_N(KK, LP, 2);    \
+    else if (gh == 4) OMNIA_GD_N(KK, LP, 4);    \
+    else OMNIA_GD_N(KK, LP, 8);                 \
+  } while (0)
+#define OMNIA_GD_K(KK)                          \
+  case KK:                                      \
+    if (Vp <= 64) OMNIA_GD_G(KK, 8);            \
+    else if (Vp <= 128) OMNIA_GD_G(KK, 16);     \
+    else OMNIA_GD_G(KK, 32);                    \
+    break
+  switch (Dp / 32) {
+    OMNIA_GD_K(1);
+    OMNIA_GD_K(2);
+    OMNIA_GD_K(3);
+    OMNIA_GD_K(4);
+    OMNIA_GD_K(6);
+    OMNIA_GD_K(8);
+    default: return -3;
+  }
+#undef OMNIA_GD_K
+#undef OMNIA_GD_G
+#undef OMNIA_GD_N
+#undef OMNIA_GD
+  if (splits > 1)
+    merge_kernel<<<T * H, 128, 0, s>>>((bf16_t*)out, part_o, part_ml, positions, H, Vp, window,
+                                       splits, sinks);
+  return (int)hipGetLastError();
+}
+
+}  // extern "C"

@@ -1,0 +1,274 @@
+// Prefill of grouped-query attention with a sliding window and attention sinks on MFMA
+// (layouts and semantics in gqa.hip; 128-row query tiles from the runner's tile list).
+//
+// Workgroup: 4 waves = HB query heads of one key/value head x RW = 4 / HB groups of 32
+// query rows, so every 64-key K / V tile staged in LDS feeds 4 waves whatever the group
+// size.  A wave is 32 rows of one head:
+//   S^T = K Q^T      lane (row l & 31, hi = l >> 5) holds 32 of its row's 64 scores
+//   O^T += V^T P^T   the lane's own scores are the B operand; V^T fragments by
+//                    ds_read_b64_tr_b16 from the row-major tile, the keys of a k-step
+//                    permuted the same way on both sides
+// Tiles go global -> LDS by LDS-DMA, two stages, one barrier a tile; tiles before the
+// block's window are not visited, tiles outside a wave's own window not computed.  The
+// sink is the initial term of the online softmax (maximum = sink, sum = 1).
+#include <type_traits>
+
+#include "common.h"
+
+using namespace omnia;
+
+namespace {
+
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+
+__device__ __forceinline__ float16v mfma32(short8 a, short8 b, float16v c) {
+  return __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, a),
+                                                 __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
+}
+
+// chunk XOR of row `row` in a [64][W] bf16 image: 16 consecutive rows, read at one
+// column, fall on 16 different 16-B slots of the banks.  What the row stride does not
+// spread by itself (W 128-multiples: nothing, 64: two rows, 32: four), the XOR does.
+template <int W>
+__device__ __forceinline__ int swz(int row) {
+  constexpr int top = W % 128 == 0 ? 3 : W % 64 == 0 ? 2 : 0;
+  const int a = top == 3 ? row & 3 : top == 2 ? (row >> 1) & 1 : 0;
+  return (a << 2) | ((row >> 2) & 3);
+}
+// byte offset of 16-B chunk ch of a row
+template <int W>
+__device__ __forceinline__ int img(int row, int ch) {
+  return row * (2 * W) + 16 * (ch ^ swz<W>(row));
+}
+
+struct Args {
+  bf16_t* out;        // [T, H, DV]
+  const bf16_t* q;    // [T, H, DK]
+  const bf16_t* kc;
+  const bf16_t* vc;
+  const int* block_tables;
+  const int* q_start;
+  const int* seq_lens;
+  const int* tile_seq;
+  const int* tile_q0;
+  const float* sinks;  // [H] or null
+  int bt_stride, n_tiles, H, G, hb_lg, page_lg, window;
+  float scale_log2;
+};
+
+template <int DK, int DV>
+__global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Args p) {
+  // two K | V stages as separate objects: reads of one cannot alias the DMA into the other
+  __shared__ __attribute__((aligned(16))) char st0[128 * (DK + DV)];
+  __shared__ __attribute__((aligned(16))) char st1[128 * (DK + DV)];
+  constexpr int kMaxPages = 1024;  // pages of the visible range staged in LDS
+  __shared__ int pg_lds[kMaxPages];
+
+  const int HB = 1 << p.hb_lg, group = p.H / p.G;
+  // blocks of one key/value head are neighbours: (head block, tile, sub-tile)
+  const int id = xcd_remap(blockIdx.x, gridDim.x);
+  const int sub = id & (HB - 1), rest = id >> p.hb_lg;
+  const int hblk = rest / p.n_tiles, tile = rest - hblk * p.n_tiles;
+  const int s = p.tile_seq[tile];
+  const int qs = p.q_start[s], qlen = p.q_start[s + 1] - qs;
+  const int rows = 128 >> p.hb_lg;  // of this block: the tile has HB sub-tiles
+  const int b0 = p.tile_q0[tile] + sub * rows;
+  if (b0 >= qlen) return;
+  const int off = p.seq_lens[s] - qlen;  // position of the portion's first row
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, ql = lane & 31, hi = lane >> 5;
+  const int h = hblk * HB + (w & (HB - 1)), kvh = hblk * HB / group;
+  const int* bt = p.block_tables + (int64_t)s * p.bt_stride;
+  const int BS = 1 << p.page_lg, pmask = BS - 1;
+
+  const int q0 = b0 + 32 * (w >> p.hb_lg);  // this wave's first row
+  const int qr = q0 + ql;
+  const bool row_ok = qr < qlen;
+  const int qr_c = min(qr, qlen - 1), qpos = off + qr_c;
+  const int wmin = off + min(q0, qlen - 1), wmax = off + min(q0 + 31, qlen - 1);
+  short8 qf[DK / 16];
+  {
+    const bf16_t* qrow = p.q + ((int64_t)(qs + qr_c) * p.H + h) * DK + 8 * hi;
+#pragma unroll
+    for (int ks = 0; ks < DK / 16; ++ks) qf[ks] = *reinterpret_cast<const short8*>(qrow + 16 * ks);
+  }
+  const int win = p.window > 0 ? p.window : 1 << 30;
+  const int kv_end = off + min(b0 + rows, qlen);
+  const int t0 = max(0, off + b0 - win + 1) >> 6, t1 = (kv_end + 63) >> 6;
+  const int pg0 = (t0 << 6) >> p.page_lg;  // first staged page
+  const int npg = min(((kv_end - 1) >> p.page_lg) - pg0 + 1, kMaxPages);
+  for (int i = tid; i < npg; i += 256) pg_lds[i] = bt[pg0 + i];
+  __syncthreads();
+
+  typedef __attribute__((address_space(3))) void* lds_ptr_t;
+  // one tensor's tile: instruction i of wave w fills 64 consecutive 16-B slots; the image's
+  // XOR is applied to the source chunk.  Keys past the end re-read the last one (masked).
+  auto dma1 = [&](int t, auto WC, const bf16_t* src, char* dst) {
+    constexpr int W = decltype(WC)::value, CPR = W / 8, N = W / 32;
+    int64_t at[N];
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      const int c = (w * N + i) * 64 + lane, row = c / CPR;
+      const int key = min(t * 64 + row, kv_end - 1);
+      const int pi = (key >> p.page_lg) - pg0;
+      const int pl = pg_lds[pi < kMaxPages ? pi : 0];
+      const int page = pi < kMaxPages ? pl : bt[pg0 + pi];
+      at[i] = ((((int64_t)page * p.G + kvh) << p.page_lg) + (key & pmask)) * W +
+              8 * ((c - row * CPR) ^ swz<W>(row));
+    }
+#pragma unroll
+    for (int i = 0; i < N; ++i)
+      __builtin_amdgcn_global_load_lds((const void*)(src + at[i]),
+                                       (lds_ptr_t)(dst + (w * N + i) * 1024), 16, 0, 0);
+  };
+  auto dma = [&](int t, auto BUF) {
+    char* st = decltype(BUF)::value ? st1 : st0;
+    dma1(t, std::integral_constant<int, DK>{}, p.kc, st);
+    dma1(t, std::integral_constant<int, DV>{}, p.vc, st + 128 * DK);
+  };
+
+  float m_run = p.sinks ? p.sinks[h] * 1.4426950408889634f : -1e30f;
+  float l_run = p.sinks ? 1.f : 0.f;
+  float16v o[DV / 32];
+#pragma unroll
+  for (int d = 0; d < DV / 32; ++d)
+#pragma unroll
+    for (int r = 0; r < 16; ++r) o[d][r] = 0.f;
+  // transposed-read roles: 16-lane group g covers columns 16 (g & 1) .. +15 of a 32-column
+  // block for the k-slot half g >> 1; lane 4 qg + pp addresses key row qg, columns 4 pp ..
+  const int g = lane >> 4, qg = (lane & 15) >> 2, pp = lane & 3;
+
+  using B0 = std::integral_constant<int, 0>;
+  using B1 = std::integral_constant<int, 1>;
+  dma(t0, B0{});
+  __syncthreads();
+  auto body = [&](int t, auto BUF) {
+    constexpr int buf = decltype(BUF)::value;
+    if (t + 1 < t1) dma(t + 1, std::integral_constant<int, 1 - buf>{});
+    const char* Kl = buf ? st1 : st0;
+    const char* Vl = Kl + 128 * DK;
+    const int k0 = t * 64;
+    if (k0 <= wmax && k0 + 63 > wmin - win) {  // wave-uniform: some row sees some key
+      float16v sa[2];
+#pragma unroll
+      for (int half = 0; half < 2; ++half) {
+#pragma unroll
+        for (int r = 0; r < 16; ++r) sa[half][r] = 0.f;
+#pragma unroll
+        for (int ks = 0; ks < DK / 16; ++ks)
+          sa[half] = mfma32(*reinterpret_cast<const short8*>(Kl + img<DK>(half * 32 + ql, 2 * ks + hi)),
+                            qf[ks], sa[half]);
+      }
+      float mloc = -INFINITY;
+      if (k0 + 63 > wmin || k0 <= wmax - win) {  // an edge crosses the tile
+        const int top = qpos - k0 - 4 * hi, bot = qpos - win + 1 - k0 - 4 * hi;
+#pragma unroll
+        for (int half = 0; half < 2; ++half)
+#pragma unroll
+          for (int r = 0; r < 16; ++r) {
+            const int kk = half * 32 + (r & 3) + 8 * (r >> 2);
+            const float v = (kk > top || kk < bot) ? -INFINITY : sa[half][r];
+            sa[half][r] = v;
+            mloc = fmaxf(mloc, v);
+          }
+      } else {
+#pragma unroll
+        for (int half = 0; half < 2; ++half)
+#pragma unroll
+          for (int r = 0; r < 16; ++r) mloc = fmaxf(mloc, sa[half][r]);
+      }
+      mloc = fmaxf(mloc, __shfl_xor(mloc, 32, 64)) * p.scale_log2;
+      // the running maximum moves only when a row's grows by more than 2^8
+      const bool grow = mloc > m_run + 8.f;
+      if (__builtin_amdgcn_ballot_w64(grow)) {
+        const float m_new = grow ? mloc : m_run;
+        const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
+        l_run *= alpha;
+#pragma unroll
+        for (int d = 0; d < DV / 32; ++d) o[d] *= alpha;
+        m_run = m_new;
+      }
+      float lsum = 0.f;
+#pragma unroll
+      for (int half = 0; half < 2; ++half)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+          const float e =
+              __builtin_amdgcn_exp2f(__builtin_fmaf(sa[half][r], p.scale_log2, -m_run));
+          sa[half][r] = e;
+          lsum += e;
+        }
+      l_run += lsum + __shfl_xor(lsum, 32, 64);
+      typedef short v4s __attribute__((ext_vector_type(4)));
+      typedef __attribute__((address_space(3))) v4s* lds_v4s;
+#pragma unroll
+      for (int st = 0; st < 4; ++st) {
+        short8 pb;
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+          pb[j] = __builtin_bit_cast(short, (__bf16)sa[st >> 1][8 * (st & 1) + j]);
+        const int kb = (st >> 1) * 32 + 16 * (st & 1) + 4 * (g >> 1) + qg;
+#pragma unroll
+        for (int d = 0; d < DV / 32; ++d) {
+          const int ch = d * 4 + 2 * (g & 1) + (pp >> 1);
+          const v4s lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+              (lds_v4s)(Vl + img<DV>(kb, ch) + 8 * (pp & 1)));
+          const v4s hv = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+              (lds_v4s)(Vl + img<DV>(kb + 8, ch) + 8 * (pp & 1)));
+          o[d] = mfma32(__builtin_shufflevector(lo, hv, 0, 1, 2, 3, 4, 5, 6, 7), pb, o[d]);
+        }
+      }
+    }
+    __syncthreads();  // the next tile landed and this one is read by all waves
+  };
+  for (int t = t0; t < t1; t += 2) {
+    body(t, B0{});
+    if (t + 1 < t1) body(t + 1, B1{});
+  }
+  if (row_ok) {
+    const float inv = 1.f / l_run;
+    bf16_t* orow = p.out + ((int64_t)(qs + qr) * p.H + h) * DV;
+#pragma unroll
+    for (int d = 0; d < DV / 32; ++d)
+#pragma unroll
+      for (int m = 0; m < 4; ++m) {
+        uint2v pk;
+        pk[0] = pack_bf2(o[d][4 * m] * inv, o[d][4 * m + 1] * inv);
+        pk[1] = pack_bf2(o[d][4 * m + 2] * inv, o[d][4 * m + 3] * inv);
+        *reinterpret_cast<uint2v*>(orow + d * 32 + 8 * m + 4 * hi) = pk;
+      }
+  }
+}
+
+}  // namespace
+
+extern "C" {
+
+int omnia_gqa_prefill(void* out, const void* q, const void* kc, const void* vc,
+                      const int* block_tables, int bt_stride, const int* q_start,
+                      const int* seq_lens, const int* tile_seq, const int* tile_q0, int n_tiles,
+                      int page, int H, int G, int Dp, int Vp, int window, float scale,
+                      const float* sinks, hipStream_t s) {
+  if (G < 1 || H % G || window < 0) return -1;
+  int page_lg = 0;
+  while (page_lg < 30 && (1 << page_lg) < page) ++page_lg;
+  if ((1 << page_lg) != page) return -2;
+  if (n_tiles == 0) return 0;
+  const int group = H / G, hb_lg = group % 4 == 0 ? 2 : group % 2 == 0 ? 1 : 0;
+  if ((int64_t)n_tiles * H > 2147483647LL) return -4;
+  Args a{(bf16_t*)out, (const bf16_t*)q, (const bf16_t*)kc, (const bf16_t*)vc, block_tables,
+         q_start, seq_lens, tile_seq, tile_q0, sinks, bt_stride, n_tiles, H, G, hb_lg, page_lg,
+         window, scale * 1.4426950408889634f};
+#define OMNIA_GQ(K, V)                                                  \
+  if (Dp == K && Vp == V) {                                             \
+    prefill_kernel<K, V><<<n_tiles * H, 256, 0, s>>>(a);                \
+    return (int)hipGetLastError();                                      \
+  }
+#define OMNIA_GQV(K) \
+  OMNIA_GQ(K, 32) OMNIA_GQ(K, 64) OMNIA_GQ(K, 96) OMNIA_GQ(K, 128) OMNIA_GQ(K, 192) OMNIA_GQ(K, 256)
+  OMNIA_GQV(32) OMNIA_GQV(64) OMNIA_GQV(96) OMNIA_GQV(128) OMNIA_GQV(192) OMNIA_GQV(256)
+#undef OMNIA_GQV
+#undef OMNIA_GQ
+  return -3;
+}
+
+}  // extern "C"

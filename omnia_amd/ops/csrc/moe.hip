@@ -8,8 +8,13 @@
 //   * moe_gemm   : grouped MFMA GEMM over the expert-sorted rows.
 //                  MODE 0: gate_up with the SwiGLU epilogue fused (a 64-column
 //                          tile = 32 gate + the matching 32 up columns)
-//                  MODE 1: down projection with the routing weight fused, rows
-//                          written back to their (token, slot) position
+//                  MODE 1: down projection with the routing weight fused (or none),
+//                          rows written back to their (token, slot) position
+//                  MODE 2: MODE 0 with a clamped GLU and the routing weight on the
+//                          expert's INPUT (W (r h) = r (W h): the epilogue scales)
+//                  fp32 models: the same modes on a plain fp32 tile
+//   * moe_route  : router logits in fp32 (never rounded), sigmoid or softmax scores,
+//                  top-k of up to 256 experts
 //   * moe_combine: out[t] = sum_j Y[t*k + j]  (deterministic, no atomics)
 // Expert parallelism: moe_align keeps only experts in [e_lo, e_hi); the caller
 // all-reduces the combined output over the EP group.
@@ -121,6 +126,103 @@ __global__ __launch_bounds__(256) void moe_router_topk_kernel(
   select_topk(mine, lane, t, E, k, renorm, ids, wts);
 }
 
+// fp32 router for any score function: logits z[e] = x . router[e] stay fp32; the k
+// largest are chosen; weights are sigmoid(z) or softmax(z), renormalised over the chosen
+// ones if asked.  One wave per token; expert e belongs to lane e & 63; EC experts'
+// dot products at a time.
+constexpr int kMaxExperts = 256;
+
+template <typename T, int EC>
+__global__ __launch_bounds__(256) void moe_route_kernel(int* __restrict__ ids,
+                                                        float* __restrict__ wts,
+                                                        const T* __restrict__ x,
+                                                        const T* __restrict__ router, int n_tok,
+                                                        int d, int E, int k, int sigmoid,
+                                                        int renorm) {
+  constexpr int NPL = kMaxExperts / 64;
+  const int lane = threadIdx.x & 63;
+  const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (t >= n_tok) return;
+  const T* xr = x + (int64_t)t * d;
+  auto load8 = [](const T* p, float (&f)[8]) {
+    if constexpr (sizeof(T) == 4) {
+      const float4v a = *reinterpret_cast<const float4v*>(p);
+      const float4v b = *reinterpret_cast<const float4v*>(p + 4);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        f[j] = a[j];
+        f[4 + j] = b[j];
+      }
+    } else {
+      const short8 v = *reinterpret_cast<const short8*>(p);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) f[j] = bf2f((uint16_t)v[j]);
+    }
+  };
+  float z[NPL];
+#pragma unroll
+  for (int i = 0; i < NPL; ++i) z[i] = -INFINITY;
+  for (int e0 = 0; e0 < E; e0 += EC) {
+    float acc[EC];
+#pragma unroll
+    for (int e = 0; e < EC; ++e) acc[e] = 0.f;
+    for (int c = lane * 8; c < d; c += 64 * 8) {
+      float xf[8];
+      load8(xr + c, xf);
+#pragma unroll
+      for (int e = 0; e < EC; ++e) {
+        float wf[8];
+        load8(router + (int64_t)min(e0 + e, E - 1) * d + c, wf);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) acc[e] += xf[j] * wf[j];
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < EC; ++e) {
+      float v = wave_sum(acc[e]);
+      if (!(v == v)) v = -INFINITY;  // NaN rows (padding) still choose distinct valid ids
+#pragma unroll
+      for (int i = 0; i < NPL; ++i)
+        if (e0 + e < E && (e0 + e) == lane + 64 * i) z[i] = v;
+    }
+  }
+  float top = -INFINITY, total = 1.f;
+  if (!sigmoid) {
+#pragma unroll
+    for (int i = 0; i < NPL; ++i) top = fmaxf(top, z[i]);
+    top = wave_max(top);
+    if (!(top > -INFINITY)) top = 0.f;
+    total = 0.f;
+#pragma unroll
+    for (int i = 0; i < NPL; ++i) total += expf(z[i] - top);
+    total = wave_sum(total);
+  }
+  unsigned taken = 0;  // bit i: this lane's expert lane + 64 i is chosen
+  float sel = 0.f, mine = 0.f;
+  for (int j = 0; j < k; ++j) {
+    float v = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < NPL; ++i)
+      if (!(taken >> i & 1) && lane + 64 * i < E) v = fmaxf(v, z[i]);
+    const float vm = wave_max(v);
+    int first = 1 << 30;  // lowest untaken expert with the largest logit
+#pragma unroll
+    for (int i = NPL - 1; i >= 0; --i)
+      if (!(taken >> i & 1) && lane + 64 * i < E && z[i] == vm) first = lane + 64 * i;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) first = min(first, __shfl_xor(first, o, 64));
+    if ((first & 63) == lane) taken |= 1u << (first >> 6);
+    const float s = sigmoid ? 1.f / (1.f + expf(-vm)) : expf(vm - top);
+    sel += s;
+    if (lane == j) mine = s;  // k <= 64: lane j keeps slot j
+    if (lane == 0) ids[(int64_t)t * k + j] = first;
+  }
+  if (lane < k) {
+    const float den = renorm ? sel : sigmoid ? 1.f : total;
+    wts[(int64_t)t * k + lane] = den > 0.f ? mine / den : 0.f;
+  }
+}
+
 // ------------------------------------------------------------------ align
 // One 1024-thread workgroup.  n = T*k assignments.  sorted has max_blocks*BM
 // entries (n = padding sentinel), blk_expert max_blocks entries.
@@ -169,19 +271,30 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(int* __restrict__ sorte
 // (ds_read_b128 fragment reads are then conflict-free across the 16 rows).
 __device__ __forceinline__ int swz(int row, int ch) { return row * 64 + ((ch ^ (row & 7)) << 3); }
 
+// clamped GLU: g = min(gate, limit), u = clamp(up, +-limit): g sigmoid(alpha g) (u + 1)
+struct Glu {
+  float alpha, limit;
+};
+__device__ __forceinline__ float clamped_glu(float g, float u, Glu c) {
+  g = fminf(g, c.limit);
+  u = fminf(fmaxf(u, -c.limit), c.limit);
+  return g * __builtin_amdgcn_rcpf(1.f + __expf(-c.alpha * g)) * (u + 1.f);
+}
+
 template <int MODE>
 __global__ __launch_bounds__(256) void moe_gemm_kernel(
     bf16_t* __restrict__ out, const bf16_t* __restrict__ A, const bf16_t* __restrict__ W,
     const int* __restrict__ sorted, const int* __restrict__ blk_expert,
     const int* __restrict__ n_blocks, const float* __restrict__ route_w, int K, int N,
-    int topk, int n_assign, int e_lo) {
+    int topk, int n_assign, int e_lo, Glu glu) {
+  constexpr bool GATED = MODE != 1;
   __shared__ __attribute__((aligned(16))) bf16_t lds[2 * 2 * BM * 64];
   const int mb = blockIdx.y;
   if (mb >= *n_blocks) return;
   const int e = blk_expert[mb] - e_lo;
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
-  const int n0 = blockIdx.x * (MODE == 0 ? 32 : 64);
-  const int w_rows = MODE == 0 ? 2 * N : N;  // rows of one expert's weight matrix
+  const int n0 = blockIdx.x * (GATED ? 32 : 64);
+  const int w_rows = GATED ? 2 * N : N;  // rows of one expert's weight matrix
   const bf16_t* We = W + (int64_t)e * w_rows * K;
 
   // per-thread staging: 2 A chunks + 2 B chunks of 16 B per k-tile
@@ -193,11 +306,11 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(
     const int c = tid + i * 256;  // 0..511
     const int row = c >> 3, ch = c & 7;
     const int flat = sorted[mb * BM + row];
-    const int64_t arow = MODE == 0 ? (flat < n_assign ? flat / topk : 0) : (int64_t)mb * BM + row;
+    const int64_t arow = GATED ? (flat < n_assign ? flat / topk : 0) : (int64_t)mb * BM + row;
     a_src[i] = A + arow * K + ch * 8;
     a_lds[i] = swz(row, ch);
     int wrow;
-    if (MODE == 0)
+    if (GATED)
       wrow = row < 32 ? n0 + row : N + n0 + (row - 32);
     else
       wrow = n0 + row;
@@ -268,7 +381,13 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(
     const int row = mb * BM + 16 * w + 4 * fq + r;
     const int flat = sorted[row];
     if (flat >= n_assign) continue;
-    if (MODE == 0) {
+    if (MODE == 2) {
+      const float wt = route_w[flat];
+#pragma unroll
+      for (int jj = 0; jj < 2; ++jj)
+        out[(int64_t)row * N + n0 + 16 * jj + fr] =
+            f2bf(clamped_glu(wt * acc[jj][r], wt * acc[jj + 2][r], glu));
+    } else if (MODE == 0) {
 #pragma unroll
       for (int jj = 0; jj < 2; ++jj) {
         const float g = acc[jj][r], u = acc[jj + 2][r];
@@ -276,9 +395,85 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(
         out[(int64_t)row * N + n0 + 16 * jj + fr] = f2bf(s * u);
       }
     } else {
-      const float wt = route_w[flat];
+      const float wt = route_w ? route_w[flat] : 1.f;
 #pragma unroll
       for (int j = 0; j < 4; ++j) out[(int64_t)flat * N + n0 + 16 * j + fr] = f2bf(wt * acc[j][r]);
+    }
+  }
+}
+
+// fp32 models: 64 x 64 tile (gated: 32 gate + the matching 32 up columns), 4 x 4 outputs a
+// thread; columns 2 tx, 2 tx + 1 and 32 + those, so a gate and its up meet in one thread
+template <int MODE>
+__global__ __launch_bounds__(256) void moe_gemm_f32_kernel(
+    float* __restrict__ out, const float* __restrict__ A, const float* __restrict__ W,
+    const int* __restrict__ sorted, const int* __restrict__ blk_expert,
+    const int* __restrict__ n_blocks, const float* __restrict__ route_w, int K, int N, int topk,
+    int n_assign, int e_lo, Glu glu) {
+  constexpr bool GATED = MODE != 1;
+  __shared__ float As[16][BM + 4], Bs[16][BM + 4];
+  const int mb = blockIdx.y;
+  if (mb >= *n_blocks) return;
+  const int n0 = blockIdx.x * (GATED ? 32 : 64);
+  const float* We = W + (int64_t)(blk_expert[mb] - e_lo) * (GATED ? 2 * N : N) * K;
+  const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4;
+  const int row = tid >> 2, kq = (tid & 3) * 4;
+  const int f0 = sorted[mb * BM + row];
+  const float* ar = A + (GATED ? (int64_t)(f0 < n_assign ? f0 / topk : 0)
+                               : (int64_t)mb * BM + row) * K + kq;
+  const int wrow = !GATED ? n0 + row : row < 32 ? n0 + row : N + n0 + row - 32;
+  const float* br = We + (int64_t)wrow * K + kq;
+  float acc[4][4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = 0.f;
+  for (int k0 = 0; k0 < K; k0 += 16) {
+    const float4v a = *reinterpret_cast<const float4v*>(ar + k0);
+    const float4v b = *reinterpret_cast<const float4v*>(br + k0);
+    __syncthreads();
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      As[kq + j][row] = a[j];
+      Bs[kq + j][row] = b[j];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int kk = 0; kk < 16; ++kk) {
+      float av[4], bv[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) av[i] = As[kk][ty * 4 + i];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) bv[j] = Bs[kk][(j >> 1) * 32 + 2 * tx + (j & 1)];
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] += av[i] * bv[j];
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int r = mb * BM + ty * 4 + i, flat = sorted[r];
+    if (flat >= n_assign) continue;
+    if (GATED) {
+      const float wt = MODE == 2 ? route_w[flat] : 1.f;
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        float g = wt * acc[i][j], u = wt * acc[i][j + 2], y;
+        if (MODE == 2) {
+          g = fminf(g, glu.limit);
+          u = fminf(fmaxf(u, -glu.limit), glu.limit);
+          y = g / (1.f + expf(-glu.alpha * g)) * (u + 1.f);
+        } else {
+          y = g / (1.f + expf(-g)) * u;
+        }
+        out[(int64_t)r * N + n0 + 2 * tx + j] = y;
+      }
+    } else {
+      const float wt = route_w ? route_w[flat] : 1.f;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        out[(int64_t)flat * N + n0 + (j >> 1) * 32 + 2 * tx + (j & 1)] = wt * acc[i][j];
     }
   }
 }
@@ -353,23 +548,54 @@ int omnia_moe_align(int* sorted, int* blk_expert, int* n_blocks, const int* ids,
   return (int)hipGetLastError();
 }
 
+// x [T, d] and router [E, d] in one dtype -> ids / wts [T, k]; fp32 logits
+int omnia_moe_route(int* ids, float* wts, const void* x, const void* router, int f32, int n_tok,
+                    int d, int E, int k, int sigmoid, int renorm, hipStream_t s) {
+  if (E < 1 || E > kMaxExperts || k < 1 || k > E || k > 64 || d % 8) return -1;
+  if (n_tok == 0) return 0;
+  const int blocks = (n_tok + 3) / 4;
+#define OMNIA_RO(TT, EC)                                                                       \
+  moe_route_kernel<TT, EC><<<blocks, 256, 0, s>>>(ids, wts, (const TT*)x, (const TT*)router,   \
+                                                  n_tok, d, E, k, sigmoid, renorm)
+#define OMNIA_ROE(TT)            \
+  do {                           \
+    if (E <= 8) OMNIA_RO(TT, 8); \
+    else OMNIA_RO(TT, 16);       \
+  } while (0)
+  if (f32) OMNIA_ROE(float);
+  else OMNIA_ROE(bf16_t);
+#undef OMNIA_ROE
+#undef OMNIA_RO
+  return (int)hipGetLastError();
+}
+
 // mode 0: out = act [max_blocks*64, N=I], A = x [T, K=d], W = [E_local, 2I, d]
 // mode 1: out = Y [T*k, N=d],            A = act [max_blocks*64, K=I], W = [E_local, d, I]
-int omnia_moe_gemm(int mode, void* out, const void* A, const void* W, const int* sorted,
+// mode 2: mode 0 with the clamped GLU (alpha, limit) of the weighted input
+int omnia_moe_gemm(int mode, void* out, const void* A, const void* W, int f32, const int* sorted,
                    const int* blk_expert, const int* n_blocks, const float* route_w, int K,
-                   int N, int topk, int n_assign, int e_lo, int max_blocks, hipStream_t s) {
-  if (K % 64) return -1;
-  if (mode == 0 ? (N % 32) : (N % 64)) return -2;
+                   int N, int topk, int n_assign, int e_lo, int max_blocks, float alpha,
+                   float limit, hipStream_t s) {
+  if (mode < 0 || mode > 2 || K % 64) return -1;
+  if (mode == 1 ? (N % 64) : (N % 32)) return -2;
+  if (mode == 2 && !route_w) return -3;
   if (max_blocks == 0) return 0;
-  dim3 grid(mode == 0 ? N / 32 : N / 64, max_blocks);
-  if (mode == 0)
-    moe_gemm_kernel<0><<<grid, 256, 0, s>>>((bf16_t*)out, (const bf16_t*)A, (const bf16_t*)W,
-                                            sorted, blk_expert, n_blocks, route_w, K, N, topk,
-                                            n_assign, e_lo);
-  else
-    moe_gemm_kernel<1><<<grid, 256, 0, s>>>((bf16_t*)out, (const bf16_t*)A, (const bf16_t*)W,
-                                            sorted, blk_expert, n_blocks, route_w, K, N, topk,
-                                            n_assign, e_lo);
+  if (max_blocks > 65535) return -4;
+  const dim3 grid(mode == 1 ? N / 64 : N / 32, max_blocks);
+  const Glu glu{alpha, limit};
+#define OMNIA_MG(KER, TT, MM)                                                                  \
+  KER<MM><<<grid, 256, 0, s>>>((TT*)out, (const TT*)A, (const TT*)W, sorted, blk_expert,       \
+                               n_blocks, route_w, K, N, topk, n_assign, e_lo, glu)
+#define OMNIA_MGM(KER, TT)                    \
+  do {                                        \
+    if (mode == 0) OMNIA_MG(KER, TT, 0);      \
+    else if (mode == 1) OMNIA_MG(KER, TT, 1); \
+    else OMNIA_MG(KER, TT, 2);                \
+  } while (0)
+  if (f32) OMNIA_MGM(moe_gemm_f32_kernel, float);
+  else OMNIA_MGM(moe_gemm_kernel, bf16_t);
+#undef OMNIA_MGM
+#undef OMNIA_MG
   return (int)hipGetLastError();
 }
 

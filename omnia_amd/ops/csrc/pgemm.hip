@@ -33,7 +33,8 @@
 //          assignments (moe_align at 256-row segments), A rows gathered by token,
 //          W = that segment's expert [Wg; Wu]; act written in sorted order
 //   EPI 6  MoE grouped down: A = act (sorted order), W = the segment's expert,
-//          each row scaled by its routing weight and scattered to Y[assignment]
+//          each row scaled by its routing weight (if given) and scattered to Y[assignment]
+//   EPI 8  EPI 5 with the routing weight on the expert's input and a clamped GLU
 //   EPI 7  EPI 1 with a bias: out = silu(g + bias[f]) * (u + bias[N + f])
 //   EPI 4  split-K partial: block (m-tile, n-tile, k-slice ks) writes its K-slice's
 //          fp32 sum, saturated to fp16, into slab ks of out[S][M][N]; the splitk.hip
@@ -87,10 +88,13 @@ struct PArgs {
   const float* route_w;
   int topk, n_assign, e_lo;
   const float* bias;     // EPI 7: fp32 [2N]
+  float glu_alpha, glu_limit;  // EPI 8
 };
 
 // a gate_up epilogue: 128 features per block tile, gate and up halves in one lane
-constexpr bool gated(int epi) { return epi == 1 || epi == 5 || epi == 7; }
+constexpr bool gated(int epi) { return epi == 1 || epi == 5 || epi == 7 || epi == 8; }
+// rows are expert-sorted assignments
+constexpr bool grouped(int epi) { return epi == 5 || epi == 6 || epi == 8; }
 
 __device__ __forceinline__ float4v mfma16(short8 a, short8 b, float4v c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a),
@@ -118,6 +122,13 @@ __device__ __forceinline__ float16v mfma32(short8 a, short8 b, float16v c) {
 }
 
 __device__ __forceinline__ float silu(float g) { return g * __builtin_amdgcn_rcpf(1.f + __expf(-g)); }
+
+// g = min(gate, limit), u = clamp(up, +-limit): g sigmoid(alpha g) (u + 1)
+__device__ __forceinline__ float clamped_glu(float g, float u, float alpha, float limit) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g * __builtin_amdgcn_rcpf(1.f + __expf(-alpha * g)) * (u + 1.f);
+}
 
 template <int N>
 __device__ __forceinline__ void wait_vm() {
@@ -240,7 +251,7 @@ template <int EPI, int VAR = 0>
 __global__ __launch_bounds__(512, 2) void pgemm_kernel(PArgs p) {
   __shared__ __attribute__((aligned(16))) bf16_t lds[LDS_ELEMS];
   constexpr int TN = gated(EPI) ? 128 : 256;  // output columns per block tile
-  constexpr bool MOE = EPI == 5 || EPI == 6;
+  constexpr bool MOE = grouped(EPI);
   // EPI 4: the K-slices are extra "m-tiles" of the L2 grouping below (blocks of
   // one slice share its x slice, blocks of one column tile its W rows)
   const int S = EPI == 4 ? p.splits : 1;
@@ -269,7 +280,7 @@ __global__ __launch_bounds__(512, 2) void pgemm_kernel(PArgs p) {
   }
   const bf16_t* Wb = p.W;
   if constexpr (MOE)
-    Wb += (int64_t)(p.blk_expert[mt] - p.e_lo) * (EPI == 5 ? 2 * p.N : p.N) * K;
+    Wb += (int64_t)(p.blk_expert[mt] - p.e_lo) * (gated(EPI) ? 2 * p.N : p.N) * K;
 
   const int tid = threadIdx.x, lane = tid & 63;
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -287,7 +298,7 @@ __global__ __launch_bounds__(512, 2) void pgemm_kernel(PArgs p) {
     for (int h = 0; h < 2; ++h) {
       int ar = m0 + h * 128 + row;
       ar = ar < p.M ? ar : p.M - 1;  // rows past the chunk: clamped copies, never stored
-      if constexpr (EPI == 5) {  // gather: the assignment's token row (padding: row 0)
+      if constexpr (MOE && gated(EPI)) {  // gather: the assignment's token row (padding: row 0)
         const int f = p.sorted[m0 + h * 128 + row];
         ar = f < p.n_assign ? f / p.topk : 0;
       }
@@ -453,12 +464,13 @@ __global__ __launch_bounds__(512, 2) void pgemm_kernel(PArgs p) {
   // ---------------------------------------------------------------- epilogue
   // lane rows: a*128 + wr*64 + m*16 + fq*4 + j ; cols: b*128 + wc*32 + n*16 + fr
   float* rs_lds = reinterpret_cast<float*>(lds + RS_OFF);
-  const bool scaled = EPI == 6 || (EPI != 2 && EPI != 7 && p.ss_in != nullptr);
+  constexpr bool ROUTED = EPI == 6 || EPI == 8;
+  const bool scaled = ROUTED || (EPI != 2 && EPI != 7 && p.ss_in != nullptr);
   if (scaled) {
     if (tid < 256) {
-      if constexpr (EPI == 6) {  // row scale = the assignment's routing weight
+      if constexpr (ROUTED) {  // row scale = the assignment's routing weight
         const int f = p.sorted[m0 + tid];
-        rs_lds[tid] = f < p.n_assign ? p.route_w[f] : 0.f;
+        rs_lds[tid] = f >= p.n_assign ? 0.f : p.route_w ? p.route_w[f] : 1.f;
       } else {
         int r = m0 + tid;
         r = r < p.M ? r : p.M - 1;
@@ -539,6 +551,11 @@ __global__ __launch_bounds__(512, 2) void pgemm_kernel(PArgs p) {
 #pragma unroll
             for (int j = 0; j < 4; ++j)
               v[j] = silu(acc[a][0][m][n][j] + bg) * (acc[a][1][m][n][j] + bu);
+          } else if constexpr (EPI == 8) {
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+              v[j] = clamped_glu(acc[a][0][m][n][j] * rs[j], acc[a][1][m][n][j] * rs[j],
+                                 p.glu_alpha, p.glu_limit);
           } else {
 #pragma unroll
             for (int j = 0; j < 4; ++j)
@@ -571,7 +588,7 @@ __global__ __launch_bounds__(512, 2) void pgemm_kernel(PArgs p) {
     PArgs q = p;
     q.out = reinterpret_cast<bf16_t*>(p.out) + (int64_t)ks * p.M * p.N;
     epi_out<4, 512>(q, stg, m0, nt, Mt, ntn, tid, lane);
-  } else if constexpr (EPI == 5) {
+  } else if constexpr (MOE && gated(EPI)) {
     epi_out<1, 512>(p, stg, m0, nt, Mt, ntn, tid, lane);
   } else {
     epi_out<EPI, 512>(p, stg, m0, nt, Mt, ntn, tid, lane);
@@ -839,7 +856,8 @@ int omnia_pgemm_splitk(void* parts, const void* X, const void* W, int M, int N, 
                        int sched, hipStream_t s);
 int omnia_pgemm_moe(int mode, void* out, const void* A, const void* W, const int* sorted,
                     const int* blk_expert, const int* n_blocks, const float* route_w, int K,
-                    int N, int topk, int n_assign, int e_lo, int max_blocks, hipStream_t s);
+                    int N, int topk, int n_assign, int e_lo, int max_blocks, float alpha,
+                    float limit, hipStream_t s);
 
 static int g_pgemm_sched = 0;  // 0: 8-wave ping-pong, 1: 4-wave (one wave per SIMD)
 
@@ -955,25 +973,29 @@ int omnia_pgemm_splitk(void* parts, const void* X, const void* W, int M, int N, 
 // MoE grouped GEMMs on the 256x256 tile (segments from omnia_moe_align with
 // bm = 256).  mode 0: act [max_blocks*256, I] = SwiGLU(x[token] . W_gu[e]^T),
 // x [T, d], W_gu [E_loc, 2I, d];  mode 1: Y[assignment] = w_route * act . W_dn[e]^T,
-// act [max_blocks*256, I], W_dn [E_loc, d, I], Y [n_assign, d].
+// act [max_blocks*256, I], W_dn [E_loc, d, I], Y [n_assign, d] (w_route null: 1);  mode 2:
+// mode 0 with the clamped GLU (alpha, limit) of the weighted input.
 int omnia_pgemm_moe(int mode, void* out, const void* A, const void* W, const int* sorted,
                     const int* blk_expert, const int* n_blocks, const float* route_w, int K,
-                    int N, int topk, int n_assign, int e_lo, int max_blocks, hipStream_t s) {
-  if (mode < 0 || mode > 1 || max_blocks < 0 || topk < 1) return -1;
+                    int N, int topk, int n_assign, int e_lo, int max_blocks, float alpha,
+                    float limit, hipStream_t s) {
+  if (mode < 0 || mode > 2 || max_blocks < 0 || topk < 1) return -1;
   if (K <= 0 || K % (2 * BK)) return -3;
-  if (N <= 0 || N % (mode == 0 ? 128 : 256)) return -4;
+  if (N <= 0 || N % (mode == 1 ? 256 : 128)) return -4;
   if ((reinterpret_cast<uintptr_t>(A) | reinterpret_cast<uintptr_t>(W) |
        reinterpret_cast<uintptr_t>(out)) & 15)
     return -5;
-  if (!sorted || !blk_expert || !n_blocks || (mode == 1 && !route_w)) return -9;
+  if (!sorted || !blk_expert || !n_blocks || (mode == 2 && !route_w)) return -9;
   if (max_blocks == 0) return 0;
-  const int64_t blocks = (int64_t)max_blocks * (N / (mode == 0 ? 128 : 256));
+  const int64_t blocks = (int64_t)max_blocks * (N / (mode == 1 ? 256 : 128));
   if (blocks > (1 << 30)) return -13;
   PArgs a{out, (const bf16_t*)A, (const bf16_t*)W, max_blocks * 256, N, K, N, nullptr, 0, 0.f,
           0.f, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, 0, 0, 0, 1, sorted,
-          blk_expert, n_blocks, route_w, topk, n_assign, e_lo};
+          blk_expert, n_blocks, route_w, topk, n_assign, e_lo, nullptr, alpha, limit};
   if (mode == 0)
     pgemm_kernel<5><<<dim3((unsigned)blocks), 512, 0, s>>>(a);
+  else if (mode == 2)
+    pgemm_kernel<8><<<dim3((unsigned)blocks), 512, 0, s>>>(a);
   else
     pgemm_kernel<6><<<dim3((unsigned)blocks), 512, 0, s>>>(a);
   return (int)hipGetLastError();

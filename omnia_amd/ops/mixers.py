@@ -1,6 +1,8 @@
-"""Front-end of the kernels behind layer-list models: Dynamic-Tanh norms fused with
-the residual (``csrc/tanh_norm.hip``), the gated delta rule (``csrc/delta.hip``)
-and latent attention (``csrc/latent.hip``).
+"""Front-end of the kernels behind layer-list models: Dynamic-Tanh and RMS norms fused
+with the residual (``csrc/tanh_norm.hip``, ``csrc/rms_residual.hip``), the gated delta
+rule (``csrc/delta.hip``), latent attention (``csrc/latent.hip``), grouped-query
+attention (``csrc/gqa.hip``, ``csrc/gqa_prefill.hip``) and clamped-GLU experts
+(``csrc/moe.hip``, ``csrc/pgemm.hip``).
 
 GPU tensors (bf16 or fp32) run the HIP kernels and nothing else; CPU tensors run
 :mod:`omnia_amd.ops.reference_mixers`."""
@@ -8,7 +10,7 @@ from __future__ import annotations
 
 import torch
 
-from . import checks, kernels
+from . import MOE_TILE256_ROWS, _moe_grouped, checks, kernels
 from . import reference_mixers as ref
 
 
@@ -59,6 +61,95 @@ def bias_swiglu(m, bias, dtype):
         kernels().bias_swiglu(out, m, bias)
         return out
     return ref.bias_swiglu(m, bias, dtype)
+
+
+# ------------------------------------------------------------------- RMS norm
+class RMSNorm:
+    """``x / sqrt(mean(x^2) + eps) * w`` over ``n`` real columns (``w`` fp32, zero on
+    the padding columns)."""
+
+    __slots__ = ("w", "inv_n", "eps")
+
+    def __init__(self, w: torch.Tensor, n: int, eps: float):
+        self.w, self.inv_n, self.eps = w, 1.0 / n, float(eps)
+
+
+def rms_embed(ids, table, vocab: int, emb: RMSNorm, pre: RMSNorm | None, src=None,
+              tok_slots=None):
+    """(fp32 residual rows ``emb(table[ids])``, first sublayer input ``pre(x)`` or x)."""
+    T, d = ids.numel(), table.shape[1]
+    if ids.is_cuda:
+        x = torch.empty(T, d, dtype=torch.float32, device=ids.device)
+        h = torch.empty(T, d, dtype=table.dtype, device=ids.device)
+        kernels().rms_embed(h, x, ids, table, vocab, emb.w, None if pre is None else pre.w,
+                            emb.inv_n, emb.eps, src, tok_slots)
+        return x, h
+    if src is not None:
+        ids = torch.where(src >= 0, tok_slots.index_select(0, src.clamp(min=0).long()), ids)
+    ok = (ids >= 0) & (ids < vocab)
+    x = table[torch.where(ok, ids, torch.zeros_like(ids)).long()].float() * ok[:, None]
+    x = ref.rms_norm(x, emb)
+    return x, (x if pre is None else ref.rms_norm(x, pre)).to(table.dtype)
+
+
+def rms_residual(x, m, post: RMSNorm, pre: RMSNorm | None, dtype, slots: bool = False):
+    """In place ``x += post(m)``; returns ``pre(x)``, or x itself, in ``dtype``.  ``m``: a
+    projection [M, d], its split-K slabs [S, M, d], or (``slots``) parts [M, S, d]."""
+    if x.is_cuda:
+        h = torch.empty(x.shape, dtype=dtype, device=x.device)
+        kernels().rms_residual(h, x, m, slots, post.w, None if pre is None else pre.w,
+                               post.inv_n, post.eps)
+        return h
+    v = m.float().sum(1) if slots else ref.slab_sum(m)
+    x += ref.rms_norm(v, post)
+    return (x if pre is None else ref.rms_norm(x, pre)).to(dtype)
+
+
+def norm_embed(ids, table, vocab: int, emb, pre, src=None, tok_slots=None):
+    """Residual rows and first sublayer input of either norm kind."""
+    if isinstance(emb or pre, TanhNorm):
+        if emb is not None:
+            raise ValueError("no embedding norm of the tanh kind")
+        return tanh_norm_embed(ids, table, vocab, pre, src, tok_slots)
+    return rms_embed(ids, table, vocab, emb, pre, src, tok_slots)
+
+
+def norm_residual(x, m, post, pre, dtype, bias=None, slots: bool = False):
+    """What follows a sublayer, of either norm kind (see the two functions above)."""
+    if isinstance(post, TanhNorm):
+        if slots or pre is None:
+            raise ValueError("tanh norms follow a projection and precede a sublayer")
+        return tanh_norm_residual(x, m, post, pre, dtype, bias)
+    if bias is not None:
+        raise ValueError("no bias under an RMS post-norm")
+    return rms_residual(x, m, post, pre, dtype, slots)
+
+
+def softcap_(logits: torch.Tensor, cap: float) -> torch.Tensor:
+    """In place ``cap tanh(logits / cap)``."""
+    if logits.is_cuda:
+        kernels().softcap(logits, cap)
+        return logits
+    return logits.copy_((cap * torch.tanh(logits.float() / cap)).to(logits.dtype))
+
+
+# -------------------------------------------------------------------- experts
+def experts(h, w: dict, spec) -> torch.Tensor:
+    """Routed clamped-GLU experts: [T, top, d], summed by the residual kernel.  The
+    weights are padded to whole tiles (``ff_pad``; d a multiple of 64)."""
+    T, d = h.shape
+    k, E, ff = spec.top, spec.experts, w["down"].shape[2]
+    if not h.is_cuda:
+        return ref.experts(h, w["router"], w["gate_up"], w["down"], spec)
+    kk = kernels()
+    ids = torch.empty(T, k, dtype=torch.int32, device=h.device)
+    wts = torch.empty(T, k, dtype=torch.float32, device=h.device)
+    kk.moe_route(ids, wts, h, w["router"], k, spec.score == "sigmoid", spec.renorm)
+    tile = h.dtype == torch.bfloat16 and T * k >= MOE_TILE256_ROWS * E and d % 256 == 0 and \
+        ff % 128 == 0
+    y = _moe_grouped(h, w["gate_up"], w["down"], ids, wts, k, E, 0, E, 256 if tile else 64,
+                     (spec.alpha, spec.limit))
+    return y.view(T, k, d)
 
 
 # ----------------------------------------------------------------- delta rule
@@ -191,4 +282,59 @@ def latent_prefill(q, kx, kr, vt, fb, spec, gate, out=None):
     kernels().latent_prefill(out.view(T, H, spec.v_pad), q.view(T, H, spec.qk_pad), kx, kr, vt,
                              fb.q_start_loc, fb.seq_lens, fb.kv_start, fb.kv_first, fb.tile_seq,
                              fb.tile_q0, spec.window, spec.scale, gate)
+    return out
+
+
+# ------------------------------------------------------ grouped-query attention
+def gqa_prep(x, w: dict, spec, pages, positions, slots, cos_sin, dtype, eps: float):
+    """Fused projection rows (or split-K slabs) -> normed, rotated queries [T, H * dim_pad];
+    writes the tokens' keys and values at ``slots`` of ``pages`` = (k, v), or, with
+    ``pages`` None, none (the layer borrows another one's)."""
+    k, v = pages if pages is not None else (None, None)
+    if x.is_cuda:
+        if pages is not None and checks.active(x):
+            checks.slots("gqa_prep", slots, k)
+        q = torch.empty(positions.numel(), spec.heads * spec.dim_pad, dtype=dtype,
+                        device=x.device)
+        kernels().gqa_prep(q, k, v, x, w["q_norm"], w.get("k_norm"), positions, slots, cos_sin,
+                           spec.heads, spec.dim, eps)
+        return q
+    return ref.gqa_prep(x, w, spec, k, v, positions, slots, cos_sin, dtype, eps)
+
+
+def gqa_attend(q, pages, block_tables, q_start, positions, spec, sinks, out=None):
+    """Generic attention (any size, bf16 / fp32): [T, H * v_pad]."""
+    if out is None:
+        out = torch.empty(positions.numel(), spec.heads * spec.v_pad, dtype=q.dtype,
+                          device=q.device)
+    args = (out, q, *pages, block_tables, q_start, positions, spec.heads, spec.window,
+            spec.scale, sinks)
+    (kernels().gqa_attend if q.is_cuda else ref.gqa_attend)(*args)
+    return out
+
+
+def gqa_decode(q, pages, block_tables, positions, spec, sinks, splits: int, out=None):
+    """bf16 decode: each row's visible keys in up to ``splits`` parts."""
+    T, H, V = positions.numel(), spec.heads, spec.v_pad
+    if out is None:
+        out = torch.empty(T, H * V, dtype=q.dtype, device=q.device)
+    po = pm = None
+    if splits > 1:
+        po = torch.empty(T * H * splits * V, dtype=torch.float32, device=q.device)
+        pm = torch.empty(T * H * splits * 2, dtype=torch.float32, device=q.device)
+    if checks.active(q):
+        checks.paged("gqa_decode", block_tables, positions + 1, pages[0], T)
+    kernels().gqa_decode(out, po, pm, q, *pages, block_tables, positions, H, spec.window,
+                         spec.scale, sinks, splits)
+    return out
+
+
+def gqa_prefill(q, pages, fb, spec, sinks, out=None):
+    """bf16 prefill portions (``fb``'s query tiles of 128 rows)."""
+    if out is None:
+        out = torch.empty(q.shape[0], spec.heads * spec.v_pad, dtype=q.dtype, device=q.device)
+    if checks.active(q):
+        checks.paged("gqa_prefill", fb.block_tables, fb.seq_lens, pages[0])
+    kernels().gqa_prefill(out, q, *pages, fb.block_tables, fb.q_start_loc, fb.seq_lens,
+                          fb.tile_seq, fb.tile_q0, spec.heads, spec.window, spec.scale, sinks)
     return out

@@ -7,7 +7,7 @@ import torch
 import torch.nn.functional as F
 
 
-def _sum(m: torch.Tensor) -> torch.Tensor:
+def slab_sum(m: torch.Tensor) -> torch.Tensor:
     return m.float().sum(0) if m.dim() == 3 else m.float()
 
 
@@ -16,7 +16,7 @@ def tanh_norm(x, alpha, w, b):
 
 
 def tanh_norm_residual(x, m, bias, a1, w1, b1, a2, w2, b2, dtype):
-    v = _sum(m)
+    v = slab_sum(m)
     if bias is not None:
         v = v + bias
     x += tanh_norm(v, a1, w1, b1)
@@ -24,7 +24,7 @@ def tanh_norm_residual(x, m, bias, a1, w1, b1, a2, w2, b2, dtype):
 
 
 def bias_swiglu(m, bias, dtype):
-    v = _sum(m) + bias
+    v = slab_sum(m) + bias
     g, u = v.chunk(2, -1)
     return (F.silu(g) * u).to(dtype)
 
@@ -161,3 +161,66 @@ def latent_attend(q, cache, block_tables, q_start, positions, H, Cp, window, sca
             p = torch.softmax(qv[t] @ rows.T * scale, -1)
             out[t] = (p @ rows[:, :Cp]).to(q.dtype)
     return out.view(T, H * Cp)
+
+
+def rms_norm(x, n):
+    return x / torch.sqrt(x.pow(2).sum(-1, keepdim=True) * n.inv_n + n.eps) * n.w
+
+
+def experts(h, router, gate_up, down, spec):
+    """[T, top, d]: the chosen experts' outputs, their weights on the inputs."""
+    T, d = h.shape
+    z = h.float() @ router.float().T
+    zt, ids = z.sort(dim=-1, descending=True, stable=True)
+    zt, ids = zt[:, :spec.top], ids[:, :spec.top]
+    if spec.score == "sigmoid":
+        wt = torch.sigmoid(zt)
+    else:
+        wt = torch.exp(zt - torch.logsumexp(z, -1, keepdim=True))
+    if spec.renorm:
+        wt = wt / wt.sum(-1, keepdim=True)
+    out = torch.zeros(T, spec.top, d, dtype=h.dtype)
+    for e in ids.unique().tolist():
+        t, j = (ids == e).nonzero(as_tuple=True)
+        v = (h[t].float() @ gate_up[e].float().T) * wt[t, j, None]
+        g, u = v.chunk(2, -1)
+        g, u = g.clamp(max=spec.limit), u.clamp(-spec.limit, spec.limit)
+        a = (g * torch.sigmoid(spec.alpha * g) * (u + 1.0)).to(h.dtype)
+        out[t, j] = (a.float() @ down[e].float().T).to(h.dtype)
+    return out
+
+
+def gqa_prep(x, w, spec, k, v, positions, slots, cos_sin, dtype, eps):
+    T, H, D, Dp, R = positions.numel(), spec.heads, spec.dim, spec.dim_pad, cos_sin.shape[1]
+    x = slab_sum(x)
+
+    def turned(z, wn, heads):
+        z = z.reshape(T, heads, Dp)
+        z = z / torch.sqrt(z.pow(2).sum(-1, keepdim=True) / D + eps) * wn
+        return torch.cat([_rotate(z[..., :R], positions, cos_sin), z[..., R:]], -1).to(dtype)
+
+    if k is not None:
+        G, page, Vp = k.shape[1], k.shape[2], v.shape[3]
+        kk = turned(x[:, H * Dp:(H + G) * Dp], w["k_norm"], G)
+        vv = x[:, (H + G) * Dp:(H + G) * Dp + G * Vp].reshape(T, G, Vp).to(dtype)
+        keep = slots >= 0
+        b, o = slots[keep] // page, slots[keep] % page
+        k[b, :, o], v[b, :, o] = kk[keep], vv[keep]
+    return turned(x[:, :H * Dp], w["q_norm"], H).reshape(T, H * Dp)
+
+
+def gqa_attend(out, q, k, v, block_tables, q_start, positions, H, window, scale, sinks):
+    T, G, page = positions.numel(), k.shape[1], k.shape[2]
+    qv = q.view(T, G, H // G, -1).float()
+    ov = out.view(T, H, -1)
+    for s, r0, n in _spans(q_start, T):
+        for t in range(r0, r0 + n):
+            pos = int(positions[t])
+            key = torch.arange(max(0, pos - window + 1) if window > 0 else 0, pos + 1)
+            b = block_tables[s, key // page].long()
+            kr, vr = k[b, :, key % page].float(), v[b, :, key % page].float()  # [n, G, w]
+            sc = torch.matmul(qv[t], kr.permute(1, 2, 0)).reshape(H, -1) * scale
+            if sinks is not None:
+                sc = torch.cat([sc, sinks[:, None]], 1)
+            p = torch.softmax(sc, -1)[:, :key.numel()].view(G, H // G, -1)
+            ov[t] = torch.matmul(p, vr.permute(1, 0, 2)).reshape(H, -1).to(q.dtype)
