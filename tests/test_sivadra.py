@@ -232,7 +232,7 @@ def test_config_and_loader_errors(models, tmp_path):
     with pytest.raises(ValueError, match="l2.mix.q"):
         load_checkpoint(sc.save(cfg, bad, tmp_path / "b"), mc)
     for edit, what in (({"type": "conv"}, "unknown mixer"),
-                       ({"mlp": {"kind": "moe"}}, "unknown feed-forward")):
+                       ({"mlp": {"kind": "gated"}}, "unknown feed-forward")):
         c = json.loads(json.dumps(cfg))
         c["layers"][0].update(edit)
         with pytest.raises(ValueError, match=what):
