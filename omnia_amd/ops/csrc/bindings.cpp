@@ -124,9 +124,10 @@ int omnia_tgemm(int mode, void* out, const void* X, const void* W, int M, int N,
 int omnia_tanh_norm_embed(void* h, float* x, const int* ids, const void* table, int f32, int T,
                           int d, int vocab, float alpha, const float* w, const float* b,
                           const int64_t* src, const int* tok_slots, hipStream_t s);
-int omnia_tanh_norm_residual(void* h, int f32, float* x, const void* m, int ptype, int S, int rows,
-                             int d, const float* bias, float a1, const float* w1, const float* b1,
-                             float a2, const float* w2, const float* b2, hipStream_t s);
+int omnia_tanh_norm_residual(void* h, int f32, float* x, const void* m, int ptype, int S,
+                             int64_t row, int64_t slab, int rows, int d, const float* bias,
+                             float a1, const float* w1, const float* b1, float a2,
+                             const float* w2, const float* b2, hipStream_t s);
 int omnia_bias_swiglu(void* out, int f32, const void* m, int ptype, int S, int rows, int inter,
                       const float* bias, hipStream_t s);
 int omnia_delta_prep(float* qn, float* kn, void* vc, float* decay, float* beta, const void* x,
@@ -153,7 +154,7 @@ int omnia_rms_embed(void* h, float* x, const int* ids, const void* table, int f3
                     const int64_t* src, const int* tok_slots, hipStream_t s);
 int omnia_rms_residual(void* h, int f32, float* x, const void* m, int ptype, int S,
                        int64_t row_stride, int64_t part_stride, int rows, int d,
-                       const float* w_post, const float* w_pre, float inv_n, float eps,
+                       const float* bias, const float* w_post, const float* w_pre, float inv_n, float eps,
                        hipStream_t s);
 int omnia_softcap(void* z, int f32, int64_t n, float cap, hipStream_t s);
 int omnia_gqa_prep(void* q, void* kc, void* vc, int f32, const void* x, int ptype, int S,
@@ -1275,17 +1276,29 @@ void tanh_norm_embed(at::Tensor h, at::Tensor x, at::Tensor ids, at::Tensor tabl
            "tanh_norm_embed");
 }
 
-void tanh_norm_residual(at::Tensor h, at::Tensor x, at::Tensor m, OptT bias, double a1,
+// m: a projection [M, d], split-K slabs [S, M, d], or (slots) per-row parts [M, S, d]
+struct ResidParts { int type; int64_t S, M, d, row, part; };
+ResidParts resid_parts(const at::Tensor& m, bool slots) {
+  const Proj p = proj(m);
+  TORCH_CHECK(!slots || m.dim() == 3, "slots [M, S, d]");
+  const int64_t S = slots ? p.M : p.S, M = slots ? m.size(0) : p.M;
+  return {p.type, S, M, p.N, slots ? S * p.N : p.N, slots ? p.N : M * p.N};
+}
+const float* opt_vecf(const OptT& t, int64_t n, const char* what) {
+  return t.has_value() && t->defined() ? vecf(*t, n, what) : nullptr;
+}
+
+void tanh_norm_residual(at::Tensor h, at::Tensor x, at::Tensor m, bool slots, OptT bias, double a1,
                         at::Tensor w1, at::Tensor b1, double a2, at::Tensor w2, at::Tensor b2) {
   const int f32 = is_f32(h, "h");
-  const Proj p = proj(m);
-  const int64_t d = p.N;
+  const ResidParts p = resid_parts(m, slots);
+  const int64_t d = p.d;
   like(h, h, p.M * d, "h");
   CHECK_RC(omnia_tanh_norm_residual(
-               h.data_ptr(), f32, outf(x, p.M * d, "x"), m.data_ptr(), p.type, p.S, p.M, d,
-               bias.has_value() && bias->defined() ? vecf(*bias, d, "bias") : nullptr, (float)a1,
-               vecf(w1, d, "w1"), vecf(b1, d, "b1"), (float)a2, vecf(w2, d, "w2"),
-               vecf(b2, d, "b2"), cur_stream()), "tanh_norm_residual");
+               h.data_ptr(), f32, outf(x, p.M * d, "x"), m.data_ptr(), p.type, p.S, p.row, p.part,
+               p.M, d, opt_vecf(bias, d, "bias"), (float)a1, vecf(w1, d, "w1"), vecf(b1, d, "b1"),
+               (float)a2, vecf(w2, d, "w2"), vecf(b2, d, "b2"), cur_stream()),
+           "tanh_norm_residual");
 }
 
 void bias_swiglu(at::Tensor out, at::Tensor m, at::Tensor bias) {
@@ -1527,10 +1540,6 @@ void latent_prefill(at::Tensor out, at::Tensor q, at::Tensor kx, at::Tensor kr, 
 }
 
 // ------------------------------------------- RMS norms around an fp32 residual stream
-const float* opt_vecf(const OptT& t, int64_t n, const char* what) {
-  return t.has_value() && t->defined() ? vecf(*t, n, what) : nullptr;
-}
-
 void rms_embed(at::Tensor h, at::Tensor x, at::Tensor ids, at::Tensor table, int64_t vocab,
                OptT w_embed, OptT w_pre, double inv_n, double eps, OptT src, OptT tok_slots) {
   const int f32 = is_f32(table, "table");
@@ -1550,16 +1559,14 @@ void rms_embed(at::Tensor h, at::Tensor x, at::Tensor ids, at::Tensor table, int
                            opt_ptr<int>(tok_slots), cur_stream()), "rms_embed");
 }
 
-// m: projection [M, d], split-K slabs [S, M, d], or (slots) per-token parts [M, S, d]
-void rms_residual(at::Tensor h, at::Tensor x, at::Tensor m, bool slots, at::Tensor w_post,
-                  OptT w_pre, double inv_n, double eps) {
+void rms_residual(at::Tensor h, at::Tensor x, at::Tensor m, bool slots, OptT bias,
+                  at::Tensor w_post, OptT w_pre, double inv_n, double eps) {
   const int f32 = is_f32(h, "h");
-  const Proj p = proj(m);
-  const int64_t d = p.N, S = slots ? p.M : p.S, M = slots ? m.size(0) : p.M;
-  TORCH_CHECK(!slots || m.dim() == 3, "slots [M, S, d]");
-  like(h, h, M * d, "h");
-  CHECK_RC(omnia_rms_residual(h.data_ptr(), f32, outf(x, M * d, "x"), m.data_ptr(), p.type, S,
-                              slots ? S * d : d, slots ? d : M * d, M, d,
+  const ResidParts p = resid_parts(m, slots);
+  const int64_t d = p.d;
+  like(h, h, p.M * d, "h");
+  CHECK_RC(omnia_rms_residual(h.data_ptr(), f32, outf(x, p.M * d, "x"), m.data_ptr(), p.type, p.S,
+                              p.row, p.part, p.M, d, opt_vecf(bias, d, "bias"),
                               vecf(w_post, d, "w_post"), opt_vecf(w_pre, d, "w_pre"),
                               (float)inv_n, (float)eps, cur_stream()), "rms_residual");
 }

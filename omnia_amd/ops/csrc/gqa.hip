@@ -63,7 +63,8 @@ __device__ __forceinline__ int find_seq(const int* q_start, int nseq, int t) {
 }
 
 // ------------------------------------------------------------------- gqa_prep
-// 1 << lg lanes own one head row of one token, 4 columns a lane and step (NC steps).
+// grid (T, groups of 256 >> lg heads): 1 << lg lanes own one head row of a token, 8
+// columns a lane and step (NC steps).
 struct PrepArgs {
   const float* wq;
   const float* wk;       // per-dimension norm weights [Dp]
@@ -71,7 +72,7 @@ struct PrepArgs {
   const int64_t* slots;  // < 0: no write (padded row)
   const float* cos_sin;  // [positions][R] = (cos[R/2] | sin[R/2])
   int64_t ldx, slab;
-  int S, T, H, G, D, Dp, Vp, R, page, lg;
+  int S, H, G, D, Dp, Vp, R, page, lg;
   float eps;
 };
 
@@ -79,40 +80,54 @@ template <typename T, typename P, int NC>
 __global__ __launch_bounds__(256) void prep_kernel(T* __restrict__ q, T* __restrict__ kc,
                                                    T* __restrict__ vc, const P* __restrict__ x,
                                                    PrepArgs a) {
-  __shared__ __attribute__((aligned(16))) float rows[256 * NC * 4];
-  const int lph = 1 << a.lg, l = threadIdx.x & (lph - 1);
+  __shared__ __attribute__((aligned(16))) float rows[256 * NC * 8];
+  const int tid = threadIdx.x, lph = 1 << a.lg, l = tid & (lph - 1), t = blockIdx.x;
   const int NH = a.H + 2 * a.G;
-  const int64_t job = ((int64_t)blockIdx.x * 256 + threadIdx.x) >> a.lg;
-  const bool live = job < (int64_t)a.T * NH;
-  const int t = live ? (int)(job / NH) : 0, hs = live ? (int)(job % NH) : 0;
+  const int hx = blockIdx.y * (256 >> a.lg) + (tid >> a.lg);
+  const bool live = hx < NH;
+  const int hs = live ? hx : 0;
   const bool isq = hs < a.H, isv = hs >= a.H + a.G;
   const int width = isv ? a.Vp : a.Dp;
   const int col = isv ? (a.H + a.G) * a.Dp + (hs - a.H - a.G) * a.Vp : hs * a.Dp;
   const P* xr = x + (int64_t)t * a.ldx + col;
-  float4v v[NC];
+  const float4v zero = {0.f, 0.f, 0.f, 0.f};
+  float4v v[NC][2];
   float ss = 0.f;
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
-    const int c = (l + (i << a.lg)) * 4;
-    v[i] = float4v{0.f, 0.f, 0.f, 0.f};
-    if (c < width) {
-      v[i] = load4(xr + c);
-      for (int s = 1; s < a.S; ++s) v[i] += load4(xr + s * a.slab + c);
+    const int c = (l + (i << a.lg)) * 8;
+    const bool in = c < width;
+    v[i][0] = in ? load4(xr + c) : zero;
+    v[i][1] = in ? load4(xr + c + 4) : zero;
+    for (int s = 1; s < a.S; s += 4) {  // four slabs in flight
+      float4v p[4][2];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) ss += v[i][j] * v[i][j];
+      for (int j = 0; j < 4; ++j) {
+        const bool has = in && s + j < a.S;
+        p[j][0] = has ? load4(xr + (s + j) * a.slab + c) : zero;
+        p[j][1] = has ? load4(xr + (s + j) * a.slab + c + 4) : zero;
+      }
+#pragma unroll
+      for (int e = 0; e < 2; ++e) v[i][e] += (p[0][e] + p[1][e]) + (p[2][e] + p[3][e]);
     }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) ss += v[i][0][j] * v[i][0][j] + v[i][1][j] * v[i][1][j];
   }
-  float* row = rows + (threadIdx.x >> a.lg << a.lg) * NC * 4;
+  const int pos = a.positions[t], half = a.R >> 1, turned = isv ? 0 : a.R;
+  const float* cs = a.cos_sin + (int64_t)pos * a.R;
+  float* row = rows + (tid >> a.lg << a.lg) * NC * 8;
   if (!isv) {
     for (int o = lph >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
     const float r = 1.f / sqrtf(ss / (float)a.D + a.eps);
     const float* w = isq ? a.wq : a.wk;
 #pragma unroll
     for (int i = 0; i < NC; ++i) {
-      const int c = (l + (i << a.lg)) * 4;
+      const int c = (l + (i << a.lg)) * 8;
       if (c < width) {
-        v[i] = v[i] * r * *reinterpret_cast<const float4v*>(w + c);
-        store4(row + c, v[i]);
+        v[i][0] = v[i][0] * r * *reinterpret_cast<const float4v*>(w + c);
+        v[i][1] = v[i][1] * r * *reinterpret_cast<const float4v*>(w + c + 4);
+        store4(row + c, v[i][0]);
+        store4(row + c + 4, v[i][1]);
       }
     }
   }
@@ -124,30 +139,54 @@ __global__ __launch_bounds__(256) void prep_kernel(T* __restrict__ q, T* __restr
   } else {
     const int64_t slot = a.slots[t];
     if (slot < 0) return;
-    const int64_t blk = slot / a.page, off = slot - blk * a.page;
+    const int blk = (int)slot / a.page, off = (int)slot - blk * a.page;
     const int g = isv ? hs - a.H - a.G : hs - a.H;
-    dst = (isv ? vc : kc) + ((blk * a.G + g) * a.page + off) * width;
+    dst = (isv ? vc : kc) + (((int64_t)blk * a.G + g) * a.page + off) * width;
   }
-  const float* cs = a.cos_sin + (int64_t)a.positions[t] * a.R;
-  const int half = a.R >> 1, turned = isv ? 0 : a.R;
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
-    const int c = (l + (i << a.lg)) * 4;
+    const int c = (l + (i << a.lg)) * 8;
     if (c >= width) continue;
-    float4v y = v[i];
     if (c < turned) {
+      if ((half & 7) == 0) {  // a chunk lies in one half of the rotated part
+        const bool first = c < half;
+        const int p = first ? c : c - half;
+        const float sg = first ? -1.f : 1.f;
+        const float* other = row + (first ? c + half : p);
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int e = c + j;
-        if (e < turned) {
-          const bool first = e < half;
-          const int p = first ? e : e - half;
-          const float other = row[first ? e + half : p];
-          y[j] = v[i][j] * cs[p] + (first ? -other : other) * cs[half + p];
+        for (int e = 0; e < 2; ++e) {
+          const float4v cv = *reinterpret_cast<const float4v*>(cs + p + 4 * e);
+          const float4v sv = *reinterpret_cast<const float4v*>(cs + half + p + 4 * e);
+          const float4v ov = *reinterpret_cast<const float4v*>(other + 4 * e);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) v[i][e][j] = v[i][e][j] * cv[j] + sg * ov[j] * sv[j];
         }
+      } else {
+#pragma unroll
+        for (int e = 0; e < 2; ++e)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            const int n = c + 4 * e + j;
+            if (n < turned) {
+              const bool first = n < half;
+              const int p = first ? n : n - half;
+              const float other = row[first ? n + half : p];
+              v[i][e][j] = v[i][e][j] * cs[p] + (first ? -other : other) * cs[half + p];
+            }
+          }
       }
     }
-    store4(dst + c, y);
+    if constexpr (sizeof(T) == 4) {
+      store4(dst + c, v[i][0]);
+      store4(dst + c + 4, v[i][1]);
+    } else {
+      uint4v k;
+      k[0] = pack_bf2(v[i][0][0], v[i][0][1]);
+      k[1] = pack_bf2(v[i][0][2], v[i][0][3]);
+      k[2] = pack_bf2(v[i][1][0], v[i][1][1]);
+      k[3] = pack_bf2(v[i][1][2], v[i][1][3]);
+      *reinterpret_cast<uint4v*>(dst + c) = k;
+    }
   }
 }
 
@@ -389,6 +428,8 @@ __global__ __launch_bounds__(128) void merge_kernel(bf16_t* __restrict__ out,
                                                     const int* __restrict__ positions, int H,
                                                     int Vp, int window, int splits,
                                                     const float* __restrict__ sinks) {
+  extern __shared__ float wt[];  // [splits]
+  __shared__ float scratch[2];
   const int bh = blockIdx.x, b = bh / H, h = bh - b * H;
   const int pos = positions[b];
   const int vis = pos + 1 - (window > 0 ? max(0, pos - window + 1) : 0);
@@ -396,15 +437,27 @@ __global__ __launch_bounds__(128) void merge_kernel(bf16_t* __restrict__ out,
   if (nparts <= 1) return;
   const float* ml = part_ml + (int64_t)bh * splits * 2;
   const float* po = part_o + (int64_t)bh * splits * Vp;
+  const int tid = threadIdx.x;
   const float sk = sinks ? sinks[h] * kLog2e : -INFINITY;
   float m = sk;
-  for (int p = 0; p < nparts; ++p) m = fmaxf(m, ml[2 * p]);
-  float tot = sinks ? exp2f(sk - m) : 0.f;
-  for (int p = 0; p < nparts; ++p) tot += exp2f(ml[2 * p] - m) * ml[2 * p + 1];
+  for (int p = tid; p < nparts; p += 128) m = fmaxf(m, ml[2 * p]);
+  m = block_max(m, scratch);
+  float tot = 0.f;
+  for (int p = tid; p < nparts; p += 128) {
+    wt[p] = exp2f(ml[2 * p] - m);
+    tot += wt[p] * ml[2 * p + 1];
+  }
+  tot = block_sum(tot, scratch) + (sinks ? exp2f(sk - m) : 0.f);  // (orders wt as well)
   const float inv = 1.f / tot;
-  for (int d = threadIdx.x; d < Vp; d += 128) {
+  for (int d = tid; d < Vp; d += 128) {
     float v = 0.f;
-    for (int p = 0; p < nparts; ++p) v += exp2f(ml[2 * p] - m) * po[(int64_t)p * Vp + d];
+    for (int p = 0; p < nparts; p += 8) {  // eight parts in flight
+      float x[8];
+#pragma unroll
+      for (int k = 0; k < 8; ++k) x[k] = po[(int64_t)min(p + k, nparts - 1) * Vp + d];
+#pragma unroll
+      for (int k = 0; k < 8; ++k) v += p + k < nparts ? wt[min(p + k, nparts - 1)] * x[k] : 0.f;
+    }
     out[(int64_t)bh * Vp + d] = f2bf(v * inv);
   }
 }
@@ -424,23 +477,23 @@ int omnia_gqa_prep(void* q, void* kc, void* vc, int f32, const void* x, int ptyp
                    int64_t slab, int64_t ldx, const float* wq, const float* wk,
                    const int* positions, const int64_t* slots, const float* cos_sin, int T, int H,
                    int G, int D, int Dp, int Vp, int R, int page, float eps, hipStream_t s) {
-  if (Dp % 4 || Vp % 4 || ldx % 4 || slab % 4 || S < 1 || R % 2 || R > D || D > Dp || page < 1)
+  if (Dp % 8 || Vp % 8 || ldx % 8 || slab % 8 || S < 1 || R % 2 || R > D || D > Dp || page < 1)
     return -1;
   const int w = Dp > Vp || G == 0 ? Dp : Vp;
   if (w > 1024) return -2;
   if (T == 0) return 0;
-  int lg = 1;
-  while (lg < 6 && (4 << lg) < w) ++lg;
-  const int64_t threads = ((int64_t)T * (H + 2 * G)) << lg;
-  PrepArgs a{wq, wk, positions, slots, cos_sin, ldx, slab, S,  T,  H,  G,
-             D,  Dp, Vp,        R,     page,    lg,  eps};
-  const dim3 grid((unsigned)((threads + 255) / 256));
+  int lg = 2;
+  while (lg < 6 && (8 << lg) < w) ++lg;
+  const PrepArgs a{wq, wk, positions, slots, cos_sin, ldx, slab, S,   H,
+                   G,  D,  Dp,        Vp,    R,       page, lg,  eps};
+  const int hpb = 256 >> lg;
+  const dim3 grid(T, (H + 2 * G + hpb - 1) / hpb);
 #define OMNIA_GP(TT, PP)                                                                       \
   do {                                                                                         \
-    if (w <= 256)                                                                              \
+    if (w <= 512)                                                                              \
       prep_kernel<TT, PP, 1><<<grid, 256, 0, s>>>((TT*)q, (TT*)kc, (TT*)vc, (const PP*)x, a);  \
     else                                                                                       \
-      prep_kernel<TT, PP, 4><<<grid, 256, 0, s>>>((TT*)q, (TT*)kc, (TT*)vc, (const PP*)x, a);  \
+      prep_kernel<TT, PP, 2><<<grid, 256, 0, s>>>((TT*)q, (TT*)kc, (TT*)vc, (const PP*)x, a);  \
   } while (0)
   if (f32) {
     if (ptype != 1) return -3;
@@ -484,7 +537,7 @@ int omnia_gqa_decode(void* out, float* part_o, float* part_ml, const void* q, co
                      const float* sinks, int splits, int max_keys, hipStream_t s) {
   const int lg = log2i(page);
   if (lg < 0 || G < 1 || H % G || Dp % 32 || Dp > 256 || Vp % 8 || Vp > 256 || splits < 1 ||
-      max_keys < 1 || window < 0 || H > 65535 || splits > 65535)
+      max_keys < 1 || window < 0 || H > 65535 || splits > 8192)
     return -1;
   if (T == 0) return 0;
   const int group = H / G, gh = group >= 5 ? 8 : group >= 3 ? 4 : group;
@@ -530,7 +583,7 @@ int omnia_gqa_decode(void* out, float* part_o, float* part_ml, const void* q, co
 #undef OMNIA_GD_N
 #undef OMNIA_GD
   if (splits > 1)
-    merge_kernel<<<T * H, 128, 0, s>>>((bf16_t*)out, part_o, part_ml, positions, H, Vp, window,
+    merge_kernel<<<T * H, 128, splits * 4, s>>>((bf16_t*)out, part_o, part_ml, positions, H, Vp, window,
                                        splits, sinks);
   return (int)hipGetLastError();
 }

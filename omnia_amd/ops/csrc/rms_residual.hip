@@ -5,13 +5,14 @@
 //
 //   rms_embed     token embedding gather [-> norm] -> fp32 residual row, and the first
 //                 sublayer's input (the residual itself, or its pre-norm)
-//   rms_residual  x += norm(sum of m's parts); h = x or pre-norm(x): what follows a
+//   rms_residual  x += norm(sum of m's parts + bias); h = x or pre-norm(x): what follows a
 //                 sublayer, in one pass.  Parts: split-K slabs of a projection, or the
 //                 slots of a token's experts
 //   softcap       logits <- cap * tanh(logits / cap), in place
 //
 // One workgroup per row; a thread keeps its columns in registers between the statistic
-// and the update.
+// and the update.  Few rows (decode): 1024 threads a row, so that a row's loads are all
+// in flight at once.
 #include "common.h"
 
 using namespace omnia;
@@ -46,8 +47,8 @@ struct Norm {
   float inv_n, eps;
 };
 
-// columns of a thread: c = (threadIdx.x + i * 256) * 4, i < NC
-template <int NC>
+// columns of a thread: c = (threadIdx.x + i * NT) * 4, i < NC
+template <int NT, int NC>
 __device__ __forceinline__ void norm_row(float4v (&v)[NC], int d, Norm n, float* scratch) {
   float ss = 0.f;
 #pragma unroll
@@ -58,19 +59,19 @@ __device__ __forceinline__ void norm_row(float4v (&v)[NC], int d, Norm n, float*
   const float r = 1.f / sqrtf(ss * n.inv_n + n.eps);
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
-    const int c = (threadIdx.x + i * 256) * 4;
+    const int c = (threadIdx.x + i * NT) * 4;
     if (c < d) v[i] = v[i] * r * *reinterpret_cast<const float4v*>(n.w + c);
   }
 }
 
-template <typename T, int NC>
-__global__ __launch_bounds__(256) void embed_kernel(T* __restrict__ h, float* __restrict__ x,
+template <typename T, int NT, int NC>
+__global__ __launch_bounds__(NT) void embed_kernel(T* __restrict__ h, float* __restrict__ x,
                                                     const int* __restrict__ ids,
                                                     const T* __restrict__ table, int d, int vocab,
                                                     Norm emb, Norm pre,
                                                     const int64_t* __restrict__ src,
                                                     const int* __restrict__ tok_slots) {
-  __shared__ float scratch[4];
+  __shared__ float scratch[NT / 64];
   const int t = blockIdx.x;
   const int64_t sl = src ? src[t] : -1;
   const int id = sl >= 0 ? tok_slots[sl] : ids[t];
@@ -79,56 +80,69 @@ __global__ __launch_bounds__(256) void embed_kernel(T* __restrict__ h, float* __
   float4v v[NC];
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
-    const int c = (threadIdx.x + i * 256) * 4;
+    const int c = (threadIdx.x + i * NT) * 4;
     v[i] = float4v{0.f, 0.f, 0.f, 0.f};
     if (ok && c < d) v[i] = load4(row + c);
   }
-  if (emb.w) norm_row<NC>(v, d, emb, scratch);
+  if (emb.w) norm_row<NT, NC>(v, d, emb, scratch);
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
-    const int c = (threadIdx.x + i * 256) * 4;
+    const int c = (threadIdx.x + i * NT) * 4;
     if (c < d) store4(x + (int64_t)t * d + c, v[i]);
   }
-  if (pre.w) norm_row<NC>(v, d, pre, scratch);
+  if (pre.w) norm_row<NT, NC>(v, d, pre, scratch);
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
-    const int c = (threadIdx.x + i * 256) * 4;
+    const int c = (threadIdx.x + i * NT) * 4;
     if (c < d) store4(h + (int64_t)t * d + c, v[i]);
   }
 }
 
-template <typename T, typename P, int NC>
-__global__ __launch_bounds__(256) void residual_kernel(T* __restrict__ h, float* __restrict__ x,
+template <typename T, typename P, int NT, int NC>
+__global__ __launch_bounds__(NT) void residual_kernel(T* __restrict__ h, float* __restrict__ x,
                                                        const P* __restrict__ m, int S,
                                                        int64_t row_stride, int64_t part_stride,
-                                                       int d, Norm post, Norm pre) {
-  __shared__ float scratch[4];
+                                                       int d, const float* __restrict__ bias,
+                                                       Norm post, Norm pre) {
+  __shared__ float scratch[NT / 64];
   const int64_t t = blockIdx.x;
   const P* mr = m + t * row_stride;
   float* xr = x + t * d;
-  float4v v[NC];
+  const float4v zero = {0.f, 0.f, 0.f, 0.f};
+  float4v v[NC], old[NC];
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
-    const int c = (threadIdx.x + i * 256) * 4;
-    v[i] = float4v{0.f, 0.f, 0.f, 0.f};
-    if (c < d) {
-      v[i] = load4(mr + c);
-      for (int s = 1; s < S; ++s) v[i] += load4(mr + s * part_stride + c);
+    const int c = (threadIdx.x + i * NT) * 4;
+    v[i] = c < d ? load4(mr + c) : zero;
+    old[i] = c < d ? *reinterpret_cast<const float4v*>(xr + c) : zero;
+    if (bias && c < d) v[i] += *reinterpret_cast<const float4v*>(bias + c);
+  }
+  for (int s = 1; s < S; s += 4) {  // four parts in flight
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+      const int c = (threadIdx.x + i * NT) * 4;
+      if (c < d) {
+        float4v p[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          p[j] = s + j < S ? load4(mr + (s + j) * part_stride + c) : zero;
+        v[i] += (p[0] + p[1]) + (p[2] + p[3]);
+      }
     }
   }
-  norm_row<NC>(v, d, post, scratch);
+  norm_row<NT, NC>(v, d, post, scratch);
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
-    const int c = (threadIdx.x + i * 256) * 4;
+    const int c = (threadIdx.x + i * NT) * 4;
     if (c < d) {
-      v[i] += *reinterpret_cast<const float4v*>(xr + c);
+      v[i] += old[i];
       store4(xr + c, v[i]);
     }
   }
-  if (pre.w) norm_row<NC>(v, d, pre, scratch);
+  if (pre.w) norm_row<NT, NC>(v, d, pre, scratch);
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
-    const int c = (threadIdx.x + i * 256) * 4;
+    const int c = (threadIdx.x + i * NT) * 4;
     if (c < d) store4(h + t * d + c, v[i]);
   }
 }
@@ -150,13 +164,17 @@ __global__ __launch_bounds__(256) void softcap_kernel(T* __restrict__ z, int64_t
 
 }  // namespace
 
-#define OMNIA_NC(K)                          \
-  do {                                       \
-    if (d <= 1024) K(1);                     \
-    else if (d <= 2048) K(2);                \
-    else if (d <= 4096) K(4);                \
-    else if (d <= 8192) K(8);                \
-    else K(16);                              \
+// (threads, chunks of 4 columns a thread) of a row
+#define OMNIA_NC(K)                                 \
+  do {                                              \
+    if (d <= 1024) K(256, 1);                       \
+    else if (rows <= 512 && d <= 4096) K(1024, 1);  \
+    else if (rows <= 512 && d <= 8192) K(1024, 2);  \
+    else if (rows <= 512) K(1024, 4);               \
+    else if (d <= 2048) K(256, 2);                  \
+    else if (d <= 4096) K(256, 4);                  \
+    else if (d <= 8192) K(256, 8);                  \
+    else K(256, 16);                                \
   } while (0)
 
 extern "C" {
@@ -167,14 +185,15 @@ int omnia_rms_embed(void* h, float* x, const int* ids, const void* table, int f3
   if (d % 4 || d < 4 || d > 16384) return -1;
   if (src && !tok_slots) return -2;
   if (T == 0) return 0;
+  const int rows = T;
   const Norm emb{we, inv_n, eps}, pre{wp, inv_n, eps};
-#define OMNIA_EM(N)                                                                             \
+#define OMNIA_EM(NT, N)                                                                            \
   do {                                                                                          \
     if (f32)                                                                                    \
-      embed_kernel<float, N><<<T, 256, 0, s>>>((float*)h, x, ids, (const float*)table, d,       \
+      embed_kernel<float, NT, N><<<T, NT, 0, s>>>((float*)h, x, ids, (const float*)table, d,       \
                                                vocab, emb, pre, src, tok_slots);                \
     else                                                                                        \
-      embed_kernel<bf16_t, N><<<T, 256, 0, s>>>((bf16_t*)h, x, ids, (const bf16_t*)table, d,    \
+      embed_kernel<bf16_t, NT, N><<<T, NT, 0, s>>>((bf16_t*)h, x, ids, (const bf16_t*)table, d,    \
                                                 vocab, emb, pre, src, tok_slots);               \
   } while (0)
   OMNIA_NC(OMNIA_EM);
@@ -185,22 +204,22 @@ int omnia_rms_embed(void* h, float* x, const int* ids, const void* table, int f3
 // ptype: storage of `m` -- 0 bf16, 1 fp32, 2 fp16 (slabs)
 int omnia_rms_residual(void* h, int f32, float* x, const void* m, int ptype, int S,
                        int64_t row_stride, int64_t part_stride, int rows, int d,
-                       const float* w_post, const float* w_pre, float inv_n, float eps,
+                       const float* bias, const float* w_post, const float* w_pre, float inv_n, float eps,
                        hipStream_t s) {
   if (d % 4 || d < 4 || d > 16384 || S < 1 || row_stride % 4 || part_stride % 4 || !w_post)
     return -1;
   if (f32 && ptype != 1) return -2;
   if (rows == 0) return 0;
   const Norm post{w_post, inv_n, eps}, pre{w_pre, inv_n, eps};
-#define OMNIA_RR(TT, PP, N)                                                                  \
-  residual_kernel<TT, PP, N><<<rows, 256, 0, s>>>((TT*)h, x, (const PP*)m, S, row_stride,    \
-                                                  part_stride, d, post, pre)
-#define OMNIA_RRN(N)                                        \
+#define OMNIA_RR(TT, PP, NT, N)                                                                 \
+  residual_kernel<TT, PP, NT, N><<<rows, NT, 0, s>>>((TT*)h, x, (const PP*)m, S, row_stride,    \
+                                                  part_stride, d, bias, post, pre)
+#define OMNIA_RRN(NT, N)                                       \
   do {                                                      \
-    if (f32) OMNIA_RR(float, float, N);                     \
-    else if (ptype == 0) OMNIA_RR(bf16_t, bf16_t, N);       \
-    else if (ptype == 1) OMNIA_RR(bf16_t, float, N);        \
-    else OMNIA_RR(bf16_t, _Float16, N);                     \
+    if (f32) OMNIA_RR(float, float, NT, N);                     \
+    else if (ptype == 0) OMNIA_RR(bf16_t, bf16_t, NT, N);       \
+    else if (ptype == 1) OMNIA_RR(bf16_t, float, NT, N);        \
+    else OMNIA_RR(bf16_t, _Float16, NT, N);                     \
   } while (0)
   OMNIA_NC(OMNIA_RRN);
 #undef OMNIA_RRN

@@ -6,7 +6,8 @@
 //                        layer's normed input
 //   tanh_norm_residual   x += norm1(m + bias); h = norm2(x): the residual update after
 //                        a sublayer and the next sublayer's input in one pass.  `m` is
-//                        a projection's bf16 / fp32 output or its S split-K slabs
+//                        a projection's bf16 / fp32 output, its S split-K slabs or S
+//                        parts per row (the slots of a token's experts)
 //   bias_swiglu          silu(g + bg) * (u + bu) of a [gate | up] projection (same
 //                        inputs as above)
 //
@@ -80,14 +81,14 @@ __global__ __launch_bounds__(256) void embed_kernel(
 
 template <typename T, typename P>
 __global__ __launch_bounds__(256) void residual_kernel(
-    T* __restrict__ h, float* __restrict__ x, const P* __restrict__ m, int S, int64_t slab,
-    int d, const float* __restrict__ bias, float a1, const float* __restrict__ w1,
+    T* __restrict__ h, float* __restrict__ x, const P* __restrict__ m, int S, int64_t row,
+    int64_t slab, int d, const float* __restrict__ bias, float a1, const float* __restrict__ w1,
     const float* __restrict__ b1, float a2, const float* __restrict__ w2,
     const float* __restrict__ b2) {
   const int c = (blockIdx.x * 256 + threadIdx.x) * 4;
   if (c >= d) return;
   const int64_t e = (int64_t)blockIdx.y * d + c;
-  float4v v = sum_slabs(m + e, S, slab);
+  float4v v = sum_slabs(m + blockIdx.y * row + c, S, slab);
   if (bias) v += *reinterpret_cast<const float4v*>(bias + c);
   const float4v r = *reinterpret_cast<const float4v*>(x + e) + norm4(v, a1, w1 + c, b1 + c);
   store4(x + e, r);
@@ -131,16 +132,16 @@ int omnia_tanh_norm_embed(void* h, float* x, const int* ids, const void* table, 
   return (int)hipGetLastError();
 }
 
-int omnia_tanh_norm_residual(void* h, int f32, float* x, const void* m, int ptype, int S, int rows,
-                             int d, const float* bias, float a1, const float* w1, const float* b1,
-                             float a2, const float* w2, const float* b2, hipStream_t s) {
-  if (d % 4 || d < 4 || S < 1 || rows > 65535) return -1;
+int omnia_tanh_norm_residual(void* h, int f32, float* x, const void* m, int ptype, int S,
+                             int64_t row, int64_t slab, int rows, int d, const float* bias,
+                             float a1, const float* w1, const float* b1, float a2,
+                             const float* w2, const float* b2, hipStream_t s) {
+  if (d % 4 || d < 4 || S < 1 || row % 4 || slab % 4 || rows > 65535) return -1;
   if (rows == 0) return 0;
   const dim3 grid((d / 4 + 255) / 256, rows);
-  const int64_t slab = (int64_t)rows * d;
 #define OMNIA_TNR(T, P)                                                                      \
-  residual_kernel<T, P><<<grid, 256, 0, s>>>((T*)h, x, (const P*)m, S, slab, d, bias, a1, w1, \
-                                             b1, a2, w2, b2)
+  residual_kernel<T, P><<<grid, 256, 0, s>>>((T*)h, x, (const P*)m, S, row, slab, d, bias, a1, \
+                                             w1, b1, a2, w2, b2)
   if (f32) {
     if (ptype != 1) return -2;
     OMNIA_TNR(float, float);

@@ -44,13 +44,16 @@ def tanh_norm_embed(ids, table, vocab: int, norm: TanhNorm, src=None, tok_slots=
     return x, ref.tanh_norm(x, *norm.args).to(table.dtype)
 
 
-def tanh_norm_residual(x, m, post: TanhNorm, pre: TanhNorm, dtype, bias=None):
+def tanh_norm_residual(x, m, post: TanhNorm, pre: TanhNorm, dtype, bias=None,
+                       slots: bool = False):
     """In place ``x += post(m + bias)``; returns ``pre(x)`` in ``dtype``.  ``m``: a
-    projection [M, N] or its split-K slabs [S, M, N]."""
+    projection [M, N], its split-K slabs [S, M, N], or (``slots``) parts [M, S, N]."""
     if x.is_cuda:
         h = torch.empty(x.shape, dtype=dtype, device=x.device)
-        kernels().tanh_norm_residual(h, x, m, bias, *post.args, *pre.args)
+        kernels().tanh_norm_residual(h, x, m, slots, bias, *post.args, *pre.args)
         return h
+    if slots:
+        m = m.float().sum(1)
     return ref.tanh_norm_residual(x, m, bias, *post.args, *pre.args, dtype)
 
 
@@ -92,15 +95,18 @@ def rms_embed(ids, table, vocab: int, emb: RMSNorm, pre: RMSNorm | None, src=Non
     return x, (x if pre is None else ref.rms_norm(x, pre)).to(table.dtype)
 
 
-def rms_residual(x, m, post: RMSNorm, pre: RMSNorm | None, dtype, slots: bool = False):
-    """In place ``x += post(m)``; returns ``pre(x)``, or x itself, in ``dtype``.  ``m``: a
+def rms_residual(x, m, post: RMSNorm, pre: RMSNorm | None, dtype, bias=None,
+                 slots: bool = False):
+    """In place ``x += post(m + bias)``; returns ``pre(x)``, or x itself, in ``dtype``.  ``m``: a
     projection [M, d], its split-K slabs [S, M, d], or (``slots``) parts [M, S, d]."""
     if x.is_cuda:
         h = torch.empty(x.shape, dtype=dtype, device=x.device)
-        kernels().rms_residual(h, x, m, slots, post.w, None if pre is None else pre.w,
+        kernels().rms_residual(h, x, m, slots, bias, post.w, None if pre is None else pre.w,
                                post.inv_n, post.eps)
         return h
     v = m.float().sum(1) if slots else ref.slab_sum(m)
+    if bias is not None:
+        v = v + bias
     x += ref.rms_norm(v, post)
     return (x if pre is None else ref.rms_norm(x, pre)).to(dtype)
 
@@ -116,13 +122,8 @@ def norm_embed(ids, table, vocab: int, emb, pre, src=None, tok_slots=None):
 
 def norm_residual(x, m, post, pre, dtype, bias=None, slots: bool = False):
     """What follows a sublayer, of either norm kind (see the two functions above)."""
-    if isinstance(post, TanhNorm):
-        if slots or pre is None:
-            raise ValueError("tanh norms follow a projection and precede a sublayer")
-        return tanh_norm_residual(x, m, post, pre, dtype, bias)
-    if bias is not None:
-        raise ValueError("no bias under an RMS post-norm")
-    return rms_residual(x, m, post, pre, dtype, slots)
+    f = tanh_norm_residual if isinstance(post, TanhNorm) else rms_residual
+    return f(x, m, post, pre, dtype, bias, slots)
 
 
 def softcap_(logits: torch.Tensor, cap: float) -> torch.Tensor:

@@ -67,11 +67,11 @@ def test_rms_residual(n, d, run):
         parts = rnd(S, M, n, g=g, scale=0.05)  # small: eps inside the root matters
         m = pad(parts.transpose(0, 1) if slots else parts)
         m = (m[0] if S == 1 else m).contiguous().to(dev, pdt)
-        wx = x0 + plain.norm_one_plus(parts.sum(0), w1, eps)
-        for pre in (None, w2):
+        for pre, bias in ((None, None), (w2, None), (None, 0.1 * w2)):
+            wx = x0 + plain.norm_one_plus(parts.sum(0) + (0 if bias is None else bias), w1, eps)
             x = pad(x0).float().to(dev)
             h = mops.norm_residual(x, m, norm(w1), None if pre is None else norm(pre), dt,
-                                   slots=slots)
+                                   None if bias is None else pad(bias).float().to(dev), slots)
             wh = wx if pre is None else plain.norm_one_plus(wx, pre, eps)
             assert rel(x[:, :n], wx) < 2e-6 and rel(h[:, :n], wh) < (
                 2e-6 if dt == torch.float32 else 3e-3)

@@ -63,6 +63,11 @@ def test_tanh_norm_residual(d, run):
                                         None if b is None else b.to(dev))
             assert x.dtype == torch.float32 and h.dtype == dt
             assert rel(x, wx) < 1e-6 and rel(h, wh) < (1e-6 if dt == torch.float32 else 4e-3)
+            if S > 1:  # the parts of a row side by side
+                x = x0.to(dev).clone()
+                h2 = mops.norm_residual(x, m.transpose(0, 1).contiguous().to(dev), *norms, dt,
+                                        None if b is None else b.to(dev), slots=True)
+                assert rel(x, wx) < 1e-6 and rel(h2, h.double()) < 4e-3
 
 
 @pytest.mark.parametrize("run", RUNS)
