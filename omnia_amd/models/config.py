@@ -12,8 +12,8 @@ import math
 from dataclasses import dataclass, field
 
 from .layers import (DESIGNS, AttentionSpec, BandSpec, DeltaSpec, DenseMLPSpec, DesignSpec,
-                     ExpertsSpec, LatentAttentionSpec, LayerSpec, RotarySpec, YarnSpec,
-                     tensor_shapes)
+                     ExpertsSpec, LatentAttentionSpec, LayerSpec, LightningSpec, ParallelSpec,
+                     RotarySpec, YarnSpec, looped, tensor_shapes)
 
 
 @dataclass(frozen=True)
@@ -38,6 +38,7 @@ class ModelConfig:
     # layer-list models (models/hybrid.py): one LayerSpec per layer; the uniform
     # head / intermediate sizes above do not apply to them
     layers: tuple = ()
+    logit_scale: float = 1.0  # the head's output times this
     logit_softcap: float = 0.0  # > 0: logits <- cap tanh(logits / cap)
     # tokenizer special ids (llama-3 layout)
     bos_token_id: int = 128000
@@ -64,12 +65,11 @@ class ModelConfig:
     def stateful(self) -> bool:
         """Some layer carries a recurrent state per sequence (beside or instead of
         cached keys): a cached prefix is usable only with the state at its end."""
-        return any(l.mixer.kind == "delta" for l in self.layers)
+        return any(l.mixer.stateful for l in self.layers)
 
     def state_bytes_per_slot(self, dtype_bytes: int = 2) -> int:
-        """Recurrent state of one sequence: fp32 matrices + convolution inputs."""
-        return sum(4 * m.heads * m.dim * m.v_state_pad + dtype_bytes * (m.conv - 1) * m.conv_channels
-                   for m in (l.mixer for l in self.layers) if m.kind == "delta")
+        """Recurrent state of one sequence."""
+        return sum(l.mixer.state_bytes(dtype_bytes) for l in self.layers if l.mixer.stateful)
 
     @property
     def design(self) -> DesignSpec:
@@ -233,11 +233,63 @@ MIXTRAL_3B = ModelConfig(name="mixtral-3b-shape", arch="mixtral", vocab_size=327
                          num_kv_heads=8, num_experts=8, experts_per_token=2, bos_token_id=256,
                          eos_token_ids=(257,))
 
+
+
+def _parallel(heads: int, kv_heads: int, dim: int, window: int, lin_heads: int, base: float,
+              keep: int = 4) -> ParallelSpec:
+    """Windowed attention with kept first tokens beside linear attention whose heads forget
+    over 2 to some thousand tokens."""
+    return ParallelSpec(
+        AttentionSpec(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, scale=dim ** -0.5,
+                      rotary=RotarySpec(dim // 2, base, interleaved=True), window=window,
+                      keep_first=keep, qk_norm=None, bias=True),
+        LightningSpec(heads=lin_heads, dim=dim, vdim=dim, decay=tuple(
+            math.exp(-2.0 ** (-1.0 - 11.0 * i / max(lin_heads - 1, 1)))
+            for i in range(lin_heads))))
+
+
+def _chunked(heads: int, kv_heads: int, dim: int, chunk: int) -> AttentionSpec:
+    return AttentionSpec(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, scale=dim ** 0.5,
+                         rotary=None, sink=False, qk_norm="unit", chunk=chunk)
+
+
+# Bisuzen: tanh pre-normed layer list of attention and linear attention side by side, chunked
+# attention without positions, gelu feed-forwards and grouped experts, looped layers
+TINY_BISUZEN = ModelConfig(
+    name="tiny-bisuzen", arch="bisuzen", vocab_size=512, hidden_size=160, num_layers=7,
+    intermediate_size=208, max_position=4096, logit_scale=0.5, bos_token_id=256,
+    eos_token_ids=(257,),
+    layers=looped((
+        LayerSpec(_parallel(6, 2, 40, 56, 3, 10000.0), DenseMLPSpec(208, "gelu_tanh", False)),
+        LayerSpec(_parallel(4, 1, 48, 32, 2, 10000.0), ExpertsSpec(
+            ff=72, experts=6, top=2, score="softmax", renorm=True, expert="gelu",
+            correction=True, groups=4, keep=2, identity=2)),
+        LayerSpec(_chunked(5, 1, 32, 48), DenseMLPSpec(144, "gelu_tanh", False)),
+        LayerSpec(_chunked(4, 2, 64, 80))), 1, 3, 2))
+# serving-sized shapes (random-init): width, depth and heads of the model named beside each
+BISUZEN_3B = ModelConfig(  # sekazen-3b
+    name="bisuzen-3b", arch="bisuzen", vocab_size=32768, hidden_size=2048, num_layers=16,
+    intermediate_size=4096, max_position=131072, logit_scale=0.25, bos_token_id=256,
+    eos_token_ids=(257,),
+    layers=(LayerSpec(_parallel(16, 8, 128, 1024, 16, 500000.0), ExpertsSpec(
+                ff=6144, experts=8, top=2, score="softmax", renorm=True, expert="gelu",
+                correction=True, groups=2, keep=1, identity=2)),
+            LayerSpec(_chunked(16, 8, 128, 4096), ExpertsSpec(
+                ff=6144, experts=8, top=2, score="softmax", renorm=True, expert="gelu",
+                correction=True, groups=2, keep=1, identity=2))) * 8)
+BISUZEN_8B = ModelConfig(  # sivadra-8b
+    name="bisuzen-8b", arch="bisuzen", vocab_size=128256, hidden_size=4096, num_layers=32,
+    intermediate_size=14336, max_position=131072, logit_scale=0.25, bos_token_id=256,
+    eos_token_ids=(257,),
+    layers=(LayerSpec(_parallel(32, 8, 128, 2048, 32, 500000.0),
+                      DenseMLPSpec(14336, "gelu_tanh", False)),) * 24
+    + (LayerSpec(_chunked(32, 8, 128, 4096), DenseMLPSpec(14336, "gelu_tanh", False)),) * 8)
+
 REGISTRY: dict[str, ModelConfig] = {
     c.name: c for c in [LLAMA3_8B, LLAMA31_8B, LLAMA3_70B, MIXTRAL_8X7B, TINY_LLAMA, TINY_MIXTRAL,
                    TINY_MIXTRAL_E8, EMBED_1B, TINY_EMBED, TINY_LLAMA_H8, TINY_SIVADRA,
                    SIVADRA_1B, SIVADRA_8B, LLAMA_1B, TINY_SEKAZEN, SEKAZEN_3B, SEKAZEN_8X7B,
-                   MIXTRAL_3B]
+                   MIXTRAL_3B, TINY_BISUZEN, BISUZEN_3B, BISUZEN_8B]
 }
 ALIASES = {
     "meta-llama/Meta-Llama-3-8B": "llama-3-8b",

@@ -2,7 +2,7 @@
 a step.
 
 ``forward(w, h, is_decode)`` returns the operands of the residual kernel that follows:
-``{"m": projection, slabs or per-slot parts, "bias": ..., "slots": ...}``.  Padding
+``{"m": projection, slabs or per-slot parts, "bias": ..., "slots": ..., ...}``.  Padding
 happens in ``pack``, as in the mixers.
 """
 from __future__ import annotations
@@ -18,8 +18,8 @@ def _up8(n: int) -> int:
     return (n + 7) // 8 * 8
 
 
-class BiasedSwiGLU:
-    """``W_down(silu(W_gate h + b) * (W_up h + b)) + b``."""
+class DenseGLU:
+    """``W_down(act(W_gate h + b) * (W_up h + b)) + b``, silu or gelu, biases or none."""
 
     def __init__(self, spec, model):
         self.spec, self.model = spec, model
@@ -36,19 +36,22 @@ class BiasedSwiGLU:
             return F.pad(t, (0, width - t.numel())).contiguous()
 
         down = get("down")
-        return {"gate_up": torch.cat([rows("gate"), rows("up")]).contiguous(),
-                "gate_up_b": torch.cat([vec("gate.b", ff), vec("up.b", ff)]),
-                "down": F.pad(down, (0, ff - down.shape[1], 0, d - down.shape[0])).contiguous(),
-                "down_b": vec("down.b", d)}
+        w = {"gate_up": torch.cat([rows("gate"), rows("up")]).contiguous(),
+             "gate_up_b": None, "down_b": None,
+             "down": F.pad(down, (0, ff - down.shape[1], 0, d - down.shape[0])).contiguous()}
+        if self.spec.bias:
+            w["gate_up_b"] = torch.cat([vec("gate.b", ff), vec("up.b", ff)])
+            w["down_b"] = vec("down.b", d)
+        return w
 
     def _act(self, h, w: dict, is_decode) -> torch.Tensor:
         """One fused prefill GEMM, or a GEMM whose bias / activation kernel also reduces
         split-K slabs."""
-        m, W, b = self.model, w["gate_up"], w["gate_up_b"]
+        m, W, b, act = self.model, w["gate_up"], w["gate_up_b"], self.spec.act
         M, K = h.shape
         N = W.shape[0]
-        if m._pgemm_ok(M, K, N // 2, is_decode, 128):
-            return ops.pgemm(1, h, W, bias=b)
+        if m._pgemm_ok(M, K, N // 2, is_decode, 128) and (b is None or act == "silu"):
+            return ops.pgemm(1, h, W, bias=b, gelu=act == "gelu_tanh")
         cfg = m._wcfg(M, N // 2, K, 1, is_decode)
         if cfg is not None:  # a tuned SwiGLU shape, as slabs (bias and activation follow)
             nw, nwaves, S = cfg
@@ -56,7 +59,7 @@ class BiasedSwiGLU:
                          out=m._parts("gu", S, M, N, m._slab_dtype(nwaves)))
         else:
             p = m._slabs("gate_up", h, W, is_decode)
-        return mops.bias_swiglu(p, b, m.dtype)
+        return mops.glu(p, b, m.dtype, act)
 
     def forward(self, w: dict, h: torch.Tensor, is_decode: bool) -> dict:
         a = self._act(h, w, is_decode)
@@ -64,7 +67,7 @@ class BiasedSwiGLU:
 
 
 class Experts:
-    """Sparse mixture of clamped GLUs (grouped MFMA kernels, no host sync)."""
+    """Sparse mixture of small feed-forwards (grouped MFMA kernels, no host sync)."""
 
     def __init__(self, spec, model):
         self.spec, self.model = spec, model
@@ -73,18 +76,26 @@ class Experts:
         s, m = self.spec, self.model
         E, ff, fp = s.experts, s.ff, s.ff_pad
         r = get("router")
-        gu = torch.zeros(E, 2 * fp, d, dtype=m.dtype, device=m.device)
+        ups = ["gate", "up"] if s.gated else ["up"]  # rows of one expert's first product
+        up = torch.zeros(E, len(ups) * fp, d, dtype=m.dtype, device=m.device)
         down = torch.zeros(E, d, fp, dtype=m.dtype, device=m.device)
         for e in range(E):
-            t = get(f"e{e}.gate")
-            gu[e, :ff, :t.shape[1]] = t
-            gu[e, fp:fp + ff, :t.shape[1]] = get(f"e{e}.up")
+            for i, n in enumerate(ups):
+                t = get(f"e{e}.{n}")
+                up[e, i * fp:i * fp + ff, :t.shape[1]] = t
             t = get(f"e{e}.down")
             down[e, :t.shape[0], :ff] = t
-        return {"router": F.pad(r, (0, d - r.shape[1])).contiguous(), "gate_up": gu, "down": down}
+        w = {"router": F.pad(r, (0, d - r.shape[1])).contiguous(), "up": up, "down": down}
+        if s.correction:
+            w["correction"] = get("correction").float().contiguous()
+        return w
 
     def forward(self, w: dict, h: torch.Tensor, is_decode: bool) -> dict:
-        return {"m": mops.experts(h, w, self.spec), "slots": True}
+        parts, ids, wts = mops.experts(h, w, self.spec)
+        out = {"m": parts, "slots": True}
+        if self.spec.identity:
+            out["identity"] = (ids, wts, h, self.spec.experts)
+        return out
 
 
-MLPS = {"dense": BiasedSwiGLU, "moe": Experts}
+MLPS = {"dense": DenseGLU, "moe": Experts}

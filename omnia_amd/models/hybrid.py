@@ -1,19 +1,20 @@
-"""Layer-list models (``ModelConfig.layers``) on the engine's paged cache: Sivadra, Sekazen.
+"""Layer-list models (``ModelConfig.layers``) on the engine's paged cache: Sivadra, Sekazen,
+Bisuzen.
 
 Every layer is ``x += post(mixer(pre(x)))`` and, with a feed-forward,
 ``x += post(ff(pre(x)))`` around an fp32 residual stream; mixers
 (:mod:`omnia_amd.models.mixers`) and feed-forwards (:mod:`omnia_amd.models.feedforward`)
-are chosen per layer, norms and head per family (``layers.DesignSpec``).  The
-post-norm, the residual update and the next sublayer's pre-norm (if the family has
-one) are one kernel behind each sublayer, which also reduces split-K slabs or sums a
-token's experts:
+are chosen per layer, norms and head per family (``layers.DesignSpec``; either norm may be
+missing).  The post-norm, the residual update and the next sublayer's pre-norm are one
+kernel behind each sublayer, which also reduces split-K slabs, sums a token's experts or
+joins the two branches of a parallel mixer:
 
     norm_embed -> [ in GEMM -> mixer kernels -> o GEMM -> norm_residual
                     (-> feed-forward -> norm_residual) ] * layers -> head GEMM
                     (-> softcap)
 
-A layer may use another layer's tensors (its pages / state are its own), or attend to
-another layer's pages.  bf16 models keep what feeds a softmax, a router or a recurrence
+A layer may use another layer's tensors (its pages / state are its own; the later passes
+of a looped layer do), or attend to another layer's pages.  bf16 models keep what feeds a softmax, a router or a recurrence
 in fp32; fp32 models run every kernel and GEMM in fp32.
 """
 from __future__ import annotations
@@ -58,6 +59,7 @@ class HybridCache:
 def random_tensor(name: str, shape: tuple, cfg: ModelConfig, gen, device) -> torch.Tensor:
     """Random-init checkpoint tensor (no checkpoint at hand), fp32."""
     leaf = name.split(".", 1)[1] if "." in name else name
+    leaf = leaf.replace("mix.left.", "mix.").replace("mix.right.", "mix.")
     if leaf.endswith("alpha"):
         return torch.full(shape, 0.5, device=device)
     if leaf == "mix.sink" or (cfg.design.norm == "rms" and leaf.startswith("norm")):
@@ -66,14 +68,14 @@ def random_tensor(name: str, shape: tuple, cfg: ModelConfig, gen, device) -> tor
         return torch.zeros(shape, device=device) if leaf.endswith(".b") else \
             torch.ones(shape, device=device)
     t = torch.empty(shape, device=device)
-    if leaf == "mix.norm":
+    if leaf in ("mix.norm", "mix.out"):
         return t.fill_(1.0)
     if leaf == "mix.A_log":
         return t.uniform_(1.0, 16.0, generator=gen).log_()
     if leaf == "mix.dt_bias":  # softplus^-1 of step sizes in [1e-3, 1e-1]
         dt = t.uniform_(math.log(1e-3), math.log(1e-1), generator=gen).exp_()
         return dt + torch.log(-torch.expm1(-dt))
-    if leaf.endswith(".b"):
+    if leaf.endswith(".b") or leaf == "mlp.correction":
         return t.zero_()
     if leaf.endswith(".conv"):
         return t.normal_(0.0, shape[1] ** -0.5, generator=gen)
@@ -148,13 +150,13 @@ class HybridModel(Projections):
             t = t.float()
             return F.pad(t, (0, d - t.numel())).contiguous()
 
-        def norm(name):
+        def norm(name, scale=1.0):
             if name is None:
                 return None
             if design.norm == "tanh":
-                return mops.TanhNorm(float(raw(name + ".alpha")), vec(raw(name)),
-                                     vec(raw(name + ".b")))
-            return mops.RMSNorm(vec(1.0 + raw(name).float()), cfg.hidden_size, cfg.rms_eps)
+                return mops.TanhNorm(float(raw(name + ".alpha")), scale * vec(raw(name)),
+                                     scale * vec(raw(name + ".b")))
+            return mops.RMSNorm(scale * vec(1.0 + raw(name).float()), cfg.hidden_size, cfg.rms_eps)
 
         def norms(p, k):
             return [norm(p + n if n else None) for n in design.sublayer_norms(k)]
@@ -162,13 +164,16 @@ class HybridModel(Projections):
         def cols(t):
             return F.pad(t, (0, d - t.shape[1])).contiguous()
 
-        w = {"embed": cols(raw("embed")), "layers": [], "final_norm": norm("final.norm"),
+        w = {"embed": cols(raw("embed")), "layers": [],
+             # the head is linear: its scale rides the norm before it
+             "final_norm": norm("final.norm", cfg.logit_scale),
              "embed_norm": norm("embed.norm") if design.embed_norm else None}
         w["head"] = w["embed"] if design.tied else cols(raw("head"))
         for i, l in enumerate(cfg.layers):
             own = i if l.weights_of is None else l.weights_of
             if own not in seen:
-                p = f"l{own}."
+                n = cfg.layers[own].index
+                p = f"l{own if n is None else n}."
                 layer = {"mix": self.mixers[i].pack(part(p + "mix."), d), "mlp": None}
                 layer["pre1"], layer["post1"] = norms(p, 1)
                 if l.mlp is not None:
@@ -207,9 +212,8 @@ class HybridModel(Projections):
                                self.w["embed_norm"], ws[0]["pre1"], fb.ids_src, fb.tok_slots)
         for i, (w, mixer, mlp) in enumerate(zip(ws, self.mixers, self.mlps)):
             after = ws[i + 1]["pre1"] if i + 1 < len(ws) else self.w["final_norm"]
-            o = mixer.forward(w["mix"], h, fb, kv.layers[i])
-            h = mops.norm_residual(x, self._slabs("o", o, w["mix"]["o"], dec), w["post1"],
-                                   w["pre2"] if mlp else after, dt)
+            h = mops.norm_residual(x, post=w["post1"], pre=w["pre2"] if mlp else after, dtype=dt,
+                                   **mixer.sublayer(w["mix"], h, fb, kv.layers[i]))
             if mlp:
                 h = mops.norm_residual(x, post=w["post2"], pre=after, dtype=dt,
                                        **mlp.forward(w["mlp"], h, dec))

@@ -9,7 +9,7 @@ the checkpoint's ``config.json`` builds them here.
 from __future__ import annotations
 
 import math
-from dataclasses import dataclass
+from dataclasses import dataclass, replace
 
 
 # head widths the MFMA prefill attention is instantiated for (latent.hip); wider
@@ -61,12 +61,14 @@ class BandSpec:
 
 @dataclass(frozen=True)
 class RotarySpec:
-    """Rotate-half rotary positions over ``dims`` dimensions."""
+    """Rotary positions over ``dims`` dimensions: pairs (i, i + dims / 2), or, if
+    ``interleaved``, neighbours (2i, 2i + 1)."""
 
     dims: int
     base: float
     yarn: YarnSpec | None = None
     bands: BandSpec | None = None
+    interleaved: bool = False
 
     def frequencies(self) -> list[float]:
         """Angle per position of every rotated pair (double precision)."""
@@ -115,6 +117,7 @@ class LatentAttentionSpec:
 
     kind = "latent_attention"
     kv_from = None
+    stateful = False
 
     # Kernel geometry: every operand is zero-padded at load (weight rows / columns)
     # so that the MFMA tiles never see a ragged edge and rows stay 16-B aligned.
@@ -164,6 +167,7 @@ class DeltaSpec:
 
     kind = "delta"
     kv_from = None
+    stateful = True
     padded_cache_width = 0  # no pages
 
     @property
@@ -182,26 +186,91 @@ class DeltaSpec:
     def v_pad(self) -> int:  # one head of the output projection's input
         return _up(self.vdim, 8)
 
+    def state_bytes(self, dtype_bytes: int) -> int:
+        """fp32 matrices and convolution inputs of one sequence."""
+        return (4 * self.heads * self.dim * self.v_state_pad
+                + dtype_bytes * (self.conv - 1) * self.conv_channels)
+
+
+@dataclass(frozen=True)
+class LightningSpec:
+    """Linear attention with one fixed ``decay`` per head: a ``dim x vdim`` fp32 state
+    ``S <- decay S + k v^T`` read as ``S^T q``, silu on q, k and v, one RMS norm over all
+    heads together and a sigmoid output gate."""
+
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple
+
+    kind = "lightning"
+    kv_from = None
+    stateful = True
+    padded_cache_width = 0  # no pages
+
+    # whole 16-B chunks of a projection row
+    @property
+    def dim_pad(self) -> int:
+        return _up(self.dim, 8)
+
+    @property
+    def v_pad(self) -> int:
+        return _up(self.vdim, 8)
+
+    @property
+    def in_cols(self) -> int:
+        """[q | k | v | gate] of one projected row."""
+        return 2 * self.heads * (self.dim_pad + self.v_pad)
+
+    def state_bytes(self, dtype_bytes: int) -> int:
+        return 4 * self.heads * self.dim_pad * self.v_pad
+
 
 @dataclass(frozen=True)
 class AttentionSpec:
     """Grouped-query attention over paged keys and values: ``kv_heads`` key/value heads
-    shared by ``heads`` query heads, per-head RMS norms of queries and keys, rotary on
-    the first ``rotary.dims`` dimensions, a sliding ``window`` (0 = the whole past) and,
-    with ``sink``, a learned number per head in the softmax denominator.  ``kv_from``:
-    the layer whose cached keys and values this one attends to instead of its own."""
+    shared by ``heads`` query heads.
+
+    ``qk_norm``: per-head RMS norms of queries and keys, with a learned ``"weight"``,
+    ``"unit"`` (none) or None.  ``rotary`` on the first ``rotary.dims`` dimensions, or
+    None.  ``bias``: on all four projections.  A query sees its last ``window`` positions
+    (0 = the whole past) and the sequence's first ``keep_first``, or, with ``chunk``, the
+    positions of its own chunk of that many up to itself.  ``sink``: a learned number per
+    head in the softmax denominator.  ``kv_from``: the layer whose cached keys and values
+    this one attends to instead of its own."""
 
     heads: int
     kv_heads: int
     dim: int
     vdim: int
     scale: float
-    rotary: RotarySpec
+    rotary: RotarySpec | None
     window: int = 0
     sink: bool = True
     kv_from: int | None = None
+    qk_norm: str | None = "weight"
+    bias: bool = False
+    keep_first: int = 0
+    chunk: int = 0
 
     kind = "attention"
+    stateful = False
+
+    @property
+    def mask(self) -> tuple[int, int, int]:
+        return self.window, self.keep_first, self.chunk
+
+    def most_visible(self, keys: int) -> int:
+        """Most keys a query sees of a context of ``keys``."""
+        if self.chunk:
+            return min(keys, self.chunk)
+        return min(keys, self.window + self.keep_first) if self.window else keys
+
+    @property
+    def in_cols(self) -> int:
+        """[q | k | v] of one projected row."""
+        own = 0 if self.kv_from is not None else self.kv_heads * (self.dim_pad + self.v_pad)
+        return self.heads * self.dim_pad + own
 
     @property
     def dim_pad(self) -> int:
@@ -218,31 +287,77 @@ class AttentionSpec:
 
 
 @dataclass(frozen=True)
+class ParallelSpec:
+    """Two mixers side by side on the same input; their outputs, each RMS-normed over the
+    model width, are averaged."""
+
+    left: object
+    right: object
+
+    kind = "parallel"
+    kv_from = None
+
+    @property
+    def stateful(self) -> bool:
+        return self.left.stateful or self.right.stateful
+
+    @property
+    def padded_cache_width(self) -> int:
+        return self.left.padded_cache_width + self.right.padded_cache_width
+
+    def state_bytes(self, dtype_bytes: int) -> int:
+        return sum(m.state_bytes(dtype_bytes) for m in (self.left, self.right) if m.stateful)
+
+
+@dataclass(frozen=True)
 class DenseMLPSpec:
-    """``W_down(silu(W_gate h + b) * (W_up h + b)) + b``."""
+    """``W_down(act(W_gate h + b) * (W_up h + b)) + b``, the biases if ``bias``; ``act``
+    is silu or the tanh form of gelu (``gelu_tanh``)."""
 
     ff: int
+    act: str = "silu"
+    bias: bool = True
 
     kind = "dense"
 
 
 @dataclass(frozen=True)
 class ExpertsSpec:
-    """Mixture of ``experts`` clamped GLUs, ``top`` per token.  Routing scores are
-    ``sigmoid`` or ``softmax`` of fp32 logits, renormalised over the chosen experts if
-    asked; a token's weight multiplies its expert's input.  Expert:
-    ``W_down(g sigmoid(alpha g) (u + 1))`` with ``g = min(W_gate h, limit)`` and
-    ``u = clamp(W_up h, -limit, limit)``."""
+    """Mixture of ``experts`` small feed-forwards, ``top`` per token.
+
+    ``expert`` "clamped_glu": ``W_down(g sigmoid(alpha g) (u + 1))`` with ``g = min(W_gate
+    h, limit)`` and ``u = clamp(W_up h, -limit, limit)``, a token's weight on its expert's
+    input; "gelu": ``W_down gelu(W_up h)`` (erf form), the weight on the output.
+
+    Routing scores are ``sigmoid`` or ``softmax`` of fp32 logits, renormalised over the
+    chosen experts if asked.  ``correction``: a learned number per expert joins the score
+    for the choice alone.  The choice is limited to the ``keep`` best of ``groups`` equal
+    groups of neighbours (a group counts as its best choice score).  The last ``identity``
+    router outputs are experts that return their input."""
 
     ff: int
     experts: int
     top: int
-    limit: float
+    limit: float = 0.0
     alpha: float = 1.702
     score: str = "sigmoid"
     renorm: bool = False
+    expert: str = "clamped_glu"
+    correction: bool = False
+    groups: int = 1
+    keep: int = 1
+    identity: int = 0
 
     kind = "moe"
+
+    @property
+    def outputs(self) -> int:
+        """Router outputs."""
+        return self.experts + self.identity
+
+    @property
+    def gated(self) -> bool:
+        return self.expert == "clamped_glu"
 
     @property
     def ff_pad(self) -> int:  # whole k-tiles of the grouped GEMMs
@@ -251,29 +366,30 @@ class ExpertsSpec:
 
 @dataclass(frozen=True)
 class LayerSpec:
-    mixer: object  # LatentAttentionSpec | DeltaSpec | AttentionSpec
+    mixer: object  # a mixer spec
     mlp: object | None = None  # DenseMLPSpec | ExpertsSpec | None
     weights_of: int | None = None  # share layer j's tensors (own cache / state)
+    index: int | None = None  # number in the checkpoint's tensor names (None: its place)
 
 
 @dataclass(frozen=True)
 class DesignSpec:
-    """What a layer-list family fixes around its layers."""
+    """What a layer-list family fixes around its layers, and which checkpoint entries
+    its ``config.json`` may hold (the same entry name can mean different mixers)."""
 
     norm: str  # "tanh": Dynamic Tanh; "rms": RMS with a weight stored around zero
     pre_norm: bool  # sublayers read the normed residual (else the residual itself)
     embed_norm: bool  # the residual starts at norm(embedding)
     tied: bool  # the embedding table is the output head
+    mixers: dict
+    mlps: dict
+    post_norm: bool = True  # a sublayer's output is normed before it is added
 
-    def sublayer_norms(self, k: int) -> tuple[str | None, str]:
+    def sublayer_norms(self, k: int) -> tuple[str | None, str | None]:
         """(pre, post) norm names of a layer's k-th sublayer (1 mixer, 2 feed-forward)."""
+        if not self.post_norm:
+            return f"norm{k}", None
         return (f"norm{k}", f"norm{k}b") if self.pre_norm else (None, f"norm{k}")
-
-
-DESIGNS = {
-    "sivadra": DesignSpec("tanh", pre_norm=True, embed_norm=False, tied=False),
-    "sekazen": DesignSpec("rms", pre_norm=False, embed_norm=True, tied=True),
-}
 
 
 # ------------------------------------------------------------ config.json reader
@@ -323,32 +439,119 @@ def _attention(c: dict) -> AttentionSpec:
     return spec
 
 
+def _grouped(spec: AttentionSpec) -> AttentionSpec:
+    if spec.kv_heads < 1 or spec.heads % spec.kv_heads:
+        raise ValueError(f"attention: {spec.heads} heads over {spec.kv_heads} k/v heads")
+    rot = spec.rotary
+    if rot is not None and (rot.dims % 2 or not 0 < rot.dims <= spec.dim):
+        raise ValueError(f"attention: rot.dims {rot.dims} of dim {spec.dim}")
+    return spec
+
+
+def _chunked_attention(c: dict) -> AttentionSpec:
+    return _grouped(AttentionSpec(
+        heads=int(c["heads"]), kv_heads=int(c["kv_heads"]), dim=int(c["dim"]),
+        vdim=int(c["vdim"]), scale=float(c["scale"]), rotary=None, sink=False, qk_norm="unit",
+        chunk=int((c.get("mask") or {}).get("size") or 0)))
+
+
+def _anchored_attention(c: dict) -> AttentionSpec:
+    mask = c.get("mask") or {}
+    rot = c.get("rot")
+    return _grouped(AttentionSpec(
+        heads=int(c["heads"]), kv_heads=int(c["kv_heads"]), dim=int(c["dim"]),
+        vdim=int(c["vdim"]), scale=float(c["scale"]),
+        rotary=replace(_rotary(rot), interleaved=True) if rot and int(rot["dims"]) else None,
+        window=int(mask.get("size") or 0), keep_first=int(mask.get("keep_first") or 0),
+        sink=True, qk_norm=None, bias=True))
+
+
+def _lightning(c: dict) -> LightningSpec:
+    spec = LightningSpec(heads=int(c["heads"]), dim=int(c["dim"]), vdim=int(c["vdim"]),
+                         decay=tuple(float(x) for x in c["decay"]))
+    if len(spec.decay) != spec.heads or not all(0.0 <= x <= 1.0 for x in spec.decay):
+        raise ValueError(f"lightning: {spec.heads} heads need as many decays in [0, 1]")
+    return spec
+
+
+def _parallel(c: dict) -> ParallelSpec:
+    return ParallelSpec(_anchored_attention(c["left"]), _lightning(c["right"]))
+
+
 def _dense(c: dict) -> DenseMLPSpec:
     return DenseMLPSpec(int(c["ff"]))
 
 
-def _experts(c: dict) -> ExpertsSpec:
-    e, r = c["expert"], c["router"]
-    spec = ExpertsSpec(ff=int(e["ff"]), experts=int(r["experts"]), top=int(r["top"]),
-                       limit=float(e["limit"]))
-    if not 1 <= spec.top <= min(spec.experts, 64) or spec.experts > 256:
-        raise ValueError(f"moe: top {spec.top} of {spec.experts} experts")
+def _dense_gelu(c: dict) -> DenseMLPSpec:
+    return DenseMLPSpec(int(c["ff"]), act="gelu_tanh", bias=False)
+
+
+def _checked(spec: ExpertsSpec) -> ExpertsSpec:
+    n, g = spec.outputs, spec.groups
+    if not 1 <= spec.top <= min(n, 64) or n > 256 or spec.experts < 1 or spec.identity < 0:
+        raise ValueError(f"moe: top {spec.top} of {n} experts")
+    if g < 1 or n % g or not 1 <= spec.keep <= g or spec.top > spec.keep * (n // g):
+        raise ValueError(f"moe: top {spec.top} in {spec.keep} of {g} groups of {n} experts")
     return spec
 
 
-MIXER_SPECS = {"latent_attention": _latent_attention, "delta": _delta, "attention": _attention}
-MLP_SPECS = {"dense": _dense, "moe": _experts}
+def _gelu_experts(c: dict) -> ExpertsSpec:
+    e, r = c["expert"], c["router"]
+    g = r.get("groups") or {"count": 1, "keep": 1}
+    return _checked(ExpertsSpec(
+        ff=int(e["ff"]), experts=int(r["experts"]), top=int(r["top"]), score="softmax",
+        renorm=True, expert="gelu", correction=True, groups=int(g["count"]), keep=int(g["keep"]),
+        identity=int(r.get("identity") or 0)))
 
 
-def parse_layers(entries: list[dict]) -> tuple[LayerSpec, ...]:
-    """``config.json`` ``layers`` -> specs.  ``weights_of`` chains are resolved to
-    the layer that owns the tensors."""
+def _experts(c: dict) -> ExpertsSpec:
+    e, r = c["expert"], c["router"]
+    return _checked(ExpertsSpec(ff=int(e["ff"]), experts=int(r["experts"]), top=int(r["top"]),
+                                limit=float(e["limit"])))
+
+
+DESIGNS = {
+    "sivadra": DesignSpec("tanh", pre_norm=True, embed_norm=False, tied=False,
+                          mixers={"latent_attention": _latent_attention, "delta": _delta},
+                          mlps={"dense": _dense}),
+    "sekazen": DesignSpec("rms", pre_norm=False, embed_norm=True, tied=True,
+                          mixers={"attention": _attention}, mlps={"moe": _experts}),
+    "bisuzen": DesignSpec("tanh", pre_norm=True, post_norm=False, embed_norm=False, tied=False,
+                          mixers={"attention": _chunked_attention, "parallel": _parallel},
+                          mlps={"dense": _dense_gelu, "moe": _gelu_experts}),
+}
+
+
+def _run_order(n: int, loop: dict | None) -> list[int]:
+    """Checkpoint layers in the order they run: ``start`` .. ``stop`` - 1 ``times`` times."""
+    if not loop:
+        return list(range(n))
+    a, b, times = int(loop["start"]), int(loop["stop"]), int(loop["times"])
+    if not 0 <= a <= b <= n or times < 1:
+        raise ValueError(f"loop {a} .. {b} x {times} of {n} layers")
+    return list(range(a)) + list(range(a, b)) * times + list(range(b, n))
+
+
+def looped(layers: tuple, start: int, stop: int, times: int) -> tuple[LayerSpec, ...]:
+    """A preset's layers with a loop unrolled, as :func:`parse_layers` does."""
     out: list[LayerSpec] = []
+    for at, i in enumerate(_run_order(len(layers), dict(start=start, stop=stop, times=times))):
+        again = at >= stop and start <= i < stop
+        out.append(replace(layers[i], weights_of=i if again else None, index=i))
+    return tuple(out)
+
+
+def parse_layers(entries: list[dict], design: DesignSpec,
+                 loop: dict | None = None) -> tuple[LayerSpec, ...]:
+    """``config.json`` ``layers`` (and ``loop``) -> the layers in the order they run.
+    ``weights_of`` chains are resolved to the layer that owns the tensors; a layer's later
+    passes use the tensors of its first, with a cache or state of their own."""
+    owners: list = []
     for i, e in enumerate(entries):
-        if e["type"] not in MIXER_SPECS:
+        if e["type"] not in design.mixers:
             raise ValueError(f"layer {i}: unknown mixer {e['type']!r}")
         mlp = e.get("mlp")
-        if mlp is not None and mlp.get("kind") not in MLP_SPECS:
+        if mlp is not None and mlp.get("kind") not in design.mlps:
             raise ValueError(f"layer {i}: unknown feed-forward {mlp.get('kind')!r}")
         owner = e.get("weights_of")
         if owner is not None:
@@ -361,8 +564,23 @@ def parse_layers(entries: list[dict]) -> tuple[LayerSpec, ...]:
                     raise ValueError(f"layer {i}: weights_of cycle")
                 seen.add(owner)
                 owner = int(entries[owner]["weights_of"])
-        out.append(LayerSpec(MIXER_SPECS[e["type"]](e["mixer"]),
-                             None if mlp is None else MLP_SPECS[mlp["kind"]](mlp), owner))
+        owners.append(owner)
+    order = _run_order(len(entries), loop)
+    first: dict = {}
+    for at, i in enumerate(order):
+        first.setdefault(i, at)
+    out: list[LayerSpec] = []
+    last: dict = {}  # latest pass of a checkpoint layer so far
+    for at, i in enumerate(order):
+        e = entries[i]
+        mixer = design.mixers[e["type"]](e["mixer"])
+        if mixer.kv_from is not None and loop:
+            mixer = replace(mixer, kv_from=last.get(mixer.kv_from, -1))
+        owner = owners[i] if owners[i] is not None else i
+        out.append(LayerSpec(
+            mixer, None if e.get("mlp") is None else design.mlps[e["mlp"]["kind"]](e["mlp"]),
+            None if first[owner] == at else first[owner], i if loop else None))
+        last[i] = at
     for i, l in enumerate(out):
         if l.weights_of is not None:
             o = out[l.weights_of]
@@ -392,12 +610,27 @@ def _mixer_shapes(m, d: int) -> dict[str, tuple]:
                 "uk": (m.heads * m.dim, m.kv_rank), "uv": (m.heads * m.vdim, m.kv_rank),
                 "g": (m.heads, d), "o": (d, m.heads * m.vdim)}
     if m.kind == "attention":
-        out = {"q": (m.heads * m.dim, d), "q.norm": (m.dim,), "o": (d, m.heads * m.vdim)}
+        out = {"q": (m.heads * m.dim, d), "o": (d, m.heads * m.vdim)}
         if m.kv_from is None:
-            out.update({"k": (m.kv_heads * m.dim, d), "k.norm": (m.dim,),
-                        "v": (m.kv_heads * m.vdim, d)})
+            out.update({"k": (m.kv_heads * m.dim, d), "v": (m.kv_heads * m.vdim, d)})
+        if m.bias:
+            out.update({n + ".b": (w[0],) for n, w in list(out.items())})
+        if m.qk_norm == "weight":
+            out["q.norm"] = (m.dim,)
+            if m.kv_from is None:
+                out["k.norm"] = (m.dim,)
         if m.sink:
             out["sink"] = (m.heads,)
+        return out
+    if m.kind == "lightning":
+        hd, hv = m.heads * m.dim, m.heads * m.vdim
+        return {"q": (hd, d), "k": (hd, d), "v": (hv, d), "g": (hv, d), "norm": (hv,),
+                "o": (d, hv)}
+    if m.kind == "parallel":
+        out = {}
+        for side, sub in (("left.", m.left), ("right.", m.right)):
+            out.update({side + n: s for n, s in _mixer_shapes(sub, d).items()})
+            out[side + "out"] = (d,)
         return out
     kd, hv = m.kv_heads * m.dim, m.heads * m.vdim
     return {"q": (kd, d), "q.conv": (kd, m.conv), "k": (kd, d), "k.conv": (kd, m.conv),
@@ -408,12 +641,18 @@ def _mixer_shapes(m, d: int) -> dict[str, tuple]:
 
 def _mlp_shapes(m, d: int) -> dict[str, tuple]:
     if m.kind == "moe":
-        out = {"router": (m.experts, d)}
+        out = {"router": (m.outputs, d)}
+        if m.correction:
+            out["correction"] = (m.outputs,)
         for e in range(m.experts):
-            out.update({f"e{e}.gate": (m.ff, d), f"e{e}.up": (m.ff, d), f"e{e}.down": (d, m.ff)})
+            if m.gated:
+                out[f"e{e}.gate"] = (m.ff, d)
+            out.update({f"e{e}.up": (m.ff, d), f"e{e}.down": (d, m.ff)})
         return out
-    return {"gate": (m.ff, d), "gate.b": (m.ff,), "up": (m.ff, d), "up.b": (m.ff,),
-            "down": (d, m.ff), "down.b": (d,)}
+    out = {"gate": (m.ff, d), "up": (m.ff, d), "down": (d, m.ff)}
+    if m.bias:
+        out.update({n + ".b": (w[0],) for n, w in list(out.items())})
+    return out
 
 
 def tensor_shapes(layers, d: int, vocab: int,
@@ -433,7 +672,7 @@ def tensor_shapes(layers, d: int, vocab: int,
     for i, l in enumerate(layers):
         if l.weights_of is not None:
             continue
-        p = f"l{i}."
+        p = f"l{i if l.index is None else l.index}."
         for k, part in ((1, l.mixer), (2, l.mlp)):
             if part is None:
                 continue

@@ -200,14 +200,16 @@ def load_checkpoint(path: str | Path, cfg: ModelConfig, tp: int = 1, rank: int =
 def _layer_list_config(c: dict, name: str) -> ModelConfig:
     from .layers import DESIGNS, parse_layers
 
-    layers = parse_layers(c["layers"])
-    vocab = int(c["vocab"])
     arch = c["architecture"].lower()
+    layers = parse_layers(c["layers"], DESIGNS[arch], c.get("loop"))
+    vocab = int(c["vocab"])
+    scale = c.get("logit_scale")
     return ModelConfig(
         name=name, arch=arch, vocab_size=vocab,
         hidden_size=int(c["width"]), num_layers=len(layers), layers=layers,
         intermediate_size=max([l.mlp.ff for l in layers if l.mlp is not None], default=0),
         rms_eps=float(c["norm"]["eps"]), logit_softcap=float(c.get("logit_softcap") or 0.0),
+        logit_scale=1.0 if scale is None else float(scale),
         tie_embeddings=DESIGNS[arch].tied,
         max_position=int(c.get("max_position", 131072)),
         bos_token_id=int(c.get("bos", min(256, vocab - 1))),

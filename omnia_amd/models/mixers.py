@@ -1,10 +1,12 @@
 """Mixers of layer-list models: how each one packs its checkpoint tensors, what it
 keeps per token or per sequence, and how it runs a step.
 
-A mixer's ``forward(w, h, fb, cache, ctx)`` takes the normed input of every row of
-a step -- decode rows first, then prefill portions -- and returns the input of its
-output projection; pages and states advance in place.  All padding happens in
-``pack`` (zero weight rows and columns), so the kernels only see aligned sizes.
+A mixer projects the (normed) input of every row of a step -- decode rows first, then
+prefill portions -- with one fused weight ``in``; ``mix(w, x, fb, cache)`` takes the
+projected rows to the input of its output projection ``o``, and pages and states advance
+in place; ``sublayer`` returns the operands of the residual kernel that follows.  All
+padding happens in ``pack`` (zero weight rows and columns), so the kernels only see
+aligned sizes.
 """
 from __future__ import annotations
 
@@ -43,13 +45,38 @@ def rotary_table(rot, positions: int, device) -> torch.Tensor:
     return (torch.cat([ang.cos(), ang.sin()], 1) * rot.magnitude).float().to(device)
 
 
-class LatentAttention:
+class Mixer:
+    cache_tensors = 0, 0  # page and state tensors of its cache entry
+    slab_input = False  # its kernels also reduce split-K slabs of a prefill projection
+    slab_decode = False  # ... of a decode step's
+
+    def __init__(self, spec, model):
+        self.spec, self.model = spec, model
+
+    def inputs(self, w: dict, h: torch.Tensor, is_decode: bool) -> torch.Tensor:
+        if self.slab_input or (is_decode and self.slab_decode):
+            return self.model._slabs("in", h, w["in"], is_decode)
+        return self.model.project(h, w["in"], is_decode)
+
+    def forward(self, w: dict, h: torch.Tensor, fb, cache) -> torch.Tensor:
+        return self.mix(w, self.inputs(w, h, fb.is_decode), fb, cache)
+
+    def output(self, w: dict, y: torch.Tensor, is_decode: bool, tag: str = "o") -> dict:
+        return {"m": self.model._slabs(tag, y, w["o"], is_decode), "bias": w.get("o_b")}
+
+    def sublayer(self, w: dict, h: torch.Tensor, fb, cache) -> dict:
+        return self.output(w, self.forward(w, h, fb, cache), fb.is_decode)
+
+
+class LatentAttention(Mixer):
     """Low-rank latent attention over one shared cached row per token.  Decode
     attends in the latent space (absorbed queries); bf16 prefill expands keys and
     values of each sequence's visible range and attends per head."""
 
+    cache_tensors = 1, 0
+
     def __init__(self, spec, model):
-        self.spec, self.model = spec, model
+        super().__init__(spec, model)
         self.table = model.rotary(spec.rotary)
         gpu16 = model.device.type == "cuda" and model.dtype == torch.bfloat16
         self.mfma_decode = gpu16 and mops.latent_decode_covers(spec)
@@ -118,10 +145,9 @@ class LatentAttention:
         vt = ops.linear(w["uv"].view(s.heads * s.v_pad, s.latent_pad), c)
         return mops.latent_prefill(q, kx, kr, vt, fb, s, gate, out)
 
-    def forward(self, w: dict, h: torch.Tensor, fb, cache) -> torch.Tensor:
+    def mix(self, w: dict, x: torch.Tensor, fb, cache) -> torch.Tensor:
         s, m = self.spec, self.model
         (pages,), _ = cache
-        x = m.project(h, w["in"], fb.is_decode)
         cq = mops.latent_prep(pages, x, w["q_norm"], w["kv_norm"], fb.positions, fb.slots,
                               self.table, s.q_rank_pad, s.latent_pad, m.cfg.rms_eps)
         q = m.project(cq, w["uq"], fb.is_decode)
@@ -129,10 +155,10 @@ class LatentAttention:
         gate = x[:, g0:g0 + s.heads]
         if fb.is_decode:
             return self._decode(w, q, gate, pages, fb.block_tables, fb.positions, None)
-        nd, T = fb.num_decode, h.shape[0]
+        nd, T = fb.num_decode, x.shape[0]
         if not nd:
             return self._prefill(w, q, gate, pages, fb, fb.positions, None)
-        out = torch.empty(T, s.heads * s.v_pad, dtype=h.dtype, device=h.device)
+        out = torch.empty(T, s.heads * s.v_pad, dtype=x.dtype, device=x.device)
         self._decode(w, q[:nd], gate[:nd], pages, fb.dec_block_tables, fb.positions[:nd],
                      out[:nd])
         if T > nd:
@@ -140,11 +166,10 @@ class LatentAttention:
         return out
 
 
-class GatedDelta:
+class GatedDelta(Mixer):
     """Gated delta rule with short convolutions; a state slot per sequence."""
 
-    def __init__(self, spec, model):
-        self.spec, self.model = spec, model
+    cache_tensors = 0, 2
 
     def pack(self, get, d: int) -> dict:
         s = self.spec
@@ -163,18 +188,17 @@ class GatedDelta:
                       torch.zeros(n_slots, s.conv - 1, s.conv_channels, dtype=m.dtype,
                                   device=m.device))
 
-    def forward(self, w: dict, h: torch.Tensor, fb, cache) -> torch.Tensor:
+    def mix(self, w: dict, x: torch.Tensor, fb, cache) -> torch.Tensor:
         s, m = self.spec, self.model
         _, (state, conv) = cache
-        x = m.project(h, w["in"], fb.is_decode)
         eps = m.cfg.rms_eps
         if fb.is_decode:
             return mops.delta_rule(x, w, s, state, conv, None, fb.positions, fb.state_slots, eps)
-        nd, T = fb.num_decode, h.shape[0]
+        nd, T = fb.num_decode, x.shape[0]
         if not nd:
             return mops.delta_rule(x, w, s, state, conv, fb.q_start_loc, fb.positions,
                                    fb.state_slots, eps)
-        y = torch.empty(T, s.heads * s.v_pad, dtype=h.dtype, device=h.device)
+        y = torch.empty(T, s.heads * s.v_pad, dtype=x.dtype, device=x.device)
         mops.delta_rule(x[:nd], w, s, state, conv, None, fb.positions[:nd], fb.state_slots[:nd],
                         eps, y[:nd])
         if T > nd:
@@ -183,13 +207,58 @@ class GatedDelta:
         return y
 
 
-class GroupedQueryAttention:
-    """Windowed attention with sinks over pages of keys and values -- its own, or (spec
-    ``kv_from``) those of an earlier layer, whose cache entry it is handed."""
+class Lightning(Mixer):
+    """Fixed-decay linear attention; a state slot per sequence."""
+
+    cache_tensors = 0, 1
+    slab_decode = True
+
+    def pack(self, get, d: int) -> dict:
+        s = self.spec
+
+        def heads(n, dim, pad):
+            t = get(n).view(s.heads, dim, -1)
+            return F.pad(t, (0, d - t.shape[2], 0, pad - dim)).reshape(s.heads * pad, d)
+
+        D, Dp, V, Vp = s.dim, s.dim_pad, s.vdim, s.v_pad
+        norm = F.pad(get("norm").float().view(s.heads, V), (0, Vp - V)).reshape(-1)
+        return {"in": _rows_to([heads("q", D, Dp), heads("k", D, Dp), heads("v", V, Vp),
+                                heads("g", V, Vp)], d),
+                "norm": norm.contiguous(), "pow": mops.decay_powers(s.decay, self.model.device),
+                "o": _head_cols(get("o"), s.heads, Vp, d)}
+
+    def alloc(self, num_blocks: int, block_size: int, n_slots: int):
+        s, m = self.spec, self.model
+        return None, (torch.zeros(n_slots, s.heads, s.dim_pad, s.v_pad, dtype=torch.float32,
+                                  device=m.device),)
+
+    def mix(self, w: dict, x: torch.Tensor, fb, cache) -> torch.Tensor:
+        s, m = self.spec, self.model
+        _, (state,) = cache
+        pos, slots, eps = fb.positions, fb.state_slots, m.cfg.rms_eps
+        if fb.is_decode:
+            return mops.lightning(x, w, s, state, None, pos, slots, eps, m.dtype)
+        nd, T = fb.num_decode, x.shape[0]
+        if not nd:
+            return mops.lightning(x, w, s, state, fb.q_start_loc, pos, slots, eps, m.dtype)
+        y = torch.empty(T, s.heads * s.v_pad, dtype=m.dtype, device=x.device)
+        mops.lightning(x[:nd], w, s, state, None, pos[:nd], slots[:nd], eps, m.dtype, y[:nd])
+        if T > nd:
+            mops.lightning(x[nd:], w, s, state, fb.q_start_loc, pos[nd:], slots[nd:], eps,
+                           m.dtype, y[nd:])
+        return y
+
+
+class GroupedQueryAttention(Mixer):
+    """Masked attention, with sinks or none, over pages of keys and values -- its own, or
+    (spec ``kv_from``) those of an earlier layer, whose cache entry it is handed."""
+
+    cache_tensors = 2, 0
+    slab_input = slab_decode = True
 
     def __init__(self, spec, model):
-        self.spec, self.model = spec, model
-        self.table = model.rotary(spec.rotary)
+        super().__init__(spec, model)
+        self.table = None if spec.rotary is None else model.rotary(spec.rotary)
         self.mfma = (model.device.type == "cuda" and model.dtype == torch.bfloat16
                      and spec.dim_pad in GQA_WIDTHS and spec.v_pad in GQA_WIDTHS)
 
@@ -202,17 +271,30 @@ class GroupedQueryAttention:
             return F.pad(t, (0, d - t.shape[2], 0, pad - dim)).reshape(count * pad, d)
 
         def norm(n):
-            return F.pad(get(n).float(), (0, s.dim_pad - s.dim)).contiguous()
+            t = get(n) if s.qk_norm == "weight" else torch.ones(s.dim, device=self.model.device)
+            return F.pad(t.float(), (0, s.dim_pad - s.dim)).contiguous()
+
+        def bias(n, count, dim, pad):
+            return F.pad(get(n + ".b").float().view(count, dim), (0, pad - dim)).reshape(-1)
 
         rows = [heads("q", s.heads, s.dim, s.dim_pad)]
         if own:
             rows += [heads("k", s.kv_heads, s.dim, s.dim_pad),
                      heads("v", s.kv_heads, s.vdim, s.v_pad)]
-        w = {"in": _rows_to(rows, d), "q_norm": norm("q.norm"),
-             "o": _head_cols(get("o"), s.heads, s.v_pad, d),
+        w = {"in": _rows_to(rows, d), "o": _head_cols(get("o"), s.heads, s.v_pad, d),
              "sink": get("sink").float().contiguous() if s.sink else None}
-        if own:
-            w["k_norm"] = norm("k.norm")
+        if s.qk_norm:
+            w["q_norm"] = norm("q.norm")
+            if own:
+                w["k_norm"] = norm("k.norm")
+        if s.bias:
+            bs = [bias("q", s.heads, s.dim, s.dim_pad)]
+            if own:
+                bs += [bias("k", s.kv_heads, s.dim, s.dim_pad),
+                       bias("v", s.kv_heads, s.vdim, s.v_pad)]
+            w["in_b"] = torch.cat(bs).contiguous()
+            ob = get("o.b").float()
+            w["o_b"] = F.pad(ob, (0, d - ob.numel())).contiguous()
         return w
 
     def alloc(self, num_blocks: int, block_size: int, n_slots: int):
@@ -227,7 +309,7 @@ class GroupedQueryAttention:
 
     def splits(self, rows: int, max_keys: int) -> int:
         s = self.spec
-        keys = min(max_keys, s.window) if s.window else max_keys
+        keys = s.most_visible(max_keys)
         groups = rows * s.kv_heads * -(-(s.heads // s.kv_heads) // 8)
         return max(1, -(-keys // self.MAX_PART),
                    min(-(-self.DECODE_GROUPS // groups), -(-keys // self.MIN_PART)))
@@ -246,23 +328,66 @@ class GroupedQueryAttention:
         return mops.gqa_attend(q, pages, fb.block_tables, fb.q_start_loc, positions, self.spec,
                                w["sink"], out)
 
-    def forward(self, w: dict, h: torch.Tensor, fb, cache) -> torch.Tensor:
+    def mix(self, w: dict, x: torch.Tensor, fb, cache) -> torch.Tensor:
         s, m = self.spec, self.model
         pages, _ = cache
-        q = mops.gqa_prep(m._slabs("in", h, w["in"], fb.is_decode), w, s,
-                          pages if s.kv_from is None else None, fb.positions, fb.slots,
+        q = mops.gqa_prep(x, w, s, pages if s.kv_from is None else None, fb.positions, fb.slots,
                           self.table, m.dtype, m.cfg.rms_eps)
         if fb.is_decode:
             return self._decode(w, q, pages, fb.block_tables, fb.positions, None)
-        nd, T = fb.num_decode, h.shape[0]
+        nd, T = fb.num_decode, fb.positions.numel()
         if not nd:
             return self._prefill(w, q, pages, fb, fb.positions, None)
-        out = torch.empty(T, s.heads * s.v_pad, dtype=h.dtype, device=h.device)
+        out = torch.empty(T, s.heads * s.v_pad, dtype=m.dtype, device=x.device)
         self._decode(w, q[:nd], pages, fb.dec_block_tables, fb.positions[:nd], out[:nd])
         if T > nd:
             self._prefill(w, q[nd:], pages, fb, fb.positions[nd:], out[nd:])
         return out
 
 
-MIXERS = {"latent_attention": LatentAttention, "delta": GatedDelta,
-          "attention": GroupedQueryAttention}
+class Parallel(Mixer):
+    """Two mixers on the same input: one fused input projection, whose columns each takes
+    its part of; their normed outputs meet in the residual kernel."""
+
+    def __init__(self, spec, model):
+        super().__init__(spec, model)
+        self.left, self.right = (MIXERS[m.kind](m, model) for m in (spec.left, spec.right))
+        both = (self.left, self.right)
+        self.slab_input = all(m.slab_input for m in both)
+        self.slab_decode = all(m.slab_decode for m in both)
+
+    def pack(self, get, d: int) -> dict:
+        sides, rows = {}, []
+        for name, m in (("left", self.left), ("right", self.right)):
+            w = m.pack(lambda n, p=name + ".": get(p + n), d)
+            rows.append(w.pop("in")[:m.spec.in_cols])
+            t = get(name + ".out").float()
+            # the mean of the two: half of each weight
+            sides[name] = w, mops.RMSNorm(F.pad(0.5 * t, (0, d - t.numel())).contiguous(),
+                                          self.model.cfg.hidden_size, self.model.cfg.rms_eps)
+        return {"in": _rows_to(rows, d), **sides}
+
+    def alloc(self, num_blocks: int, block_size: int, n_slots: int):
+        pages, states = (), ()
+        for m in (self.left, self.right):
+            p, s = m.alloc(num_blocks, block_size, n_slots)
+            pages, states = pages + (p or ()), states + (s or ())
+        return pages or None, states or None
+
+    def sublayer(self, w: dict, h: torch.Tensor, fb, cache) -> dict:
+        x = self.inputs(w, h, fb.is_decode)
+        pages, states = cache
+        np, ns, at, out = 0, 0, 0, []
+        for name, m in (("left", self.left), ("right", self.right)):
+            sub, norm = w[name]
+            kp, ks = m.cache_tensors
+            part = (pages[np:np + kp] if kp else None, states[ns:ns + ks] if ks else None)
+            y = m.mix(sub, x[..., at:at + m.spec.in_cols], fb, part)
+            o = m.output(sub, y, fb.is_decode, "o_" + name)
+            out.append((o["m"], o["bias"], norm))
+            np, ns, at = np + kp, ns + ks, at + m.spec.in_cols
+        return {"branches": out}
+
+
+MIXERS = {"latent_attention": LatentAttention, "delta": GatedDelta, "lightning": Lightning,
+          "attention": GroupedQueryAttention, "parallel": Parallel}

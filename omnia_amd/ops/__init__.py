@@ -368,13 +368,14 @@ def pgemm(epi: int, x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None =
           ss_in: torch.Tensor | None = None, inv_d: float = 0.0, eps: float = 0.0,
           ss_out: torch.Tensor | None = None, positions=None, cos_sin=None, k_cache=None,
           v_cache=None, slots=None, hq: int = 0, hkv: int = 0, block_size: int = 0,
-          bias: torch.Tensor | None = None):
+          bias: torch.Tensor | None = None, gelu: bool = False):
     """Prefill GEMM ``x @ w.T`` with a fused epilogue (``csrc/pgemm.hip``).
 
     ``ss_in`` ([M, n] fp32 partial row sums of squares of ``x``) scales row r by
     ``rsqrt(sum(ss_in[r]) * inv_d + eps)`` -- RMSNorm with the norm weight folded
     into ``w``.  epi 0: out = scaled GEMM; 1: out = silu(g) * u with
-    ``w = [Wg; Wu]`` (``bias`` fp32 [2N], unscaled only: ``silu(g + bg) * (u + bu)``);
+    ``w = [Wg; Wu]`` (``bias`` fp32 [2N], unscaled only: ``silu(g + bg) * (u + bu)``;
+    ``gelu``, unscaled only: ``gelu_tanh(g) * u``);
     2: ``out`` is the residual, updated in place (out += GEMM)
     with ``ss_out[r, t]`` = sum of squares of its new 256-column slice t;
     3: QKV -> RoPE'd q in ``out`` [M, hq*128], RoPE'd k and v written to the
@@ -387,7 +388,7 @@ def pgemm(epi: int, x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None =
         if epi == 3 and checks.active(x):
             checks.slots("pgemm qkv", slots, k_cache)
         kernels().pgemm(epi, out, x.contiguous(), w, ss_in, inv_d, eps, ss_out, positions,
-                        cos_sin, k_cache, v_cache, slots, hq, hkv, block_size, bias)
+                        cos_sin, k_cache, v_cache, slots, hq, hkv, block_size, bias, gelu)
         return out
     h = x.float() @ w.float().t()
     if bias is not None:
@@ -397,7 +398,8 @@ def pgemm(epi: int, x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None =
     if epi == 0:
         out.copy_(h.to(out.dtype))
     elif epi == 1:
-        out.copy_((F.silu(h[:, :N]) * h[:, N:]).to(out.dtype))
+        a = F.gelu(h[:, :N], approximate="tanh") if gelu else F.silu(h[:, :N])
+        out.copy_((a * h[:, N:]).to(out.dtype))
     elif epi == 2:
         new = (out.float() + h.to(out.dtype).float()).to(out.dtype)
         out.copy_(new)
@@ -735,11 +737,13 @@ MOE_LIBRARY_ROWS = 1024  # mean rows/expert above which eager calls use hipBLASL
 MOE_TILE256_ROWS = int(os.environ.get("OMNIA_MOE_TILE256_ROWS", "512"))
 
 
-def _moe_grouped(x, w_gu, w_down, ids, wts, k, n_experts, e_lo, e_hi, bm, glu=None):
+def _moe_grouped(x, w_gu, w_down, ids, wts, k, n_experts, e_lo, e_hi, bm, glu=None,
+                 gelu: bool = False):
     """Grouped expert FFN over device-sorted assignments, no host sync: Y [T*k, d]
     (row t*k + j = slot j of token t, routing weight applied; other experts' rows
     unwritten).  ``bm`` 256: the 256x256 MFMA prefill tile; 64: moe.hip.  ``glu`` =
-    (alpha, limit): clamped GLU experts whose INPUT takes the routing weight."""
+    (alpha, limit): clamped GLU experts whose INPUT takes the routing weight; ``gelu``:
+    ungated experts (``w_gu`` [E, I, d])."""
     kk = kernels()
     n = ids.numel()
     mb = kk.moe_max_blocks(n, e_hi - e_lo, bm)
@@ -754,7 +758,7 @@ def _moe_grouped(x, w_gu, w_down, ids, wts, k, n_experts, e_lo, e_hi, bm, glu=No
         gemm(2, act, x, w_gu, sorted_ids, blk, nblk, wts.view(-1), k, n, e_lo, *glu)
         gemm(1, Y, act, w_down, sorted_ids, blk, nblk, None, k, n, e_lo)
         return Y
-    gemm(0, act, x, w_gu, sorted_ids, blk, nblk, None, k, n, e_lo)
+    gemm(3 if gelu else 0, act, x, w_gu, sorted_ids, blk, nblk, None, k, n, e_lo)
     gemm(1, Y, act, w_down, sorted_ids, blk, nblk, wts.view(-1), k, n, e_lo)
     return Y
 

@@ -7,12 +7,15 @@
 #include <c10/hip/HIPStream.h>
 #include <hip/hip_runtime.h>
 
+// the layout of mask.h's struct: (window, kept first positions, chunk)
+struct Mask { int window, keep, chunk; };
+
 extern "C" {
 int omnia_pgemm(int epi, void* out, const void* X, const void* W, int M, int N, int K, int ldo,
                 const float* ss_in, int ss_in_n, float inv_d, float eps, float* ss_out,
                 const int* positions, const float* cos_sin, void* k_cache, void* v_cache,
                 const int64_t* slots, int hq, int hkv, int block_size, const float* bias,
-                hipStream_t s);
+                int gelu, hipStream_t s);
 int omnia_row_sumsq(float* ss, const void* x, int rows, int d, int64_t stride, hipStream_t s);
 int omnia_ar_alltoall(void* out, const void* in, void* const* regions, int* epochs, int* err,
                       int64_t chunk, int64_t slot_bytes, int rank, int world, hipStream_t s);
@@ -82,7 +85,8 @@ int omnia_moe_router_topk(int* ids, float* wts, const void* x, const void* route
 int omnia_moe_align(int* sorted, int* blk_expert, int* n_blocks, const int* ids, int n, int E,
                     int e_lo, int e_hi, int max_blocks, int bm, hipStream_t s);
 int omnia_moe_route(int* ids, float* wts, const void* x, const void* router, int f32, int n_tok,
-                    int d, int E, int k, int sigmoid, int renorm, hipStream_t s);
+                    int d, int E, int k, int sigmoid, int renorm, const float* corr, int groups,
+                    int keep, hipStream_t s);
 int omnia_moe_gemm(int mode, void* out, const void* A, const void* W, int f32, const int* sorted,
                    const int* blk_expert, const int* n_blocks, const float* route_w, int K, int N,
                    int topk, int n_assign, int e_lo, int max_blocks, float alpha, float limit,
@@ -127,9 +131,27 @@ int omnia_tanh_norm_embed(void* h, float* x, const int* ids, const void* table, 
 int omnia_tanh_norm_residual(void* h, int f32, float* x, const void* m, int ptype, int S,
                              int64_t row, int64_t slab, int rows, int d, const float* bias,
                              float a1, const float* w1, const float* b1, float a2,
-                             const float* w2, const float* b2, hipStream_t s);
-int omnia_bias_swiglu(void* out, int f32, const void* m, int ptype, int S, int rows, int inter,
-                      const float* bias, hipStream_t s);
+                             const float* w2, const float* b2, const int* ids, const float* wts,
+                             const void* in, int first, hipStream_t s);
+int omnia_glu(void* out, int f32, const void* m, int ptype, int S, int rows, int inter,
+              const float* bias, int gelu, hipStream_t s);
+int omnia_branch_residual(void* h, int f32, float* x, int rows, int d, const void* a, int at,
+                          int aS, int64_t arow, int64_t aslab, const float* abias,
+                          const float* aw, const void* b, int bt, int bS, int64_t brow,
+                          int64_t bslab, const float* bbias, const float* bw, float inv_n,
+                          float eps, float alpha, const float* nw, const float* nb,
+                          hipStream_t s);
+int omnia_lightning_pow_cols();
+int64_t omnia_lightning_scratch(int n_rows, int nseq, int H, int Dp, int Vp);
+int omnia_lightning_step(float* o, float* state, const void* x, int ptype, int S, int64_t ld,
+                         int64_t slab, const float* pw, const int* positions, const int* slots,
+                         int T, int H, int Dp, int Vp, hipStream_t s);
+int omnia_lightning_scan(float* o, float* state, float* seg, const void* x, int f32, int64_t ldx,
+                         const float* pw, const int* q_start, int nseq, const int* positions,
+                         const int* slots, int n_rows, int H, int Dp, int Vp, hipStream_t s);
+int omnia_lightning_norm(void* y, int f32, const float* o, const void* x, int ptype, int S,
+                         int64_t ld, int64_t slab, int goff, const float* w, int T, int n,
+                         float inv_n, float eps, hipStream_t s);
 int omnia_delta_prep(float* qn, float* kn, void* vc, float* decay, float* beta, const void* x,
                      int f32, int64_t ldx, const void* conv_w, const void* conv_state,
                      const float* a_log, const float* dt_bias, const int* q_start, int nseq,
@@ -159,20 +181,21 @@ int omnia_rms_residual(void* h, int f32, float* x, const void* m, int ptype, int
 int omnia_softcap(void* z, int f32, int64_t n, float cap, hipStream_t s);
 int omnia_gqa_prep(void* q, void* kc, void* vc, int f32, const void* x, int ptype, int S,
                    int64_t slab, int64_t ldx, const float* wq, const float* wk,
-                   const int* positions, const int64_t* slots, const float* cos_sin, int T, int H,
-                   int G, int D, int Dp, int Vp, int R, int page, float eps, hipStream_t s);
+                   const float* bias, const int* positions, const int64_t* slots,
+                   const float* cos_sin, int pairs, int T, int H, int G, int D, int Dp, int Vp,
+                   int R, int page, float eps, hipStream_t s);
 int omnia_gqa_attend(void* out, int f32, const void* q, const void* kc, const void* vc,
                      const int* block_tables, int bt_stride, const int* q_start, int nseq,
                      const int* positions, int T, int page, int H, int G, int Dp, int Vp,
-                     int window, float scale, const float* sinks, hipStream_t s);
+                     Mask mask, float scale, const float* sinks, hipStream_t s);
 int omnia_gqa_decode(void* out, float* part_o, float* part_ml, const void* q, const void* kc,
                      const void* vc, const int* block_tables, int bt_stride, const int* positions,
-                     int T, int page, int H, int G, int Dp, int Vp, int window, float scale,
-                     const float* sinks, int splits, int max_keys, hipStream_t s);
+                     int T, int page, int H, int G, int Dp, int Vp, Mask mask, float scale,
+                     const float* sinks, int splits, int max_ctx, hipStream_t s);
 int omnia_gqa_prefill(void* out, const void* q, const void* kc, const void* vc,
                       const int* block_tables, int bt_stride, const int* q_start,
                       const int* seq_lens, const int* tile_seq, const int* tile_q0, int n_tiles,
-                      int page, int H, int G, int Dp, int Vp, int window, float scale,
+                      int page, int H, int G, int Dp, int Vp, Mask mask, float scale,
                       const float* sinks, hipStream_t s);
 int omnia_latent_prep(void* cq, void* cache, const void* x, int f32, int64_t ldx, const float* wq,
                       const float* wc, const int* positions, const int64_t* slots,
@@ -630,7 +653,7 @@ void pgemm_moe(int64_t mode, at::Tensor out, at::Tensor A, at::Tensor W, at::Ten
   TORCH_CHECK(A.size(-1) == K && K % 128 == 0, "K mismatch / K % 128");
   int N;
   if (mode != 1) {
-    N = W.size(1) / 2;
+    N = mode == 3 ? W.size(1) : W.size(1) / 2;
     TORCH_CHECK(N % 128 == 0 && out.size(0) == (int64_t)mb * 256 && out.size(1) == N,
                 "act [max_blocks*256, I]");
     TORCH_CHECK(A.size(0) * topk == n_assign, "x rows * topk == n_assign");
@@ -648,7 +671,8 @@ void pgemm_moe(int64_t mode, at::Tensor out, at::Tensor A, at::Tensor W, at::Ten
 
 // router: fp32 logits, sigmoid / softmax scores; x [T, d] and router [E, d] bf16 or fp32
 void moe_route(at::Tensor ids, at::Tensor wts, at::Tensor x, at::Tensor router, int64_t k,
-               bool sigmoid, bool renorm) {
+               bool sigmoid, bool renorm, c10::optional<at::Tensor> corr, int64_t groups,
+               int64_t keep) {
   CHECK_GPU(x); CHECK_I32(ids);
   const bool f32 = x.scalar_type() == at::kFloat;
   TORCH_CHECK((f32 || x.scalar_type() == at::kBFloat16) && router.scalar_type() == x.scalar_type(),
@@ -660,9 +684,12 @@ void moe_route(at::Tensor ids, at::Tensor wts, at::Tensor x, at::Tensor router, 
   TORCH_CHECK(ids.numel() == (int64_t)T * k && wts.numel() == (int64_t)T * k && wts.is_cuda() &&
               wts.scalar_type() == at::kFloat && ids.is_contiguous() && wts.is_contiguous(),
               "ids/wts [T, k]");
+  if (corr.has_value())
+    TORCH_CHECK(corr->is_cuda() && corr->scalar_type() == at::kFloat && corr->is_contiguous() &&
+                corr->numel() == E, "correction fp32 [E]");
   CHECK_RC(omnia_moe_route(ids.data_ptr<int>(), wts.data_ptr<float>(), x.data_ptr(),
                            router.data_ptr(), f32, T, x.size(1), E, k, sigmoid, renorm,
-                           cur_stream()), "moe_route");
+                           opt_ptr<float>(corr), groups, keep, cur_stream()), "moe_route");
 }
 
 // modes in moe.hip; A, W and out all bf16 or all fp32
@@ -685,7 +712,7 @@ void moe_gemm(int64_t mode, at::Tensor out, at::Tensor A, at::Tensor W, at::Tens
                 route_w->scalar_type() == at::kFloat, "route weights fp32 [T*k]");
   int N;
   if (mode != 1) {
-    N = W.size(1) / 2;
+    N = mode == 3 ? W.size(1) : W.size(1) / 2;
     TORCH_CHECK(N % 32 == 0 && out.size(0) == (int64_t)mb * 64 && out.size(1) == N,
                 "act [max_blocks*64, I]");
     TORCH_CHECK(A.size(0) * topk == n_assign, "x rows * topk == n_assign");
@@ -832,7 +859,7 @@ void pgemm(int64_t epi, at::Tensor out, at::Tensor x, at::Tensor W,
            c10::optional<at::Tensor> ss_out, c10::optional<at::Tensor> positions,
            c10::optional<at::Tensor> cos_sin, c10::optional<at::Tensor> k_cache,
            c10::optional<at::Tensor> v_cache, c10::optional<at::Tensor> slots, int64_t hq,
-           int64_t hkv, int64_t block_size, c10::optional<at::Tensor> bias) {
+           int64_t hkv, int64_t block_size, c10::optional<at::Tensor> bias, bool gelu) {
   CHECK_GPU(x); CHECK_BF16(x); CHECK_BF16(W); CHECK_BF16(out);
   TORCH_CHECK(x.dim() == 2 && W.dim() == 2 && out.dim() == 2, "2-D operands");
   TORCH_CHECK(x.is_contiguous() && W.is_contiguous(), "contiguous x / W");
@@ -895,7 +922,7 @@ void pgemm(int64_t epi, at::Tensor out, at::Tensor x, at::Tensor W,
   if (M == 0) return;
   CHECK_RC(omnia_pgemm((int)epi, out.data_ptr(), x.data_ptr(), W.data_ptr(), M, N, K,
                        out.stride(0), ssi, ssn, (float)inv_d, (float)eps, sso, pos, cs, kc, vc, sl,
-                       (int)hq, (int)hkv, (int)block_size, bp, cur_stream()),
+                       (int)hq, (int)hkv, (int)block_size, bp, gelu, cur_stream()),
            "pgemm");
 }
 
@@ -1245,16 +1272,18 @@ int64_t rows2(const at::Tensor& t, int64_t T, int64_t width, const char* what) {
   return t.stride(0);
 }
 
-// a projection: [M, N] in bf16 / fp32, or split-K slabs [S, M, N] in fp32 / fp16
-struct Proj { int type, S; int64_t M, N; };
-Proj proj(const at::Tensor& m) {
+// a projection: [M, N] in bf16 / fp32, or split-K slabs [S, M, N] in fp32 / fp16; rows may
+// be columns of a wider projection (row stride ld, slab stride slab)
+struct Proj { int type, S; int64_t M, N, ld, slab; };
+Proj proj(const at::Tensor& m, bool strided = false) {
   CHECK_GPU(m);
-  TORCH_CHECK(m.is_contiguous() && (m.dim() == 2 || m.dim() == 3), "projection [M, N] or [S, M, N]");
+  const bool p = m.dim() == 3;
+  TORCH_CHECK((m.dim() == 2 || p) && (strided ? m.stride(-1) == 1 : m.is_contiguous()),
+              "projection [M, N] or [S, M, N]");
   const auto st = m.scalar_type();
   TORCH_CHECK(st == at::kBFloat16 || st == at::kFloat || st == at::kHalf, "projection dtype");
-  const bool p = m.dim() == 3;
   return {st == at::kBFloat16 ? 0 : st == at::kFloat ? 1 : 2, p ? (int)m.size(0) : 1,
-          p ? m.size(1) : m.size(0), m.size(-1)};
+          p ? m.size(1) : m.size(0), m.size(-1), m.stride(-2), p ? m.stride(0) : 0};
 }
 
 void tanh_norm_embed(at::Tensor h, at::Tensor x, at::Tensor ids, at::Tensor table, int64_t vocab,
@@ -1288,26 +1317,112 @@ const float* opt_vecf(const OptT& t, int64_t n, const char* what) {
   return t.has_value() && t->defined() ? vecf(*t, n, what) : nullptr;
 }
 
+// w1 null: no post-norm.  ids / wts [M, S], in [M, d]: parts of identity experts (ids >=
+// first) stand for wts * in
 void tanh_norm_residual(at::Tensor h, at::Tensor x, at::Tensor m, bool slots, OptT bias, double a1,
-                        at::Tensor w1, at::Tensor b1, double a2, at::Tensor w2, at::Tensor b2) {
+                        OptT w1, OptT b1, double a2, at::Tensor w2, at::Tensor b2, OptT ids,
+                        OptT wts, OptT in, int64_t first) {
   const int f32 = is_f32(h, "h");
   const ResidParts p = resid_parts(m, slots);
   const int64_t d = p.d;
   like(h, h, p.M * d, "h");
+  const float* w1p = opt_vecf(w1, d, "w1");
+  TORCH_CHECK(!w1p || (b1.has_value() && b1->defined()), "w1 comes with b1");
+  const int* idp = nullptr;
+  if (ids.has_value() && ids->defined()) {
+    TORCH_CHECK(slots && wts.has_value() && in.has_value(), "identity parts: slots, wts, in");
+    idp = veci(*ids, p.M * p.S, "ids");
+    vecf(*wts, p.M * p.S, "wts");
+    like(*in, h, p.M * d, "in");
+  }
   CHECK_RC(omnia_tanh_norm_residual(
                h.data_ptr(), f32, outf(x, p.M * d, "x"), m.data_ptr(), p.type, p.S, p.row, p.part,
-               p.M, d, opt_vecf(bias, d, "bias"), (float)a1, vecf(w1, d, "w1"), vecf(b1, d, "b1"),
-               (float)a2, vecf(w2, d, "w2"), vecf(b2, d, "b2"), cur_stream()),
+               p.M, d, opt_vecf(bias, d, "bias"), (float)a1, w1p, opt_vecf(b1, d, "b1"),
+               (float)a2, vecf(w2, d, "w2"), vecf(b2, d, "b2"), idp,
+               idp ? wts->data_ptr<float>() : nullptr, idp ? in->data_ptr() : nullptr, first,
+               cur_stream()),
            "tanh_norm_residual");
 }
 
-void bias_swiglu(at::Tensor out, at::Tensor m, at::Tensor bias) {
+// x += rms(a + abias) aw + rms(b + bbias) bw; h = x (nw null), RMS (nb null) or tanh norm
+void branch_residual(at::Tensor h, at::Tensor x, at::Tensor a, OptT abias, at::Tensor aw,
+                     at::Tensor b, OptT bbias, at::Tensor bw, double inv_n, double eps,
+                     double alpha, OptT nw, OptT nb) {
+  const int f32 = is_f32(h, "h");
+  const Proj pa = proj(a), pb = proj(b);
+  const int64_t M = pa.M, d = pa.N;
+  TORCH_CHECK(pb.M == M && pb.N == d, "branches of one shape");
+  like(h, h, M * d, "h");
+  CHECK_RC(omnia_branch_residual(
+               h.data_ptr(), f32, outf(x, M * d, "x"), M, d, a.data_ptr(), pa.type, pa.S, pa.ld,
+               pa.slab, opt_vecf(abias, d, "abias"), vecf(aw, d, "aw"), b.data_ptr(), pb.type,
+               pb.S, pb.ld, pb.slab, opt_vecf(bbias, d, "bbias"), vecf(bw, d, "bw"), (float)inv_n,
+               (float)eps, (float)alpha, opt_vecf(nw, d, "nw"), opt_vecf(nb, d, "nb"),
+               cur_stream()),
+           "branch_residual");
+}
+
+// act(g + bg) * (u + bu): silu, or the tanh form of gelu
+void glu(at::Tensor out, at::Tensor m, OptT bias, bool gelu) {
   const int f32 = is_f32(out, "out");
   const Proj p = proj(m);
   TORCH_CHECK(p.N % 2 == 0, "gate | up columns");
   like(out, out, p.M * (p.N / 2), "out");
-  CHECK_RC(omnia_bias_swiglu(out.data_ptr(), f32, m.data_ptr(), p.type, p.S, p.M, p.N / 2,
-                             vecf(bias, p.N, "bias"), cur_stream()), "bias_swiglu");
+  CHECK_RC(omnia_glu(out.data_ptr(), f32, m.data_ptr(), p.type, p.S, p.M, p.N / 2,
+                     opt_vecf(bias, p.N, "bias"), gelu, cur_stream()), "glu");
+}
+
+// ------------------------------------------------------- fixed-decay linear attention
+// state fp32 [slots, H, Dp, Vp]; pw [H, pow cols]; x rows [q | k | v | g] (possibly slabs)
+struct Lightning { int64_t H, Dp, Vp, cols; };
+Lightning lightning_sizes(const at::Tensor& state, const at::Tensor& pw, const Proj& p,
+                          int64_t T, const at::Tensor& o) {
+  TORCH_CHECK(state.is_cuda() && state.scalar_type() == at::kFloat && state.is_contiguous() &&
+              state.dim() == 4, "state fp32 [slots, H, Dp, Vp]");
+  const int64_t H = state.size(1), Dp = state.size(2), Vp = state.size(3);
+  vecf(pw, H * omnia_lightning_pow_cols(), "pw");
+  TORCH_CHECK(p.M == T && p.N >= 2 * H * (Dp + Vp), "projection rows [q | k | v | g]");
+  vecf(o, T * H * Vp, "o");
+  return {H, Dp, Vp, 2 * H * (Dp + Vp)};
+}
+
+void lightning_step(at::Tensor o, at::Tensor state, at::Tensor x, at::Tensor pw,
+                    at::Tensor positions, at::Tensor slots) {
+  const Proj p = proj(x, true);
+  const int64_t T = positions.numel();
+  const Lightning l = lightning_sizes(state, pw, p, T, o);
+  CHECK_RC(omnia_lightning_step(o.data_ptr<float>(), state.data_ptr<float>(), x.data_ptr(), p.type,
+                                p.S, p.ld, p.slab, pw.data_ptr<float>(),
+                                veci(positions, T, "positions"), veci(slots, T, "slots"), T, l.H,
+                                l.Dp, l.Vp, cur_stream()), "lightning_step");
+}
+
+void lightning_scan(at::Tensor o, at::Tensor state, OptT seg, at::Tensor x, at::Tensor pw,
+                    at::Tensor q_start, at::Tensor positions, at::Tensor slots) {
+  const int f32 = is_f32(x, "x");
+  const Proj p = proj(x, true);
+  const int64_t T = positions.numel(), nseq = slots.numel();
+  TORCH_CHECK(p.S == 1 && x.dim() == 2, "plain projection rows");
+  const Lightning l = lightning_sizes(state, pw, p, T, o);
+  const int64_t need = omnia_lightning_scratch(T, nseq, l.H, l.Dp, l.Vp);
+  CHECK_RC(omnia_lightning_scan(o.data_ptr<float>(), state.data_ptr<float>(),
+                                need ? outf(seg.value(), need, "seg") : nullptr, x.data_ptr(), f32,
+                                p.ld, pw.data_ptr<float>(), veci(q_start, nseq + 1, "q_start"),
+                                nseq, veci(positions, T, "positions"),
+                                veci(slots, nseq, "slots"), T, l.H, l.Dp, l.Vp, cur_stream()),
+           "lightning_scan");
+}
+
+void lightning_norm(at::Tensor y, at::Tensor o, at::Tensor x, int64_t goff, at::Tensor w,
+                    double inv_n, double eps) {
+  const int f32 = is_f32(y, "y");
+  const Proj p = proj(x, true);
+  const int64_t n = w.numel();
+  TORCH_CHECK(p.N >= goff + n, "gate columns");
+  like(y, y, p.M * n, "y");
+  CHECK_RC(omnia_lightning_norm(y.data_ptr(), f32, vecf(o, p.M * n, "o"), x.data_ptr(), p.type,
+                                p.S, p.ld, p.slab, goff, vecf(w, n, "w"), p.M, n, (float)inv_n,
+                                (float)eps, cur_stream()), "lightning_norm");
 }
 
 // rows of a step: q_start null = decode (row = sequence), else prefill portions
@@ -1587,16 +1702,19 @@ void check_kv(const at::Tensor& k, const at::Tensor& v, const at::Tensor& ref) {
 }
 
 // x: [T, (H*Dp | G*Dp | G*Vp) + padding] or its slabs; k / v pages absent: q only
-void gqa_prep(at::Tensor q, OptT k, OptT v, at::Tensor x, at::Tensor wq, OptT wk,
-              at::Tensor positions, at::Tensor slots, at::Tensor cos_sin, int64_t H, int64_t D,
-              double eps) {
+// wq null: no norms; cos_sin null: no rotation; pairs: neighbours turn together
+void gqa_prep(at::Tensor q, OptT k, OptT v, at::Tensor x, OptT wq, OptT wk, OptT bias,
+              at::Tensor positions, at::Tensor slots, OptT cos_sin, bool pairs, int64_t H,
+              int64_t D, int64_t Dp, double eps) {
   const int f32 = is_f32(q, "q");
-  const Proj p = proj(x);
-  const int64_t T = positions.numel(), R = cos_sin.size(1), Dp = wq.numel();
+  const Proj p = proj(x, true);
+  const bool rot = cos_sin.has_value() && cos_sin->defined();
+  const int64_t T = positions.numel(), R = rot ? cos_sin->size(1) : 0;
+  const float* wqp = opt_vecf(wq, Dp, "wq");
   const bool own = k.has_value() && k->defined();
   int64_t G = 0, Vp = 0, page = 1;
   if (own) {
-    TORCH_CHECK(v.has_value() && wk.has_value(), "k pages come with v pages and a k norm");
+    TORCH_CHECK(v.has_value() && (!wqp || wk.has_value()), "k pages come with v pages and a k norm");
     check_kv(*k, *v, q);
     G = k->size(1);
     page = k->size(2);
@@ -1609,9 +1727,10 @@ void gqa_prep(at::Tensor q, OptT k, OptT v, at::Tensor x, at::Tensor wq, OptT wk
               slots.numel() == T, "slots int64 [T]");
   CHECK_RC(omnia_gqa_prep(q.data_ptr(), own ? k->data_ptr() : nullptr,
                           own ? v->data_ptr() : nullptr, f32, x.data_ptr(), p.type, p.S,
-                          p.M * p.N, p.N, vecf(wq, Dp, "wq"),
-                          own ? vecf(*wk, Dp, "wk") : nullptr, veci(positions, T, "positions"),
-                          slots.data_ptr<int64_t>(), rot_table(cos_sin, R), T, H, G, D, Dp, Vp, R,
+                          p.slab, p.ld, wqp, own && wqp ? vecf(*wk, Dp, "wk") : nullptr,
+                          opt_vecf(bias, H * Dp + G * (Dp + Vp), "bias"),
+                          veci(positions, T, "positions"), slots.data_ptr<int64_t>(),
+                          rot ? rot_table(*cos_sin, R) : nullptr, pairs, T, H, G, D, Dp, Vp, R,
                           page, (float)eps, cur_stream()), "gqa_prep");
 }
 
@@ -1627,8 +1746,13 @@ KV kv_sizes(const at::Tensor& out, const at::Tensor& q, const at::Tensor& k, con
   return s;
 }
 
+using MaskT = std::tuple<int64_t, int64_t, int64_t>;  // (window, kept first, chunk)
+Mask mask_of(const MaskT& m) {
+  return {(int)std::get<0>(m), (int)std::get<1>(m), (int)std::get<2>(m)};
+}
+
 void gqa_attend(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor block_tables,
-                OptT q_start, at::Tensor positions, int64_t H, int64_t window, double scale,
+                OptT q_start, at::Tensor positions, int64_t H, MaskT mask, double scale,
                 OptT sinks) {
   const int f32 = is_f32(q, "q");
   const int64_t T = positions.numel();
@@ -1638,13 +1762,14 @@ void gqa_attend(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::Te
   CHECK_RC(omnia_gqa_attend(out.data_ptr(), f32, q.data_ptr(), k.data_ptr(), v.data_ptr(),
                             tables(block_tables, nseq), block_tables.stride(0),
                             pre ? veci(*q_start, nseq + 1, "q_start") : nullptr, nseq,
-                            veci(positions, T, "positions"), T, s.page, H, s.G, s.Dp, s.Vp, window,
-                            (float)scale, opt_ptr<float>(sinks), cur_stream()), "gqa_attend");
+                            veci(positions, T, "positions"), T, s.page, H, s.G, s.Dp, s.Vp,
+                            mask_of(mask), (float)scale, opt_ptr<float>(sinks), cur_stream()),
+           "gqa_attend");
 }
 
 void gqa_decode(at::Tensor out, OptT part_o, OptT part_ml, at::Tensor q, at::Tensor k,
                 at::Tensor v, at::Tensor block_tables, at::Tensor positions, int64_t H,
-                int64_t window, double scale, OptT sinks, int64_t splits) {
+                MaskT mask, double scale, OptT sinks, int64_t splits) {
   CHECK_GPU(q); CHECK_BF16(q);
   const int64_t T = positions.numel();
   const KV s = kv_sizes(out, q, k, v, T, H, sinks);
@@ -1654,19 +1779,18 @@ void gqa_decode(at::Tensor out, OptT part_o, OptT part_ml, at::Tensor q, at::Ten
     po = outf(*part_o, T * H * splits * s.Vp, "part_o");
     pm = outf(*part_ml, T * H * splits * 2, "part_ml");
   }
-  // a row's context fits its block-table row, so no row sees more keys than this
-  int64_t keys = block_tables.size(1) * s.page;
-  if (window > 0 && window < keys) keys = window;
+  const int64_t ctx = block_tables.size(1) * s.page;  // a row's context fits its table row
   CHECK_RC(omnia_gqa_decode(out.data_ptr(), po, pm, q.data_ptr(), k.data_ptr(), v.data_ptr(),
                             tables(block_tables, T), block_tables.stride(0),
-                            veci(positions, T, "positions"), T, s.page, H, s.G, s.Dp, s.Vp, window,
-                            (float)scale, opt_ptr<float>(sinks), splits, keys, cur_stream()),
+                            veci(positions, T, "positions"), T, s.page, H, s.G, s.Dp, s.Vp,
+                            mask_of(mask), (float)scale, opt_ptr<float>(sinks), splits, ctx,
+                            cur_stream()),
            "gqa_decode");
 }
 
 void gqa_prefill(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor block_tables,
                  at::Tensor q_start, at::Tensor seq_lens, at::Tensor tile_seq, at::Tensor tile_q0,
-                 int64_t H, int64_t window, double scale, OptT sinks) {
+                 int64_t H, MaskT mask, double scale, OptT sinks) {
   CHECK_GPU(q); CHECK_BF16(q);
   TORCH_CHECK(q.dim() == 2, "q [T, H*Dp]");
   const KV s = kv_sizes(out, q, k, v, q.size(0), H, sinks);
@@ -1675,8 +1799,8 @@ void gqa_prefill(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::T
                              tables(block_tables, nseq), block_tables.stride(0),
                              veci(q_start, nseq + 1, "q_start"), veci(seq_lens, nseq, "seq_lens"),
                              veci(tile_seq, nt, "tile_seq"), veci(tile_q0, nt, "tile_q0"), nt,
-                             s.page, H, s.G, s.Dp, s.Vp, window, (float)scale,
-                             opt_ptr<float>(sinks), cur_stream()), "gqa_prefill");
+                             s.page, H, s.G, s.Dp, s.Vp, mask_of(mask),
+                             (float)scale, opt_ptr<float>(sinks), cur_stream()), "gqa_prefill");
 }
 
 }  // namespace
@@ -1693,7 +1817,13 @@ PYBIND11_MODULE(_omnia_kernels, m) {
   m.def("gqa_decode", &gqa_decode);
   m.def("gqa_prefill", &gqa_prefill);
   m.def("tanh_norm_residual", &tanh_norm_residual);
-  m.def("bias_swiglu", &bias_swiglu);
+  m.def("branch_residual", &branch_residual);
+  m.def("glu", &glu);
+  m.def("lightning_step", &lightning_step);
+  m.def("lightning_scan", &lightning_scan);
+  m.def("lightning_norm", &lightning_norm);
+  m.def("lightning_pow_cols", &omnia_lightning_pow_cols);
+  m.def("lightning_scratch", &omnia_lightning_scratch);
   m.def("delta_prep", &delta_prep);
   m.def("delta_step", &delta_step);
   m.def("delta_scan", &delta_scan);
@@ -1733,7 +1863,9 @@ PYBIND11_MODULE(_omnia_kernels, m) {
         py::arg("sorted"), py::arg("blk_expert"), py::arg("n_blocks"), py::arg("route_w"),
         py::arg("topk"), py::arg("n_assign"), py::arg("e_lo"), py::arg("alpha") = 0.0,
         py::arg("limit") = 0.0);
-  m.def("moe_route", &moe_route);
+  m.def("moe_route", &moe_route, py::arg("ids"), py::arg("wts"), py::arg("x"), py::arg("router"),
+        py::arg("k"), py::arg("sigmoid"), py::arg("renorm"), py::arg("corr") = py::none(),
+        py::arg("groups") = 1, py::arg("keep") = 1);
   m.def("moe_align", &moe_align);
   m.def("moe_gemm", &moe_gemm, py::arg("mode"), py::arg("out"), py::arg("A"), py::arg("W"),
         py::arg("sorted"), py::arg("blk_expert"), py::arg("n_blocks"), py::arg("route_w"),

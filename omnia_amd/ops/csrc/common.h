@@ -46,6 +46,14 @@ __device__ __forceinline__ float sigmoidf_(float x) {
   return __builtin_amdgcn_rcpf(1.f + __expf(-x));
 }
 __device__ __forceinline__ float siluf_(float x) { return x * sigmoidf_(x); }
+// gelu, tanh form: 0.5 x (1 + tanh(y)) = x sigmoid(2 y)
+__device__ __forceinline__ float gelu_tanh_(float x) {
+  return x * sigmoidf_(1.5957691216057308f * (x + 0.044715f * x * x * x));
+}
+// gelu, erf form
+__device__ __forceinline__ float gelu_erf_(float x) {
+  return 0.5f * x * (1.f + erff(x * 0.7071067811865476f));
+}
 
 // sum over the 16 lanes of a DPP row, result in every lane of the row
 template <int CTRL>

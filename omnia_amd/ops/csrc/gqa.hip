@@ -4,19 +4,20 @@
 //
 //   k pages [num_pages][G][page][Dp], v pages [num_pages][G][page][Vp]
 //
-// Query head h reads key/value head h / (H / G).  A query at position i sees keys j with
-// 0 <= i - j < window (window 0: all); the softmax denominator of head h also holds
-// exp(sink[h]) (sinks null: none).  Scores, softmax and norms are fp32.
+// Query head h reads key/value head h / (H / G).  A query sees the keys its Mask names (a
+// window with kept first keys, a chunk, or all; mask.h); the softmax denominator of head h
+// also holds exp(sink[h]) (sinks null: none).  Scores, softmax and norms are fp32.
 //
 //   gqa_prep     one fused projection row [q (H*Dp) | k (G*Dp) | v (G*Vp)] (or its split-K
-//                slabs) -> per-head RMS norm of q and k, rotate-half rotary on the first R
-//                dimensions, q rows out, k / v rows into the pages.  G = 0: q only (a layer
-//                that attends to another layer's pages)
+//                slabs) -> + bias, per-head RMS norm of q and k, rotary on the first R
+//                dimensions (halves or neighbours paired), q rows out, k / v rows into the
+//                pages; bias, norm and rotation each if asked.  G = 0: q only (a layer that
+//                attends to another layer's pages)
 //   gqa_attend   generic attention (any size, bf16 or fp32), decode and prefill
 //   gqa_decode   bf16 decode: Q K^T on MFMA, P V on the VALU, the visible keys cut into
 //                equal parts on the device, + gqa_merge
 //   gqa_prefill  bf16 prefill (gqa_prefill.hip)
-#include "common.h"
+#include "mask.h"
 
 using namespace omnia;
 
@@ -67,12 +68,13 @@ __device__ __forceinline__ int find_seq(const int* q_start, int nseq, int t) {
 // columns a lane and step (NC steps).
 struct PrepArgs {
   const float* wq;
-  const float* wk;       // per-dimension norm weights [Dp]
+  const float* wk;       // per-dimension norm weights [Dp]; wq null: no norm
+  const float* bias;     // per projection column, or null
   const int* positions;
   const int64_t* slots;  // < 0: no write (padded row)
   const float* cos_sin;  // [positions][R] = (cos[R/2] | sin[R/2])
   int64_t ldx, slab;
-  int S, H, G, D, Dp, Vp, R, page, lg;
+  int S, H, G, D, Dp, Vp, R, page, lg, pairs;  // pairs: neighbours turn together
   float eps;
 };
 
@@ -110,13 +112,26 @@ __global__ __launch_bounds__(256) void prep_kernel(T* __restrict__ q, T* __restr
 #pragma unroll
       for (int e = 0; e < 2; ++e) v[i][e] += (p[0][e] + p[1][e]) + (p[2][e] + p[3][e]);
     }
+    if (a.bias && in) {
+      v[i][0] += load4(a.bias + col + c);
+      v[i][1] += load4(a.bias + col + c + 4);
+    }
 #pragma unroll
     for (int j = 0; j < 4; ++j) ss += v[i][0][j] * v[i][0][j] + v[i][1][j] * v[i][1][j];
   }
   const int pos = a.positions[t], half = a.R >> 1, turned = isv ? 0 : a.R;
   const float* cs = a.cos_sin + (int64_t)pos * a.R;
   float* row = rows + (tid >> a.lg << a.lg) * NC * 8;
-  if (!isv) {
+  if (!isv && !a.wq) {
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+      const int c = (l + (i << a.lg)) * 8;
+      if (c < width) {
+        store4(row + c, v[i][0]);
+        store4(row + c + 4, v[i][1]);
+      }
+    }
+  } else if (!isv) {
     for (int o = lph >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
     const float r = 1.f / sqrtf(ss / (float)a.D + a.eps);
     const float* w = isq ? a.wq : a.wk;
@@ -148,7 +163,19 @@ __global__ __launch_bounds__(256) void prep_kernel(T* __restrict__ q, T* __restr
     const int c = (l + (i << a.lg)) * 8;
     if (c >= width) continue;
     if (c < turned) {
-      if ((half & 7) == 0) {  // a chunk lies in one half of the rotated part
+      if (a.pairs) {
+#pragma unroll
+        for (int e = 0; e < 2; ++e)
+#pragma unroll
+          for (int j = 0; j < 4; j += 2) {
+            const int n = c + 4 * e + j, p = n >> 1;
+            if (n < turned) {
+              const float x0 = v[i][e][j], x1 = v[i][e][j + 1];
+              v[i][e][j] = x0 * cs[p] - x1 * cs[half + p];
+              v[i][e][j + 1] = x1 * cs[p] + x0 * cs[half + p];
+            }
+          }
+      } else if ((half & 7) == 0) {  // a chunk lies in one half of the rotated part
         const bool first = c < half;
         const int p = first ? c : c - half;
         const float sg = first ? -1.f : 1.f;
@@ -198,7 +225,7 @@ __global__ __launch_bounds__(256) void attend_kernel(
     T* __restrict__ out, const T* __restrict__ q, const T* __restrict__ kc,
     const T* __restrict__ vc, const int* __restrict__ block_tables, int bt_stride,
     const int* __restrict__ q_start, int nseq, const int* __restrict__ positions, int page, int H,
-    int G, int Dp, int Vp, int window, float scale, const float* __restrict__ sinks) {
+    int G, int Dp, int Vp, Mask mask, float scale, const float* __restrict__ sinks) {
   extern __shared__ float sm[];
   float* qs = sm;        // [Dp]
   float* acc = qs + Dp;  // [Vp]
@@ -208,16 +235,17 @@ __global__ __launch_bounds__(256) void attend_kernel(
   const int s = q_start ? find_seq(q_start, nseq, t) : t;
   const int* bt = block_tables + (int64_t)s * bt_stride;
   const int pos = positions[t];
-  const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+  const int lo = mask.lo(pos), kp = mask.kept(lo), vis = kp + pos + 1 - lo;
   const T* qr = q + ((int64_t)t * H + h) * Dp;
   for (int i = tid; i < Dp; i += 256) qs[i] = ldf(qr + i);
   for (int i = tid; i < Vp; i += 256) acc[i] = 0.f;
-  auto at = [&](int key) {  // row index of a key in the pages
+  auto at = [&](int i) {  // row in the pages of the i-th visible key
+    const int key = i < kp ? i : lo + i - kp;
     return ((int64_t)bt[key / page] * G + g) * page + key % page;
   };
   float m = sinks ? sinks[h] : -INFINITY, l = sinks ? 1.f : 0.f;
-  for (int k0 = lo; k0 <= pos; k0 += 256) {
-    const int n = min(256, pos + 1 - k0);
+  for (int k0 = 0; k0 < vis; k0 += 256) {
+    const int n = min(256, vis - k0);
     __syncthreads();
     float sc = -INFINITY;
     if (tid < n) {
@@ -243,8 +271,8 @@ __global__ __launch_bounds__(256) void attend_kernel(
 }
 
 // ----------------------------------------------------------------- gqa_decode
-// The visible keys of a row, [lo, pos], in parts of part_len keys: decided on the device
-// from the live length, so one captured graph splits every context evenly.
+// The visible keys of a row (kept ones, then its window) in parts of part_len keys: decided
+// on the device from the live length, so one captured graph splits every context evenly.
 constexpr int MIN_PART = 64;
 
 __device__ __forceinline__ int part_len(int n, int splits) {
@@ -263,7 +291,7 @@ __global__ __launch_bounds__(64 * NW) void decode_kernel(
     bf16_t* __restrict__ out, float* __restrict__ part_o, float* __restrict__ part_ml,
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
     const int* __restrict__ block_tables, int bt_stride, const int* __restrict__ positions, int H,
-    int G, int nch, int page_lg, int Vp, int window, float scale_log2,
+    int G, int nch, int page_lg, int Vp, Mask mask, float scale_log2,
     const float* __restrict__ sinks, int cap) {
   constexpr int Dp = 32 * KK, UG = KK > 4 ? 2 : 4, U = 4, TG = 64 / LPR;
   extern __shared__ __attribute__((aligned(16))) char smem[];
@@ -274,16 +302,21 @@ __global__ __launch_bounds__(64 * NW) void decode_kernel(
   const int b = blockIdx.x, g = blockIdx.y / nch, ch0 = blockIdx.y % nch, part = blockIdx.z;
   const int group = H / G, h0 = g * group + ch0 * GH, hn = min(GH, group - ch0 * GH);
   const int pos = positions[b];
-  const int lo = window > 0 ? max(0, pos - window + 1) : 0;
-  const int vis = pos + 1 - lo, splits = gridDim.z;
+  const int lo = mask.lo(pos), kept = mask.kept(lo);
+  const int vis = kept + pos + 1 - lo, splits = gridDim.z;
   const int pl = part_len(vis, splits);
-  const int p0 = lo + part * pl;
-  if (p0 > pos) return;
-  const int n = min(pl, pos + 1 - p0), nparts = (vis + pl - 1) / pl;
+  const int p0 = part * pl;
+  if (p0 >= vis) return;
+  const int n = min(pl, vis - p0), nparts = (vis + pl - 1) / pl;
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, pmask = (1 << page_lg) - 1;
-  const int pg0 = p0 >> page_lg, npg = ((p0 + n - 1) >> page_lg) - pg0 + 1;
-  for (int i = tid; i < npg; i += 64 * NW)
-    pages[i] = block_tables[(int64_t)b * bt_stride + pg0 + i];
+  // the part's kept keys p0 .. and, from index nk on, window keys w0 ..; their pages lie
+  // behind one another in LDS
+  const int nk = max(0, min(kept - p0, n)), w0 = lo + max(0, p0 - kept);
+  const int ka = p0 >> page_lg, nkp = nk > 0 ? ((p0 + nk - 1) >> page_lg) - ka + 1 : 0;
+  const int wa = w0 >> page_lg;
+  const int nwp = n > nk ? ((w0 + n - nk - 1) >> page_lg) - wa + 1 : 0;
+  for (int i = tid; i < nkp + nwp; i += 64 * NW)
+    pages[i] = block_tables[(int64_t)b * bt_stride + (i < nkp ? ka + i : wa + i - nkp)];
 
   short8 qf[KK];
   {
@@ -294,8 +327,10 @@ __global__ __launch_bounds__(64 * NW) void decode_kernel(
   }
   __syncthreads();
   auto at = [&](int i) {  // row of the part's i-th key
-    const int key = p0 + i;
-    return (((int64_t)pages[(key >> page_lg) - pg0] * G + g) << page_lg) + (key & pmask);
+    const bool k = i < nk;
+    const int key = k ? p0 + i : w0 + i - nk;
+    return (((int64_t)pages[(key >> page_lg) - (k ? ka : wa - nkp)] * G + g) << page_lg) +
+           (key & pmask);
   };
   const int ngroups = (n + 15) / 16;
   for (int grp0 = w; grp0 < ngroups; grp0 += NW * UG) {
@@ -426,13 +461,13 @@ __global__ __launch_bounds__(128) void merge_kernel(bf16_t* __restrict__ out,
                                                     const float* __restrict__ part_o,
                                                     const float* __restrict__ part_ml,
                                                     const int* __restrict__ positions, int H,
-                                                    int Vp, int window, int splits,
+                                                    int Vp, Mask mask, int splits,
                                                     const float* __restrict__ sinks) {
   extern __shared__ float wt[];  // [splits]
   __shared__ float scratch[2];
   const int bh = blockIdx.x, b = bh / H, h = bh - b * H;
   const int pos = positions[b];
-  const int vis = pos + 1 - (window > 0 ? max(0, pos - window + 1) : 0);
+  const int lo = mask.lo(pos), vis = mask.kept(lo) + pos + 1 - lo;
   const int pl = part_len(vis, splits), nparts = (vis + pl - 1) / pl;
   if (nparts <= 1) return;
   const float* ml = part_ml + (int64_t)bh * splits * 2;
@@ -475,8 +510,9 @@ extern "C" {
 // ptype: storage of x -- 0 bf16, 1 fp32, 2 fp16 (slabs)
 int omnia_gqa_prep(void* q, void* kc, void* vc, int f32, const void* x, int ptype, int S,
                    int64_t slab, int64_t ldx, const float* wq, const float* wk,
-                   const int* positions, const int64_t* slots, const float* cos_sin, int T, int H,
-                   int G, int D, int Dp, int Vp, int R, int page, float eps, hipStream_t s) {
+                   const float* bias, const int* positions, const int64_t* slots,
+                   const float* cos_sin, int pairs, int T, int H, int G, int D, int Dp, int Vp,
+                   int R, int page, float eps, hipStream_t s) {
   if (Dp % 8 || Vp % 8 || ldx % 8 || slab % 8 || S < 1 || R % 2 || R > D || D > Dp || page < 1)
     return -1;
   const int w = Dp > Vp || G == 0 ? Dp : Vp;
@@ -484,8 +520,8 @@ int omnia_gqa_prep(void* q, void* kc, void* vc, int f32, const void* x, int ptyp
   if (T == 0) return 0;
   int lg = 2;
   while (lg < 6 && (8 << lg) < w) ++lg;
-  const PrepArgs a{wq, wk, positions, slots, cos_sin, ldx, slab, S,   H,
-                   G,  D,  Dp,        Vp,    R,       page, lg,  eps};
+  const PrepArgs a{wq, wk, bias, positions, slots, cos_sin, ldx, slab,  S,  H,
+                   G,  D,  Dp,   Vp,        R,     page,    lg,  pairs, eps};
   const int hpb = 256 >> lg;
   const dim3 grid(T, (H + 2 * G + hpb - 1) / hpb);
 #define OMNIA_GP(TT, PP)                                                                       \
@@ -512,8 +548,8 @@ int omnia_gqa_prep(void* q, void* kc, void* vc, int f32, const void* x, int ptyp
 int omnia_gqa_attend(void* out, int f32, const void* q, const void* kc, const void* vc,
                      const int* block_tables, int bt_stride, const int* q_start, int nseq,
                      const int* positions, int T, int page, int H, int G, int Dp, int Vp,
-                     int window, float scale, const float* sinks, hipStream_t s) {
-  if (G < 1 || H % G || page < 1 || window < 0) return -1;
+                     Mask mask, float scale, const float* sinks, hipStream_t s) {
+  if (G < 1 || H % G || page < 1 || !mask.ok()) return -1;
   if (T == 0) return 0;
   const size_t lds = (size_t)(Dp + Vp + 256 + 8) * 4;
   if (lds > 64 * 1024 || H > 65535) return -2;
@@ -521,23 +557,24 @@ int omnia_gqa_attend(void* out, int f32, const void* q, const void* kc, const vo
   if (f32)
     attend_kernel<float><<<grid, 256, lds, s>>>((float*)out, (const float*)q, (const float*)kc,
                                                 (const float*)vc, block_tables, bt_stride, q_start,
-                                                nseq, positions, page, H, G, Dp, Vp, window, scale,
+                                                nseq, positions, page, H, G, Dp, Vp, mask, scale,
                                                 sinks);
   else
     attend_kernel<bf16_t><<<grid, 256, lds, s>>>(
         (bf16_t*)out, (const bf16_t*)q, (const bf16_t*)kc, (const bf16_t*)vc, block_tables,
-        bt_stride, q_start, nseq, positions, page, H, G, Dp, Vp, window, scale, sinks);
+        bt_stride, q_start, nseq, positions, page, H, G, Dp, Vp, mask, scale, sinks);
   return (int)hipGetLastError();
 }
 
-// max_keys: no row sees more keys than this (sizes the score tile)
+// max_ctx: no context is longer than this (sizes the score tile)
 int omnia_gqa_decode(void* out, float* part_o, float* part_ml, const void* q, const void* kc,
                      const void* vc, const int* block_tables, int bt_stride, const int* positions,
-                     int T, int page, int H, int G, int Dp, int Vp, int window, float scale,
-                     const float* sinks, int splits, int max_keys, hipStream_t s) {
+                     int T, int page, int H, int G, int Dp, int Vp, Mask mask, float scale,
+                     const float* sinks, int splits, int max_ctx, hipStream_t s) {
+  const int max_keys = mask.ok() ? mask.most(max_ctx) : 0;
   const int lg = log2i(page);
   if (lg < 0 || G < 1 || H % G || Dp % 32 || Dp > 256 || Vp % 8 || Vp > 256 || splits < 1 ||
-      max_keys < 1 || window < 0 || H > 65535 || splits > 8192)
+      max_keys < 1 || H > 65535 || splits > 8192)
     return -1;
   if (T == 0) return 0;
   const int group = H / G, gh = group >= 5 ? 8 : group >= 3 ? 4 : group;
@@ -547,13 +584,13 @@ int omnia_gqa_decode(void* out, float* part_o, float* part_ml, const void* q, co
   // two-wave workgroups once there are enough of them to keep the chip's loads in flight
   const int nw = (int64_t)T * G * nch * splits >= 1024 ? 2 : 4;
   const int tile = gh * cap > nw * gh * Vp ? gh * cap : nw * gh * Vp;
-  const size_t lds = 64 + (size_t)tile * 4 + (size_t)(cap / page + 2) * 4;
+  const size_t lds = 64 + (size_t)tile * 4 + (size_t)(cap / page + 4) * 4;
   if (lds > 96 * 1024) return -2;
   const dim3 grid(T, G * nch, splits);
 #define OMNIA_GD(KK, LP, GH, NN)                                                               \
   decode_kernel<KK, LP, GH, NN><<<grid, 64 * NN, lds, s>>>(                                    \
       (bf16_t*)out, part_o, part_ml, (const bf16_t*)q, (const bf16_t*)kc, (const bf16_t*)vc,   \
-      block_tables, bt_stride, positions, H, G, nch, lg, Vp, window, scale * kLog2e, sinks, cap)
+      block_tables, bt_stride, positions, H, G, nch, lg, Vp, mask, scale * kLog2e, sinks, cap)
 #define OMNIA_GD_N(KK, LP, GH) \
   do { if (nw == 2) OMNIA_GD(KK, LP, GH, 2); else OMNIA_GD(KK, LP, GH, 4); } while (0)
 #define OMNIA_GD_G(KK, LP)                      \
@@ -583,7 +620,7 @@ int omnia_gqa_decode(void* out, float* part_o, float* part_ml, const void* q, co
 #undef OMNIA_GD_N
 #undef OMNIA_GD
   if (splits > 1)
-    merge_kernel<<<T * H, 128, splits * 4, s>>>((bf16_t*)out, part_o, part_ml, positions, H, Vp, window,
+    merge_kernel<<<T * H, 128, splits * 4, s>>>((bf16_t*)out, part_o, part_ml, positions, H, Vp, mask,
                                        splits, sinks);
   return (int)hipGetLastError();
 }

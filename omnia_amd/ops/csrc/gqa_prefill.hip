@@ -8,12 +8,13 @@
 //   O^T += V^T P^T   the lane's own scores are the B operand; V^T fragments by
 //                    ds_read_b64_tr_b16 from the row-major tile, the keys of a k-step
 //                    permuted the same way on both sides
-// Tiles go global -> LDS by LDS-DMA, two stages, one barrier a tile; tiles before the
-// block's window are not visited, tiles outside a wave's own window not computed.  The
+// Tiles go global -> LDS by LDS-DMA, two stages, one barrier a tile; the tiles of kept first
+// keys come before those of the block's window, the ones between are not visited, and tiles
+// of which a wave sees nothing are not computed.  The
 // sink is the initial term of the online softmax (maximum = sink, sum = 1).
 #include <type_traits>
 
-#include "common.h"
+#include "mask.h"
 
 using namespace omnia;
 
@@ -52,7 +53,8 @@ struct Args {
   const int* tile_seq;
   const int* tile_q0;
   const float* sinks;  // [H] or null
-  int bt_stride, n_tiles, H, G, hb_lg, page_lg, window;
+  int bt_stride, n_tiles, H, G, hb_lg, page_lg;
+  Mask mask;
   float scale_log2;
 };
 
@@ -91,12 +93,18 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
 #pragma unroll
     for (int ks = 0; ks < DK / 16; ++ks) qf[ks] = *reinterpret_cast<const short8*>(qrow + 16 * ks);
   }
-  const int win = p.window > 0 ? p.window : 1 << 30;
+  const int keep = p.mask.keep, qlo = p.mask.lo(qpos);
+  const int lo_min = p.mask.lo(wmin), lo_max = p.mask.lo(wmax);
   const int kv_end = off + min(b0 + rows, qlen);
-  const int t0 = max(0, off + b0 - win + 1) >> 6, t1 = (kv_end + 63) >> 6;
-  const int pg0 = (t0 << 6) >> p.page_lg;  // first staged page
-  const int npg = min(((kv_end - 1) >> p.page_lg) - pg0 + 1, kMaxPages);
-  for (int i = tid; i < npg; i += 256) pg_lds[i] = bt[pg0 + i];
+  // visited tiles: [0, tk) with kept keys, then the window's [t0, t1)
+  const int t0 = p.mask.lo(off + b0) >> 6, t1 = (kv_end + 63) >> 6;
+  const int tk = min((keep + 63) >> 6, t0), nt = tk + t1 - t0;
+  auto tile_of = [&](int j) { return j < tk ? j : t0 + j - tk; };
+  // staged pages: those of the kept tiles, then the window's from pg0 on
+  const int nkp = ((tk << 6) + BS - 1) >> p.page_lg;
+  const int pg0 = (t0 << 6) >> p.page_lg;
+  const int npg = min(nkp + ((kv_end - 1) >> p.page_lg) - pg0 + 1, kMaxPages);
+  for (int i = tid; i < npg; i += 256) pg_lds[i] = bt[i < nkp ? i : pg0 + i - nkp];
   __syncthreads();
 
   typedef __attribute__((address_space(3))) void* lds_ptr_t;
@@ -109,9 +117,9 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
     for (int i = 0; i < N; ++i) {
       const int c = (w * N + i) * 64 + lane, row = c / CPR;
       const int key = min(t * 64 + row, kv_end - 1);
-      const int pi = (key >> p.page_lg) - pg0;
+      const int pi = (key >> p.page_lg) - (t < tk ? 0 : pg0 - nkp);
       const int pl = pg_lds[pi < kMaxPages ? pi : 0];
-      const int page = pi < kMaxPages ? pl : bt[pg0 + pi];
+      const int page = pi < kMaxPages ? pl : bt[key >> p.page_lg];
       at[i] = ((((int64_t)page * p.G + kvh) << p.page_lg) + (key & pmask)) * W +
               8 * ((c - row * CPR) ^ swz<W>(row));
     }
@@ -139,15 +147,16 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
 
   using B0 = std::integral_constant<int, 0>;
   using B1 = std::integral_constant<int, 1>;
-  dma(t0, B0{});
+  dma(tile_of(0), B0{});
   __syncthreads();
-  auto body = [&](int t, auto BUF) {
+  auto body = [&](int j, auto BUF) {
     constexpr int buf = decltype(BUF)::value;
-    if (t + 1 < t1) dma(t + 1, std::integral_constant<int, 1 - buf>{});
+    const int t = tile_of(j);
+    if (j + 1 < nt) dma(tile_of(j + 1), std::integral_constant<int, 1 - buf>{});
     const char* Kl = buf ? st1 : st0;
     const char* Vl = Kl + 128 * DK;
     const int k0 = t * 64;
-    if (k0 <= wmax && k0 + 63 > wmin - win) {  // wave-uniform: some row sees some key
+    if (k0 <= wmax && (k0 + 63 >= lo_min || k0 < keep)) {  // wave-uniform: some row sees some key
       float16v sa[2];
 #pragma unroll
       for (int half = 0; half < 2; ++half) {
@@ -159,14 +168,14 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
                             qf[ks], sa[half]);
       }
       float mloc = -INFINITY;
-      if (k0 + 63 > wmin || k0 <= wmax - win) {  // an edge crosses the tile
-        const int top = qpos - k0 - 4 * hi, bot = qpos - win + 1 - k0 - 4 * hi;
+      if (k0 + 63 > wmin || (k0 < lo_max && k0 + 63 >= keep)) {  // an edge crosses the tile
+        const int top = qpos - k0 - 4 * hi, bot = qlo - k0 - 4 * hi, kp = keep - k0 - 4 * hi;
 #pragma unroll
         for (int half = 0; half < 2; ++half)
 #pragma unroll
           for (int r = 0; r < 16; ++r) {
             const int kk = half * 32 + (r & 3) + 8 * (r >> 2);
-            const float v = (kk > top || kk < bot) ? -INFINITY : sa[half][r];
+            const float v = (kk > top || (kk < bot && kk >= kp)) ? -INFINITY : sa[half][r];
             sa[half][r] = v;
             mloc = fmaxf(mloc, v);
           }
@@ -220,9 +229,9 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
     }
     __syncthreads();  // the next tile landed and this one is read by all waves
   };
-  for (int t = t0; t < t1; t += 2) {
-    body(t, B0{});
-    if (t + 1 < t1) body(t + 1, B1{});
+  for (int j = 0; j < nt; j += 2) {
+    body(j, B0{});
+    if (j + 1 < nt) body(j + 1, B1{});
   }
   if (row_ok) {
     const float inv = 1.f / l_run;
@@ -246,9 +255,9 @@ extern "C" {
 int omnia_gqa_prefill(void* out, const void* q, const void* kc, const void* vc,
                       const int* block_tables, int bt_stride, const int* q_start,
                       const int* seq_lens, const int* tile_seq, const int* tile_q0, int n_tiles,
-                      int page, int H, int G, int Dp, int Vp, int window, float scale,
+                      int page, int H, int G, int Dp, int Vp, Mask mask, float scale,
                       const float* sinks, hipStream_t s) {
-  if (G < 1 || H % G || window < 0) return -1;
+  if (G < 1 || H % G || !mask.ok()) return -1;
   int page_lg = 0;
   while (page_lg < 30 && (1 << page_lg) < page) ++page_lg;
   if ((1 << page_lg) != page) return -2;
@@ -257,7 +266,7 @@ int omnia_gqa_prefill(void* out, const void* q, const void* kc, const void* vc,
   if ((int64_t)n_tiles * H > 2147483647LL) return -4;
   Args a{(bf16_t*)out, (const bf16_t*)q, (const bf16_t*)kc, (const bf16_t*)vc, block_tables,
          q_start, seq_lens, tile_seq, tile_q0, sinks, bt_stride, n_tiles, H, G, hb_lg, page_lg,
-         window, scale * 1.4426950408889634f};
+         mask, scale * 1.4426950408889634f};
 #define OMNIA_GQ(K, V)                                                  \
   if (Dp == K && Vp == V) {                                             \
     prefill_kernel<K, V><<<n_tiles * H, 256, 0, s>>>(a);                \

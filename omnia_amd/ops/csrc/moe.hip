@@ -12,9 +12,11 @@
 //                          rows written back to their (token, slot) position
 //                  MODE 2: MODE 0 with a clamped GLU and the routing weight on the
 //                          expert's INPUT (W (r h) = r (W h): the epilogue scales)
+//                  MODE 3: ungated experts, gelu (erf form) of the up projection
 //                  fp32 models: the same modes on a plain fp32 tile
 //   * moe_route  : router logits in fp32 (never rounded), sigmoid or softmax scores,
-//                  top-k of up to 256 experts
+//                  top-k of up to 256 experts, if asked by corrected scores and within the
+//                  best groups of neighbours
 //   * moe_combine: out[t] = sum_j Y[t*k + j]  (deterministic, no atomics)
 // Expert parallelism: moe_align keeps only experts in [e_lo, e_hi); the caller
 // all-reduces the combined output over the EP group.
@@ -128,9 +130,12 @@ __global__ __launch_bounds__(256) void moe_router_topk_kernel(
 
 // fp32 router for any score function: logits z[e] = x . router[e] stay fp32; the k
 // largest are chosen; weights are sigmoid(z) or softmax(z), renormalised over the chosen
-// ones if asked.  One wave per token; expert e belongs to lane e & 63; EC experts'
-// dot products at a time.
+// ones if asked.  With a correction the choice goes by score + correction (weights stay the
+// plain scores); with groups, experts outside the `keep` groups of E / groups neighbours
+// with the largest choice score are out of the choice.  One wave per token; expert e
+// belongs to lane e & 63; EC experts' dot products at a time.
 constexpr int kMaxExperts = 256;
+constexpr float kRenormEps = 1e-20f;
 
 template <typename T, int EC>
 __global__ __launch_bounds__(256) void moe_route_kernel(int* __restrict__ ids,
@@ -138,7 +143,10 @@ __global__ __launch_bounds__(256) void moe_route_kernel(int* __restrict__ ids,
                                                         const T* __restrict__ x,
                                                         const T* __restrict__ router, int n_tok,
                                                         int d, int E, int k, int sigmoid,
-                                                        int renorm) {
+                                                        int renorm,
+                                                        const float* __restrict__ corr,
+                                                        int groups, int keep) {
+  __shared__ float pick[4][kMaxExperts];  // a token's choice scores, then its groups'
   constexpr int NPL = kMaxExperts / 64;
   const int lane = threadIdx.x & 63;
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
@@ -196,30 +204,82 @@ __global__ __launch_bounds__(256) void moe_route_kernel(int* __restrict__ ids,
 #pragma unroll
     for (int i = 0; i < NPL; ++i) total += expf(z[i] - top);
     total = wave_sum(total);
+    if (!(total > 0.f)) total = 1.f;
   }
-  unsigned taken = 0;  // bit i: this lane's expert lane + 64 i is chosen
+  // choice score of this lane's experts: monotone in the logit without a correction
+  float c[NPL];
+  unsigned taken = 0;  // bit i: this lane's expert lane + 64 i is chosen, or out of the choice
+#pragma unroll
+  for (int i = 0; i < NPL; ++i) {
+    c[i] = z[i];
+    const int e = lane + 64 * i;
+    if (corr && e < E) {
+      c[i] = (sigmoid ? 1.f / (1.f + expf(-z[i])) : expf(z[i] - top) / total) + corr[e];
+      if (!(c[i] == c[i])) c[i] = -INFINITY;
+    }
+  }
+  if (groups > 1) {
+    const int wv = threadIdx.x >> 6, per = E / groups;
+#pragma unroll
+    for (int i = 0; i < NPL; ++i)
+      if (lane + 64 * i < E) pick[wv][lane + 64 * i] = c[i];
+    __builtin_amdgcn_wave_barrier();
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // this wave's LDS writes
+    float gs[NPL];
+#pragma unroll
+    for (int i = 0; i < NPL; ++i) {
+      gs[i] = -INFINITY;
+      const int g = lane + 64 * i;
+      if (g < groups)
+        for (int j = 0; j < per; ++j) gs[i] = fmaxf(gs[i], pick[wv][g * per + j]);
+    }
+    __builtin_amdgcn_wave_barrier();
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+#pragma unroll
+    for (int i = 0; i < NPL; ++i)
+      if (lane + 64 * i < groups) pick[wv][lane + 64 * i] = gs[i];
+    __builtin_amdgcn_wave_barrier();
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+#pragma unroll
+    for (int i = 0; i < NPL; ++i) {
+      const int e = lane + 64 * i;
+      if (e >= E) continue;
+      const int g = e / per;
+      const float mine_g = pick[wv][g];
+      int better = 0;  // groups ahead of this expert's (lower index wins ties)
+      for (int j = 0; j < groups; ++j) {
+        const float o = pick[wv][j];
+        better += o > mine_g || (o == mine_g && j < g);
+      }
+      if (better >= keep) taken |= 1u << i;
+    }
+  }
   float sel = 0.f, mine = 0.f;
   for (int j = 0; j < k; ++j) {
     float v = -INFINITY;
 #pragma unroll
     for (int i = 0; i < NPL; ++i)
-      if (!(taken >> i & 1) && lane + 64 * i < E) v = fmaxf(v, z[i]);
+      if (!(taken >> i & 1) && lane + 64 * i < E) v = fmaxf(v, c[i]);
     const float vm = wave_max(v);
-    int first = 1 << 30;  // lowest untaken expert with the largest logit
+    int first = 1 << 30;  // lowest untaken expert with the largest choice score
 #pragma unroll
     for (int i = NPL - 1; i >= 0; --i)
-      if (!(taken >> i & 1) && lane + 64 * i < E && z[i] == vm) first = lane + 64 * i;
+      if (!(taken >> i & 1) && lane + 64 * i < E && c[i] == vm) first = lane + 64 * i;
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) first = min(first, __shfl_xor(first, o, 64));
     if ((first & 63) == lane) taken |= 1u << (first >> 6);
-    const float s = sigmoid ? 1.f / (1.f + expf(-vm)) : expf(vm - top);
+    float zf = -INFINITY;  // the chosen expert's logit
+#pragma unroll
+    for (int i = 0; i < NPL; ++i)
+      if (first == lane + 64 * i) zf = z[i];
+    zf = __shfl(zf, first & 63, 64);
+    const float s = sigmoid ? 1.f / (1.f + expf(-zf)) : expf(zf - top) / total;
     sel += s;
     if (lane == j) mine = s;  // k <= 64: lane j keeps slot j
     if (lane == 0) ids[(int64_t)t * k + j] = first;
   }
   if (lane < k) {
-    const float den = renorm ? sel : sigmoid ? 1.f : total;
-    wts[(int64_t)t * k + lane] = den > 0.f ? mine / den : 0.f;
+    wts[(int64_t)t * k + lane] = renorm ? mine / (sel + kRenormEps) : mine;
   }
 }
 
@@ -287,7 +347,7 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(
     const int* __restrict__ sorted, const int* __restrict__ blk_expert,
     const int* __restrict__ n_blocks, const float* __restrict__ route_w, int K, int N,
     int topk, int n_assign, int e_lo, Glu glu) {
-  constexpr bool GATED = MODE != 1;
+  constexpr bool GATED = MODE == 0 || MODE == 2, GATHER = MODE != 1;
   __shared__ __attribute__((aligned(16))) bf16_t lds[2 * 2 * BM * 64];
   const int mb = blockIdx.y;
   if (mb >= *n_blocks) return;
@@ -306,7 +366,7 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(
     const int c = tid + i * 256;  // 0..511
     const int row = c >> 3, ch = c & 7;
     const int flat = sorted[mb * BM + row];
-    const int64_t arow = GATED ? (flat < n_assign ? flat / topk : 0) : (int64_t)mb * BM + row;
+    const int64_t arow = GATHER ? (flat < n_assign ? flat / topk : 0) : (int64_t)mb * BM + row;
     a_src[i] = A + arow * K + ch * 8;
     a_lds[i] = swz(row, ch);
     int wrow;
@@ -394,6 +454,10 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(
         const float s = g * __builtin_amdgcn_rcpf(1.f + __expf(-g));
         out[(int64_t)row * N + n0 + 16 * jj + fr] = f2bf(s * u);
       }
+    } else if (MODE == 3) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        out[(int64_t)row * N + n0 + 16 * j + fr] = f2bf(gelu_erf_(acc[j][r]));
     } else {
       const float wt = route_w ? route_w[flat] : 1.f;
 #pragma unroll
@@ -410,7 +474,7 @@ __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(
     const int* __restrict__ sorted, const int* __restrict__ blk_expert,
     const int* __restrict__ n_blocks, const float* __restrict__ route_w, int K, int N, int topk,
     int n_assign, int e_lo, Glu glu) {
-  constexpr bool GATED = MODE != 1;
+  constexpr bool GATED = MODE == 0 || MODE == 2, GATHER = MODE != 1;
   __shared__ float As[16][BM + 4], Bs[16][BM + 4];
   const int mb = blockIdx.y;
   if (mb >= *n_blocks) return;
@@ -419,7 +483,7 @@ __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(
   const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4;
   const int row = tid >> 2, kq = (tid & 3) * 4;
   const int f0 = sorted[mb * BM + row];
-  const float* ar = A + (GATED ? (int64_t)(f0 < n_assign ? f0 / topk : 0)
+  const float* ar = A + (GATHER ? (int64_t)(f0 < n_assign ? f0 / topk : 0)
                                : (int64_t)mb * BM + row) * K + kq;
   const int wrow = !GATED ? n0 + row : row < 32 ? n0 + row : N + n0 + row - 32;
   const float* br = We + (int64_t)wrow * K + kq;
@@ -469,6 +533,10 @@ __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(
         }
         out[(int64_t)r * N + n0 + 2 * tx + j] = y;
       }
+    } else if (MODE == 3) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        out[(int64_t)r * N + n0 + (j >> 1) * 32 + 2 * tx + (j & 1)] = gelu_erf_(acc[i][j]);
     } else {
       const float wt = route_w ? route_w[flat] : 1.f;
 #pragma unroll
@@ -548,15 +616,18 @@ int omnia_moe_align(int* sorted, int* blk_expert, int* n_blocks, const int* ids,
   return (int)hipGetLastError();
 }
 
-// x [T, d] and router [E, d] in one dtype -> ids / wts [T, k]; fp32 logits
+// x [T, d] and router [E, d] in one dtype -> ids / wts [T, k]; fp32 logits; corr [E] or null
 int omnia_moe_route(int* ids, float* wts, const void* x, const void* router, int f32, int n_tok,
-                    int d, int E, int k, int sigmoid, int renorm, hipStream_t s) {
+                    int d, int E, int k, int sigmoid, int renorm, const float* corr, int groups,
+                    int keep, hipStream_t s) {
   if (E < 1 || E > kMaxExperts || k < 1 || k > E || k > 64 || d % 8) return -1;
+  if (groups < 1 || E % groups || keep < 1 || keep > groups || k > keep * (E / groups)) return -2;
   if (n_tok == 0) return 0;
   const int blocks = (n_tok + 3) / 4;
 #define OMNIA_RO(TT, EC)                                                                       \
   moe_route_kernel<TT, EC><<<blocks, 256, 0, s>>>(ids, wts, (const TT*)x, (const TT*)router,   \
-                                                  n_tok, d, E, k, sigmoid, renorm)
+                                                  n_tok, d, E, k, sigmoid, renorm, corr,       \
+                                                  groups, keep)
 #define OMNIA_ROE(TT)            \
   do {                           \
     if (E <= 8) OMNIA_RO(TT, 8); \
@@ -572,16 +643,18 @@ int omnia_moe_route(int* ids, float* wts, const void* x, const void* router, int
 // mode 0: out = act [max_blocks*64, N=I], A = x [T, K=d], W = [E_local, 2I, d]
 // mode 1: out = Y [T*k, N=d],            A = act [max_blocks*64, K=I], W = [E_local, d, I]
 // mode 2: mode 0 with the clamped GLU (alpha, limit) of the weighted input
+// mode 3: mode 0 ungated, gelu(x W^T) with W = [E_local, I, d]
 int omnia_moe_gemm(int mode, void* out, const void* A, const void* W, int f32, const int* sorted,
                    const int* blk_expert, const int* n_blocks, const float* route_w, int K,
                    int N, int topk, int n_assign, int e_lo, int max_blocks, float alpha,
                    float limit, hipStream_t s) {
-  if (mode < 0 || mode > 2 || K % 64) return -1;
-  if (mode == 1 ? (N % 64) : (N % 32)) return -2;
+  if (mode < 0 || mode > 3 || K % 64) return -1;
+  const bool gated = mode == 0 || mode == 2;
+  if (N % (gated ? 32 : 64)) return -2;
   if (mode == 2 && !route_w) return -3;
   if (max_blocks == 0) return 0;
   if (max_blocks > 65535) return -4;
-  const dim3 grid(mode == 1 ? N / 64 : N / 32, max_blocks);
+  const dim3 grid(N / (gated ? 32 : 64), max_blocks);
   const Glu glu{alpha, limit};
 #define OMNIA_MG(KER, TT, MM)                                                                  \
   KER<MM><<<grid, 256, 0, s>>>((TT*)out, (const TT*)A, (const TT*)W, sorted, blk_expert,       \
@@ -590,7 +663,8 @@ int omnia_moe_gemm(int mode, void* out, const void* A, const void* W, int f32, c
   do {                                        \
     if (mode == 0) OMNIA_MG(KER, TT, 0);      \
     else if (mode == 1) OMNIA_MG(KER, TT, 1); \
-    else OMNIA_MG(KER, TT, 2);                \
+    else if (mode == 2) OMNIA_MG(KER, TT, 2); \
+    else OMNIA_MG(KER, TT, 3);                \
   } while (0)
   if (f32) OMNIA_MGM(moe_gemm_f32_kernel, float);
   else OMNIA_MGM(moe_gemm_kernel, bf16_t);

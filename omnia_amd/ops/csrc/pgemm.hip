@@ -36,6 +36,8 @@
 //          each row scaled by its routing weight (if given) and scattered to Y[assignment]
 //   EPI 8  EPI 5 with the routing weight on the expert's input and a clamped GLU
 //   EPI 7  EPI 1 with a bias: out = silu(g + bias[f]) * (u + bias[N + f])
+//   EPI 9  EPI 1 with the tanh form of gelu, unscaled: out = gelu(g) * u
+//   EPI 10 EPI 5 ungated: gelu (erf form) of the up projection, W = that segment's expert Wu
 //   EPI 4  split-K partial: block (m-tile, n-tile, k-slice ks) writes its K-slice's
 //          fp32 sum, saturated to fp16, into slab ks of out[S][M][N]; the splitk.hip
 //          consumers reduce the slabs (decode projections at M <= 256: one m-tile,
@@ -92,9 +94,13 @@ struct PArgs {
 };
 
 // a gate_up epilogue: 128 features per block tile, gate and up halves in one lane
-constexpr bool gated(int epi) { return epi == 1 || epi == 5 || epi == 7 || epi == 8; }
+constexpr bool gated(int epi) {
+  return epi == 1 || epi == 5 || epi == 7 || epi == 8 || epi == 9;
+}
 // rows are expert-sorted assignments
-constexpr bool grouped(int epi) { return epi == 5 || epi == 6 || epi == 8; }
+constexpr bool grouped(int epi) { return epi == 5 || epi == 6 || epi == 8 || epi == 10; }
+// A rows are token rows gathered by assignment
+constexpr bool gathered(int epi) { return epi == 5 || epi == 8 || epi == 10; }
 
 __device__ __forceinline__ float4v mfma16(short8 a, short8 b, float4v c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a),
@@ -298,7 +304,7 @@ __global__ __launch_bounds__(512, 2) void pgemm_kernel(PArgs p) {
     for (int h = 0; h < 2; ++h) {
       int ar = m0 + h * 128 + row;
       ar = ar < p.M ? ar : p.M - 1;  // rows past the chunk: clamped copies, never stored
-      if constexpr (MOE && gated(EPI)) {  // gather: the assignment's token row (padding: row 0)
+      if constexpr (gathered(EPI)) {  // gather: the assignment's token row (padding: row 0)
         const int f = p.sorted[m0 + h * 128 + row];
         ar = f < p.n_assign ? f / p.topk : 0;
       }
@@ -465,7 +471,8 @@ __global__ __launch_bounds__(512, 2) void pgemm_kernel(PArgs p) {
   // lane rows: a*128 + wr*64 + m*16 + fq*4 + j ; cols: b*128 + wc*32 + n*16 + fr
   float* rs_lds = reinterpret_cast<float*>(lds + RS_OFF);
   constexpr bool ROUTED = EPI == 6 || EPI == 8;
-  const bool scaled = ROUTED || (EPI != 2 && EPI != 7 && p.ss_in != nullptr);
+  constexpr bool UNSCALED = EPI == 2 || EPI == 7 || EPI == 9 || EPI == 10;
+  const bool scaled = ROUTED || (!UNSCALED && p.ss_in != nullptr);
   if (scaled) {
     if (tid < 256) {
       if constexpr (ROUTED) {  // row scale = the assignment's routing weight
@@ -551,6 +558,10 @@ __global__ __launch_bounds__(512, 2) void pgemm_kernel(PArgs p) {
 #pragma unroll
             for (int j = 0; j < 4; ++j)
               v[j] = silu(acc[a][0][m][n][j] + bg) * (acc[a][1][m][n][j] + bu);
+          } else if constexpr (EPI == 9) {
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+              v[j] = gelu_tanh_(acc[a][0][m][n][j]) * acc[a][1][m][n][j];
           } else if constexpr (EPI == 8) {
 #pragma unroll
             for (int j = 0; j < 4; ++j)
@@ -576,7 +587,11 @@ __global__ __launch_bounds__(512, 2) void pgemm_kernel(PArgs p) {
         for (int b = 0; b < 2; ++b)
 #pragma unroll
           for (int n = 0; n < 2; ++n) {
-            const float4v v = acc[a][b][m][n];
+            float4v v = acc[a][b][m][n];
+            if constexpr (EPI == 10) {
+#pragma unroll
+              for (int j = 0; j < 4; ++j) v[j] = gelu_erf_(v[j]);
+            }
             put(row0, b * 128 + wc * 32 + n * 16 + fr, v[0] * rs[0], v[1] * rs[1], v[2] * rs[2],
                 v[3] * rs[3]);
           }
@@ -590,6 +605,8 @@ __global__ __launch_bounds__(512, 2) void pgemm_kernel(PArgs p) {
     epi_out<4, 512>(q, stg, m0, nt, Mt, ntn, tid, lane);
   } else if constexpr (MOE && gated(EPI)) {
     epi_out<1, 512>(p, stg, m0, nt, Mt, ntn, tid, lane);
+  } else if constexpr (EPI == 10) {
+    epi_out<0, 512>(p, stg, m0, nt, Mt, ntn, tid, lane);
   } else {
     epi_out<EPI, 512>(p, stg, m0, nt, Mt, ntn, tid, lane);
   }
@@ -871,9 +888,10 @@ int omnia_pgemm(int epi, void* out, const void* X, const void* W, int M, int N, 
                 const float* ss_in, int ss_in_n, float inv_d, float eps, float* ss_out,
                 const int* positions, const float* cos_sin, void* k_cache, void* v_cache,
                 const int64_t* slots, int hq, int hkv, int block_size, const float* bias,
-                hipStream_t s) {
+                int gelu, hipStream_t s) {
   if (epi < 0 || epi > 3) return -1;
   if (bias && (epi != 1 || ss_in)) return -14;
+  if (gelu && (epi != 1 || ss_in || bias)) return -15;
   if (M < 1) return -2;
   if (K <= 0 || K % (2 * BK)) return -3;  // whole iterations of two K-tiles
   const int tn = epi == 1 ? 128 : 256;
@@ -902,6 +920,10 @@ int omnia_pgemm(int epi, void* out, const void* X, const void* W, int M, int N, 
   const dim3 grid((unsigned)blocks);
   if (bias) {
     pgemm_kernel<7><<<grid, 512, 0, s>>>(a);
+    return (int)hipGetLastError();
+  }
+  if (gelu) {
+    pgemm_kernel<9><<<grid, 512, 0, s>>>(a);
     return (int)hipGetLastError();
   }
   if (g_pgemm_sched == 1) {
@@ -974,20 +996,22 @@ int omnia_pgemm_splitk(void* parts, const void* X, const void* W, int M, int N, 
 // bm = 256).  mode 0: act [max_blocks*256, I] = SwiGLU(x[token] . W_gu[e]^T),
 // x [T, d], W_gu [E_loc, 2I, d];  mode 1: Y[assignment] = w_route * act . W_dn[e]^T,
 // act [max_blocks*256, I], W_dn [E_loc, d, I], Y [n_assign, d] (w_route null: 1);  mode 2:
-// mode 0 with the clamped GLU (alpha, limit) of the weighted input.
+// mode 0 with the clamped GLU (alpha, limit) of the weighted input;  mode 3: mode 0
+// ungated, gelu(x . W^T), W [E_loc, I, d].
 int omnia_pgemm_moe(int mode, void* out, const void* A, const void* W, const int* sorted,
                     const int* blk_expert, const int* n_blocks, const float* route_w, int K,
                     int N, int topk, int n_assign, int e_lo, int max_blocks, float alpha,
                     float limit, hipStream_t s) {
-  if (mode < 0 || mode > 2 || max_blocks < 0 || topk < 1) return -1;
+  if (mode < 0 || mode > 3 || max_blocks < 0 || topk < 1) return -1;
+  const int tn = mode == 0 || mode == 2 ? 128 : 256;
   if (K <= 0 || K % (2 * BK)) return -3;
-  if (N <= 0 || N % (mode == 1 ? 256 : 128)) return -4;
+  if (N <= 0 || N % tn) return -4;
   if ((reinterpret_cast<uintptr_t>(A) | reinterpret_cast<uintptr_t>(W) |
        reinterpret_cast<uintptr_t>(out)) & 15)
     return -5;
   if (!sorted || !blk_expert || !n_blocks || (mode == 2 && !route_w)) return -9;
   if (max_blocks == 0) return 0;
-  const int64_t blocks = (int64_t)max_blocks * (N / (mode == 1 ? 256 : 128));
+  const int64_t blocks = (int64_t)max_blocks * (N / tn);
   if (blocks > (1 << 30)) return -13;
   PArgs a{out, (const bf16_t*)A, (const bf16_t*)W, max_blocks * 256, N, K, N, nullptr, 0, 0.f,
           0.f, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, 0, 0, 0, 1, sorted,
@@ -996,6 +1020,8 @@ int omnia_pgemm_moe(int mode, void* out, const void* A, const void* W, const int
     pgemm_kernel<5><<<dim3((unsigned)blocks), 512, 0, s>>>(a);
   else if (mode == 2)
     pgemm_kernel<8><<<dim3((unsigned)blocks), 512, 0, s>>>(a);
+  else if (mode == 3)
+    pgemm_kernel<10><<<dim3((unsigned)blocks), 512, 0, s>>>(a);
   else
     pgemm_kernel<6><<<dim3((unsigned)blocks), 512, 0, s>>>(a);
   return (int)hipGetLastError();

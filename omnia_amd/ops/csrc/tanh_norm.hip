@@ -5,11 +5,13 @@
 //   tanh_norm_embed      token embedding gather -> fp32 residual row, and the first
 //                        layer's normed input
 //   tanh_norm_residual   x += norm1(m + bias); h = norm2(x): the residual update after
-//                        a sublayer and the next sublayer's input in one pass.  `m` is
-//                        a projection's bf16 / fp32 output, its S split-K slabs or S
-//                        parts per row (the slots of a token's experts)
-//   bias_swiglu          silu(g + bg) * (u + bu) of a [gate | up] projection (same
-//                        inputs as above)
+//                        a sublayer and the next sublayer's input in one pass (norm1: or
+//                        none).  `m` is a projection's bf16 / fp32 output, its S split-K
+//                        slabs or S parts per row (the slots of a token's experts, where
+//                        an identity expert's slot stands for its weight times the
+//                        sublayer's input and holds nothing)
+//   glu                  act(g + bg) * (u + bu) of a [gate | up] projection (same inputs
+//                        as above), act = silu or the tanh form of gelu; biases if given
 //
 // The residual stream is fp32.  All are memory-bound; because the norm has no
 // reduction there is no row ownership: threads cover the flat [rows, d] matrix,
@@ -61,6 +63,20 @@ __device__ __forceinline__ float4v norm4(float4v x, float alpha, const float* w,
   return y;
 }
 
+struct Post {  // norm of the sublayer's output; w null: none
+  float alpha;
+  const float* w;
+  const float* b;
+};
+// identity experts among the parts of a row: those with ids >= first
+template <typename T>
+struct Identity {
+  const int* ids;  // [rows, S]; null: none
+  const float* wts;
+  const T* in;  // [rows, d]
+  int first;
+};
+
 template <typename T>
 __global__ __launch_bounds__(256) void embed_kernel(
     T* __restrict__ h, float* __restrict__ x, const int* __restrict__ ids,
@@ -82,33 +98,44 @@ __global__ __launch_bounds__(256) void embed_kernel(
 template <typename T, typename P>
 __global__ __launch_bounds__(256) void residual_kernel(
     T* __restrict__ h, float* __restrict__ x, const P* __restrict__ m, int S, int64_t row,
-    int64_t slab, int d, const float* __restrict__ bias, float a1, const float* __restrict__ w1,
-    const float* __restrict__ b1, float a2, const float* __restrict__ w2,
-    const float* __restrict__ b2) {
+    int64_t slab, int d, const float* __restrict__ bias, Post post, Identity<T> idn, float a2,
+    const float* __restrict__ w2, const float* __restrict__ b2) {
   const int c = (blockIdx.x * 256 + threadIdx.x) * 4;
   if (c >= d) return;
   const int64_t e = (int64_t)blockIdx.y * d + c;
-  float4v v = sum_slabs(m + blockIdx.y * row + c, S, slab);
+  const P* mr = m + blockIdx.y * row + c;
+  float4v v;
+  if (idn.ids) {
+    const float4v hv = load4(idn.in + e);
+    const int* ids = idn.ids + (int64_t)blockIdx.y * S;
+    const float* wts = idn.wts + (int64_t)blockIdx.y * S;
+    v = float4v{0.f, 0.f, 0.f, 0.f};
+    for (int s = 0; s < S; ++s) v += ids[s] < idn.first ? load4(mr + s * slab) : hv * wts[s];
+  } else {
+    v = sum_slabs(mr, S, slab);
+  }
   if (bias) v += *reinterpret_cast<const float4v*>(bias + c);
-  const float4v r = *reinterpret_cast<const float4v*>(x + e) + norm4(v, a1, w1 + c, b1 + c);
+  if (post.w) v = norm4(v, post.alpha, post.w + c, post.b + c);
+  const float4v r = *reinterpret_cast<const float4v*>(x + e) + v;
   store4(x + e, r);
   store4(h + e, norm4(r, a2, w2 + c, b2 + c));
 }
 
-template <typename T, typename P>
-__global__ __launch_bounds__(256) void bias_swiglu_kernel(T* __restrict__ out,
-                                                          const P* __restrict__ m, int S,
-                                                          int64_t slab, int inter,
-                                                          const float* __restrict__ bias) {
+template <typename T, typename P, int ACT>
+__global__ __launch_bounds__(256) void glu_kernel(T* __restrict__ out, const P* __restrict__ m,
+                                                  int S, int64_t slab, int inter,
+                                                  const float* __restrict__ bias) {
   const int c = (blockIdx.x * 256 + threadIdx.x) * 4;
   if (c >= inter) return;
   const P* row = m + (int64_t)blockIdx.y * 2 * inter;
-  const float4v g = sum_slabs(row + c, S, slab) + *reinterpret_cast<const float4v*>(bias + c);
-  const float4v u = sum_slabs(row + inter + c, S, slab) +
-                    *reinterpret_cast<const float4v*>(bias + inter + c);
+  float4v g = sum_slabs(row + c, S, slab), u = sum_slabs(row + inter + c, S, slab);
+  if (bias) {
+    g += *reinterpret_cast<const float4v*>(bias + c);
+    u += *reinterpret_cast<const float4v*>(bias + inter + c);
+  }
   float4v o;
 #pragma unroll
-  for (int j = 0; j < 4; ++j) o[j] = siluf_(g[j]) * u[j];
+  for (int j = 0; j < 4; ++j) o[j] = (ACT ? gelu_tanh_(g[j]) : siluf_(g[j])) * u[j];
   store4(out + (int64_t)blockIdx.y * inter + c, o);
 }
 
@@ -135,13 +162,17 @@ int omnia_tanh_norm_embed(void* h, float* x, const int* ids, const void* table, 
 int omnia_tanh_norm_residual(void* h, int f32, float* x, const void* m, int ptype, int S,
                              int64_t row, int64_t slab, int rows, int d, const float* bias,
                              float a1, const float* w1, const float* b1, float a2,
-                             const float* w2, const float* b2, hipStream_t s) {
+                             const float* w2, const float* b2, const int* ids, const float* wts,
+                             const void* in, int first, hipStream_t s) {
+  if (ids && (!wts || !in)) return -3;
   if (d % 4 || d < 4 || S < 1 || row % 4 || slab % 4 || rows > 65535) return -1;
   if (rows == 0) return 0;
   const dim3 grid((d / 4 + 255) / 256, rows);
 #define OMNIA_TNR(T, P)                                                                      \
-  residual_kernel<T, P><<<grid, 256, 0, s>>>((T*)h, x, (const P*)m, S, row, slab, d, bias, a1, \
-                                             w1, b1, a2, w2, b2)
+  residual_kernel<T, P><<<grid, 256, 0, s>>>((T*)h, x, (const P*)m, S, row, slab, d, bias,     \
+                                             Post{a1, w1, b1},                                 \
+                                             Identity<T>{ids, wts, (const T*)in, first}, a2,   \
+                                             w2, b2)
   if (f32) {
     if (ptype != 1) return -2;
     OMNIA_TNR(float, float);
@@ -156,25 +187,31 @@ int omnia_tanh_norm_residual(void* h, int f32, float* x, const void* m, int ptyp
   return (int)hipGetLastError();
 }
 
-int omnia_bias_swiglu(void* out, int f32, const void* m, int ptype, int S, int rows, int inter,
-                      const float* bias, hipStream_t s) {
+int omnia_glu(void* out, int f32, const void* m, int ptype, int S, int rows, int inter,
+              const float* bias, int gelu, hipStream_t s) {
   if (inter % 4 || inter < 4 || S < 1 || rows > 65535) return -1;
   if (rows == 0) return 0;
   const dim3 grid((inter / 4 + 255) / 256, rows);
   const int64_t slab = (int64_t)rows * 2 * inter;
-#define OMNIA_BSW(T, P) \
-  bias_swiglu_kernel<T, P><<<grid, 256, 0, s>>>((T*)out, (const P*)m, S, slab, inter, bias)
+#define OMNIA_GLU_A(T, P, A) \
+  glu_kernel<T, P, A><<<grid, 256, 0, s>>>((T*)out, (const P*)m, S, slab, inter, bias)
+#define OMNIA_GLU(T, P)                                           \
+  do {                                                            \
+    if (gelu) OMNIA_GLU_A(T, P, 1);                               \
+    else OMNIA_GLU_A(T, P, 0);                                    \
+  } while (0)
   if (f32) {
     if (ptype != 1) return -2;
-    OMNIA_BSW(float, float);
+    OMNIA_GLU(float, float);
   } else if (ptype == 0) {
-    OMNIA_BSW(bf16_t, bf16_t);
+    OMNIA_GLU(bf16_t, bf16_t);
   } else if (ptype == 1) {
-    OMNIA_BSW(bf16_t, float);
+    OMNIA_GLU(bf16_t, float);
   } else {
-    OMNIA_BSW(bf16_t, _Float16);
+    OMNIA_GLU(bf16_t, _Float16);
   }
-#undef OMNIA_BSW
+#undef OMNIA_GLU
+#undef OMNIA_GLU_A
   return (int)hipGetLastError();
 }
 

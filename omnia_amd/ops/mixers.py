@@ -1,7 +1,8 @@
 """Front-end of the kernels behind layer-list models: Dynamic-Tanh and RMS norms fused
-with the residual (``csrc/tanh_norm.hip``, ``csrc/rms_residual.hip``), the gated delta
-rule (``csrc/delta.hip``), latent attention (``csrc/latent.hip``), grouped-query
-attention (``csrc/gqa.hip``, ``csrc/gqa_prefill.hip``) and clamped-GLU experts
+with the residual (``csrc/tanh_norm.hip``, ``csrc/rms_residual.hip``,
+``csrc/branch_residual.hip``), the gated delta rule (``csrc/delta.hip``), fixed-decay
+linear attention (``csrc/lightning.hip``), latent attention (``csrc/latent.hip``),
+grouped-query attention (``csrc/gqa.hip``, ``csrc/gqa_prefill.hip``) and routed experts
 (``csrc/moe.hip``, ``csrc/pgemm.hip``).
 
 GPU tensors (bf16 or fp32) run the HIP kernels and nothing else; CPU tensors run
@@ -44,26 +45,30 @@ def tanh_norm_embed(ids, table, vocab: int, norm: TanhNorm, src=None, tok_slots=
     return x, ref.tanh_norm(x, *norm.args).to(table.dtype)
 
 
-def tanh_norm_residual(x, m, post: TanhNorm, pre: TanhNorm, dtype, bias=None,
-                       slots: bool = False):
-    """In place ``x += post(m + bias)``; returns ``pre(x)`` in ``dtype``.  ``m``: a
-    projection [M, N], its split-K slabs [S, M, N], or (``slots``) parts [M, S, N]."""
+def tanh_norm_residual(x, m, post: TanhNorm | None, pre: TanhNorm, dtype, bias=None,
+                       slots: bool = False, identity=None):
+    """In place ``x += post(m + bias)`` (no post: ``m + bias`` itself); returns ``pre(x)`` in
+    ``dtype``.  ``m``: a projection [M, N], its split-K slabs [S, M, N], or (``slots``)
+    parts [M, S, N], where ``identity`` = (ids [M, S], weights [M, S], input [M, N], first)
+    makes the parts with ids >= first stand for weight * input."""
     if x.is_cuda:
         h = torch.empty(x.shape, dtype=dtype, device=x.device)
-        kernels().tanh_norm_residual(h, x, m, slots, bias, *post.args, *pre.args)
+        kernels().tanh_norm_residual(h, x, m, slots, bias,
+                                     *(post.args if post else (0.0, None, None)), *pre.args,
+                                     *(identity or (None, None, None, 0)))
         return h
     if slots:
-        m = m.float().sum(1)
-    return ref.tanh_norm_residual(x, m, bias, *post.args, *pre.args, dtype)
+        m = ref.slot_sum(m, identity)
+    return ref.tanh_norm_residual(x, m, bias, post, *pre.args, dtype)
 
 
-def bias_swiglu(m, bias, dtype):
-    """``silu(g + bg) * (u + bu)`` of a [gate | up] projection (or its slabs)."""
+def glu(m, bias, dtype, act: str = "silu"):
+    """``act(g + bg) * (u + bu)`` of a [gate | up] projection (or its slabs)."""
     if m.is_cuda:
         out = torch.empty(m.shape[-2], m.shape[-1] // 2, dtype=dtype, device=m.device)
-        kernels().bias_swiglu(out, m, bias)
+        kernels().glu(out, m, bias, act == "gelu_tanh")
         return out
-    return ref.bias_swiglu(m, bias, dtype)
+    return ref.glu(m, bias, dtype, act)
 
 
 # ------------------------------------------------------------------- RMS norm
@@ -120,10 +125,36 @@ def norm_embed(ids, table, vocab: int, emb, pre, src=None, tok_slots=None):
     return rms_embed(ids, table, vocab, emb, pre, src, tok_slots)
 
 
-def norm_residual(x, m, post, pre, dtype, bias=None, slots: bool = False):
-    """What follows a sublayer, of either norm kind (see the two functions above)."""
-    f = tanh_norm_residual if isinstance(post, TanhNorm) else rms_residual
-    return f(x, m, post, pre, dtype, bias, slots)
+def branch_residual(x, branches, pre, dtype):
+    """In place ``x += sum of norm(m + bias)`` over two branches (m, bias, RMSNorm), m a
+    projection or its slabs; returns ``pre(x)`` (either kind, None: x) in ``dtype``."""
+    (a, ab, an), (b, bb, bn) = branches
+    if x.is_cuda:
+        h = torch.empty(x.shape, dtype=dtype, device=x.device)
+        alpha, nw, nb = pre.args if isinstance(pre, TanhNorm) else (
+            0.0, None if pre is None else pre.w, None)
+        kernels().branch_residual(h, x, a, ab, an.w, b, bb, bn.w, an.inv_n, an.eps, alpha, nw, nb)
+        return h
+    for m, bias, norm in branches:
+        v = ref.slab_sum(m)
+        x += ref.rms_norm(v if bias is None else v + bias, norm)
+    if isinstance(pre, TanhNorm):
+        return ref.tanh_norm(x, *pre.args).to(dtype)
+    return (x if pre is None else ref.rms_norm(x, pre)).to(dtype)
+
+
+def norm_residual(x, m=None, post=None, pre=None, dtype=None, bias=None, slots: bool = False,
+                  identity=None, branches=None):
+    """What follows a sublayer, of either norm kind (see the functions above)."""
+    if branches is not None:
+        if post is not None:
+            raise ValueError("branches carry their own norms")
+        return branch_residual(x, branches, pre, dtype)
+    if isinstance(post or pre, TanhNorm):
+        return tanh_norm_residual(x, m, post, pre, dtype, bias, slots, identity)
+    if post is None or identity is not None:
+        raise ValueError("RMS residual steps need a post-norm and no identity parts")
+    return rms_residual(x, m, post, pre, dtype, bias, slots)
 
 
 def softcap_(logits: torch.Tensor, cap: float) -> torch.Tensor:
@@ -135,22 +166,27 @@ def softcap_(logits: torch.Tensor, cap: float) -> torch.Tensor:
 
 
 # -------------------------------------------------------------------- experts
-def experts(h, w: dict, spec) -> torch.Tensor:
-    """Routed clamped-GLU experts: [T, top, d], summed by the residual kernel.  The
-    weights are padded to whole tiles (``ff_pad``; d a multiple of 64)."""
+def experts(h, w: dict, spec):
+    """Routed experts: (parts [T, top, d], ids, weights), the parts summed by the residual
+    kernel; those of identity experts (ids >= spec.experts) are not written.  The weights
+    are padded to whole tiles (``ff_pad``; d a multiple of 64)."""
     T, d = h.shape
-    k, E, ff = spec.top, spec.experts, w["down"].shape[2]
+    k, E, ff = spec.top, spec.outputs, w["down"].shape[2]
+    corr = w.get("correction")
     if not h.is_cuda:
-        return ref.experts(h, w["router"], w["gate_up"], w["down"], spec)
+        ids, wts = ref.route(h, w["router"], spec, corr)
+        return ref.experts(h, ids, wts, w["up"], w["down"], spec), ids, wts
     kk = kernels()
     ids = torch.empty(T, k, dtype=torch.int32, device=h.device)
     wts = torch.empty(T, k, dtype=torch.float32, device=h.device)
-    kk.moe_route(ids, wts, h, w["router"], k, spec.score == "sigmoid", spec.renorm)
+    kk.moe_route(ids, wts, h, w["router"], k, spec.score == "sigmoid", spec.renorm, corr,
+                 spec.groups, spec.keep)
+    # column tiles of the 256-row prefill GEMM: 128 gate and up columns, or 256
     tile = h.dtype == torch.bfloat16 and T * k >= MOE_TILE256_ROWS * E and d % 256 == 0 and \
-        ff % 128 == 0
-    y = _moe_grouped(h, w["gate_up"], w["down"], ids, wts, k, E, 0, E, 256 if tile else 64,
-                     (spec.alpha, spec.limit))
-    return y.view(T, k, d)
+        ff % (128 if spec.gated else 256) == 0
+    y = _moe_grouped(h, w["up"], w["down"], ids, wts, k, E, 0, spec.experts, 256 if tile else 64,
+                     (spec.alpha, spec.limit) if spec.gated else None, not spec.gated)
+    return y.view(T, k, d), ids, wts
 
 
 # ----------------------------------------------------------------- delta rule
@@ -195,6 +231,39 @@ def delta_rule(x, w: dict, spec, state, conv_state, q_start, positions, slots, e
     kk.delta_scan(o, state, conv_state, rec, qn, kn, vc, decay, beta, x, q_start, positions, slots, KH,
                   H, D, Dp, V, taps)
     kk.delta_norm(y, o, x, C, w["norm"], H, V, Vs, Vp, eps)
+    return y
+
+
+# ---------------------------------------------------- fixed-decay linear attention
+def decay_powers(decay, device) -> torch.Tensor:
+    """fp32 [heads, 32]: a^0 .. a^16, then a^64, a^128, a^256, ... (double precision)."""
+    n = torch.tensor([*range(17), *(64 << i for i in range(15))], dtype=torch.float64)
+    a = torch.tensor(decay, dtype=torch.float64)
+    return torch.pow(a[:, None], n).float().to(device)
+
+
+def lightning(x, w: dict, spec, state, q_start, positions, slots, eps: float, dtype,
+              out: torch.Tensor | None = None) -> torch.Tensor:
+    """Linear attention over one set of rows: decode (``q_start`` None, one row per
+    sequence) or prefill portions.  ``x`` rows are projections [q | k | v | gate], of a
+    decode step also their split-K slabs; states of ``slots`` advance in place.  Returns
+    [T, heads * v_pad], the output projection's input."""
+    T, H, Dp, Vp = positions.numel(), spec.heads, spec.dim_pad, spec.v_pad
+    n, inv_n, goff = H * Vp, 1.0 / (H * spec.vdim), H * (2 * Dp + Vp)
+    y = torch.empty(T, n, dtype=dtype, device=x.device) if out is None else out
+    if not x.is_cuda:
+        return y.copy_(ref.lightning(x, w, spec, state, q_start, positions, slots, eps))
+    kk, dev = kernels(), x.device
+    if checks.active(x):
+        checks.state_slots("lightning", slots, state)
+    o = torch.empty(T, H, Vp, dtype=torch.float32, device=dev)
+    if q_start is None:
+        kk.lightning_step(o, state, x, w["pow"], positions, slots)
+    else:
+        need = kk.lightning_scratch(T, slots.numel(), H, Dp, Vp)
+        seg = torch.empty(need, dtype=torch.float32, device=dev) if need else None
+        kk.lightning_scan(o, state, seg, x, w["pow"], q_start, positions, slots)
+    kk.lightning_norm(y, o, x, goff, w["norm"], inv_n, eps)
     return y
 
 
@@ -288,8 +357,8 @@ def latent_prefill(q, kx, kr, vt, fb, spec, gate, out=None):
 
 # ------------------------------------------------------ grouped-query attention
 def gqa_prep(x, w: dict, spec, pages, positions, slots, cos_sin, dtype, eps: float):
-    """Fused projection rows (or split-K slabs) -> normed, rotated queries [T, H * dim_pad];
-    writes the tokens' keys and values at ``slots`` of ``pages`` = (k, v), or, with
+    """Fused projection rows (or split-K slabs) -> queries [T, H * dim_pad], with bias, norm
+    and rotation as the spec says; writes the tokens' keys and values at ``slots`` of ``pages`` = (k, v), or, with
     ``pages`` None, none (the layer borrows another one's)."""
     k, v = pages if pages is not None else (None, None)
     if x.is_cuda:
@@ -297,8 +366,9 @@ def gqa_prep(x, w: dict, spec, pages, positions, slots, cos_sin, dtype, eps: flo
             checks.slots("gqa_prep", slots, k)
         q = torch.empty(positions.numel(), spec.heads * spec.dim_pad, dtype=dtype,
                         device=x.device)
-        kernels().gqa_prep(q, k, v, x, w["q_norm"], w.get("k_norm"), positions, slots, cos_sin,
-                           spec.heads, spec.dim, eps)
+        kernels().gqa_prep(q, k, v, x, w.get("q_norm"), w.get("k_norm"), w.get("in_b"), positions,
+                           slots, cos_sin, spec.rotary is not None and spec.rotary.interleaved,
+                           spec.heads, spec.dim, spec.dim_pad, eps)
         return q
     return ref.gqa_prep(x, w, spec, k, v, positions, slots, cos_sin, dtype, eps)
 
@@ -308,7 +378,7 @@ def gqa_attend(q, pages, block_tables, q_start, positions, spec, sinks, out=None
     if out is None:
         out = torch.empty(positions.numel(), spec.heads * spec.v_pad, dtype=q.dtype,
                           device=q.device)
-    args = (out, q, *pages, block_tables, q_start, positions, spec.heads, spec.window,
+    args = (out, q, *pages, block_tables, q_start, positions, spec.heads, spec.mask,
             spec.scale, sinks)
     (kernels().gqa_attend if q.is_cuda else ref.gqa_attend)(*args)
     return out
@@ -325,7 +395,7 @@ def gqa_decode(q, pages, block_tables, positions, spec, sinks, splits: int, out=
         pm = torch.empty(T * H * splits * 2, dtype=torch.float32, device=q.device)
     if checks.active(q):
         checks.paged("gqa_decode", block_tables, positions + 1, pages[0], T)
-    kernels().gqa_decode(out, po, pm, q, *pages, block_tables, positions, H, spec.window,
+    kernels().gqa_decode(out, po, pm, q, *pages, block_tables, positions, H, spec.mask,
                          spec.scale, sinks, splits)
     return out
 
@@ -337,5 +407,5 @@ def gqa_prefill(q, pages, fb, spec, sinks, out=None):
     if checks.active(q):
         checks.paged("gqa_prefill", fb.block_tables, fb.seq_lens, pages[0])
     kernels().gqa_prefill(out, q, *pages, fb.block_tables, fb.q_start_loc, fb.seq_lens,
-                          fb.tile_seq, fb.tile_q0, spec.heads, spec.window, spec.scale, sinks)
+                          fb.tile_seq, fb.tile_q0, spec.heads, spec.mask, spec.scale, sinks)
     return out

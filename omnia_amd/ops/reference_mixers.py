@@ -15,18 +15,29 @@ def tanh_norm(x, alpha, w, b):
     return torch.tanh(alpha * x) * w + b
 
 
-def tanh_norm_residual(x, m, bias, a1, w1, b1, a2, w2, b2, dtype):
+def slot_sum(m, identity):
+    """Parts [M, S, N] summed; identity parts stand for weight * input."""
+    m = m.float()
+    if identity is not None:
+        ids, wts, inp, first = identity
+        m = torch.where((ids >= first)[..., None], wts[..., None] * inp.float()[:, None], m)
+    return m.sum(1)
+
+
+def tanh_norm_residual(x, m, bias, post, a2, w2, b2, dtype):
     v = slab_sum(m)
     if bias is not None:
         v = v + bias
-    x += tanh_norm(v, a1, w1, b1)
+    x += v if post is None else tanh_norm(v, *post.args)
     return tanh_norm(x, a2, w2, b2).to(dtype)
 
 
-def bias_swiglu(m, bias, dtype):
-    v = slab_sum(m) + bias
+def glu(m, bias, dtype, act):
+    v = slab_sum(m)
+    if bias is not None:
+        v = v + bias
     g, u = v.chunk(2, -1)
-    return (F.silu(g) * u).to(dtype)
+    return ((F.gelu(g, approximate="tanh") if act == "gelu_tanh" else F.silu(g)) * u).to(dtype)
 
 
 def _spans(q_start, n):
@@ -101,6 +112,27 @@ def delta_norm(o, x, zoff, norm_w, H, V, Vp, eps):
     return F.pad(y, (0, Vp - V)).to(x.dtype).reshape(T, H * Vp)
 
 
+def lightning(x, w, spec, state, q_start, positions, slots, eps):
+    T, H, Dp, Vp = positions.numel(), spec.heads, spec.dim_pad, spec.v_pad
+    x = slab_sum(x)[:, :spec.in_cols]
+    q, k, v, g = x.split([H * Dp, H * Dp, H * Vp, H * Vp], 1)
+    q, k, v = (F.silu(t).view(T, H, -1) for t in (q, k, v))
+    a = w["pow"][:, 1, None, None]
+    o = torch.zeros(T, H, Vp)
+    for s, r0, n in _spans(q_start, T):
+        slot = int(slots[s])
+        if slot < 0:
+            continue
+        S = torch.zeros(H, Dp, Vp) if int(positions[r0]) == 0 else state[slot].clone()
+        for t in range(r0, r0 + n):
+            S = S * a + k[t][:, :, None] * v[t][:, None, :]
+            o[t] = torch.matmul(q[t][:, None], S)[:, 0]
+        state[slot] = S
+    o = o.view(T, H * Vp)
+    o = o / torch.sqrt(o.pow(2).sum(-1, keepdim=True) / (H * spec.vdim) + eps) * w["norm"]
+    return o * torch.sigmoid(g)
+
+
 def _rotate(v, positions, cos_sin):
     half = v.shape[-1] // 2
     cs = cos_sin[positions.long()]
@@ -167,56 +199,93 @@ def rms_norm(x, n):
     return x / torch.sqrt(x.pow(2).sum(-1, keepdim=True) * n.inv_n + n.eps) * n.w
 
 
-def experts(h, router, gate_up, down, spec):
-    """[T, top, d]: the chosen experts' outputs, their weights on the inputs."""
-    T, d = h.shape
+def route(h, router, spec, corr=None):
+    """(ids int32 [T, top], weights fp32 [T, top])."""
     z = h.float() @ router.float().T
-    zt, ids = z.sort(dim=-1, descending=True, stable=True)
-    zt, ids = zt[:, :spec.top], ids[:, :spec.top]
-    if spec.score == "sigmoid":
-        wt = torch.sigmoid(zt)
-    else:
-        wt = torch.exp(zt - torch.logsumexp(z, -1, keepdim=True))
+    s = torch.sigmoid(z) if spec.score == "sigmoid" else torch.softmax(z, -1)
+    c = z if corr is None else s + corr
+    if spec.groups > 1:
+        best = c.view(c.shape[0], spec.groups, -1).amax(-1)
+        order = best.sort(dim=-1, descending=True, stable=True).indices[:, spec.keep:]
+        out = torch.zeros_like(best, dtype=torch.bool).scatter_(1, order, True)
+        c = c.masked_fill(out.repeat_interleave(c.shape[1] // spec.groups, 1), float("-inf"))
+    ids = c.sort(dim=-1, descending=True, stable=True).indices[:, :spec.top]
+    wt = s.gather(1, ids)
     if spec.renorm:
-        wt = wt / wt.sum(-1, keepdim=True)
+        wt = wt / (wt.sum(-1, keepdim=True) + 1e-20)
+    return ids.int(), wt
+
+
+def experts(h, ids, wts, up, down, spec):
+    """[T, top, d]: the chosen experts' weighted outputs (clamped GLUs take the weight on
+    their input)."""
+    T, d = h.shape
     out = torch.zeros(T, spec.top, d, dtype=h.dtype)
     for e in ids.unique().tolist():
+        if e >= spec.experts:
+            continue
         t, j = (ids == e).nonzero(as_tuple=True)
-        v = (h[t].float() @ gate_up[e].float().T) * wt[t, j, None]
-        g, u = v.chunk(2, -1)
-        g, u = g.clamp(max=spec.limit), u.clamp(-spec.limit, spec.limit)
-        a = (g * torch.sigmoid(spec.alpha * g) * (u + 1.0)).to(h.dtype)
-        out[t, j] = (a.float() @ down[e].float().T).to(h.dtype)
+        v, wt = h[t].float() @ up[e].float().T, wts[t, j, None]
+        if spec.gated:
+            g, u = (v * wt).chunk(2, -1)
+            g, u = g.clamp(max=spec.limit), u.clamp(-spec.limit, spec.limit)
+            a, wt = g * torch.sigmoid(spec.alpha * g) * (u + 1.0), 1.0
+        else:
+            a = F.gelu(v)
+        out[t, j] = (a.to(h.dtype).float() @ down[e].float().T * wt).to(h.dtype)
     return out
 
 
+def _rotate_pairs(v, positions, cos_sin):
+    """Neighbours (2i, 2i + 1) turn together."""
+    half = v.shape[-1] // 2
+    cs = cos_sin[positions.long()][:, None]
+    c, s = cs[..., :half], cs[..., half:]
+    a, b = v[..., 0::2], v[..., 1::2]
+    return torch.stack([a * c - b * s, b * c + a * s], -1).flatten(-2)
+
+
 def gqa_prep(x, w, spec, k, v, positions, slots, cos_sin, dtype, eps):
-    T, H, D, Dp, R = positions.numel(), spec.heads, spec.dim, spec.dim_pad, cos_sin.shape[1]
+    T, H, D, Dp = positions.numel(), spec.heads, spec.dim, spec.dim_pad
+    R = 0 if cos_sin is None else cos_sin.shape[1]
     x = slab_sum(x)
+    if w.get("in_b") is not None:
+        x = x[:, :w["in_b"].numel()] + w["in_b"]
 
     def turned(z, wn, heads):
         z = z.reshape(T, heads, Dp)
-        z = z / torch.sqrt(z.pow(2).sum(-1, keepdim=True) / D + eps) * wn
-        return torch.cat([_rotate(z[..., :R], positions, cos_sin), z[..., R:]], -1).to(dtype)
+        if wn is not None:
+            z = z / torch.sqrt(z.pow(2).sum(-1, keepdim=True) / D + eps) * wn
+        if R:
+            turn = _rotate_pairs if spec.rotary.interleaved else _rotate
+            z = torch.cat([turn(z[..., :R], positions, cos_sin), z[..., R:]], -1)
+        return z.to(dtype)
 
     if k is not None:
         G, page, Vp = k.shape[1], k.shape[2], v.shape[3]
-        kk = turned(x[:, H * Dp:(H + G) * Dp], w["k_norm"], G)
+        kk = turned(x[:, H * Dp:(H + G) * Dp], w.get("k_norm"), G)
         vv = x[:, (H + G) * Dp:(H + G) * Dp + G * Vp].reshape(T, G, Vp).to(dtype)
         keep = slots >= 0
         b, o = slots[keep] // page, slots[keep] % page
         k[b, :, o], v[b, :, o] = kk[keep], vv[keep]
-    return turned(x[:, :H * Dp], w["q_norm"], H).reshape(T, H * Dp)
+    return turned(x[:, :H * Dp], w.get("q_norm"), H).reshape(T, H * Dp)
 
 
-def gqa_attend(out, q, k, v, block_tables, q_start, positions, H, window, scale, sinks):
+def _visible(pos, mask):
+    window, first, chunk = mask
+    if chunk:
+        return torch.arange(pos // chunk * chunk, pos + 1)
+    lo = max(0, pos - window + 1) if window > 0 else 0
+    return torch.cat([torch.arange(0, min(first, lo)), torch.arange(lo, pos + 1)])
+
+
+def gqa_attend(out, q, k, v, block_tables, q_start, positions, H, mask, scale, sinks):
     T, G, page = positions.numel(), k.shape[1], k.shape[2]
     qv = q.view(T, G, H // G, -1).float()
     ov = out.view(T, H, -1)
     for s, r0, n in _spans(q_start, T):
         for t in range(r0, r0 + n):
-            pos = int(positions[t])
-            key = torch.arange(max(0, pos - window + 1) if window > 0 else 0, pos + 1)
+            key = _visible(int(positions[t]), mask)
             b = block_tables[s, key // page].long()
             kr, vr = k[b, :, key % page].float(), v[b, :, key % page].float()  # [n, G, w]
             sc = torch.matmul(qv[t], kr.permute(1, 2, 0)).reshape(H, -1) * scale

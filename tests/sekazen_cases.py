@@ -117,7 +117,7 @@ def weights(cfg, seed=0):
     def rnd(shape):
         return torch.randn(shape, generator=g, dtype=torch.float64)
 
-    for n, shape in tensor_shapes(parse_layers(cfg["layers"]), cfg["width"], cfg["vocab"],
+    for n, shape in tensor_shapes(parse_layers(cfg["layers"], DESIGNS["sekazen"]), cfg["width"], cfg["vocab"],
                                   DESIGNS["sekazen"]).items():
         leaf = n.split(".")[-1]
         if leaf == "sink":

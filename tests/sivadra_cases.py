@@ -73,11 +73,11 @@ CASES = {
 
 def weights(cfg, seed=0):
     """name -> float64 tensor, bf16-representable."""
-    from omnia_amd.models.layers import parse_layers, tensor_shapes
+    from omnia_amd.models.layers import DESIGNS, parse_layers, tensor_shapes
 
     g = torch.Generator().manual_seed(seed)
     W = {}
-    for n, shape in tensor_shapes(parse_layers(cfg["layers"]), cfg["width"],
+    for n, shape in tensor_shapes(parse_layers(cfg["layers"], DESIGNS["sivadra"]), cfg["width"],
                                   cfg["vocab"]).items():
         t = torch.randn(shape, generator=g, dtype=torch.float64)
         leaf = n.split(".")[-1]
