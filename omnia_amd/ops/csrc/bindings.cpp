@@ -678,7 +678,7 @@ void moe_route(at::Tensor ids, at::Tensor wts, at::Tensor x, at::Tensor router, 
   TORCH_CHECK((f32 || x.scalar_type() == at::kBFloat16) && router.scalar_type() == x.scalar_type(),
               "x and router: bf16 or fp32");
   TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && router.is_cuda() && router.dim() == 2 &&
-              router.is_contiguous() && router.size(1) == x.size(1) && x.size(1) % 8 == 0,
+              router.is_contiguous() && router.size(1) == x.size(1),
               "x [T, d], router [E, d]");
   const int T = x.size(0), E = router.size(0);
   TORCH_CHECK(ids.numel() == (int64_t)T * k && wts.numel() == (int64_t)T * k && wts.is_cuda() &&

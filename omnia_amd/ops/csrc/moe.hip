@@ -128,159 +128,214 @@ __global__ __launch_bounds__(256) void moe_router_topk_kernel(
   select_topk(mine, lane, t, E, k, renorm, ids, wts);
 }
 
-// fp32 router for any score function: logits z[e] = x . router[e] stay fp32; the k
-// largest are chosen; weights are sigmoid(z) or softmax(z), renormalised over the chosen
-// ones if asked.  With a correction the choice goes by score + correction (weights stay the
-// plain scores); with groups, experts outside the `keep` groups of E / groups neighbours
-// with the largest choice score are out of the choice.  One wave per token; expert e
-// belongs to lane e & 63; EC experts' dot products at a time.
+// Router for any score function: logits z[e] = x . router[e] accumulate and stay in fp32;
+// weights are sigmoid(z) or softmax(z), renormalised over the chosen ones if asked.  The k
+// largest choice scores are chosen: z, or with a correction score + correction (weights stay
+// the plain scores); with groups, experts outside the `keep` groups of E / groups neighbours
+// with the largest choice score are out of the choice.  Lower numbers win ties.
 constexpr int kMaxExperts = 256;
 constexpr float kRenormEps = 1e-20f;
 
-template <typename T, int EC>
-__global__ __launch_bounds__(256) void moe_route_kernel(int* __restrict__ ids,
-                                                        float* __restrict__ wts,
-                                                        const T* __restrict__ x,
-                                                        const T* __restrict__ router, int n_tok,
-                                                        int d, int E, int k, int sigmoid,
-                                                        int renorm,
-                                                        const float* __restrict__ corr,
-                                                        int groups, int keep) {
-  __shared__ float pick[4][kMaxExperts];  // a token's choice scores, then its groups'
-  constexpr int NPL = kMaxExperts / 64;
-  const int lane = threadIdx.x & 63;
-  const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (t >= n_tok) return;
-  const T* xr = x + (int64_t)t * d;
-  auto load8 = [](const T* p, float (&f)[8]) {
-    if constexpr (sizeof(T) == 4) {
-      const float4v a = *reinterpret_cast<const float4v*>(p);
-      const float4v b = *reinterpret_cast<const float4v*>(p + 4);
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        f[j] = a[j];
-        f[4 + j] = b[j];
-      }
-    } else {
-      const short8 v = *reinterpret_cast<const short8*>(p);
-#pragma unroll
-      for (int j = 0; j < 8; ++j) f[j] = bf2f((uint16_t)v[j]);
-    }
+struct Route {
+  int* ids;    // [T, k]
+  float* wts;  // [T, k]
+  const float* corr;
+  int E, k, sigmoid, renorm, groups, keep;
+};
+
+// One token by LPT lanes (l of them), NPL experts a lane; its E logits lie in the LDS row
+// zc, which ends as the choice scores.  Every expert counts the experts ahead of it: its
+// rank is its slot.
+template <int LPT, int NPL>
+__device__ __forceinline__ void choose(float* zc, int l, int64_t t, const Route& a) {
+  auto sync = [] {  // LDS of one wave
+    __builtin_amdgcn_wave_barrier();
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
   };
-  float z[NPL];
+  float z[NPL], s[NPL], c[NPL], top = -INFINITY;
 #pragma unroll
-  for (int i = 0; i < NPL; ++i) z[i] = -INFINITY;
-  for (int e0 = 0; e0 < E; e0 += EC) {
+  for (int i = 0; i < NPL; ++i) {
+    const int e = l + LPT * i;
+    z[i] = e < a.E ? zc[e] : -INFINITY;
+    if (!(z[i] == z[i])) z[i] = -INFINITY;  // NaN rows (padding) still get distinct valid ids
+    top = fmaxf(top, z[i]);
+  }
+  if (a.sigmoid) {
+#pragma unroll
+    for (int i = 0; i < NPL; ++i) s[i] = 1.f / (1.f + expf(-z[i]));
+  } else {
+#pragma unroll
+    for (int o = LPT / 2; o > 0; o >>= 1) top = fmaxf(top, __shfl_xor(top, o, 64));
+    if (!(top > -INFINITY)) top = 0.f;
+    float total = 0.f;
+#pragma unroll
+    for (int i = 0; i < NPL; ++i) {
+      s[i] = expf(z[i] - top);
+      total += s[i];
+    }
+#pragma unroll
+    for (int o = LPT / 2; o > 0; o >>= 1) total += __shfl_xor(total, o, 64);
+    if (!(total > 0.f)) total = 1.f;
+#pragma unroll
+    for (int i = 0; i < NPL; ++i) s[i] /= total;
+  }
+#pragma unroll
+  for (int i = 0; i < NPL; ++i) {
+    const int e = l + LPT * i;
+    c[i] = a.corr && e < a.E ? s[i] + a.corr[e] : z[i];
+    if (e < a.E) zc[e] = c[i];
+  }
+  sync();
+  if (a.groups > 1) {
+    const int per = a.E / a.groups;
+    int better[NPL], grp[NPL];
+    float own[NPL];
+#pragma unroll
+    for (int i = 0; i < NPL; ++i) {
+      grp[i] = min((l + LPT * i) / per, a.groups - 1);
+      better[i] = 0;
+      own[i] = -INFINITY;
+      for (int j = 0; j < per; ++j) own[i] = fmaxf(own[i], zc[grp[i] * per + j]);
+    }
+    for (int g = 0; g < a.groups; ++g) {
+      float m = -INFINITY;
+      for (int j = 0; j < per; ++j) m = fmaxf(m, zc[g * per + j]);
+#pragma unroll
+      for (int i = 0; i < NPL; ++i) better[i] += m > own[i] || (m == own[i] && g < grp[i]);
+    }
+    sync();
+#pragma unroll
+    for (int i = 0; i < NPL; ++i) {
+      if (better[i] >= a.keep) c[i] = -INFINITY;
+      if (l + LPT * i < a.E) zc[l + LPT * i] = c[i];
+    }
+    sync();
+  }
+  int rank[NPL];
+#pragma unroll
+  for (int i = 0; i < NPL; ++i) rank[i] = 0;
+  for (int e = 0; e < a.E; ++e) {
+    const float v = zc[e];
+#pragma unroll
+    for (int i = 0; i < NPL; ++i) rank[i] += v > c[i] || (v == c[i] && e < l + LPT * i);
+  }
+  float sel = 0.f;
+#pragma unroll
+  for (int i = 0; i < NPL; ++i)
+    if (l + LPT * i < a.E && rank[i] < a.k) sel += s[i];
+#pragma unroll
+  for (int o = LPT / 2; o > 0; o >>= 1) sel += __shfl_xor(sel, o, 64);
+#pragma unroll
+  for (int i = 0; i < NPL; ++i)
+    if (l + LPT * i < a.E && rank[i] < a.k) {
+      a.ids[t * a.k + rank[i]] = l + LPT * i;
+      a.wts[t * a.k + rank[i]] = a.renorm ? s[i] / (sel + kRenormEps) : s[i];
+    }
+}
+
+// bf16: 16 tokens a workgroup of 8 waves, logits on MFMA (exact products, fp32 sums).  Up
+// to 64 experts the waves split the width and meet in LDS; past that each wave has its own
+// tiles of 16 experts.
+template <int NT>
+__global__ __launch_bounds__(512) void moe_route_kernel(const bf16_t* __restrict__ x,
+                                                        const bf16_t* __restrict__ router,
+                                                        int n_tok, int d, Route a) {
+  constexpr bool SPLIT = NT <= 4;
+  constexpr int TPW = SPLIT ? NT : NT / 8;  // expert tiles of a wave
+  constexpr int ZS = 16 * NT + 4;
+  __shared__ float part[SPLIT ? 8 * 16 * ZS : 16 * ZS];
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+  const int t0 = blockIdx.x * 16, c16 = lane & 15, g4 = lane >> 4;
+  const bf16_t* xr = x + (int64_t)min(t0 + c16, n_tok - 1) * d + 8 * g4;
+  const bf16_t* rr[TPW];
+#pragma unroll
+  for (int i = 0; i < TPW; ++i)
+    rr[i] = router + (int64_t)min((SPLIT ? i : w * TPW + i) * 16 + c16, a.E - 1) * d + 8 * g4;
+  const int nk = d / 32, per = SPLIT ? (nk + 7) / 8 : nk;
+  const int k0 = SPLIT ? w * per : 0, k1 = min(nk, k0 + per);
+  float4v acc[TPW];
+#pragma unroll
+  for (int i = 0; i < TPW; ++i) acc[i] = float4v{0.f, 0.f, 0.f, 0.f};
+  constexpr int U = TPW == 1 ? 8 : 4;
+  for (int k = k0; k < k1; k += U) {  // U steps of loads in flight; past the end: the last
+    short8 av[U], bv[TPW][U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int at = 32 * min(k + u, k1 - 1);
+      av[u] = *reinterpret_cast<const short8*>(xr + at);
+#pragma unroll
+      for (int i = 0; i < TPW; ++i) bv[i][u] = *reinterpret_cast<const short8*>(rr[i] + at);
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      if (k + u >= k1) break;
+#pragma unroll
+      for (int i = 0; i < TPW; ++i) acc[i] = mfma16(av[u], bv[i][u], acc[i]);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < TPW; ++i)
+#pragma unroll
+    for (int r = 0; r < 4; ++r)  // token 4 g4 + r, expert 16 tile + c16
+      part[(SPLIT ? w * 16 * ZS : 0) + (4 * g4 + r) * ZS + (SPLIT ? i : w * TPW + i) * 16 + c16] =
+          acc[i][r];
+  __syncthreads();
+  if (SPLIT) {
+    for (int i = tid; i < 16 * 16 * NT; i += 512) {
+      const int at = i / (16 * NT) * ZS + i % (16 * NT);
+      float v = 0.f;
+#pragma unroll
+      for (int k = 0; k < 8; ++k) v += part[k * 16 * ZS + at];
+      part[at] = v;
+    }
+    __syncthreads();
+  }
+  if constexpr (NT == 1) {  // four tokens a wave, 16 lanes each
+    const int tt = 4 * w + g4;
+    if (w < 4 && t0 + 4 * w < n_tok)  // a token past the end repeats the last one
+      choose<16, 1>(part + tt * ZS, c16, min(t0 + tt, n_tok - 1), a);
+  } else {
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int tt = 2 * w + i;
+      if (t0 + tt < n_tok) choose<64, (NT + 3) / 4>(part + tt * ZS, lane, t0 + tt, a);
+    }
+  }
+}
+
+// fp32: one wave per token, EC experts' dot products at a time
+template <int EC>
+__global__ __launch_bounds__(256) void moe_route_f32_kernel(const float* __restrict__ x,
+                                                            const float* __restrict__ router,
+                                                            int n_tok, int d, Route a) {
+  __shared__ float zs[4][kMaxExperts];
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  const int t = blockIdx.x * 4 + w;
+  if (t >= n_tok) return;
+  const float* xr = x + (int64_t)t * d;
+  for (int e0 = 0; e0 < a.E; e0 += EC) {
     float acc[EC];
 #pragma unroll
     for (int e = 0; e < EC; ++e) acc[e] = 0.f;
-    for (int c = lane * 8; c < d; c += 64 * 8) {
-      float xf[8];
-      load8(xr + c, xf);
+    for (int c = lane * 4; c < d; c += 256) {
+      const float4v xv = *reinterpret_cast<const float4v*>(xr + c);
 #pragma unroll
       for (int e = 0; e < EC; ++e) {
-        float wf[8];
-        load8(router + (int64_t)min(e0 + e, E - 1) * d + c, wf);
+        const float4v wv =
+            *reinterpret_cast<const float4v*>(router + (int64_t)min(e0 + e, a.E - 1) * d + c);
 #pragma unroll
-        for (int j = 0; j < 8; ++j) acc[e] += xf[j] * wf[j];
+        for (int j = 0; j < 4; ++j) acc[e] += xv[j] * wv[j];
       }
     }
 #pragma unroll
     for (int e = 0; e < EC; ++e) {
-      float v = wave_sum(acc[e]);
-      if (!(v == v)) v = -INFINITY;  // NaN rows (padding) still choose distinct valid ids
-#pragma unroll
-      for (int i = 0; i < NPL; ++i)
-        if (e0 + e < E && (e0 + e) == lane + 64 * i) z[i] = v;
+      const float v = wave_sum(acc[e]);
+      if (lane == 0 && e0 + e < a.E) zs[w][e0 + e] = v;
     }
   }
-  float top = -INFINITY, total = 1.f;
-  if (!sigmoid) {
-#pragma unroll
-    for (int i = 0; i < NPL; ++i) top = fmaxf(top, z[i]);
-    top = wave_max(top);
-    if (!(top > -INFINITY)) top = 0.f;
-    total = 0.f;
-#pragma unroll
-    for (int i = 0; i < NPL; ++i) total += expf(z[i] - top);
-    total = wave_sum(total);
-    if (!(total > 0.f)) total = 1.f;
-  }
-  // choice score of this lane's experts: monotone in the logit without a correction
-  float c[NPL];
-  unsigned taken = 0;  // bit i: this lane's expert lane + 64 i is chosen, or out of the choice
-#pragma unroll
-  for (int i = 0; i < NPL; ++i) {
-    c[i] = z[i];
-    const int e = lane + 64 * i;
-    if (corr && e < E) {
-      c[i] = (sigmoid ? 1.f / (1.f + expf(-z[i])) : expf(z[i] - top) / total) + corr[e];
-      if (!(c[i] == c[i])) c[i] = -INFINITY;
-    }
-  }
-  if (groups > 1) {
-    const int wv = threadIdx.x >> 6, per = E / groups;
-#pragma unroll
-    for (int i = 0; i < NPL; ++i)
-      if (lane + 64 * i < E) pick[wv][lane + 64 * i] = c[i];
-    __builtin_amdgcn_wave_barrier();
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // this wave's LDS writes
-    float gs[NPL];
-#pragma unroll
-    for (int i = 0; i < NPL; ++i) {
-      gs[i] = -INFINITY;
-      const int g = lane + 64 * i;
-      if (g < groups)
-        for (int j = 0; j < per; ++j) gs[i] = fmaxf(gs[i], pick[wv][g * per + j]);
-    }
-    __builtin_amdgcn_wave_barrier();
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-#pragma unroll
-    for (int i = 0; i < NPL; ++i)
-      if (lane + 64 * i < groups) pick[wv][lane + 64 * i] = gs[i];
-    __builtin_amdgcn_wave_barrier();
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-#pragma unroll
-    for (int i = 0; i < NPL; ++i) {
-      const int e = lane + 64 * i;
-      if (e >= E) continue;
-      const int g = e / per;
-      const float mine_g = pick[wv][g];
-      int better = 0;  // groups ahead of this expert's (lower index wins ties)
-      for (int j = 0; j < groups; ++j) {
-        const float o = pick[wv][j];
-        better += o > mine_g || (o == mine_g && j < g);
-      }
-      if (better >= keep) taken |= 1u << i;
-    }
-  }
-  float sel = 0.f, mine = 0.f;
-  for (int j = 0; j < k; ++j) {
-    float v = -INFINITY;
-#pragma unroll
-    for (int i = 0; i < NPL; ++i)
-      if (!(taken >> i & 1) && lane + 64 * i < E) v = fmaxf(v, c[i]);
-    const float vm = wave_max(v);
-    int first = 1 << 30;  // lowest untaken expert with the largest choice score
-#pragma unroll
-    for (int i = NPL - 1; i >= 0; --i)
-      if (!(taken >> i & 1) && lane + 64 * i < E && c[i] == vm) first = lane + 64 * i;
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) first = min(first, __shfl_xor(first, o, 64));
-    if ((first & 63) == lane) taken |= 1u << (first >> 6);
-    float zf = -INFINITY;  // the chosen expert's logit
-#pragma unroll
-    for (int i = 0; i < NPL; ++i)
-      if (first == lane + 64 * i) zf = z[i];
-    zf = __shfl(zf, first & 63, 64);
-    const float s = sigmoid ? 1.f / (1.f + expf(-zf)) : expf(zf - top) / total;
-    sel += s;
-    if (lane == j) mine = s;  // k <= 64: lane j keeps slot j
-    if (lane == 0) ids[(int64_t)t * k + j] = first;
-  }
-  if (lane < k) {
-    wts[(int64_t)t * k + lane] = renorm ? mine / (sel + kRenormEps) : mine;
-  }
+  __builtin_amdgcn_wave_barrier();
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  choose<64, kMaxExperts / 64>(zs[w], lane, t, a);
 }
 
 // ------------------------------------------------------------------ align
@@ -620,22 +675,21 @@ int omnia_moe_align(int* sorted, int* blk_expert, int* n_blocks, const int* ids,
 int omnia_moe_route(int* ids, float* wts, const void* x, const void* router, int f32, int n_tok,
                     int d, int E, int k, int sigmoid, int renorm, const float* corr, int groups,
                     int keep, hipStream_t s) {
-  if (E < 1 || E > kMaxExperts || k < 1 || k > E || k > 64 || d % 8) return -1;
+  if (E < 1 || E > kMaxExperts || k < 1 || k > E || k > 64 || d % (f32 ? 4 : 32)) return -1;
   if (groups < 1 || E % groups || keep < 1 || keep > groups || k > keep * (E / groups)) return -2;
   if (n_tok == 0) return 0;
-  const int blocks = (n_tok + 3) / 4;
-#define OMNIA_RO(TT, EC)                                                                       \
-  moe_route_kernel<TT, EC><<<blocks, 256, 0, s>>>(ids, wts, (const TT*)x, (const TT*)router,   \
-                                                  n_tok, d, E, k, sigmoid, renorm, corr,       \
-                                                  groups, keep)
-#define OMNIA_ROE(TT)            \
-  do {                           \
-    if (E <= 8) OMNIA_RO(TT, 8); \
-    else OMNIA_RO(TT, 16);       \
-  } while (0)
-  if (f32) OMNIA_ROE(float);
-  else OMNIA_ROE(bf16_t);
-#undef OMNIA_ROE
+  const Route a{ids, wts, corr, E, k, sigmoid, renorm, groups, keep};
+  if (f32) {
+    moe_route_f32_kernel<16><<<(n_tok + 3) / 4, 256, 0, s>>>((const float*)x, (const float*)router,
+                                                             n_tok, d, a);
+    return (int)hipGetLastError();
+  }
+  const int blocks = (n_tok + 15) / 16;
+#define OMNIA_RO(NT)                                                                           \
+  moe_route_kernel<NT><<<blocks, 512, 0, s>>>((const bf16_t*)x, (const bf16_t*)router, n_tok, d, a)
+  if (E <= 16) OMNIA_RO(1);
+  else if (E <= 64) OMNIA_RO(4);
+  else OMNIA_RO(16);
 #undef OMNIA_RO
   return (int)hipGetLastError();
 }

@@ -492,7 +492,7 @@ def test_router_scores(run):
         down = torch.zeros(E, d, 64)
         for e in range(E):
             down[e, e] = 1.0
-        y = mops.experts(h, {"router": router, "gate_up": gu, "down": down}, spec)
+        y, _, _ = mops.experts(h, {"router": router, "up": gu, "down": down}, spec)
         assert [int(v) for v in y[0].abs().argmax(-1)] == [11, 10, 9]
         return
     from omnia_amd.ops import kernels

@@ -89,13 +89,13 @@ def test_tanh_norm_embed(run):
 
 
 @pytest.mark.parametrize("run", RUNS)
-def test_bias_swiglu(run):
+def test_glu(run):
     dev, dt = run
     g = gen(4)
     for S, pdt in ((1, dt), (4, torch.float32)):
         m, b = rnd(S, 5, 2 * 88, g=g).to(pdt), torch.randn(2 * 88, generator=g)
         v = m.double().sum(0) + b.double()
-        got = mops.bias_swiglu((m if S > 1 else m[0]).to(dev), b.to(dev), dt)
+        got = mops.glu((m if S > 1 else m[0]).to(dev), b.to(dev), dt)
         assert rel(got, plain.silu(v[:, :88]) * v[:, 88:]) < (2e-6 if dt == torch.float32 else 4e-3)
 
 
