@@ -541,6 +541,11 @@ def looped(layers: tuple, start: int, stop: int, times: int) -> tuple[LayerSpec,
     return tuple(out)
 
 
+def _tensors_of(mixer):
+    """The mixer without which layer it borrows from: passes of a loop differ in that."""
+    return mixer if mixer.kv_from is None else replace(mixer, kv_from=-1)
+
+
 def parse_layers(entries: list[dict], design: DesignSpec,
                  loop: dict | None = None) -> tuple[LayerSpec, ...]:
     """``config.json`` ``layers`` (and ``loop``) -> the layers in the order they run.
@@ -584,7 +589,7 @@ def parse_layers(entries: list[dict], design: DesignSpec,
     for i, l in enumerate(out):
         if l.weights_of is not None:
             o = out[l.weights_of]
-            if (o.mixer, o.mlp) != (l.mixer, l.mlp):
+            if (_tensors_of(o.mixer), o.mlp) != (_tensors_of(l.mixer), l.mlp):
                 raise ValueError(f"layer {i} differs from layer {l.weights_of} whose "
                                  "weights it uses")
         j = l.mixer.kv_from

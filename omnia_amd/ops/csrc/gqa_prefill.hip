@@ -58,7 +58,8 @@ struct Args {
   float scale_log2;
 };
 
-template <int DK, int DV>
+// KEEP: windows hold the sequence's first p.mask.keep keys as well
+template <int DK, int DV, bool KEEP>
 __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Args p) {
   // two K | V stages as separate objects: reads of one cannot alias the DMA into the other
   __shared__ __attribute__((aligned(16))) char st0[128 * (DK + DV)];
@@ -93,13 +94,13 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
 #pragma unroll
     for (int ks = 0; ks < DK / 16; ++ks) qf[ks] = *reinterpret_cast<const short8*>(qrow + 16 * ks);
   }
-  const int keep = p.mask.keep, qlo = p.mask.lo(qpos);
+  const int keep = KEEP ? p.mask.keep : 0, qlo = p.mask.lo(qpos);
   const int lo_min = p.mask.lo(wmin), lo_max = p.mask.lo(wmax);
   const int kv_end = off + min(b0 + rows, qlen);
   // visited tiles: [0, tk) with kept keys, then the window's [t0, t1)
   const int t0 = p.mask.lo(off + b0) >> 6, t1 = (kv_end + 63) >> 6;
-  const int tk = min((keep + 63) >> 6, t0), nt = tk + t1 - t0;
-  auto tile_of = [&](int j) { return j < tk ? j : t0 + j - tk; };
+  const int tk = KEEP ? min((keep + 63) >> 6, t0) : 0, nt = tk + t1 - t0;
+  auto tile_of = [&](int j) { return KEEP && j < tk ? j : t0 + j - tk; };
   // staged pages: those of the kept tiles, then the window's from pg0 on
   const int nkp = ((tk << 6) + BS - 1) >> p.page_lg;
   const int pg0 = (t0 << 6) >> p.page_lg;
@@ -117,7 +118,7 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
     for (int i = 0; i < N; ++i) {
       const int c = (w * N + i) * 64 + lane, row = c / CPR;
       const int key = min(t * 64 + row, kv_end - 1);
-      const int pi = (key >> p.page_lg) - (t < tk ? 0 : pg0 - nkp);
+      const int pi = (key >> p.page_lg) - (KEEP && t < tk ? 0 : pg0 - nkp);
       const int pl = pg_lds[pi < kMaxPages ? pi : 0];
       const int page = pi < kMaxPages ? pl : bt[key >> p.page_lg];
       at[i] = ((((int64_t)page * p.G + kvh) << p.page_lg) + (key & pmask)) * W +
@@ -156,7 +157,7 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
     const char* Kl = buf ? st1 : st0;
     const char* Vl = Kl + 128 * DK;
     const int k0 = t * 64;
-    if (k0 <= wmax && (k0 + 63 >= lo_min || k0 < keep)) {  // wave-uniform: some row sees some key
+    if (k0 <= wmax && (k0 + 63 >= lo_min || (KEEP && k0 < keep))) {  // wave-uniform: some row sees some key
       float16v sa[2];
 #pragma unroll
       for (int half = 0; half < 2; ++half) {
@@ -168,14 +169,14 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
                             qf[ks], sa[half]);
       }
       float mloc = -INFINITY;
-      if (k0 + 63 > wmin || (k0 < lo_max && k0 + 63 >= keep)) {  // an edge crosses the tile
+      if (k0 + 63 > wmin || (k0 < lo_max && (!KEEP || k0 + 63 >= keep))) {  // an edge crosses the tile
         const int top = qpos - k0 - 4 * hi, bot = qlo - k0 - 4 * hi, kp = keep - k0 - 4 * hi;
 #pragma unroll
         for (int half = 0; half < 2; ++half)
 #pragma unroll
           for (int r = 0; r < 16; ++r) {
             const int kk = half * 32 + (r & 3) + 8 * (r >> 2);
-            const float v = (kk > top || (kk < bot && kk >= kp)) ? -INFINITY : sa[half][r];
+            const float v = (kk > top || (kk < bot && (!KEEP || kk >= kp))) ? -INFINITY : sa[half][r];
             sa[half][r] = v;
             mloc = fmaxf(mloc, v);
           }
@@ -269,7 +270,10 @@ int omnia_gqa_prefill(void* out, const void* q, const void* kc, const void* vc,
          mask, scale * 1.4426950408889634f};
 #define OMNIA_GQ(K, V)                                                  \
   if (Dp == K && Vp == V) {                                             \
-    prefill_kernel<K, V><<<n_tiles * H, 256, 0, s>>>(a);                \
+    if (mask.window > 0 && mask.chunk == 0 && mask.keep > 0)            \
+      prefill_kernel<K, V, true><<<n_tiles * H, 256, 0, s>>>(a);        \
+    else                                                                \
+      prefill_kernel<K, V, false><<<n_tiles * H, 256, 0, s>>>(a);       \
     return (int)hipGetLastError();                                      \
   }
 #define OMNIA_GQV(K) \

@@ -22,7 +22,7 @@ struct Mask {
     return window > 0 ? max(0, p - window + 1) : 0;
   }
   // kept keys before a window that starts at lo
-  __device__ __forceinline__ int kept(int lo) const { return min(keep, lo); }
+  __device__ __forceinline__ int kept(int lo) const { return chunk > 0 ? 0 : min(keep, lo); }
 };
 
 }  // namespace omnia
