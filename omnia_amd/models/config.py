@@ -256,7 +256,7 @@ def _chunked(heads: int, kv_heads: int, dim: int, chunk: int) -> AttentionSpec:
 # Bisuzen: tanh pre-normed layer list of attention and linear attention side by side, chunked
 # attention without positions, gelu feed-forwards and grouped experts, looped layers
 TINY_BISUZEN = ModelConfig(
-    name="tiny-bisuzen", arch="bisuzen", vocab_size=512, hidden_size=160, num_layers=7,
+    name="tiny-bisuzen", arch="bisuzen", vocab_size=512, hidden_size=160, num_layers=6,
     intermediate_size=208, max_position=4096, logit_scale=0.5, bos_token_id=256,
     eos_token_ids=(257,),
     layers=looped((
