@@ -31,7 +31,11 @@ struct Next {  // w null: identity; b null: RMS, else tanh
   const float* b;
 };
 
+// PT: the storage type if both branches have it, else -1 (looked up: slower, since every
+// load is then waited for in its own branch)
+template <int PT>
 __device__ __forceinline__ float4v load4(const void* base, int type, int64_t at) {
+  if constexpr (PT >= 0) type = PT;
   if (type == 1) return *reinterpret_cast<const float4v*>((const float*)base + at);
   if (type == 2) {
     const half4v h = *reinterpret_cast<const half4v*>((const _Float16*)base + at);
@@ -50,7 +54,7 @@ __device__ __forceinline__ void store4(bf16_t* p, float4v v) {
 }
 
 // columns of a thread: c = (threadIdx.x + i * NT) * 4, i < NC
-template <typename T, int NT, int NC>
+template <typename T, int PT, int NT, int NC>
 __global__ __launch_bounds__(NT) void branch_kernel(T* __restrict__ h, float* __restrict__ x,
                                                     int d, Branch ba, Branch bb, float inv_n,
                                                     float eps, Next next) {
@@ -63,8 +67,8 @@ __global__ __launch_bounds__(NT) void branch_kernel(T* __restrict__ h, float* __
   for (int i = 0; i < NC; ++i) {
     const int c = (tid + i * NT) * 4;
     const bool in = c < d;
-    a[i] = in ? load4(ba.m, ba.type, t * ba.row + c) : zero;
-    b[i] = in ? load4(bb.m, bb.type, t * bb.row + c) : zero;
+    a[i] = in ? load4<PT>(ba.m, ba.type, t * ba.row + c) : zero;
+    b[i] = in ? load4<PT>(bb.m, bb.type, t * bb.row + c) : zero;
     old[i] = in ? *reinterpret_cast<const float4v*>(x + t * d + c) : zero;
   }
   auto slabs = [&](float4v (&v)[NC], const Branch& p) {
@@ -76,7 +80,7 @@ __global__ __launch_bounds__(NT) void branch_kernel(T* __restrict__ h, float* __
           float4v q[4];
 #pragma unroll
           for (int j = 0; j < 4; ++j)
-            q[j] = s + j < p.S ? load4(p.m, p.type, (s + j) * p.slab + t * p.row + c) : zero;
+            q[j] = s + j < p.S ? load4<PT>(p.m, p.type, (s + j) * p.slab + t * p.row + c) : zero;
           v[i] += (q[0] + q[1]) + (q[2] + q[3]);
         }
       }
@@ -165,19 +169,20 @@ extern "C" int omnia_branch_residual(void* h, int f32, float* x, int rows, int d
                                      const float* bw, float inv_n, float eps, float alpha,
                                      const float* nw, const float* nb, hipStream_t s) {
   if (d % 4 || d < 4 || d > 16384 || aS < 1 || bS < 1 || arow % 4 || aslab % 4 || brow % 4 ||
-      bslab % 4 || !aw || !bw)
+      bslab % 4 || !aw || !bw || (f32 && (at != 1 || bt != 1)))
     return -1;
   if (rows == 0) return 0;
   const Branch ba{a, at, aS, arow, aslab, abias, aw}, bb{b, bt, bS, brow, bslab, bbias, bw};
   const Next next{alpha, nw, nb};
-#define OMNIA_BR(NT, NC)                                                                     \
-  do {                                                                                       \
-    if (f32)                                                                                 \
-      branch_kernel<float, NT, NC><<<rows, NT, 0, s>>>((float*)h, x, d, ba, bb, inv_n, eps,  \
-                                                       next);                                \
-    else                                                                                     \
-      branch_kernel<bf16_t, NT, NC><<<rows, NT, 0, s>>>((bf16_t*)h, x, d, ba, bb, inv_n,     \
-                                                        eps, next);                          \
+#define OMNIA_BRP(TT, PT, NT, NC) \
+  branch_kernel<TT, PT, NT, NC><<<rows, NT, 0, s>>>((TT*)h, x, d, ba, bb, inv_n, eps, next)
+#define OMNIA_BR(NT, NC)                                        \
+  do {                                                          \
+    if (f32) OMNIA_BRP(float, 1, NT, NC);                       \
+    else if (at != bt) OMNIA_BRP(bf16_t, -1, NT, NC);           \
+    else if (at == 0) OMNIA_BRP(bf16_t, 0, NT, NC);             \
+    else if (at == 1) OMNIA_BRP(bf16_t, 1, NT, NC);             \
+    else OMNIA_BRP(bf16_t, 2, NT, NC);                          \
   } while (0)
   if (d <= 1024) OMNIA_BR(256, 1);
   else if (rows <= 512 && d <= 4096) OMNIA_BR(1024, 1);
@@ -186,5 +191,6 @@ extern "C" int omnia_branch_residual(void* h, int f32, float* x, int rows, int d
   else if (d <= 8192) OMNIA_BR(1024, 2);
   else OMNIA_BR(1024, 4);
 #undef OMNIA_BR
+#undef OMNIA_BRP
   return (int)hipGetLastError();
 }

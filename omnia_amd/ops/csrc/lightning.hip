@@ -234,7 +234,7 @@ struct Scan {
 // B operand of the next product as it stands: k-step r takes dimension (token)
 // 4 (lane >> 4) + r, and the A side is read in that order.  32 tokens a step.
 template <typename T, int ND, int NC, bool OUT>
-__global__ __launch_bounds__(256) void scan_kernel(const T* __restrict__ x, Scan p) {
+__global__ __launch_bounds__(256, ND <= 8 ? 2 : 1) void scan_kernel(const T* __restrict__ x, Scan p) {
   constexpr int DW = 16 * ND, KS = DW + 4, PS = 20;
   constexpr int NL = 32 * DW / 4 / 256;  // 4-element chunks a thread holds of 32 rows
   __shared__ __attribute__((aligned(16))) float kb[32 * KS];
