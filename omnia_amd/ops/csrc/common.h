@@ -50,6 +50,14 @@ __device__ __forceinline__ float siluf_(float x) { return x * sigmoidf_(x); }
 __device__ __forceinline__ float gelu_tanh_(float x) {
   return x * sigmoidf_(1.5957691216057308f * (x + 0.044715f * x * x * x));
 }
+// gelu, erf form, for 16-bit results: max(x, 0) - |x| e, e = 0.5 erfc(|x| / sqrt(2)) by
+// Abramowitz and Stegun 7.1.26 (|error| of erf < 1.5e-7), its constants scaled to |x|
+__device__ __forceinline__ float gelu_erf16_(float x) {
+  const float a = fabsf(x), t = __builtin_amdgcn_rcpf(1.f + 0.23164189f * a);
+  const float p = ((((0.5307027145f * t - 0.7265760135f) * t + 0.7107068705f) * t -
+                    0.142248368f) * t + 0.127414796f) * t;
+  return fmaxf(x, 0.f) - a * p * __builtin_amdgcn_exp2f(-0.7213475204f * x * x);
+}
 // gelu, erf form
 __device__ __forceinline__ float gelu_erf_(float x) {
   return 0.5f * x * (1.f + erff(x * 0.7071067811865476f));

@@ -20,15 +20,17 @@
 // State of sequence slot s: state[s][h][Dp][Vp] fp32.  A sequence whose first row of this
 // launch is at position 0 starts from zeros, whatever its slot held: slots are never
 // cleared.  A negative slot (padded graph row) reads and writes no state.  Everything in
-// the recurrence is fp32, the products too (fp32 MFMA).
+// the recurrence is fp32.  The products of fp32 models are fp32 MFMA; bf16 models round q,
+// k and v to bf16 and split every fp32 operand (state, decayed scores and values) into
+// three bf16 parts that hold all its bits, so that bf16 MFMA multiplies it unrounded.
 #include "common.h"
 
 using namespace omnia;
 
 namespace {
 
-constexpr int kPow = 32;     // a row of the power table: a^0 .. a^16, then a^(64 * 2^i)
-constexpr int kPowSeg = 17;  // first of the latter
+constexpr int kPow = 48;     // a row of the power table: a^0 .. a^32, then a^(64 * 2^i)
+constexpr int kPowSeg = 33;  // first of the latter
 
 // projection rows or their split-K slabs
 struct Src {
@@ -234,7 +236,8 @@ struct Scan {
 // B operand of the next product as it stands: k-step r takes dimension (token)
 // 4 (lane >> 4) + r, and the A side is read in that order.  32 tokens a step.
 template <typename T, int ND, int NC, bool OUT>
-__global__ __launch_bounds__(256, ND <= 8 ? 2 : 1) void scan_kernel(const T* __restrict__ x, Scan p) {
+__global__ __launch_bounds__(256, ND <= 8 ? 2 : 1) void scan_kernel(const T* __restrict__ x,
+                                                                   Scan p) {
   constexpr int DW = 16 * ND, KS = DW + 4, PS = 20;
   constexpr int NL = 32 * DW / 4 / 256;  // 4-element chunks a thread holds of 32 rows
   __shared__ __attribute__((aligned(16))) float kb[32 * KS];
@@ -373,17 +376,21 @@ __global__ __launch_bounds__(256, ND <= 8 ? 2 : 1) void scan_kernel(const T* __r
         const float* p0 = pb + 2 * b * 16 * PS + c16 * PS + 4 * g4;
         const float4v pa = *reinterpret_cast<const float4v*>(p0) +
                            *reinterpret_cast<const float4v*>(p0 + 16 * PS);
+        float4v ov[NC];
+#pragma unroll
+        for (int c = 0; c < NC; ++c) ov[c] = G * (qs[c][0] + qs[c][1]);
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+          for (int c = 0; c < NC; ++c) ov[c] = mfma4(pa[r], v[b][c][r], ov[c]);
 #pragma unroll
         for (int c = 0; c < NC; ++c) {
-          float4v ov = G * (qs[c][0] + qs[c][1]);
-#pragma unroll
-          for (int r = 0; r < 4; ++r) ov = mfma4(pa[r], v[b][c][r], ov);
           const int col = col0 + 16 * c;
           if (col < Vp) {
             float* op = p.o + ((int64_t)(row0 + t0 + 16 * b + 4 * g4) * H + h) * Vp + col;
 #pragma unroll
             for (int r = 0; r < 4; ++r)
-              if (4 * g4 + r < m) op[(int64_t)r * H * Vp] = ov[r];
+              if (4 * g4 + r < m) op[(int64_t)r * H * Vp] = ov[c][r];
           }
         }
       }
@@ -396,19 +403,281 @@ __global__ __launch_bounds__(256, ND <= 8 ? 2 : 1) void scan_kernel(const T* __r
       }
 #pragma unroll
       for (int c = 0; c < NC; ++c) v[b][c] *= e;
+      // two key tiles at a time: independent products between dependent ones
 #pragma unroll
-      for (int j = 0; j < ND; ++j) {
-        float ka[4];
+      for (int j = 0; j < ND; j += 2) {
+        float ka[2][4];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) ka[r] = k0[(4 * g4 + r) * KS + 16 * j + c16];
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) ka[i][r] = k0[(4 * g4 + r) * KS + 16 * (j + i) + c16];
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+          for (int c = 0; c < NC; ++c) S[j + i][c] *= am;
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+          for (int i = 0; i < 2; ++i)
+#pragma unroll
+            for (int c = 0; c < NC; ++c) S[j + i][c] = mfma4(ka[i][r], v[b][c][r], S[j + i][c]);
+      }
+    }
+  }
+  if (slot < 0 || (OUT && !last)) return;
+  float* to = OUT ? p.state + ((int64_t)slot * H + h) * Dp * Vp
+                  : p.seg + ((int64_t)id * H + h) * Dp * Vp;
+#pragma unroll
+  for (int j = 0; j < ND; ++j)
+#pragma unroll
+    for (int c = 0; c < NC; ++c)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int d = 16 * j + 4 * g4 + r, col = col0 + 16 * c;
+        if (d < Dp && col < Vp) to[(int64_t)d * Vp + col] = S[j][c][r];
+      }
+}
+
+// ------------------------------------------- the same scan on bf16 MFMA (bf16 models)
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+__device__ __forceinline__ float4v mfma16(short8 a, short8 b, float4v c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a),
+                                                 __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
+}
+// eight fp32 values as three bf16 parts of 8 bits each (their sum is the value)
+struct Split {
+  short8 part[3];
+};
+__device__ __forceinline__ Split split8(float4v lo, float4v hi) {
+  Split s;
+#pragma unroll
+  for (int k = 0; k < 3; ++k)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const uint32_t a = __float_as_uint(lo[j]), b = __float_as_uint(hi[j]);
+      s.part[k][j] = (short)(a >> 16);
+      s.part[k][4 + j] = (short)(b >> 16);
+      lo[j] -= __uint_as_float(a & 0xffff0000u);
+      hi[j] -= __uint_as_float(b & 0xffff0000u);
+    }
+  return s;
+}
+
+// As scan_kernel, 32 tokens a block, two LDS buffers and one barrier a block.  Products
+// over 32 key dimensions (or tokens) take, in lane group g4 = lane >> 4, the dimensions
+// 4 g4 + r of one 16-tile and of the next (r < 4): what the state's accumulators hold.  The
+// scores are made transposed (row i, column t), which is the A operand of P V as it stands.
+template <int ND, int NC, bool OUT>
+__global__ __launch_bounds__(256, ND <= 8 ? 2 : 1) void scan16_kernel(const bf16_t* __restrict__ x, Scan p) {
+  constexpr int DW = 16 * ND, KS = DW + 8, NJ = ND / 2;
+  constexpr int NL = 32 * DW / 4 / 256;
+  struct Buf {
+    bf16_t k[32 * KS], q[OUT ? 32 * KS : 8];
+  };
+  __shared__ __attribute__((aligned(16))) Buf buf[2];
+  const int id = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
+  int lo = 0, hi = p.nseq - 1;
+  while (lo < hi) {
+    const int mid = (lo + hi + 1) >> 1;
+    if (seg_base(p.q_start, mid, p.L) <= id) lo = mid; else hi = mid - 1;
+  }
+  const int j0 = (id - seg_base(p.q_start, lo, p.L)) * p.L;
+  const int all = p.q_start[lo + 1] - p.q_start[lo], n = min(p.L, all - j0);
+  const int slot = p.slots[lo];
+  const bool last = j0 + p.L >= all;
+  if (n <= 0 || (!OUT && (last || slot < 0))) return;
+  const int row0 = p.q_start[lo] + j0;
+  const int lane = tid & 63, w = tid >> 6, c16 = lane & 15, g4 = lane >> 4;
+  const int Dp = p.Dp, Vp = p.Vp, H = p.H;
+  const int col0 = (blockIdx.z * 4 + w) * 16 * NC + c16;
+  const float* pw = p.pw + h * kPow;
+  const float4v zero = {0.f, 0.f, 0.f, 0.f};
+
+  float4v S[ND][NC];
+  {
+    const float* from = nullptr;
+    if (OUT && slot >= 0) {
+      if (all > p.L) from = p.seg + ((int64_t)id * H + h) * Dp * Vp;
+      else if (p.positions[row0] != 0) from = p.state + ((int64_t)slot * H + h) * Dp * Vp;
+    }
+#pragma unroll
+    for (int j = 0; j < ND; ++j)
+#pragma unroll
+      for (int c = 0; c < NC; ++c)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int d = 16 * j + 4 * g4 + r, col = col0 + 16 * c;
+          S[j][c][r] = (from && d < Dp && col < Vp) ? from[(int64_t)d * Vp + col] : 0.f;
+        }
+  }
+  // decays of this lane's places: outputs a^(t+1) and values a^(31-t) at t = 4 g4 + r (+ 16),
+  // scores a^(t-i) at t = c16, i = 4 g4 + r of one tile and of the one before
+  float4v G[2], E[2], Pd, Po;
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int t = 4 * g4 + r;
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      G[b][r] = pw[16 * b + t + 1];
+      E[b][r] = pw[31 - 16 * b - t];
+    }
+    Pd[r] = c16 >= t ? pw[max(c16 - t, 0)] : 0.f;
+    Po[r] = pw[16 + c16 - t];
+  }
+  const float a32 = pw[32];
+
+  const bf16_t* kx = x + (int64_t)row0 * p.ldx + (int64_t)H * Dp + h * Dp;
+  const bf16_t* qx = x + (int64_t)row0 * p.ldx + h * Dp;
+  const bf16_t* vx = x + (int64_t)row0 * p.ldx + (int64_t)2 * H * Dp + h * Vp;
+  short4v kreg[NL], qreg[OUT ? NL : 1];
+  bf16_t vreg[2][NC][4];
+  // unconditional loads: rows past the end re-read the last one, columns past the head its
+  // last ones (zeroed when they are used)
+  auto gload = [&](int t0) {
+#pragma unroll
+    for (int i = 0; i < NL; ++i) {
+      const int e = i * 256 + tid, tt = min(t0 + e / (DW / 4), n - 1);
+      const int64_t at = (int64_t)tt * p.ldx + min(e % (DW / 4) * 4, Dp - 4);
+      kreg[i] = *reinterpret_cast<const short4v*>(kx + at);
+      if (OUT) qreg[i] = *reinterpret_cast<const short4v*>(qx + at);
+    }
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const bf16_t* vr = vx + (int64_t)min(t0 + 16 * b + 4 * g4 + r, n - 1) * p.ldx;
+#pragma unroll
+        for (int c = 0; c < NC; ++c) vreg[b][c][r] = vr[min(col0 + 16 * c, Vp - 1)];
+      }
+  };
+  auto lwrite = [&](Buf& B, int t0) {
+#pragma unroll
+    for (int i = 0; i < NL; ++i) {
+      const int e = i * 256 + tid, tt = e / (DW / 4), d4 = e % (DW / 4) * 4;
+      const bool in = d4 < Dp && t0 + tt < n;
+      auto put = [&](bf16_t* to, short4v v) {
+        const float4v f = silu4(Raw4<bf16_t>::f(v));
+        uint2v o;
+        o[0] = in ? pack_bf2(f[0], f[1]) : 0u;
+        o[1] = in ? pack_bf2(f[2], f[3]) : 0u;
+        *reinterpret_cast<uint2v*>(to + tt * KS + d4) = o;
+      };
+      put(B.k, kreg[i]);
+      if constexpr (OUT) put(B.q, qreg[i]);
+    }
+  };
+  typedef short v4s __attribute__((ext_vector_type(4)));
+  typedef __attribute__((address_space(3))) v4s* lds_v4s;
+  auto frag = [&](const bf16_t* base, int tile, int jj) {  // rows of a tile, 32 dimensions
+    const bf16_t* at = base + (16 * tile + c16) * KS + 32 * jj + 4 * g4;
+    return __builtin_shufflevector(*reinterpret_cast<const v4s*>(at),
+                                   *reinterpret_cast<const v4s*>(at + 16), 0, 1, 2, 3, 4, 5, 6, 7);
+  };
+
+  gload(0);
+  lwrite(buf[0], 0);
+  const int nblk = (n + 31) / 32;
+  for (int bi = 0; bi < nblk; ++bi) {
+    const int t0 = 32 * bi, m = n - t0;
+    Buf& B = buf[bi & 1];
+    short8 vb[NC];  // values at tokens 4 g4 + r (+ 16)
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int c = 0; c < NC; ++c)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const bool in = 16 * b + 4 * g4 + r < m && col0 + 16 * c < Vp;
+          vb[c][4 * b + r] = in ? (short)f2bf(siluf_(bf2f(vreg[b][c][r]))) : (short)0;
+        }
+    // this block's operands are complete, and every wave is done with the other buffer
+    __syncthreads();
+    if (bi + 1 < nblk) gload(t0 + 32);
+    if constexpr (OUT) {
+      float4v s00 = zero, s10 = zero, s11 = zero;  // scores of (t tile, i tile), transposed
+#pragma unroll
+      for (int jj = 0; jj < NJ; ++jj) {
+        const short8 k0 = frag(B.k, 0, jj), k1 = frag(B.k, 1, jj);
+        const short8 q0 = frag(B.q, 0, jj), q1 = frag(B.q, 1, jj);
+        s00 = mfma16(k0, q0, s00);
+        s10 = mfma16(k0, q1, s10);
+        s11 = mfma16(k1, q1, s11);
+      }
+      __builtin_amdgcn_sched_barrier(0);  // registers: the scores first
+      const Split p0 = split8(s00 * Pd, zero), p1 = split8(s10 * Po, s11 * Pd);
+      float4v o[2][NC];
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int c = 0; c < NC; ++c) o[b][c] = zero;
+#pragma unroll
+      for (int jj = 0; jj < NJ; ++jj) {
+        const short8 qf[2] = {frag(B.q, 0, jj), frag(B.q, 1, jj)};
 #pragma unroll
         for (int c = 0; c < NC; ++c) {
-          S[j][c] *= am;
+          const Split st = split8(S[2 * jj][c], S[2 * jj + 1][c]);
 #pragma unroll
-          for (int r = 0; r < 4; ++r) S[j][c] = mfma4(ka[r], v[b][c][r], S[j][c]);
+          for (int k = 0; k < 3; ++k)
+#pragma unroll
+            for (int b = 0; b < 2; ++b) o[b][c] = mfma16(qf[b], st.part[k], o[b][c]);
+        }
+      }
+#pragma unroll
+      for (int c = 0; c < NC; ++c) {
+#pragma unroll
+        for (int b = 0; b < 2; ++b) o[b][c] *= G[b];
+#pragma unroll
+        for (int k = 0; k < 3; ++k) {
+          o[0][c] = mfma16(p0.part[k], vb[c], o[0][c]);
+          o[1][c] = mfma16(p1.part[k], vb[c], o[1][c]);
+        }
+        const int col = col0 + 16 * c;
+        if (col < Vp) {
+#pragma unroll
+          for (int b = 0; b < 2; ++b) {
+            float* op = p.o + ((int64_t)(row0 + t0 + 16 * b + 4 * g4) * H + h) * Vp + col;
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+              if (16 * b + 4 * g4 + r < m) op[(int64_t)r * H * Vp] = o[b][c][r];
+          }
         }
       }
     }
+    float4v e[2] = {E[0], E[1]};
+    float am = a32;
+    if (m < 32) {
+      am = pw[m];
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int t = 16 * b + 4 * g4 + r;
+          e[b][r] = t < m ? pw[max(m - 1 - t, 0)] : 0.f;
+        }
+    }
+    Split vs[NC];
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+      float4v v[2];
+#pragma unroll
+      for (int r = 0; r < 8; ++r) v[r >> 2][r & 3] = bf2f((uint16_t)vb[c][r]);
+      vs[c] = split8(v[0] * e[0], v[1] * e[1]);
+    }
+#pragma unroll
+    for (int j = 0; j < ND; ++j) {
+      // keys transposed: this lane's dimension 16 j + c16 at tokens 4 g4 + r (+ 16)
+      const bf16_t* at = B.k + (4 * g4 + (c16 >> 2)) * KS + 16 * j + 4 * (c16 & 3);
+      const v4s lo4 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_v4s)at);
+      const v4s hi4 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_v4s)(at + 16 * KS));
+      const short8 kt = __builtin_shufflevector(lo4, hi4, 0, 1, 2, 3, 4, 5, 6, 7);
+#pragma unroll
+      for (int c = 0; c < NC; ++c) S[j][c] *= am;
+#pragma unroll
+      for (int k = 0; k < 3; ++k)
+#pragma unroll
+        for (int c = 0; c < NC; ++c) S[j][c] = mfma16(kt, vs[c].part[k], S[j][c]);
+    }
+    if (bi + 1 < nblk) lwrite(buf[(bi + 1) & 1], t0 + 32);
   }
   if (slot < 0 || (OUT && !last)) return;
   float* to = OUT ? p.state + ((int64_t)slot * H + h) * Dp * Vp
@@ -505,30 +774,35 @@ int any(float* o, float* state, Src x, const float* pw, const int* q_start, int 
   return (int)hipGetLastError();
 }
 
-template <typename T>
-int scan(const void* x, const Scan& p, int n_rows, int pow_at, hipStream_t s) {
+int scan(const void* x, int f32, const Scan& p, int n_rows, int pow_at, hipStream_t s) {
   const bool split = n_rows > p.L;  // else every portion is one segment
-  const int segs = n_rows / p.L + p.nseq, nc = p.Vp <= 64 ? 1 : 2;
+  const int segs = n_rows / p.L + p.nseq, nc = p.Vp <= 64 || p.Dp > 128 ? 1 : 2;
   const dim3 grid(segs, p.H, (p.Vp + 64 * nc - 1) / (64 * nc));
   const dim3 cgrid(p.nseq, p.H, (p.Dp * p.Vp + 1023) / 1024);
-#define OMNIA_LS(ND, NC)                                                        \
-  do {                                                                          \
-    if (split) {                                                                \
-      scan_kernel<T, ND, NC, false><<<grid, 256, 0, s>>>((const T*)x, p);       \
-      chain_kernel<<<cgrid, 256, 0, s>>>(p, pow_at);                            \
-    }                                                                           \
-    scan_kernel<T, ND, NC, true><<<grid, 256, 0, s>>>((const T*)x, p);          \
-    return (int)hipGetLastError();                                              \
+#define OMNIA_LSK(OUT, ND, NC)                                                            \
+  do {                                                                                    \
+    if (f32) scan_kernel<float, ND, NC, OUT><<<grid, 256, 0, s>>>((const float*)x, p);    \
+    else scan16_kernel<ND, NC, OUT><<<grid, 256, 0, s>>>((const bf16_t*)x, p);            \
+  } while (0)
+#define OMNIA_LS(ND, NC)                                \
+  do {                                                  \
+    if (split) {                                        \
+      OMNIA_LSK(false, ND, NC);                         \
+      chain_kernel<<<cgrid, 256, 0, s>>>(p, pow_at);    \
+    }                                                   \
+    OMNIA_LSK(true, ND, NC);                            \
+    return (int)hipGetLastError();                      \
   } while (0)
 #define OMNIA_LSD(ND)                   \
   if (p.Dp <= 16 * ND) {                \
     if (nc == 1) OMNIA_LS(ND, 1);       \
     else OMNIA_LS(ND, 2);               \
   }
-  OMNIA_LSD(2) OMNIA_LSD(4) OMNIA_LSD(8) OMNIA_LSD(16)
+  OMNIA_LSD(2) OMNIA_LSD(4) OMNIA_LSD(8)
+  OMNIA_LS(16, 1);
 #undef OMNIA_LSD
 #undef OMNIA_LS
-  return -5;
+#undef OMNIA_LSK
 }
 
 // segment length of n_rows rows: enough workgroups to fill the chip, no shorter than 128
@@ -584,7 +858,7 @@ int omnia_lightning_scan(float* o, float* state, float* seg, const void* x, int 
   while ((64 << (pow_at - kPowSeg)) < L) ++pow_at;
   if (pow_at >= kPow || (n_rows > L && !seg)) return -2;
   const Scan p{o, state, seg, pw, q_start, positions, slots, ldx, nseq, H, Dp, Vp, L};
-  return f32 ? scan<float>(x, p, n_rows, pow_at, s) : scan<bf16_t>(x, p, n_rows, pow_at, s);
+  return scan(x, f32, p, n_rows, pow_at, s);
 }
 
 // w [n] fp32, n = H * Vp; inv_n counts the real columns

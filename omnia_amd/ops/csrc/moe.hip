@@ -512,7 +512,7 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(
     } else if (MODE == 3) {
 #pragma unroll
       for (int j = 0; j < 4; ++j)
-        out[(int64_t)row * N + n0 + 16 * j + fr] = f2bf(gelu_erf_(acc[j][r]));
+        out[(int64_t)row * N + n0 + 16 * j + fr] = f2bf(gelu_erf16_(acc[j][r]));
     } else {
       const float wt = route_w ? route_w[flat] : 1.f;
 #pragma unroll

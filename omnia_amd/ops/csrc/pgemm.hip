@@ -590,7 +590,7 @@ __global__ __launch_bounds__(512, 2) void pgemm_kernel(PArgs p) {
             float4v v = acc[a][b][m][n];
             if constexpr (EPI == 10) {
 #pragma unroll
-              for (int j = 0; j < 4; ++j) v[j] = gelu_erf_(v[j]);
+              for (int j = 0; j < 4; ++j) v[j] = gelu_erf16_(v[j]);
             }
             put(row0, b * 128 + wc * 32 + n * 16 + fr, v[0] * rs[0], v[1] * rs[1], v[2] * rs[2],
                 v[3] * rs[3]);

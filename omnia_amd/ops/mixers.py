@@ -236,8 +236,8 @@ def delta_rule(x, w: dict, spec, state, conv_state, q_start, positions, slots, e
 
 # ---------------------------------------------------- fixed-decay linear attention
 def decay_powers(decay, device) -> torch.Tensor:
-    """fp32 [heads, 32]: a^0 .. a^16, then a^64, a^128, a^256, ... (double precision)."""
-    n = torch.tensor([*range(17), *(64 << i for i in range(15))], dtype=torch.float64)
+    """fp32 [heads, 48]: a^0 .. a^32, then a^64, a^128, a^256, ... (double precision)."""
+    n = torch.tensor([*range(33), *(64 << i for i in range(15))], dtype=torch.float64)
     a = torch.tensor(decay, dtype=torch.float64)
     return torch.pow(a[:, None], n).float().to(device)
 
