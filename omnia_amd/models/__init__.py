@@ -1,5 +1,5 @@
 """Model families served by the in-node engine (Llama-3 dense, Mixtral MoE, and the
-layer lists Sivadra and Sekazen)."""
+layer lists Sivadra, Sekazen and Bisuzen)."""
 from .config import REGISTRY, ModelConfig, resolve  # noqa: F401
 
 
