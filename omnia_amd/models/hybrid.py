@@ -14,8 +14,8 @@ joins the two branches of a parallel mixer:
                     (-> softcap)
 
 A layer may use another layer's tensors (its pages / state are its own; the later passes
-of a looped layer do), or attend to another layer's pages.  bf16 models keep what feeds a softmax, a router or a recurrence
-in fp32; fp32 models run every kernel and GEMM in fp32.
+of a looped layer do), or attend to another layer's pages.  bf16 models keep what feeds a
+softmax, a router or a recurrence in fp32; fp32 models run every kernel and GEMM in fp32.
 """
 from __future__ import annotations
 

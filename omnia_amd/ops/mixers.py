@@ -358,7 +358,8 @@ def latent_prefill(q, kx, kr, vt, fb, spec, gate, out=None):
 # ------------------------------------------------------ grouped-query attention
 def gqa_prep(x, w: dict, spec, pages, positions, slots, cos_sin, dtype, eps: float):
     """Fused projection rows (or split-K slabs) -> queries [T, H * dim_pad], with bias, norm
-    and rotation as the spec says; writes the tokens' keys and values at ``slots`` of ``pages`` = (k, v), or, with
+    and rotation as the spec says; writes the tokens' keys and values at ``slots`` of
+    ``pages`` = (k, v), or, with
     ``pages`` None, none (the layer borrows another one's)."""
     k, v = pages if pages is not None else (None, None)
     if x.is_cuda:
