@@ -244,7 +244,7 @@ def _parallel(heads: int, kv_heads: int, dim: int, window: int, lin_heads: int, 
                       rotary=RotarySpec(dim // 2, base, interleaved=True), window=window,
                       keep_first=keep, qk_norm=None, bias=True),
         LightningSpec(heads=lin_heads, dim=dim, vdim=dim, decay=tuple(
-            math.exp(-2.0 ** (-1.0 - 11.0 * i / max(lin_heads - 1, 1)))
+            1.0 - 2.0 ** (-1.0 - 11.0 * i / max(lin_heads - 1, 1))
             for i in range(lin_heads))))
 
 
