@@ -13,7 +13,7 @@ from dataclasses import dataclass, field
 
 from .layers import (DESIGNS, AttentionSpec, BandSpec, DeltaSpec, DenseMLPSpec, DesignSpec,
                      ExpertsSpec, LatentAttentionSpec, LayerSpec, LightningSpec, ParallelSpec,
-                     RotarySpec, YarnSpec, looped, tensor_shapes)
+                     RotarySpec, TemperatureSpec, YarnSpec, looped, tensor_shapes)
 
 
 @dataclass(frozen=True)
@@ -38,6 +38,7 @@ class ModelConfig:
     # layer-list models (models/hybrid.py): one LayerSpec per layer; the uniform
     # head / intermediate sizes above do not apply to them
     layers: tuple = ()
+    embed_scale: float = 1.0  # the residual starts at the embedding times this
     logit_scale: float = 1.0  # the head's output times this
     logit_softcap: float = 0.0  # > 0: logits <- cap tanh(logits / cap)
     # tokenizer special ids (llama-3 layout)
@@ -242,7 +243,7 @@ def _parallel(heads: int, kv_heads: int, dim: int, window: int, lin_heads: int, 
     return ParallelSpec(
         AttentionSpec(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, scale=dim ** -0.5,
                       rotary=RotarySpec(dim // 2, base, interleaved=True), window=window,
-                      keep_first=keep, qk_norm=None, bias=True),
+                      keep_first=keep, qk_norm=None, bias="qkvo"),
         LightningSpec(heads=lin_heads, dim=dim, vdim=dim, decay=tuple(
             1.0 - 2.0 ** (-1.0 - 11.0 * i / max(lin_heads - 1, 1))
             for i in range(lin_heads))))
@@ -250,7 +251,7 @@ def _parallel(heads: int, kv_heads: int, dim: int, window: int, lin_heads: int, 
 
 def _chunked(heads: int, kv_heads: int, dim: int, chunk: int) -> AttentionSpec:
     return AttentionSpec(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, scale=dim ** 0.5,
-                         rotary=None, sink=False, qk_norm="unit", chunk=chunk)
+                         rotary=None, sink=None, qk_norm="unit", chunk=chunk)
 
 
 # Bisuzen: tanh pre-normed layer list of attention and linear attention side by side, chunked
@@ -285,11 +286,64 @@ BISUZEN_8B = ModelConfig(  # sivadra-8b
                       DenseMLPSpec(14336, "gelu_tanh", False)),) * 24
     + (LayerSpec(_chunked(32, 8, 128, 4096), DenseMLPSpec(14336, "gelu_tanh", False)),) * 8)
 
+
+
+def _biased(heads: int, kv_heads: int, dim: int, every: float) -> AttentionSpec:
+    """Attention whose positions are a query temperature and a distance bias."""
+    return AttentionSpec(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, scale=dim ** -0.5,
+                         rotary=None, sink="zero", qk_norm=None, bias="qkv", softcap=30.0,
+                         distance_bias=True, gate=True,
+                         temperature=TemperatureSpec(0.1, every))
+
+
+def _latent(heads: int, q_rank: int, base: float) -> LatentAttentionSpec:
+    return LatentAttentionSpec(heads=heads, dim=128, rot_dim=64, vdim=128, q_rank=q_rank,
+                               kv_rank=512, scale=192 ** -0.5,
+                               rotary=RotarySpec(64, base, interleaved=True))
+
+
+def _shared(ff: int, experts: int, top: int, shared: int) -> ExpertsSpec:
+    return ExpertsSpec(ff=ff, experts=experts, top=top, score="softmax", renorm=True,
+                       expert="glu", router_bias=True, shared=DenseMLPSpec(shared, bias=False))
+
+
+# Tarunex: layer list whose mixer and feed-forward run side by side on one residual: capped
+# attention with a distance bias, latent attention, experts beside a shared one, and a loop
+# that every pass enters with the embedding and a vector of its own
+TINY_TARUNEX = ModelConfig(
+    name="tiny-tarunex", arch="tarunex", vocab_size=512, hidden_size=160, num_layers=6,
+    intermediate_size=72, max_position=4096, rms_eps=1e-5, embed_scale=8.0, logit_scale=0.5,
+    logit_softcap=25.0, bos_token_id=256, eos_token_ids=(257,),
+    layers=looped((
+        LayerSpec(_biased(6, 2, 40, 96), _shared(72, 6, 2, 88)),
+        LayerSpec(LatentAttentionSpec(
+            heads=5, dim=40, rot_dim=12, vdim=48, q_rank=56, kv_rank=72, scale=0.14,
+            rotary=RotarySpec(12, 20000.0, interleaved=True)), _shared(56, 5, 1, 40)),
+        LayerSpec(_biased(4, 1, 32, 64), _shared(72, 6, 3, 88)),
+        LayerSpec(_biased(4, 4, 64, 128))), 1, 3, 2))
+# serving-sized shapes (random-init): width, heads, layers run and active feed-forward of the
+# model named beside each
+TARUNEX_3B = ModelConfig(  # sekazen-3b
+    name="tarunex-3b", arch="tarunex", vocab_size=32768, hidden_size=2048, num_layers=16,
+    intermediate_size=3072, max_position=131072, embed_scale=8.0, logit_scale=0.25,
+    logit_softcap=30.0, bos_token_id=256, eos_token_ids=(257,),
+    layers=looped(((LayerSpec(_biased(16, 8, 128, 8192), _shared(3072, 8, 2, 2048)),) * 3
+                   + (LayerSpec(_latent(16, 1024, 500000.0), _shared(3072, 8, 2, 2048)),)) * 3,
+                  4, 8, 2))
+TARUNEX_8B = ModelConfig(  # sivadra-8b
+    name="tarunex-8b", arch="tarunex", vocab_size=128256, hidden_size=4096, num_layers=32,
+    intermediate_size=7168, max_position=131072, embed_scale=8.0, logit_scale=0.25,
+    logit_softcap=30.0, bos_token_id=256, eos_token_ids=(257,),
+    layers=looped(((LayerSpec(_biased(32, 8, 128, 8192), _shared(7168, 3, 1, 7168)),)
+                   + (LayerSpec(_latent(32, 1536, 500000.0), _shared(7168, 3, 1, 7168)),)) * 10,
+                  4, 16, 2))
+
 REGISTRY: dict[str, ModelConfig] = {
     c.name: c for c in [LLAMA3_8B, LLAMA31_8B, LLAMA3_70B, MIXTRAL_8X7B, TINY_LLAMA, TINY_MIXTRAL,
                    TINY_MIXTRAL_E8, EMBED_1B, TINY_EMBED, TINY_LLAMA_H8, TINY_SIVADRA,
                    SIVADRA_1B, SIVADRA_8B, LLAMA_1B, TINY_SEKAZEN, SEKAZEN_3B, SEKAZEN_8X7B,
-                   MIXTRAL_3B, TINY_BISUZEN, BISUZEN_3B, BISUZEN_8B]
+                   MIXTRAL_3B, TINY_BISUZEN, BISUZEN_3B, BISUZEN_8B, TINY_TARUNEX,
+                   TARUNEX_3B, TARUNEX_8B]
 }
 ALIASES = {
     "meta-llama/Meta-Llama-3-8B": "llama-3-8b",

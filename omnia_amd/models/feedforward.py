@@ -21,8 +21,8 @@ def _up8(n: int) -> int:
 class DenseGLU:
     """``W_down(act(W_gate h + b) * (W_up h + b)) + b``, silu or gelu, biases or none."""
 
-    def __init__(self, spec, model):
-        self.spec, self.model = spec, model
+    def __init__(self, spec, model, tag: str = ""):
+        self.spec, self.model, self.tag = spec, model, tag
 
     def pack(self, get, d: int) -> dict:
         ff = _up8(self.spec.ff)
@@ -56,21 +56,24 @@ class DenseGLU:
         if cfg is not None:  # a tuned SwiGLU shape, as slabs (bias and activation follow)
             nw, nwaves, S = cfg
             p = m._wgemm(2, h, W, S, nw, nwaves,
-                         out=m._parts("gu", S, M, N, m._slab_dtype(nwaves)))
+                         out=m._parts(self.tag + "gu", S, M, N, m._slab_dtype(nwaves)))
         else:
-            p = m._slabs("gate_up", h, W, is_decode)
+            p = m._slabs(self.tag + "gate_up", h, W, is_decode)
         return mops.glu(p, b, m.dtype, act)
 
     def forward(self, w: dict, h: torch.Tensor, is_decode: bool) -> dict:
         a = self._act(h, w, is_decode)
-        return {"m": self.model._slabs("down", a, w["down"], is_decode), "bias": w["down_b"]}
+        return {"m": self.model._slabs(self.tag + "down", a, w["down"], is_decode),
+                "bias": w["down_b"]}
 
 
 class Experts:
-    """Sparse mixture of small feed-forwards (grouped MFMA kernels, no host sync)."""
+    """Sparse mixture of small feed-forwards (grouped MFMA kernels, no host sync), with a
+    shared one for every token if asked."""
 
     def __init__(self, spec, model):
         self.spec, self.model = spec, model
+        self.shared = None if spec.shared is None else DenseGLU(spec.shared, model, "shared_")
 
     def pack(self, get, d: int) -> dict:
         s, m = self.spec, self.model
@@ -88,6 +91,10 @@ class Experts:
         w = {"router": F.pad(r, (0, d - r.shape[1])).contiguous(), "up": up, "down": down}
         if s.correction:
             w["correction"] = get("correction").float().contiguous()
+        if s.router_bias:
+            w["router_b"] = get("router.b").float().contiguous()
+        if self.shared is not None:
+            w["shared"] = self.shared.pack(lambda n: get("shared." + n), d)
         return w
 
     def forward(self, w: dict, h: torch.Tensor, is_decode: bool) -> dict:
@@ -95,6 +102,8 @@ class Experts:
         out = {"m": parts, "slots": True}
         if self.spec.identity:
             out["identity"] = (ids, wts, h, self.spec.experts)
+        if self.shared is not None:
+            out["shared"] = self.shared.forward(w["shared"], h, is_decode)["m"]
         return out
 
 

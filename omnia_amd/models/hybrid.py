@@ -1,5 +1,5 @@
 """Layer-list models (``ModelConfig.layers``) on the engine's paged cache: Sivadra, Sekazen,
-Bisuzen.
+Bisuzen, Tarunex.
 
 Every layer is ``x += post(mixer(pre(x)))`` and, with a feed-forward,
 ``x += post(ff(pre(x)))`` around an fp32 residual stream; mixers
@@ -12,6 +12,10 @@ joins the two branches of a parallel mixer:
     norm_embed -> [ in GEMM -> mixer kernels -> o GEMM -> norm_residual
                     (-> feed-forward -> norm_residual) ] * layers -> head GEMM
                     (-> softcap)
+
+In a family with ``joined`` sublayers a layer is ``x += mixer(norm1(x)) + ff(norm2(x))``: one
+kernel behind both adds their outputs (a token's experts and the shared one among them),
+what a loop's pass enters with, and writes the next layer's two inputs.
 
 A layer may use another layer's tensors (its pages / state are its own; the later passes
 of a looped layer do), or attend to another layer's pages.  bf16 models keep what feeds a
@@ -62,6 +66,8 @@ def random_tensor(name: str, shape: tuple, cfg: ModelConfig, gen, device) -> tor
     leaf = leaf.replace("mix.left.", "mix.").replace("mix.right.", "mix.")
     if leaf.endswith("alpha"):
         return torch.full(shape, 0.5, device=device)
+    if leaf in ("mix.r1", "mix.r2"):
+        return torch.empty(shape, device=device).uniform_(0.05, 1.0, generator=gen)
     if leaf == "mix.sink" or (cfg.design.norm == "rms" and leaf.startswith("norm")):
         return torch.zeros(shape, device=device)  # norm weights stored around zero
     if leaf.startswith("norm") or name.startswith("final.") or leaf.endswith(".norm"):
@@ -109,6 +115,9 @@ class HybridModel(Projections):
         self.mixers = [MIXERS[l.mixer.kind](l.mixer, self) for l in cfg.layers]
         self.mlps = [None if l.mlp is None else MLPS[l.mlp.kind](l.mlp, self)
                      for l in cfg.layers]
+        if cfg.design.joined and any("o" in getattr(l.mixer, "bias", "") or
+                                     getattr(l.mlp, "bias", False) for l in cfg.layers):
+            raise ValueError(f"{cfg.name}: joined sublayers have no output biases")
         self.w = self._pack(weights if weights is not None else self._random())
         ops.dgemm_prepare(self.device)
 
@@ -156,6 +165,8 @@ class HybridModel(Projections):
             if design.norm == "tanh":
                 return mops.TanhNorm(float(raw(name + ".alpha")), scale * vec(raw(name)),
                                      scale * vec(raw(name + ".b")))
+            if design.norm == "rms_scalar":
+                return mops.RMSNorm(None, cfg.hidden_size, cfg.rms_eps, scale * float(raw(name)))
             return mops.RMSNorm(scale * vec(1.0 + raw(name).float()), cfg.hidden_size, cfg.rms_eps)
 
         def norms(p, k):
@@ -169,6 +180,8 @@ class HybridModel(Projections):
              "final_norm": norm("final.norm", cfg.logit_scale),
              "embed_norm": norm("embed.norm") if design.embed_norm else None}
         w["head"] = w["embed"] if design.tied else cols(raw("head"))
+        if design.pass_inputs and any(l.starts is not None for l in cfg.layers):
+            w["step"] = [vec(t) for t in raw("loop.step")]
         for i, l in enumerate(cfg.layers):
             own = i if l.weights_of is None else l.weights_of
             if own not in seen:
@@ -203,10 +216,54 @@ class HybridModel(Projections):
         m = self._proj(tag, x, w, is_decode)
         return m.t if isinstance(m, Parts) else m
 
+    def temperature(self, t) -> torch.Tensor:
+        if t not in self._tables:
+            self._tables[t] = mops.temperature_table(t, self.cfg.max_position, self.device)
+        return self._tables[t]
+
+    def _pass_input(self, fb, i: int) -> mops.PassInput | None:
+        """What joins the residual before layer ``i``: at the first layer the embedding, and
+        where a loop's pass starts its inputs."""
+        t = None
+        if self.cfg.design.pass_inputs and i < len(self.cfg.layers):
+            t = self.cfg.layers[i].starts
+        if i and t is None:
+            return None
+        return mops.PassInput(fb.input_ids, self.w["embed"], self.cfg.vocab_size,
+                              self.cfg.embed_scale if i == 0 or t else 0.0,
+                              None if t is None else self.w["step"][t], fb.ids_src, fb.tok_slots)
+
+    def _run_joined(self, fb, kv: HybridCache, trace: list | None) -> torch.Tensor:
+        ws, dt, dec = self.w["layers"], self.dtype, fb.is_decode
+        x = torch.empty(fb.input_ids.numel(), self.d, dtype=torch.float32, device=self.device)
+
+        def norms(i):  # of layer i's sublayers, or the final one
+            if i == len(ws):
+                return [self.w["final_norm"]]
+            return [ws[i]["pre1"]] + ([ws[i]["pre2"]] if self.mlps[i] else [])
+
+        h = mops.joined_residual(x, [], norms(0), dt, self._pass_input(fb, 0), fresh=True)
+        for i, (w, mixer, mlp) in enumerate(zip(ws, self.mixers, self.mlps)):
+            parts = [(mixer.sublayer(w["mix"], h[0], fb, kv.layers[i])["m"], False)]
+            if mlp:
+                f = mlp.forward(w["mlp"], h[1], dec)
+                parts.append((f["m"], f.get("slots", False)))
+                if "shared" in f:
+                    parts.append((f["shared"], False))
+            enter = self._pass_input(fb, i + 1)
+            if trace is not None:
+                mops.joined_residual(x, parts, norms(i + 1), dt)
+                trace.append(x[:, :self.cfg.hidden_size].clone())
+                parts = []
+            h = mops.joined_residual(x, parts, norms(i + 1), dt, enter)
+        return h[0]
+
     def run_layers(self, fb, kv: HybridCache, trace: list | None = None) -> torch.Tensor:
         """Final-normed rows of the step; ``trace`` receives the residual stream after
         every layer (tests)."""
         self._min_rows = self.PGEMM_MIXED_MIN_ROWS if fb.num_decode else self.PGEMM_MIN_ROWS
+        if self.cfg.design.joined:
+            return self._run_joined(fb, kv, trace)
         ws, dt, dec = self.w["layers"], self.dtype, fb.is_decode
         x, h = mops.norm_embed(fb.input_ids, self.w["embed"], self.cfg.vocab_size,
                                self.w["embed_norm"], ws[0]["pre1"], fb.ids_src, fb.tok_slots)

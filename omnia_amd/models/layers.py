@@ -98,6 +98,17 @@ class RotarySpec:
 
 
 @dataclass(frozen=True)
+class TemperatureSpec:
+    """Queries grow with their position p: times ``1 + coef ln(floor((p + 1) / every) + 1)``."""
+
+    coef: float
+    every: float
+
+    def factor(self, p: int) -> float:
+        return 1.0 + self.coef * math.log(math.floor((p + 1) / self.every) + 1.0)
+
+
+@dataclass(frozen=True)
 class LatentAttentionSpec:
     """Attention over a low-rank latent: per token the cache holds one normed
     latent of ``kv_rank`` numbers (every head's unrotated key and value are
@@ -233,11 +244,17 @@ class AttentionSpec:
 
     ``qk_norm``: per-head RMS norms of queries and keys, with a learned ``"weight"``,
     ``"unit"`` (none) or None.  ``rotary`` on the first ``rotary.dims`` dimensions, or
-    None.  ``bias``: on all four projections.  A query sees its last ``window`` positions
-    (0 = the whole past) and the sequence's first ``keep_first``, or, with ``chunk``, the
-    positions of its own chunk of that many up to itself.  ``sink``: a learned number per
-    head in the softmax denominator.  ``kv_from``: the layer whose cached keys and values
-    this one attends to instead of its own."""
+    None.  ``bias``: letters of the projections (q, k, v, o) that have one.  A query sees its
+    last ``window`` positions (0 = the whole past) and the sequence's first ``keep_first``,
+    or, with ``chunk``, the positions of its own chunk of that many up to itself.  ``sink``:
+    a number per head in the softmax denominator beside the scores, ``"learned"``, ``"zero"``
+    (one is added to the denominator) or None.  ``kv_from``: the layer whose cached keys and
+    values this one attends to instead of its own.
+
+    ``temperature`` scales queries by position.  Scores are capped, ``softcap tanh(s /
+    softcap)`` (0: not), then lose ``r1 ln(1 + r2 (i - j))`` with two learned numbers per
+    head (``distance_bias``).  ``gate``: a head's output times a sigmoid of the layer's
+    input."""
 
     heads: int
     kv_heads: int
@@ -246,12 +263,16 @@ class AttentionSpec:
     scale: float
     rotary: RotarySpec | None
     window: int = 0
-    sink: bool = True
+    sink: str | None = "learned"
     kv_from: int | None = None
     qk_norm: str | None = "weight"
-    bias: bool = False
+    bias: str = ""
     keep_first: int = 0
     chunk: int = 0
+    temperature: TemperatureSpec | None = None
+    softcap: float = 0.0
+    distance_bias: bool = False
+    gate: bool = False
 
     kind = "attention"
     stateful = False
@@ -268,7 +289,11 @@ class AttentionSpec:
 
     @property
     def in_cols(self) -> int:
-        """[q | k | v] of one projected row."""
+        """[q | k | v | gate] of one projected row."""
+        return self.qkv_cols + (self.heads if self.gate else 0)
+
+    @property
+    def qkv_cols(self) -> int:
         own = 0 if self.kv_from is not None else self.kv_heads * (self.dim_pad + self.v_pad)
         return self.heads * self.dim_pad + own
 
@@ -327,13 +352,15 @@ class ExpertsSpec:
 
     ``expert`` "clamped_glu": ``W_down(g sigmoid(alpha g) (u + 1))`` with ``g = min(W_gate
     h, limit)`` and ``u = clamp(W_up h, -limit, limit)``, a token's weight on its expert's
-    input; "gelu": ``W_down gelu(W_up h)`` (erf form), the weight on the output.
+    input; "glu": ``W_down(silu(W_gate h) * (W_up h))`` and "gelu": ``W_down gelu(W_up h)``
+    (erf form), the weight on the output.
 
-    Routing scores are ``sigmoid`` or ``softmax`` of fp32 logits, renormalised over the
-    chosen experts if asked.  ``correction``: a learned number per expert joins the score
-    for the choice alone.  The choice is limited to the ``keep`` best of ``groups`` equal
-    groups of neighbours (a group counts as its best choice score).  The last ``identity``
-    router outputs are experts that return their input."""
+    Routing scores are ``sigmoid`` or ``softmax`` of fp32 logits (``router_bias``: with a
+    learned number per expert in them), renormalised over the chosen experts if asked.
+    ``correction``: a learned number per expert joins the score for the choice alone.  The
+    choice is limited to the ``keep`` best of ``groups`` equal groups of neighbours (a group
+    counts as its best choice score).  The last ``identity`` router outputs are experts that
+    return their input.  ``shared``: a feed-forward that every token passes as well."""
 
     ff: int
     experts: int
@@ -347,6 +374,8 @@ class ExpertsSpec:
     groups: int = 1
     keep: int = 1
     identity: int = 0
+    router_bias: bool = False
+    shared: DenseMLPSpec | None = None
 
     kind = "moe"
 
@@ -357,7 +386,8 @@ class ExpertsSpec:
 
     @property
     def gated(self) -> bool:
-        return self.expert == "clamped_glu"
+        """An expert's first product has gate and up halves."""
+        return self.expert != "gelu"
 
     @property
     def ff_pad(self) -> int:  # whole k-tiles of the grouped GEMMs
@@ -370,6 +400,7 @@ class LayerSpec:
     mlp: object | None = None  # DenseMLPSpec | ExpertsSpec | None
     weights_of: int | None = None  # share layer j's tensors (own cache / state)
     index: int | None = None  # number in the checkpoint's tensor names (None: its place)
+    starts: int | None = None  # number of the loop's pass that starts with this layer
 
 
 @dataclass(frozen=True)
@@ -377,13 +408,17 @@ class DesignSpec:
     """What a layer-list family fixes around its layers, and which checkpoint entries
     its ``config.json`` may hold (the same entry name can mean different mixers)."""
 
-    norm: str  # "tanh": Dynamic Tanh; "rms": RMS with a weight stored around zero
+    norm: str  # "tanh": Dynamic Tanh; "rms": RMS with a weight stored around zero;
+    #            "rms_scalar": RMS with one number for all coordinates
     pre_norm: bool  # sublayers read the normed residual (else the residual itself)
     embed_norm: bool  # the residual starts at norm(embedding)
     tied: bool  # the embedding table is the output head
     mixers: dict
     mlps: dict
     post_norm: bool = True  # a sublayer's output is normed before it is added
+    joined: bool = False  # mixer and feed-forward read the same residual, each normed by
+    #                       its own norm, and their outputs are added together
+    pass_inputs: bool = False  # before a loop's pass t: + the embedding (t > 0), + step[t]
 
     def sublayer_norms(self, k: int) -> tuple[str | None, str | None]:
         """(pre, post) norm names of a layer's k-th sublayer (1 mixer, 2 feed-forward)."""
@@ -451,8 +486,24 @@ def _grouped(spec: AttentionSpec) -> AttentionSpec:
 def _chunked_attention(c: dict) -> AttentionSpec:
     return _grouped(AttentionSpec(
         heads=int(c["heads"]), kv_heads=int(c["kv_heads"]), dim=int(c["dim"]),
-        vdim=int(c["vdim"]), scale=float(c["scale"]), rotary=None, sink=False, qk_norm="unit",
+        vdim=int(c["vdim"]), scale=float(c["scale"]), rotary=None, sink=None, qk_norm="unit",
         chunk=int((c.get("mask") or {}).get("size") or 0)))
+
+
+def _biased_attention(c: dict) -> AttentionSpec:
+    t, cap = c.get("q_temp"), float(c.get("softcap") or 0.0)
+    if cap < 0.0 or (t and not float(t["every"]) > 0.0):
+        raise ValueError(f"attention: softcap {cap}, q_temp {t}")
+    return _grouped(AttentionSpec(
+        heads=int(c["heads"]), kv_heads=int(c["kv_heads"]), dim=int(c["dim"]),
+        vdim=int(c["vdim"]), scale=float(c["scale"]), rotary=None, sink="zero", qk_norm=None,
+        bias="qkv", softcap=cap, distance_bias=True, gate=True,
+        temperature=TemperatureSpec(float(t["coef"]), float(t["every"])) if t else None))
+
+
+def _paired_latent_attention(c: dict) -> LatentAttentionSpec:
+    spec = _latent_attention(c)
+    return replace(spec, rotary=replace(spec.rotary, interleaved=True))
 
 
 def _anchored_attention(c: dict) -> AttentionSpec:
@@ -463,7 +514,7 @@ def _anchored_attention(c: dict) -> AttentionSpec:
         vdim=int(c["vdim"]), scale=float(c["scale"]),
         rotary=replace(_rotary(rot), interleaved=True) if rot and int(rot["dims"]) else None,
         window=int(mask.get("size") or 0), keep_first=int(mask.get("keep_first") or 0),
-        sink=True, qk_norm=None, bias=True))
+        qk_norm=None, bias="qkvo"))
 
 
 def _lightning(c: dict) -> LightningSpec:
@@ -504,6 +555,14 @@ def _gelu_experts(c: dict) -> ExpertsSpec:
         identity=int(r.get("identity") or 0)))
 
 
+def _shared_experts(c: dict) -> ExpertsSpec:
+    e, r, s = c["expert"], c["router"], c.get("shared")
+    return _checked(ExpertsSpec(
+        ff=int(e["ff"]), experts=int(r["experts"]), top=int(r["top"]), score="softmax",
+        renorm=True, expert="glu", router_bias=True,
+        shared=DenseMLPSpec(int(s["ff"]), bias=False) if s else None))
+
+
 def _experts(c: dict) -> ExpertsSpec:
     e, r = c["expert"], c["router"]
     return _checked(ExpertsSpec(ff=int(e["ff"]), experts=int(r["experts"]), top=int(r["top"]),
@@ -519,6 +578,11 @@ DESIGNS = {
     "bisuzen": DesignSpec("tanh", pre_norm=True, post_norm=False, embed_norm=False, tied=False,
                           mixers={"attention": _chunked_attention, "parallel": _parallel},
                           mlps={"dense": _dense_gelu, "moe": _gelu_experts}),
+    "tarunex": DesignSpec("rms_scalar", pre_norm=True, post_norm=False, embed_norm=False,
+                          tied=False, joined=True, pass_inputs=True,
+                          mixers={"attention": _biased_attention,
+                                  "latent_attention": _paired_latent_attention},
+                          mlps={"moe": _shared_experts}),
 }
 
 
@@ -532,12 +596,23 @@ def _run_order(n: int, loop: dict | None) -> list[int]:
     return list(range(a)) + list(range(a, b)) * times + list(range(b, n))
 
 
+def _passes(n: int, loop: dict | None) -> dict[int, int]:
+    """Place in the run order -> number of the pass that starts there."""
+    if not loop:
+        return {}
+    a, b = int(loop["start"]), int(loop["stop"])
+    return {a + t * (b - a): t for t in range(int(loop["times"]))} if b > a else {}
+
+
 def looped(layers: tuple, start: int, stop: int, times: int) -> tuple[LayerSpec, ...]:
     """A preset's layers with a loop unrolled, as :func:`parse_layers` does."""
     out: list[LayerSpec] = []
-    for at, i in enumerate(_run_order(len(layers), dict(start=start, stop=stop, times=times))):
+    loop = dict(start=start, stop=stop, times=times)
+    starts = _passes(len(layers), loop)
+    for at, i in enumerate(_run_order(len(layers), loop)):
         again = at >= stop and start <= i < stop
-        out.append(replace(layers[i], weights_of=i if again else None, index=i))
+        out.append(replace(layers[i], weights_of=i if again else None, index=i,
+                           starts=starts.get(at)))
     return tuple(out)
 
 
@@ -574,6 +649,7 @@ def parse_layers(entries: list[dict], design: DesignSpec,
     first: dict = {}
     for at, i in enumerate(order):
         first.setdefault(i, at)
+    starts = _passes(len(entries), loop)
     out: list[LayerSpec] = []
     last: dict = {}  # latest pass of a checkpoint layer so far
     for at, i in enumerate(order):
@@ -584,7 +660,8 @@ def parse_layers(entries: list[dict], design: DesignSpec,
         owner = owners[i] if owners[i] is not None else i
         out.append(LayerSpec(
             mixer, None if e.get("mlp") is None else design.mlps[e["mlp"]["kind"]](e["mlp"]),
-            None if first[owner] == at else first[owner], i if loop else None))
+            None if first[owner] == at else first[owner], i if loop else None,
+            starts.get(at)))
         last[i] = at
     for i, l in enumerate(out):
         if l.weights_of is not None:
@@ -618,13 +695,16 @@ def _mixer_shapes(m, d: int) -> dict[str, tuple]:
         out = {"q": (m.heads * m.dim, d), "o": (d, m.heads * m.vdim)}
         if m.kv_from is None:
             out.update({"k": (m.kv_heads * m.dim, d), "v": (m.kv_heads * m.vdim, d)})
-        if m.bias:
-            out.update({n + ".b": (w[0],) for n, w in list(out.items())})
+        out.update({n + ".b": (w[0],) for n, w in list(out.items()) if n in m.bias})
+        if m.distance_bias:
+            out.update({"r1": (m.heads,), "r2": (m.heads,)})
+        if m.gate:
+            out["g"] = (m.heads, d)
         if m.qk_norm == "weight":
             out["q.norm"] = (m.dim,)
             if m.kv_from is None:
                 out["k.norm"] = (m.dim,)
-        if m.sink:
+        if m.sink == "learned":
             out["sink"] = (m.heads,)
         return out
     if m.kind == "lightning":
@@ -647,12 +727,16 @@ def _mixer_shapes(m, d: int) -> dict[str, tuple]:
 def _mlp_shapes(m, d: int) -> dict[str, tuple]:
     if m.kind == "moe":
         out = {"router": (m.outputs, d)}
+        if m.router_bias:
+            out["router.b"] = (m.outputs,)
         if m.correction:
             out["correction"] = (m.outputs,)
         for e in range(m.experts):
             if m.gated:
                 out[f"e{e}.gate"] = (m.ff, d)
             out.update({f"e{e}.up": (m.ff, d), f"e{e}.down": (d, m.ff)})
+        if m.shared is not None:
+            out.update({"shared." + n: s for n, s in _mlp_shapes(m.shared, d).items()})
         return out
     out = {"gate": (m.ff, d), "up": (m.ff, d), "down": (d, m.ff)}
     if m.bias:
@@ -669,9 +753,13 @@ def tensor_shapes(layers, d: int, vocab: int,
             return {}
         if design.norm == "tanh":
             return {name: (d,), name + ".b": (d,), name + ".alpha": ()}
-        return {name: (d,)}
+        return {name: () if design.norm == "rms_scalar" else (d,)}
 
     out = {"embed": (vocab, d)}
+    if design.pass_inputs:
+        times = sum(l.starts is not None for l in layers)
+        if times:
+            out["loop.step"] = (times, d)
     if design.embed_norm:
         out.update(norm("embed.norm"))
     for i, l in enumerate(layers):

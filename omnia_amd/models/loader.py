@@ -203,13 +203,14 @@ def _layer_list_config(c: dict, name: str) -> ModelConfig:
     arch = c["architecture"].lower()
     layers = parse_layers(c["layers"], DESIGNS[arch], c.get("loop"))
     vocab = int(c["vocab"])
-    scale = c.get("logit_scale")
+    scale, embed = c.get("logit_scale"), (c.get("embedding") or {}).get("scale")
     return ModelConfig(
         name=name, arch=arch, vocab_size=vocab,
         hidden_size=int(c["width"]), num_layers=len(layers), layers=layers,
         intermediate_size=max([l.mlp.ff for l in layers if l.mlp is not None], default=0),
         rms_eps=float(c["norm"]["eps"]), logit_softcap=float(c.get("logit_softcap") or 0.0),
         logit_scale=1.0 if scale is None else float(scale),
+        embed_scale=1.0 if embed is None else float(embed),
         tie_embeddings=DESIGNS[arch].tied,
         max_position=int(c.get("max_position", 131072)),
         bos_token_id=int(c.get("bos", min(256, vocab - 1))),

@@ -89,9 +89,12 @@ class LatentAttention(Mixer):
         H, D, R, C = s.heads, s.dim, s.rot_dim, s.kv_rank
         dkv = get("dkv")
         uq = get("uq").view(H, D + R, s.q_rank)
+        kr, qr = dkv[C:], uq[:, D:]
+        if s.rotary.interleaved:  # neighbours to halves: scores do not see a common order
+            kr, qr = (torch.cat([t[..., 0::2, :], t[..., 1::2, :]], -2) for t in (kr, qr))
         wq = uq.new_zeros(H, s.qk_pad, s.q_rank_pad)
         wq[:, :D, :s.q_rank] = uq[:, :D]
-        wq[:, s.dim_pad:s.dim_pad + R, :s.q_rank] = uq[:, D:]
+        wq[:, s.dim_pad:s.dim_pad + R, :s.q_rank] = qr
         uk = F.pad(get("uk").view(H, D, C), (0, s.latent_pad - C, 0, s.dim_pad - D))
         # absorbed form: whole 32-wide k-steps (the columns past dim_pad meet the rotated
         # part of the query row with zero weight)
@@ -99,7 +102,7 @@ class LatentAttention(Mixer):
         uv = F.pad(get("uv").view(H, s.vdim, C), (0, s.latent_pad - C, 0, s.v_pad - s.vdim))
         return {
             "in": _rows_to([_pad2(get("dq"), s.q_rank_pad, d), _pad2(dkv[:C], s.latent_pad, d),
-                            _pad2(dkv[C:], s.rot_pad, d), _pad2(get("g"), H, d)], d),
+                            _pad2(kr, s.rot_pad, d), _pad2(get("g"), H, d)], d),
             "q_norm": get("dq.norm").float(), "kv_norm": get("dkv.norm").float(),
             "uq": wq.view(H * s.qk_pad, s.q_rank_pad),
             "uk_absorb": ua.transpose(1, 2).contiguous(),  # [H, latent, dim]
@@ -250,8 +253,9 @@ class Lightning(Mixer):
 
 
 class GroupedQueryAttention(Mixer):
-    """Masked attention, with sinks or none, over pages of keys and values -- its own, or
-    (spec ``kv_from``) those of an earlier layer, whose cache entry it is handed."""
+    """Masked attention over pages of keys and values -- its own, or (spec ``kv_from``) those
+    of an earlier layer, whose cache entry it is handed; with or without sinks, query
+    temperature, capped scores, distance bias and gated heads."""
 
     cache_tensors = 2, 0
     slab_input = slab_decode = True
@@ -259,6 +263,7 @@ class GroupedQueryAttention(Mixer):
     def __init__(self, spec, model):
         super().__init__(spec, model)
         self.table = None if spec.rotary is None else model.rotary(spec.rotary)
+        self.temp = None if spec.temperature is None else model.temperature(spec.temperature)
         self.mfma = (model.device.type == "cuda" and model.dtype == torch.bfloat16
                      and spec.dim_pad in GQA_WIDTHS and spec.v_pad in GQA_WIDTHS)
 
@@ -275,24 +280,32 @@ class GroupedQueryAttention(Mixer):
             return F.pad(t.float(), (0, s.dim_pad - s.dim)).contiguous()
 
         def bias(n, count, dim, pad):
+            if n not in s.bias:
+                return torch.zeros(count * pad, device=self.model.device)
             return F.pad(get(n + ".b").float().view(count, dim), (0, pad - dim)).reshape(-1)
 
         rows = [heads("q", s.heads, s.dim, s.dim_pad)]
         if own:
             rows += [heads("k", s.kv_heads, s.dim, s.dim_pad),
                      heads("v", s.kv_heads, s.vdim, s.v_pad)]
+        if s.gate:
+            rows.append(_pad2(get("g"), s.heads, d))
         w = {"in": _rows_to(rows, d), "o": _head_cols(get("o"), s.heads, s.v_pad, d),
-             "sink": get("sink").float().contiguous() if s.sink else None}
+             "sink": get("sink").float().contiguous() if s.sink == "learned" else
+             torch.zeros(s.heads, device=self.model.device) if s.sink else None}
+        if s.distance_bias:
+            w["dist"] = torch.stack([get("r1").float(), get("r2").float()]).contiguous()
         if s.qk_norm:
             w["q_norm"] = norm("q.norm")
             if own:
                 w["k_norm"] = norm("k.norm")
-        if s.bias:
+        if set(s.bias) & set("qkv"):
             bs = [bias("q", s.heads, s.dim, s.dim_pad)]
             if own:
                 bs += [bias("k", s.kv_heads, s.dim, s.dim_pad),
                        bias("v", s.kv_heads, s.vdim, s.v_pad)]
             w["in_b"] = torch.cat(bs).contiguous()
+        if "o" in s.bias:
             ob = get("o.b").float()
             w["o_b"] = F.pad(ob, (0, d - ob.numel())).contiguous()
         return w
@@ -314,34 +327,36 @@ class GroupedQueryAttention(Mixer):
         return max(1, -(-keys // self.MAX_PART),
                    min(-(-self.DECODE_GROUPS // groups), -(-keys // self.MIN_PART)))
 
-    def _decode(self, w, q, pages, bt, positions, out):
-        page = pages[0].shape[2]
+    def _decode(self, w, q, pages, bt, positions, out, gate=None):
+        page, more = pages[0].shape[2], dict(out=out, dist=w.get("dist"), gate=gate)
         if self.mfma and page & (page - 1) == 0:
             return mops.gqa_decode(q, pages, bt, positions, self.spec, w["sink"],
-                                   self.splits(q.shape[0], bt.shape[1] * page), out)
-        return mops.gqa_attend(q, pages, bt, None, positions, self.spec, w["sink"], out)
+                                   self.splits(q.shape[0], bt.shape[1] * page), **more)
+        return mops.gqa_attend(q, pages, bt, None, positions, self.spec, w["sink"], **more)
 
-    def _prefill(self, w, q, pages, fb, positions, out):
-        page = pages[0].shape[2]
+    def _prefill(self, w, q, pages, fb, positions, out, gate=None):
+        page, more = pages[0].shape[2], dict(out=out, dist=w.get("dist"), gate=gate)
         if self.mfma and page & (page - 1) == 0:
-            return mops.gqa_prefill(q, pages, fb, self.spec, w["sink"], out)
+            return mops.gqa_prefill(q, pages, fb, self.spec, w["sink"], **more)
         return mops.gqa_attend(q, pages, fb.block_tables, fb.q_start_loc, positions, self.spec,
-                               w["sink"], out)
+                               w["sink"], **more)
 
     def mix(self, w: dict, x: torch.Tensor, fb, cache) -> torch.Tensor:
         s, m = self.spec, self.model
         pages, _ = cache
-        q = mops.gqa_prep(x, w, s, pages if s.kv_from is None else None, fb.positions, fb.slots,
-                          self.table, m.dtype, m.cfg.rms_eps)
-        if fb.is_decode:
-            return self._decode(w, q, pages, fb.block_tables, fb.positions, None)
         nd, T = fb.num_decode, fb.positions.numel()
+        gate = torch.empty(T, s.heads, dtype=torch.float32, device=x.device) if s.gate else None
+        q = mops.gqa_prep(x, w, s, pages if s.kv_from is None else None, fb.positions, fb.slots,
+                          self.table, m.dtype, m.cfg.rms_eps, self.temp, gate)
+        if fb.is_decode:
+            return self._decode(w, q, pages, fb.block_tables, fb.positions, None, gate)
         if not nd:
-            return self._prefill(w, q, pages, fb, fb.positions, None)
+            return self._prefill(w, q, pages, fb, fb.positions, None, gate)
         out = torch.empty(T, s.heads * s.v_pad, dtype=m.dtype, device=x.device)
-        self._decode(w, q[:nd], pages, fb.dec_block_tables, fb.positions[:nd], out[:nd])
+        gd, gp = (None, None) if gate is None else (gate[:nd], gate[nd:])
+        self._decode(w, q[:nd], pages, fb.dec_block_tables, fb.positions[:nd], out[:nd], gd)
         if T > nd:
-            self._prefill(w, q[nd:], pages, fb, fb.positions[nd:], out[nd:])
+            self._prefill(w, q[nd:], pages, fb, fb.positions[nd:], out[nd:], gp)
         return out
 
 

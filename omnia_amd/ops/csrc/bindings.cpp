@@ -9,6 +9,8 @@
 
 // the layout of mask.h's struct: (window, kept first positions, chunk)
 struct Mask { int window, keep, chunk; };
+// of score.h's: (scale, cap, r1, r2)
+struct Score { float scale, cap; const float *r1, *r2; };
 
 extern "C" {
 int omnia_pgemm(int epi, void* out, const void* X, const void* W, int M, int N, int K, int ldo,
@@ -86,7 +88,7 @@ int omnia_moe_align(int* sorted, int* blk_expert, int* n_blocks, const int* ids,
                     int e_lo, int e_hi, int max_blocks, int bm, hipStream_t s);
 int omnia_moe_route(int* ids, float* wts, const void* x, const void* router, int f32, int n_tok,
                     int d, int E, int k, int sigmoid, int renorm, const float* corr, int groups,
-                    int keep, hipStream_t s);
+                    int keep, const float* bias, hipStream_t s);
 int omnia_moe_gemm(int mode, void* out, const void* A, const void* W, int f32, const int* sorted,
                    const int* blk_expert, const int* n_blocks, const float* route_w, int K, int N,
                    int topk, int n_assign, int e_lo, int max_blocks, float alpha, float limit,
@@ -183,20 +185,29 @@ int omnia_gqa_prep(void* q, void* kc, void* vc, int f32, const void* x, int ptyp
                    int64_t slab, int64_t ldx, const float* wq, const float* wk,
                    const float* bias, const int* positions, const int64_t* slots,
                    const float* cos_sin, int pairs, int T, int H, int G, int D, int Dp, int Vp,
-                   int R, int page, float eps, hipStream_t s);
+                   int R, int page, float eps, const float* temp, float* gate, hipStream_t s);
 int omnia_gqa_attend(void* out, int f32, const void* q, const void* kc, const void* vc,
                      const int* block_tables, int bt_stride, const int* q_start, int nseq,
                      const int* positions, int T, int page, int H, int G, int Dp, int Vp,
-                     Mask mask, float scale, const float* sinks, hipStream_t s);
+                     Mask mask, Score score, const float* sinks, const float* gate,
+                     hipStream_t s);
 int omnia_gqa_decode(void* out, float* part_o, float* part_ml, const void* q, const void* kc,
                      const void* vc, const int* block_tables, int bt_stride, const int* positions,
-                     int T, int page, int H, int G, int Dp, int Vp, Mask mask, float scale,
-                     const float* sinks, int splits, int max_ctx, hipStream_t s);
+                     int T, int page, int H, int G, int Dp, int Vp, Mask mask, Score score,
+                     const float* sinks, const float* gate, int splits, int max_ctx,
+                     hipStream_t s);
 int omnia_gqa_prefill(void* out, const void* q, const void* kc, const void* vc,
                       const int* block_tables, int bt_stride, const int* q_start,
                       const int* seq_lens, const int* tile_seq, const int* tile_q0, int n_tiles,
-                      int page, int H, int G, int Dp, int Vp, Mask mask, float scale,
-                      const float* sinks, hipStream_t s);
+                      int page, int H, int G, int Dp, int Vp, Mask mask, Score score,
+                      const float* sinks, const float* gate, hipStream_t s);
+int omnia_joined_residual(void* h1, void* h2, int f32, float* x, int fresh, int rows, int d,
+                          const void* am, int at, int aS, int64_t arow, int64_t apart,
+                          const void* bm, int bS, int64_t brow, int64_t bpart, const void* cm,
+                          int ct, int cS, int64_t crow, int64_t cpart, const int* ids,
+                          const void* table, int vocab, float scale, const float* step,
+                          const int64_t* src, const int* tok_slots, const float* w1, float g1,
+                          const float* w2, float g2, float inv_n, float eps, hipStream_t s);
 int omnia_latent_prep(void* cq, void* cache, const void* x, int f32, int64_t ldx, const float* wq,
                       const float* wc, const int* positions, const int64_t* slots,
                       const float* cos_sin, int T, int Q, int Qp, int C, int Cp, int R, int Lp,
@@ -672,7 +683,7 @@ void pgemm_moe(int64_t mode, at::Tensor out, at::Tensor A, at::Tensor W, at::Ten
 // router: fp32 logits, sigmoid / softmax scores; x [T, d] and router [E, d] bf16 or fp32
 void moe_route(at::Tensor ids, at::Tensor wts, at::Tensor x, at::Tensor router, int64_t k,
                bool sigmoid, bool renorm, c10::optional<at::Tensor> corr, int64_t groups,
-               int64_t keep) {
+               int64_t keep, c10::optional<at::Tensor> bias) {
   CHECK_GPU(x); CHECK_I32(ids);
   const bool f32 = x.scalar_type() == at::kFloat;
   TORCH_CHECK((f32 || x.scalar_type() == at::kBFloat16) && router.scalar_type() == x.scalar_type(),
@@ -687,9 +698,13 @@ void moe_route(at::Tensor ids, at::Tensor wts, at::Tensor x, at::Tensor router, 
   if (corr.has_value())
     TORCH_CHECK(corr->is_cuda() && corr->scalar_type() == at::kFloat && corr->is_contiguous() &&
                 corr->numel() == E, "correction fp32 [E]");
+  if (bias.has_value())
+    TORCH_CHECK(bias->is_cuda() && bias->scalar_type() == at::kFloat && bias->is_contiguous() &&
+                bias->numel() == E, "bias fp32 [E]");
   CHECK_RC(omnia_moe_route(ids.data_ptr<int>(), wts.data_ptr<float>(), x.data_ptr(),
                            router.data_ptr(), f32, T, x.size(1), E, k, sigmoid, renorm,
-                           opt_ptr<float>(corr), groups, keep, cur_stream()), "moe_route");
+                           opt_ptr<float>(corr), groups, keep, opt_ptr<float>(bias),
+                           cur_stream()), "moe_route");
 }
 
 // modes in moe.hip; A, W and out all bf16 or all fp32
@@ -1362,6 +1377,69 @@ void branch_residual(at::Tensor h, at::Tensor x, at::Tensor a, OptT abias, at::T
            "branch_residual");
 }
 
+// x (+)= parts + scale * table[token] + step; h1 / h2 = rms(x) g w.  Parts: [M, d], slabs
+// [S, M, d], or (slots) [M, S, d]; table null: no embedding
+void joined_residual(at::Tensor h1, OptT h2, at::Tensor x, bool fresh, OptT m0, bool slots0,
+                     OptT m1, bool slots1, OptT m2, bool slots2, OptT ids, OptT table,
+                     int64_t vocab, double scale, OptT step, OptT src, OptT tok_slots, OptT w1,
+                     double g1, OptT w2, double g2, double inv_n, double eps) {
+  const int f32 = is_f32(h1, "h1");
+  TORCH_CHECK(x.dim() == 2 && x.size(0) == h1.size(0) && x.size(1) == h1.size(1), "x [M, d]");
+  const int64_t M = x.size(0), d = x.size(1);
+  like(h1, h1, M * d, "h1");
+  const bool two = h2.has_value() && h2->defined();
+  if (two) like(*h2, h1, M * d, "h2");
+  // kernel slots a, b, c: b takes a part stored in the model's type, expert slots first
+  const int own = f32 ? 1 : 0;
+  const OptT* ms[3] = {&m0, &m1, &m2};
+  const bool sl[3] = {slots0, slots1, slots2};
+  ResidParts p[3];
+  int n = 0, at_b = -1;
+  const void* ptr[3];
+  for (int i = 0; i < 3; ++i) {
+    if (!ms[i]->has_value() || !(*ms[i])->defined()) continue;
+    p[n] = resid_parts(**ms[i], sl[i]);
+    TORCH_CHECK(p[n].M == M && p[n].d == d, "part [M, d]");
+    ptr[n] = (*ms[i])->data_ptr();
+    if (p[n].type == own && (at_b < 0 || sl[i])) at_b = n;
+    ++n;
+  }
+  TORCH_CHECK(n < 3 || at_b >= 0, "one of three parts is stored in the model's type");
+  const ResidParts none{own, 0, M, d, 0, 0};
+  ResidParts k[3] = {none, none, none};
+  const void* kp[3] = {nullptr, nullptr, nullptr};
+  for (int i = 0, at = 0; i < n; ++i) {
+    const int to = i == at_b ? 1 : at;
+    if (i != at_b) at += 2;
+    k[to] = p[i];
+    kp[to] = ptr[i];
+  }
+  const void* tp = nullptr;
+  const int* idp = nullptr;
+  const int64_t* sp = nullptr;
+  if (table.has_value() && table->defined() && scale != 0.0) {
+    TORCH_CHECK(table->is_cuda() && table->dim() == 2 && table->is_contiguous() &&
+                table->scalar_type() == h1.scalar_type() && table->size(0) >= vocab &&
+                table->size(1) == d && ids.has_value(), "table [V, d] with ids");
+    tp = table->data_ptr();
+    idp = veci(*ids, M, "ids");
+    if (src.has_value() && src->defined()) {
+      TORCH_CHECK(src->is_cuda() && src->scalar_type() == at::kLong && src->is_contiguous() &&
+                  src->numel() == M && tok_slots.has_value(), "src int64 [M] with tok_slots");
+      CHECK_I32(*tok_slots);
+      sp = src->data_ptr<int64_t>();
+    }
+  }
+  CHECK_RC(omnia_joined_residual(
+               h1.data_ptr(), two ? h2->data_ptr() : nullptr, f32, outf(x, M * d, "x"), fresh, M,
+               d, kp[0], k[0].type, k[0].S, k[0].row, k[0].part, kp[1], k[1].S, k[1].row,
+               k[1].part, kp[2], k[2].type, k[2].S, k[2].row, k[2].part, idp, tp, vocab,
+               (float)scale, opt_vecf(step, d, "step"), sp, opt_ptr<int>(tok_slots),
+               opt_vecf(w1, d, "w1"), (float)g1, opt_vecf(w2, d, "w2"), (float)g2, (float)inv_n,
+               (float)eps, cur_stream()),
+           "joined_residual");
+}
+
 // act(g + bg) * (u + bu): silu, or the tanh form of gelu
 void glu(at::Tensor out, at::Tensor m, OptT bias, bool gelu) {
   const int f32 = is_f32(out, "out");
@@ -1702,10 +1780,11 @@ void check_kv(const at::Tensor& k, const at::Tensor& v, const at::Tensor& ref) {
 }
 
 // x: [T, (H*Dp | G*Dp | G*Vp) + padding] or its slabs; k / v pages absent: q only
-// wq null: no norms; cos_sin null: no rotation; pairs: neighbours turn together
+// wq null: no norms; cos_sin null: no rotation; pairs: neighbours turn together; temp
+// [positions] or null; gate [T, H] or null: H more columns behind v
 void gqa_prep(at::Tensor q, OptT k, OptT v, at::Tensor x, OptT wq, OptT wk, OptT bias,
               at::Tensor positions, at::Tensor slots, OptT cos_sin, bool pairs, int64_t H,
-              int64_t D, int64_t Dp, double eps) {
+              int64_t D, int64_t Dp, double eps, OptT temp, OptT gate) {
   const int f32 = is_f32(q, "q");
   const Proj p = proj(x, true);
   const bool rot = cos_sin.has_value() && cos_sin->defined();
@@ -1721,7 +1800,9 @@ void gqa_prep(at::Tensor q, OptT k, OptT v, at::Tensor x, OptT wq, OptT wk, OptT
     Vp = v->size(3);
     TORCH_CHECK(k->size(3) == Dp, "k page width");
   }
-  TORCH_CHECK(p.M == T && p.N >= H * Dp + G * (Dp + Vp), "projection row width");
+  float* gp = nullptr;
+  if (gate.has_value() && gate->defined()) gp = outf(*gate, T * H, "gate");
+  TORCH_CHECK(p.M == T && p.N >= H * Dp + G * (Dp + Vp) + (gp ? H : 0), "projection row width");
   like(q, q, T * H * Dp, "q");
   TORCH_CHECK(slots.is_cuda() && slots.scalar_type() == at::kLong && slots.is_contiguous() &&
               slots.numel() == T, "slots int64 [T]");
@@ -1731,7 +1812,10 @@ void gqa_prep(at::Tensor q, OptT k, OptT v, at::Tensor x, OptT wq, OptT wk, OptT
                           opt_vecf(bias, H * Dp + G * (Dp + Vp), "bias"),
                           veci(positions, T, "positions"), slots.data_ptr<int64_t>(),
                           rot ? rot_table(*cos_sin, R) : nullptr, pairs, T, H, G, D, Dp, Vp, R,
-                          page, (float)eps, cur_stream()), "gqa_prep");
+                          page, (float)eps,
+                          temp.has_value() && temp->defined() ?
+                              vecf(*temp, temp->numel(), "temp") : nullptr, gp, cur_stream()),
+           "gqa_prep");
 }
 
 struct KV { int64_t G, page, Dp, Vp; };
@@ -1751,9 +1835,16 @@ Mask mask_of(const MaskT& m) {
   return {(int)std::get<0>(m), (int)std::get<1>(m), (int)std::get<2>(m)};
 }
 
+// dist [2, H]: the heads' distance biases (r1 | r2), or null
+Score score_of(double scale, double cap, const OptT& dist, int64_t H) {
+  const float* r = opt_vecf(dist, 2 * H, "dist");
+  TORCH_CHECK(cap >= 0, "cap");
+  return {(float)scale, (float)cap, r, r ? r + H : nullptr};
+}
+
 void gqa_attend(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor block_tables,
                 OptT q_start, at::Tensor positions, int64_t H, MaskT mask, double scale,
-                OptT sinks) {
+                OptT sinks, double cap, OptT dist, OptT gate) {
   const int f32 = is_f32(q, "q");
   const int64_t T = positions.numel();
   const KV s = kv_sizes(out, q, k, v, T, H, sinks);
@@ -1763,13 +1854,15 @@ void gqa_attend(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::Te
                             tables(block_tables, nseq), block_tables.stride(0),
                             pre ? veci(*q_start, nseq + 1, "q_start") : nullptr, nseq,
                             veci(positions, T, "positions"), T, s.page, H, s.G, s.Dp, s.Vp,
-                            mask_of(mask), (float)scale, opt_ptr<float>(sinks), cur_stream()),
+                            mask_of(mask), score_of(scale, cap, dist, H),
+                            opt_ptr<float>(sinks), opt_vecf(gate, T * H, "gate"), cur_stream()),
            "gqa_attend");
 }
 
 void gqa_decode(at::Tensor out, OptT part_o, OptT part_ml, at::Tensor q, at::Tensor k,
                 at::Tensor v, at::Tensor block_tables, at::Tensor positions, int64_t H,
-                MaskT mask, double scale, OptT sinks, int64_t splits) {
+                MaskT mask, double scale, OptT sinks, int64_t splits, double cap, OptT dist,
+                OptT gate) {
   CHECK_GPU(q); CHECK_BF16(q);
   const int64_t T = positions.numel();
   const KV s = kv_sizes(out, q, k, v, T, H, sinks);
@@ -1783,14 +1876,16 @@ void gqa_decode(at::Tensor out, OptT part_o, OptT part_ml, at::Tensor q, at::Ten
   CHECK_RC(omnia_gqa_decode(out.data_ptr(), po, pm, q.data_ptr(), k.data_ptr(), v.data_ptr(),
                             tables(block_tables, T), block_tables.stride(0),
                             veci(positions, T, "positions"), T, s.page, H, s.G, s.Dp, s.Vp,
-                            mask_of(mask), (float)scale, opt_ptr<float>(sinks), splits, ctx,
+                            mask_of(mask), score_of(scale, cap, dist, H),
+                            opt_ptr<float>(sinks), opt_vecf(gate, T * H, "gate"), splits, ctx,
                             cur_stream()),
            "gqa_decode");
 }
 
 void gqa_prefill(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor block_tables,
                  at::Tensor q_start, at::Tensor seq_lens, at::Tensor tile_seq, at::Tensor tile_q0,
-                 int64_t H, MaskT mask, double scale, OptT sinks) {
+                 int64_t H, MaskT mask, double scale, OptT sinks, double cap, OptT dist,
+                 OptT gate) {
   CHECK_GPU(q); CHECK_BF16(q);
   TORCH_CHECK(q.dim() == 2, "q [T, H*Dp]");
   const KV s = kv_sizes(out, q, k, v, q.size(0), H, sinks);
@@ -1800,7 +1895,9 @@ void gqa_prefill(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::T
                              veci(q_start, nseq + 1, "q_start"), veci(seq_lens, nseq, "seq_lens"),
                              veci(tile_seq, nt, "tile_seq"), veci(tile_q0, nt, "tile_q0"), nt,
                              s.page, H, s.G, s.Dp, s.Vp, mask_of(mask),
-                             (float)scale, opt_ptr<float>(sinks), cur_stream()), "gqa_prefill");
+                             score_of(scale, cap, dist, H), opt_ptr<float>(sinks),
+                             opt_vecf(gate, q.size(0) * H, "gate"), cur_stream()),
+           "gqa_prefill");
 }
 
 }  // namespace
@@ -1818,6 +1915,7 @@ PYBIND11_MODULE(_omnia_kernels, m) {
   m.def("gqa_prefill", &gqa_prefill);
   m.def("tanh_norm_residual", &tanh_norm_residual);
   m.def("branch_residual", &branch_residual);
+  m.def("joined_residual", &joined_residual);
   m.def("glu", &glu);
   m.def("lightning_step", &lightning_step);
   m.def("lightning_scan", &lightning_scan);
@@ -1865,7 +1963,7 @@ PYBIND11_MODULE(_omnia_kernels, m) {
         py::arg("limit") = 0.0);
   m.def("moe_route", &moe_route, py::arg("ids"), py::arg("wts"), py::arg("x"), py::arg("router"),
         py::arg("k"), py::arg("sigmoid"), py::arg("renorm"), py::arg("corr") = py::none(),
-        py::arg("groups") = 1, py::arg("keep") = 1);
+        py::arg("groups") = 1, py::arg("keep") = 1, py::arg("bias") = py::none());
   m.def("moe_align", &moe_align);
   m.def("moe_gemm", &moe_gemm, py::arg("mode"), py::arg("out"), py::arg("A"), py::arg("W"),
         py::arg("sorted"), py::arg("blk_expert"), py::arg("n_blocks"), py::arg("route_w"),

@@ -5,19 +5,23 @@
 //   k pages [num_pages][G][page][Dp], v pages [num_pages][G][page][Vp]
 //
 // Query head h reads key/value head h / (H / G).  A query sees the keys its Mask names (a
-// window with kept first keys, a chunk, or all; mask.h); the softmax denominator of head h
-// also holds exp(sink[h]) (sinks null: none).  Scores, softmax and norms are fp32.
+// window with kept first keys, a chunk, or all; mask.h); scores may be capped and lose a
+// distance bias (score.h); the softmax denominator of head h also holds exp(sink[h]) (sinks
+// null: none); a head's output may be multiplied by a gate [T][H].  Scores, softmax, norms
+// and gates are fp32.
 //
 //   gqa_prep     one fused projection row [q (H*Dp) | k (G*Dp) | v (G*Vp)] (or its split-K
 //                slabs) -> + bias, per-head RMS norm of q and k, rotary on the first R
-//                dimensions (halves or neighbours paired), q rows out, k / v rows into the
-//                pages; bias, norm and rotation each if asked.  G = 0: q only (a layer that
-//                attends to another layer's pages)
+//                dimensions (halves or neighbours paired), q rows out (times a factor of
+//                their position), k / v rows into the pages; bias, norm, rotation and factor
+//                each if asked.  G = 0: q only (a layer that attends to another layer's
+//                pages).  Gate columns behind v: their sigmoid, fp32
 //   gqa_attend   generic attention (any size, bf16 or fp32), decode and prefill
 //   gqa_decode   bf16 decode: Q K^T on MFMA, P V on the VALU, the visible keys cut into
 //                equal parts on the device, + gqa_merge
 //   gqa_prefill  bf16 prefill (gqa_prefill.hip)
 #include "mask.h"
+#include "score.h"
 
 using namespace omnia;
 
@@ -73,6 +77,8 @@ struct PrepArgs {
   const int* positions;
   const int64_t* slots;  // < 0: no write (padded row)
   const float* cos_sin;  // [positions][R] = (cos[R/2] | sin[R/2])
+  const float* temp;     // [positions] factors of the queries, or null
+  float* gate;           // [T][H], or null
   int64_t ldx, slab;
   int S, H, G, D, Dp, Vp, R, page, lg, pairs;  // pairs: neighbours turn together
   float eps;
@@ -91,6 +97,14 @@ __global__ __launch_bounds__(256) void prep_kernel(T* __restrict__ q, T* __restr
   const bool isq = hs < a.H, isv = hs >= a.H + a.G;
   const int width = isv ? a.Vp : a.Dp;
   const int col = isv ? (a.H + a.G) * a.Dp + (hs - a.H - a.G) * a.Vp : hs * a.Dp;
+  if (a.gate && blockIdx.y == gridDim.y - 1) {
+    const P* gr = x + (int64_t)t * a.ldx + (a.H + a.G) * a.Dp + a.G * a.Vp;
+    for (int i = tid; i < a.H; i += 256) {
+      float z = 0.f;
+      for (int s = 0; s < a.S; ++s) z += ldf(gr + s * a.slab + i);
+      a.gate[(int64_t)t * a.H + i] = 1.f / (1.f + expf(-z));
+    }
+  }
   const P* xr = x + (int64_t)t * a.ldx + col;
   const float4v zero = {0.f, 0.f, 0.f, 0.f};
   float4v v[NC][2];
@@ -121,6 +135,7 @@ __global__ __launch_bounds__(256) void prep_kernel(T* __restrict__ q, T* __restr
   }
   const int pos = a.positions[t], half = a.R >> 1, turned = isv ? 0 : a.R;
   const float* cs = a.cos_sin + (int64_t)pos * a.R;
+  const float factor = a.temp && isq ? a.temp[pos] : 1.f;
   float* row = rows + (tid >> a.lg << a.lg) * NC * 8;
   if (!isv && !a.wq) {
 #pragma unroll
@@ -203,6 +218,8 @@ __global__ __launch_bounds__(256) void prep_kernel(T* __restrict__ q, T* __restr
           }
       }
     }
+    v[i][0] *= factor;
+    v[i][1] *= factor;
     if constexpr (sizeof(T) == 4) {
       store4(dst + c, v[i][0]);
       store4(dst + c + 4, v[i][1]);
@@ -225,7 +242,8 @@ __global__ __launch_bounds__(256) void attend_kernel(
     T* __restrict__ out, const T* __restrict__ q, const T* __restrict__ kc,
     const T* __restrict__ vc, const int* __restrict__ block_tables, int bt_stride,
     const int* __restrict__ q_start, int nseq, const int* __restrict__ positions, int page, int H,
-    int G, int Dp, int Vp, Mask mask, float scale, const float* __restrict__ sinks) {
+    int G, int Dp, int Vp, Mask mask, Score score, const float* __restrict__ sinks,
+    const float* __restrict__ gate) {
   extern __shared__ float sm[];
   float* qs = sm;        // [Dp]
   float* acc = qs + Dp;  // [Vp]
@@ -249,10 +267,11 @@ __global__ __launch_bounds__(256) void attend_kernel(
     __syncthreads();
     float sc = -INFINITY;
     if (tid < n) {
-      const T* row = kc + at(k0 + tid) * Dp;
+      const int i0 = k0 + tid, key = i0 < kp ? i0 : lo + i0 - kp;
+      const T* row = kc + at(i0) * Dp;
       float a = 0.f;
       for (int i = 0; i < Dp; ++i) a += qs[i] * ldf(row + i);
-      sc = a * scale;
+      sc = score(a, h, pos - key);
     }
     const float mn = fmaxf(m, block_max(sc, scratch));
     const float e = tid < n ? expf(sc - mn) : 0.f;
@@ -267,7 +286,8 @@ __global__ __launch_bounds__(256) void attend_kernel(
       acc[c] = a;
     }
   }
-  for (int c = tid; c < Vp; c += 256) stf(out + ((int64_t)t * H + h) * Vp + c, acc[c] / l);
+  const float inv = (gate ? gate[(int64_t)t * H + h] : 1.f) / l;
+  for (int c = tid; c < Vp; c += 256) stf(out + ((int64_t)t * H + h) * Vp + c, acc[c] * inv);
 }
 
 // ----------------------------------------------------------------- gqa_decode
@@ -284,15 +304,16 @@ __device__ __forceinline__ int part_len(int n, int splits) {
 // the group's end recomputes the last one and is not written).
 //   1 scores   each wave takes groups of 16 keys: K rows as the MFMA A operand, Q^T
 //              (16 columns, GH real) as B; UG groups of loads in flight
-//   2 softmax  per head over the part, in LDS
+//   2 softmax  per head over the part, in LDS; caps and distance biases here, where every
+//              lane has a key
 //   3 P V      64 / LPR value rows a wave and step, U steps of loads in flight
 template <int KK, int LPR, int GH, int NW>
 __global__ __launch_bounds__(64 * NW) void decode_kernel(
     bf16_t* __restrict__ out, float* __restrict__ part_o, float* __restrict__ part_ml,
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
     const int* __restrict__ block_tables, int bt_stride, const int* __restrict__ positions, int H,
-    int G, int nch, int page_lg, int Vp, Mask mask, float scale_log2,
-    const float* __restrict__ sinks, int cap) {
+    int G, int nch, int page_lg, int Vp, Mask mask, Score2 score,
+    const float* __restrict__ sinks, const float* __restrict__ gate, int cap) {
   constexpr int Dp = 32 * KK, UG = KK > 4 ? 2 : 4, U = 4, TG = 64 / LPR;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   float* stat = reinterpret_cast<float*>(smem);  // [2 * GH], padded to 16
@@ -354,7 +375,7 @@ __global__ __launch_bounds__(64 * NW) void decode_kernel(
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int i = grp * 16 + 4 * (lane >> 4) + r;
-          if (i < n) scores[c * cap + i] = acc[r] * scale_log2;
+          if (i < n) scores[c * cap + i] = acc[r] * score.mul;
         }
       }
     }
@@ -376,7 +397,20 @@ __global__ __launch_bounds__(64 * NW) void decode_kernel(
   __syncthreads();
   for (int c = w; c < GH; c += NW) {
     float m = -INFINITY;
-    for (int i = lane; i < n; i += 64) m = fmaxf(m, scores[c * cap + i]);
+    if (score.cap > 0.f || score.r1) {
+      const int h = h0 + min(c, hn - 1);
+      const float r1 = score.r1 ? score.r1[h] : 0.f, r2 = score.r1 ? score.r2[h] : 0.f;
+      for (int i = lane; i < n; i += 64) {
+        float s = scores[c * cap + i];
+        if (score.cap > 0.f) s = score.squash(s);
+        const int key = i < nk ? p0 + i : w0 + i - nk;
+        s -= r1 * log2_(__builtin_fmaf(r2, (float)(pos - key), 1.f));
+        scores[c * cap + i] = s;
+        m = fmaxf(m, s);
+      }
+    } else {
+      for (int i = lane; i < n; i += 64) m = fmaxf(m, scores[c * cap + i]);
+    }
     m = wave_max(m);
     float s = 0.f;
     for (int i = lane; i < n; i += 64) {
@@ -444,6 +478,7 @@ __global__ __launch_bounds__(64 * NW) void decode_kernel(
       } else {
         v = v / s;
       }
+      if (gate) v *= gate[(int64_t)b * H + h];
       out[((int64_t)b * H + h) * Vp + d] = f2bf(v);
     } else {
       const int64_t slot = ((int64_t)b * H + h) * splits + part;
@@ -462,7 +497,8 @@ __global__ __launch_bounds__(128) void merge_kernel(bf16_t* __restrict__ out,
                                                     const float* __restrict__ part_ml,
                                                     const int* __restrict__ positions, int H,
                                                     int Vp, Mask mask, int splits,
-                                                    const float* __restrict__ sinks) {
+                                                    const float* __restrict__ sinks,
+                                                    const float* __restrict__ gate) {
   extern __shared__ float wt[];  // [splits]
   __shared__ float scratch[2];
   const int bh = blockIdx.x, b = bh / H, h = bh - b * H;
@@ -483,7 +519,7 @@ __global__ __launch_bounds__(128) void merge_kernel(bf16_t* __restrict__ out,
     tot += wt[p] * ml[2 * p + 1];
   }
   tot = block_sum(tot, scratch) + (sinks ? exp2f(sk - m) : 0.f);  // (orders wt as well)
-  const float inv = 1.f / tot;
+  const float inv = (gate ? gate[bh] : 1.f) / tot;
   for (int d = tid; d < Vp; d += 128) {
     float v = 0.f;
     for (int p = 0; p < nparts; p += 8) {  // eight parts in flight
@@ -512,7 +548,7 @@ int omnia_gqa_prep(void* q, void* kc, void* vc, int f32, const void* x, int ptyp
                    int64_t slab, int64_t ldx, const float* wq, const float* wk,
                    const float* bias, const int* positions, const int64_t* slots,
                    const float* cos_sin, int pairs, int T, int H, int G, int D, int Dp, int Vp,
-                   int R, int page, float eps, hipStream_t s) {
+                   int R, int page, float eps, const float* temp, float* gate, hipStream_t s) {
   if (Dp % 8 || Vp % 8 || ldx % 8 || slab % 8 || S < 1 || R % 2 || R > D || D > Dp || page < 1)
     return -1;
   const int w = Dp > Vp || G == 0 ? Dp : Vp;
@@ -520,8 +556,8 @@ int omnia_gqa_prep(void* q, void* kc, void* vc, int f32, const void* x, int ptyp
   if (T == 0) return 0;
   int lg = 2;
   while (lg < 6 && (8 << lg) < w) ++lg;
-  const PrepArgs a{wq, wk, bias, positions, slots, cos_sin, ldx, slab,  S,  H,
-                   G,  D,  Dp,   Vp,        R,     page,    lg,  pairs, eps};
+  const PrepArgs a{wq, wk, bias, positions, slots, cos_sin, temp, gate, ldx, slab, S,
+                   H,  G,  D,    Dp,        Vp,    R,       page, lg,  pairs, eps};
   const int hpb = 256 >> lg;
   const dim3 grid(T, (H + 2 * G + hpb - 1) / hpb);
 #define OMNIA_GP(TT, PP)                                                                       \
@@ -548,8 +584,9 @@ int omnia_gqa_prep(void* q, void* kc, void* vc, int f32, const void* x, int ptyp
 int omnia_gqa_attend(void* out, int f32, const void* q, const void* kc, const void* vc,
                      const int* block_tables, int bt_stride, const int* q_start, int nseq,
                      const int* positions, int T, int page, int H, int G, int Dp, int Vp,
-                     Mask mask, float scale, const float* sinks, hipStream_t s) {
-  if (G < 1 || H % G || page < 1 || !mask.ok()) return -1;
+                     Mask mask, Score score, const float* sinks, const float* gate,
+                     hipStream_t s) {
+  if (G < 1 || H % G || page < 1 || !mask.ok() || !score.ok()) return -1;
   if (T == 0) return 0;
   const size_t lds = (size_t)(Dp + Vp + 256 + 8) * 4;
   if (lds > 64 * 1024 || H > 65535) return -2;
@@ -557,24 +594,25 @@ int omnia_gqa_attend(void* out, int f32, const void* q, const void* kc, const vo
   if (f32)
     attend_kernel<float><<<grid, 256, lds, s>>>((float*)out, (const float*)q, (const float*)kc,
                                                 (const float*)vc, block_tables, bt_stride, q_start,
-                                                nseq, positions, page, H, G, Dp, Vp, mask, scale,
-                                                sinks);
+                                                nseq, positions, page, H, G, Dp, Vp, mask, score,
+                                                sinks, gate);
   else
     attend_kernel<bf16_t><<<grid, 256, lds, s>>>(
         (bf16_t*)out, (const bf16_t*)q, (const bf16_t*)kc, (const bf16_t*)vc, block_tables,
-        bt_stride, q_start, nseq, positions, page, H, G, Dp, Vp, mask, scale, sinks);
+        bt_stride, q_start, nseq, positions, page, H, G, Dp, Vp, mask, score, sinks, gate);
   return (int)hipGetLastError();
 }
 
 // max_ctx: no context is longer than this (sizes the score tile)
 int omnia_gqa_decode(void* out, float* part_o, float* part_ml, const void* q, const void* kc,
                      const void* vc, const int* block_tables, int bt_stride, const int* positions,
-                     int T, int page, int H, int G, int Dp, int Vp, Mask mask, float scale,
-                     const float* sinks, int splits, int max_ctx, hipStream_t s) {
+                     int T, int page, int H, int G, int Dp, int Vp, Mask mask, Score score,
+                     const float* sinks, const float* gate, int splits, int max_ctx,
+                     hipStream_t s) {
   const int max_keys = mask.ok() ? mask.most(max_ctx) : 0;
   const int lg = log2i(page);
   if (lg < 0 || G < 1 || H % G || Dp % 32 || Dp > 256 || Vp % 8 || Vp > 256 || splits < 1 ||
-      max_keys < 1 || H > 65535 || splits > 8192)
+      max_keys < 1 || H > 65535 || splits > 8192 || !score.ok())
     return -1;
   if (T == 0) return 0;
   const int group = H / G, gh = group >= 5 ? 8 : group >= 3 ? 4 : group;
@@ -587,10 +625,11 @@ int omnia_gqa_decode(void* out, float* part_o, float* part_ml, const void* q, co
   const size_t lds = 64 + (size_t)tile * 4 + (size_t)(cap / page + 4) * 4;
   if (lds > 96 * 1024) return -2;
   const dim3 grid(T, G * nch, splits);
+  const Score2 sc(score);
 #define OMNIA_GD(KK, LP, GH, NN)                                                               \
   decode_kernel<KK, LP, GH, NN><<<grid, 64 * NN, lds, s>>>(                                    \
       (bf16_t*)out, part_o, part_ml, (const bf16_t*)q, (const bf16_t*)kc, (const bf16_t*)vc,   \
-      block_tables, bt_stride, positions, H, G, nch, lg, Vp, mask, scale * kLog2e, sinks, cap)
+      block_tables, bt_stride, positions, H, G, nch, lg, Vp, mask, sc, sinks, gate, cap)
 #define OMNIA_GD_N(KK, LP, GH) \
   do { if (nw == 2) OMNIA_GD(KK, LP, GH, 2); else OMNIA_GD(KK, LP, GH, 4); } while (0)
 #define OMNIA_GD_G(KK, LP)                      \
@@ -621,7 +660,7 @@ int omnia_gqa_decode(void* out, float* part_o, float* part_ml, const void* q, co
 #undef OMNIA_GD
   if (splits > 1)
     merge_kernel<<<T * H, 128, splits * 4, s>>>((bf16_t*)out, part_o, part_ml, positions, H, Vp, mask,
-                                       splits, sinks);
+                                       splits, sinks, gate);
   return (int)hipGetLastError();
 }
 

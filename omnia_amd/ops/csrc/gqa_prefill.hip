@@ -11,10 +11,13 @@
 // Tiles go global -> LDS by LDS-DMA, two stages, one barrier a tile; the tiles of kept first
 // keys come before those of the block's window, the ones between are not visited, and tiles
 // of which a wave sees nothing are not computed.  The
-// sink is the initial term of the online softmax (maximum = sink, sum = 1).
+// sink is the initial term of the online softmax (maximum = sink, sum = 1).  Caps and
+// distance biases (score.h) are applied to the score tile in registers; the head's gate joins
+// the last division.
 #include <type_traits>
 
 #include "mask.h"
+#include "score.h"
 
 using namespace omnia;
 
@@ -53,13 +56,15 @@ struct Args {
   const int* tile_seq;
   const int* tile_q0;
   const float* sinks;  // [H] or null
+  const float* gate;   // [T, H] or null
   int bt_stride, n_tiles, H, G, hb_lg, page_lg;
   Mask mask;
-  float scale_log2;
+  Score2 score;
 };
 
-// KEEP: windows hold the sequence's first p.mask.keep keys as well
-template <int DK, int DV, bool KEEP>
+// KEEP: windows hold the sequence's first p.mask.keep keys as well.  SHAPED: scores are
+// capped or lose a distance bias
+template <int DK, int DV, bool KEEP, bool SHAPED>
 __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Args p) {
   // two K | V stages as separate objects: reads of one cannot alias the DMA into the other
   __shared__ __attribute__((aligned(16))) char st0[128 * (DK + DV)];
@@ -135,6 +140,9 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
     dma1(t, std::integral_constant<int, DV>{}, p.vc, st + 128 * DK);
   };
 
+  const float r1 = SHAPED && p.score.r1 ? p.score.r1[h] : 0.f;
+  const float r2 = SHAPED && p.score.r1 ? p.score.r2[h] : 0.f;
+  const float to2 = SHAPED ? 1.f : p.score.mul;  // the tile's scores to base 2
   float m_run = p.sinks ? p.sinks[h] * 1.4426950408889634f : -1e30f;
   float l_run = p.sinks ? 1.f : 0.f;
   float16v o[DV / 32];
@@ -168,6 +176,29 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
           sa[half] = mfma32(*reinterpret_cast<const short8*>(Kl + img<DK>(half * 32 + ql, 2 * ks + hi)),
                             qf[ks], sa[half]);
       }
+      if constexpr (SHAPED) {
+        const bool capped = p.score.cap > 0.f;
+        const float one = __builtin_fmaf(r2, (float)(qpos - k0 - 4 * hi), 1.f);
+#pragma unroll
+        for (int half = 0; half < 2; ++half)
+#pragma unroll
+          for (int r = 0; r < 16; ++r) sa[half][r] *= p.score.mul;
+        if (capped) {
+#pragma unroll
+          for (int half = 0; half < 2; ++half)
+#pragma unroll
+            for (int r = 0; r < 16; ++r) sa[half][r] = p.score.squash(sa[half][r]);
+        }
+        if (p.score.r1) {  // keys ahead of the row: not a number, masked below
+#pragma unroll
+          for (int half = 0; half < 2; ++half)
+#pragma unroll
+            for (int r = 0; r < 16; ++r) {
+              const float kk = half * 32 + (r & 3) + 8 * (r >> 2);
+              sa[half][r] = __builtin_fmaf(-r1, log2_(__builtin_fmaf(-kk, r2, one)), sa[half][r]);
+            }
+        }
+      }
       float mloc = -INFINITY;
       if (k0 + 63 > wmin || (k0 < lo_max && (!KEEP || k0 + 63 >= keep))) {  // an edge crosses the tile
         const int top = qpos - k0 - 4 * hi, bot = qlo - k0 - 4 * hi, kp = keep - k0 - 4 * hi;
@@ -186,7 +217,7 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
 #pragma unroll
           for (int r = 0; r < 16; ++r) mloc = fmaxf(mloc, sa[half][r]);
       }
-      mloc = fmaxf(mloc, __shfl_xor(mloc, 32, 64)) * p.scale_log2;
+      mloc = fmaxf(mloc, __shfl_xor(mloc, 32, 64)) * to2;
       // the running maximum moves only when a row's grows by more than 2^8
       const bool grow = mloc > m_run + 8.f;
       if (__builtin_amdgcn_ballot_w64(grow)) {
@@ -202,8 +233,8 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
       for (int half = 0; half < 2; ++half)
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
-          const float e =
-              __builtin_amdgcn_exp2f(__builtin_fmaf(sa[half][r], p.scale_log2, -m_run));
+          const float e = __builtin_amdgcn_exp2f(
+              SHAPED ? sa[half][r] - m_run : __builtin_fmaf(sa[half][r], to2, -m_run));
           sa[half][r] = e;
           lsum += e;
         }
@@ -235,7 +266,7 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
     if (j + 1 < nt) body(j + 1, B1{});
   }
   if (row_ok) {
-    const float inv = 1.f / l_run;
+    const float inv = (p.gate ? p.gate[(int64_t)(qs + qr) * p.H + h] : 1.f) / l_run;
     bf16_t* orow = p.out + ((int64_t)(qs + qr) * p.H + h) * DV;
 #pragma unroll
     for (int d = 0; d < DV / 32; ++d)
@@ -256,9 +287,9 @@ extern "C" {
 int omnia_gqa_prefill(void* out, const void* q, const void* kc, const void* vc,
                       const int* block_tables, int bt_stride, const int* q_start,
                       const int* seq_lens, const int* tile_seq, const int* tile_q0, int n_tiles,
-                      int page, int H, int G, int Dp, int Vp, Mask mask, float scale,
-                      const float* sinks, hipStream_t s) {
-  if (G < 1 || H % G || !mask.ok()) return -1;
+                      int page, int H, int G, int Dp, int Vp, Mask mask, Score score,
+                      const float* sinks, const float* gate, hipStream_t s) {
+  if (G < 1 || H % G || !mask.ok() || !score.ok()) return -1;
   int page_lg = 0;
   while (page_lg < 30 && (1 << page_lg) < page) ++page_lg;
   if ((1 << page_lg) != page) return -2;
@@ -266,14 +297,19 @@ int omnia_gqa_prefill(void* out, const void* q, const void* kc, const void* vc,
   const int group = H / G, hb_lg = group % 4 == 0 ? 2 : group % 2 == 0 ? 1 : 0;
   if ((int64_t)n_tiles * H > 2147483647LL) return -4;
   Args a{(bf16_t*)out, (const bf16_t*)q, (const bf16_t*)kc, (const bf16_t*)vc, block_tables,
-         q_start, seq_lens, tile_seq, tile_q0, sinks, bt_stride, n_tiles, H, G, hb_lg, page_lg,
-         mask, scale * 1.4426950408889634f};
+         q_start, seq_lens, tile_seq, tile_q0, sinks, gate, bt_stride, n_tiles, H, G, hb_lg,
+         page_lg, mask, Score2(score)};
+  const bool keep = mask.window > 0 && mask.chunk == 0 && mask.keep > 0;
 #define OMNIA_GQ(K, V)                                                  \
   if (Dp == K && Vp == V) {                                             \
-    if (mask.window > 0 && mask.chunk == 0 && mask.keep > 0)            \
-      prefill_kernel<K, V, true><<<n_tiles * H, 256, 0, s>>>(a);        \
+    if (!score.plain() && keep)                                         \
+      prefill_kernel<K, V, true, true><<<n_tiles * H, 256, 0, s>>>(a);  \
+    else if (!score.plain())                                            \
+      prefill_kernel<K, V, false, true><<<n_tiles * H, 256, 0, s>>>(a); \
+    else if (keep)                                                      \
+      prefill_kernel<K, V, true, false><<<n_tiles * H, 256, 0, s>>>(a); \
     else                                                                \
-      prefill_kernel<K, V, false><<<n_tiles * H, 256, 0, s>>>(a);       \
+      prefill_kernel<K, V, false, false><<<n_tiles * H, 256, 0, s>>>(a);\
     return (int)hipGetLastError();                                      \
   }
 #define OMNIA_GQV(K) \

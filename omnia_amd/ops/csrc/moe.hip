@@ -128,7 +128,7 @@ __global__ __launch_bounds__(256) void moe_router_topk_kernel(
   select_topk(mine, lane, t, E, k, renorm, ids, wts);
 }
 
-// Router for any score function: logits z[e] = x . router[e] accumulate and stay in fp32;
+// Router for any score function: logits z[e] = x . router[e] (+ bias[e]) stay in fp32;
 // weights are sigmoid(z) or softmax(z), renormalised over the chosen ones if asked.  The k
 // largest choice scores are chosen: z, or with a correction score + correction (weights stay
 // the plain scores); with groups, experts outside the `keep` groups of E / groups neighbours
@@ -140,6 +140,7 @@ struct Route {
   int* ids;    // [T, k]
   float* wts;  // [T, k]
   const float* corr;
+  const float* bias;  // [E] added to the logits, or null
   int E, k, sigmoid, renorm, groups, keep;
 };
 
@@ -156,7 +157,7 @@ __device__ __forceinline__ void choose(float* zc, int l, int64_t t, const Route&
 #pragma unroll
   for (int i = 0; i < NPL; ++i) {
     const int e = l + LPT * i;
-    z[i] = e < a.E ? zc[e] : -INFINITY;
+    z[i] = e < a.E ? zc[e] + (a.bias ? a.bias[e] : 0.f) : -INFINITY;
     if (!(z[i] == z[i])) z[i] = -INFINITY;  // NaN rows (padding) still get distinct valid ids
     top = fmaxf(top, z[i]);
   }
@@ -671,14 +672,15 @@ int omnia_moe_align(int* sorted, int* blk_expert, int* n_blocks, const int* ids,
   return (int)hipGetLastError();
 }
 
-// x [T, d] and router [E, d] in one dtype -> ids / wts [T, k]; fp32 logits; corr [E] or null
+// x [T, d] and router [E, d] in one dtype -> ids / wts [T, k]; fp32 logits; corr, bias [E] or
+// null
 int omnia_moe_route(int* ids, float* wts, const void* x, const void* router, int f32, int n_tok,
                     int d, int E, int k, int sigmoid, int renorm, const float* corr, int groups,
-                    int keep, hipStream_t s) {
+                    int keep, const float* bias, hipStream_t s) {
   if (E < 1 || E > kMaxExperts || k < 1 || k > E || k > 64 || d % (f32 ? 4 : 32)) return -1;
   if (groups < 1 || E % groups || keep < 1 || keep > groups || k > keep * (E / groups)) return -2;
   if (n_tok == 0) return 0;
-  const Route a{ids, wts, corr, E, k, sigmoid, renorm, groups, keep};
+  const Route a{ids, wts, corr, bias, E, k, sigmoid, renorm, groups, keep};
   if (f32) {
     moe_route_f32_kernel<16><<<(n_tok + 3) / 4, 256, 0, s>>>((const float*)x, (const float*)router,
                                                              n_tok, d, a);

@@ -1,6 +1,6 @@
 """Front-end of the kernels behind layer-list models: Dynamic-Tanh and RMS norms fused
 with the residual (``csrc/tanh_norm.hip``, ``csrc/rms_residual.hip``,
-``csrc/branch_residual.hip``), the gated delta rule (``csrc/delta.hip``), fixed-decay
+``csrc/branch_residual.hip``, ``csrc/joined_residual.hip``), the gated delta rule (``csrc/delta.hip``), fixed-decay
 linear attention (``csrc/lightning.hip``), latent attention (``csrc/latent.hip``),
 grouped-query attention (``csrc/gqa.hip``, ``csrc/gqa_prefill.hip``) and routed experts
 (``csrc/moe.hip``, ``csrc/pgemm.hip``).
@@ -73,13 +73,13 @@ def glu(m, bias, dtype, act: str = "silu"):
 
 # ------------------------------------------------------------------- RMS norm
 class RMSNorm:
-    """``x / sqrt(mean(x^2) + eps) * w`` over ``n`` real columns (``w`` fp32, zero on
-    the padding columns)."""
+    """``x / sqrt(mean(x^2) + eps) * gain * w`` over ``n`` real columns (``w`` fp32, zero on
+    the padding columns, or None: ``gain`` alone)."""
 
-    __slots__ = ("w", "inv_n", "eps")
+    __slots__ = ("w", "gain", "inv_n", "eps")
 
-    def __init__(self, w: torch.Tensor, n: int, eps: float):
-        self.w, self.inv_n, self.eps = w, 1.0 / n, float(eps)
+    def __init__(self, w: torch.Tensor | None, n: int, eps: float, gain: float = 1.0):
+        self.w, self.gain, self.inv_n, self.eps = w, float(gain), 1.0 / n, float(eps)
 
 
 def rms_embed(ids, table, vocab: int, emb: RMSNorm, pre: RMSNorm | None, src=None,
@@ -143,6 +143,51 @@ def branch_residual(x, branches, pre, dtype):
     return (x if pre is None else ref.rms_norm(x, pre)).to(dtype)
 
 
+class PassInput:
+    """What a pass of a looped stretch adds to the residual before its first layer: ``scale``
+    times the embedding of each row's token (``scale`` 0: nothing), and ``step`` [d] (fp32,
+    or None).  ``ids`` / ``src`` / ``tok_slots``: the rows' tokens, as
+    :func:`omnia_amd.ops.embedding`."""
+
+    __slots__ = ("ids", "table", "vocab", "scale", "step", "src", "tok_slots")
+
+    def __init__(self, ids, table, vocab: int, scale: float, step=None, src=None, tok_slots=None):
+        self.ids, self.table, self.vocab, self.scale = ids, table, vocab, float(scale)
+        self.step, self.src, self.tok_slots = step, src, tok_slots
+
+
+def joined_residual(x, parts, pres, dtype, enter: PassInput | None = None, fresh: bool = False):
+    """In place ``x += sum of parts`` and what a pass enters with (``fresh``: x starts from
+    zero); returns one normed row set in ``dtype`` for each of ``pres`` (one or two RMS
+    norms of one mean).  ``parts``: up to three (m, slots): a projection [M, d], its split-K
+    slabs [S, M, d], or (slots) per-row parts [M, S, d]."""
+    if x.is_cuda:
+        out = [torch.empty(x.shape, dtype=dtype, device=x.device) for _ in pres]
+        p = list(parts) + [(None, False)] * (3 - len(parts))
+        e = (enter.ids, enter.table, enter.vocab, enter.scale, enter.step, enter.src,
+             enter.tok_slots) if enter else (None, None, 0, 0.0, None, None, None)
+        a, b = pres[0], pres[-1]
+        kernels().joined_residual(out[0], out[1] if len(out) > 1 else None, x, fresh, *p[0],
+                                  *p[1], *p[2], *e, a.w, a.gain, b.w, b.gain, a.inv_n, a.eps)
+        return out
+    if fresh:
+        x.zero_()
+    for m, slots in parts:
+        x += m.float().sum(1) if slots else ref.slab_sum(m)
+    if enter is not None:
+        if enter.scale:
+            ids = enter.ids
+            if enter.src is not None:
+                ids = torch.where(enter.src >= 0, enter.tok_slots.index_select(
+                    0, enter.src.clamp(min=0).long()), ids)
+            ok = (ids >= 0) & (ids < enter.vocab)
+            x += enter.scale * enter.table[torch.where(
+                ok, ids, torch.zeros_like(ids)).long()].float() * ok[:, None]
+        if enter.step is not None:
+            x += enter.step
+    return [ref.rms_norm(x, n).to(dtype) for n in pres]
+
+
 def norm_residual(x, m=None, post=None, pre=None, dtype=None, bias=None, slots: bool = False,
                   identity=None, branches=None):
     """What follows a sublayer, of either norm kind (see the functions above)."""
@@ -172,20 +217,21 @@ def experts(h, w: dict, spec):
     are padded to whole tiles (``ff_pad``; d a multiple of 64)."""
     T, d = h.shape
     k, E, ff = spec.top, spec.outputs, w["down"].shape[2]
-    corr = w.get("correction")
+    corr, bias = w.get("correction"), w.get("router_b")
     if not h.is_cuda:
-        ids, wts = ref.route(h, w["router"], spec, corr)
+        ids, wts = ref.route(h, w["router"], spec, corr, bias)
         return ref.experts(h, ids, wts, w["up"], w["down"], spec), ids, wts
     kk = kernels()
     ids = torch.empty(T, k, dtype=torch.int32, device=h.device)
     wts = torch.empty(T, k, dtype=torch.float32, device=h.device)
     kk.moe_route(ids, wts, h, w["router"], k, spec.score == "sigmoid", spec.renorm, corr,
-                 spec.groups, spec.keep)
+                 spec.groups, spec.keep, bias)
     # column tiles of the 256-row prefill GEMM: 128 gate and up columns, or 256
     tile = h.dtype == torch.bfloat16 and T * k >= MOE_TILE256_ROWS * E and d % 256 == 0 and \
         ff % (128 if spec.gated else 256) == 0
     y = _moe_grouped(h, w["up"], w["down"], ids, wts, k, E, 0, spec.experts, 256 if tile else 64,
-                     (spec.alpha, spec.limit) if spec.gated else None, not spec.gated)
+                     (spec.alpha, spec.limit) if spec.expert == "clamped_glu" else None,
+                     not spec.gated)
     return y.view(T, k, d), ids, wts
 
 
@@ -356,11 +402,19 @@ def latent_prefill(q, kx, kr, vt, fb, spec, gate, out=None):
 
 
 # ------------------------------------------------------ grouped-query attention
-def gqa_prep(x, w: dict, spec, pages, positions, slots, cos_sin, dtype, eps: float):
-    """Fused projection rows (or split-K slabs) -> queries [T, H * dim_pad], with bias, norm
-    and rotation as the spec says; writes the tokens' keys and values at ``slots`` of
-    ``pages`` = (k, v), or, with
-    ``pages`` None, none (the layer borrows another one's)."""
+def temperature_table(t, positions: int, device) -> torch.Tensor:
+    """fp32 [positions]: a query's factor at each position (double precision)."""
+    p = torch.arange(1, positions + 1, dtype=torch.float64)
+    return (1.0 + t.coef * torch.log(torch.floor(p / t.every) + 1.0)).float().to(device)
+
+
+def gqa_prep(x, w: dict, spec, pages, positions, slots, cos_sin, dtype, eps: float, temp=None,
+             gate=None):
+    """Fused projection rows (or split-K slabs) -> queries [T, H * dim_pad], with bias, norm,
+    rotation and temperature (``temp``: :func:`temperature_table`) as the spec says; writes
+    the tokens' keys and values at ``slots`` of ``pages`` = (k, v), or, with ``pages`` None,
+    none (the layer borrows another one's).  ``gate`` [T, H] fp32 receives the sigmoid of
+    the row's gate columns."""
     k, v = pages if pages is not None else (None, None)
     if x.is_cuda:
         if pages is not None and checks.active(x):
@@ -369,23 +423,27 @@ def gqa_prep(x, w: dict, spec, pages, positions, slots, cos_sin, dtype, eps: flo
                         device=x.device)
         kernels().gqa_prep(q, k, v, x, w.get("q_norm"), w.get("k_norm"), w.get("in_b"), positions,
                            slots, cos_sin, spec.rotary is not None and spec.rotary.interleaved,
-                           spec.heads, spec.dim, spec.dim_pad, eps)
+                           spec.heads, spec.dim, spec.dim_pad, eps, temp, gate)
         return q
-    return ref.gqa_prep(x, w, spec, k, v, positions, slots, cos_sin, dtype, eps)
+    return ref.gqa_prep(x, w, spec, k, v, positions, slots, cos_sin, dtype, eps, temp, gate)
 
 
-def gqa_attend(q, pages, block_tables, q_start, positions, spec, sinks, out=None):
+# ``dist`` [2, H] fp32: the heads' distance biases (r1, r2), or None; ``gate`` [T, H] fp32:
+# factors of the head outputs, or None
+def gqa_attend(q, pages, block_tables, q_start, positions, spec, sinks, out=None, dist=None,
+               gate=None):
     """Generic attention (any size, bf16 / fp32): [T, H * v_pad]."""
     if out is None:
         out = torch.empty(positions.numel(), spec.heads * spec.v_pad, dtype=q.dtype,
                           device=q.device)
     args = (out, q, *pages, block_tables, q_start, positions, spec.heads, spec.mask,
-            spec.scale, sinks)
+            spec.scale, sinks, spec.softcap, dist, gate)
     (kernels().gqa_attend if q.is_cuda else ref.gqa_attend)(*args)
     return out
 
 
-def gqa_decode(q, pages, block_tables, positions, spec, sinks, splits: int, out=None):
+def gqa_decode(q, pages, block_tables, positions, spec, sinks, splits: int, out=None, dist=None,
+               gate=None):
     """bf16 decode: each row's visible keys in up to ``splits`` parts."""
     T, H, V = positions.numel(), spec.heads, spec.v_pad
     if out is None:
@@ -397,16 +455,17 @@ def gqa_decode(q, pages, block_tables, positions, spec, sinks, splits: int, out=
     if checks.active(q):
         checks.paged("gqa_decode", block_tables, positions + 1, pages[0], T)
     kernels().gqa_decode(out, po, pm, q, *pages, block_tables, positions, H, spec.mask,
-                         spec.scale, sinks, splits)
+                         spec.scale, sinks, splits, spec.softcap, dist, gate)
     return out
 
 
-def gqa_prefill(q, pages, fb, spec, sinks, out=None):
+def gqa_prefill(q, pages, fb, spec, sinks, out=None, dist=None, gate=None):
     """bf16 prefill portions (``fb``'s query tiles of 128 rows)."""
     if out is None:
         out = torch.empty(q.shape[0], spec.heads * spec.v_pad, dtype=q.dtype, device=q.device)
     if checks.active(q):
         checks.paged("gqa_prefill", fb.block_tables, fb.seq_lens, pages[0])
     kernels().gqa_prefill(out, q, *pages, fb.block_tables, fb.q_start_loc, fb.seq_lens,
-                          fb.tile_seq, fb.tile_q0, spec.heads, spec.mask, spec.scale, sinks)
+                          fb.tile_seq, fb.tile_q0, spec.heads, spec.mask, spec.scale, sinks,
+                          spec.softcap, dist, gate)
     return out

@@ -196,12 +196,15 @@ def latent_attend(q, cache, block_tables, q_start, positions, H, Cp, window, sca
 
 
 def rms_norm(x, n):
-    return x / torch.sqrt(x.pow(2).sum(-1, keepdim=True) * n.inv_n + n.eps) * n.w
+    x = x / torch.sqrt(x.pow(2).sum(-1, keepdim=True) * n.inv_n + n.eps) * n.gain
+    return x if n.w is None else x * n.w
 
 
-def route(h, router, spec, corr=None):
+def route(h, router, spec, corr=None, bias=None):
     """(ids int32 [T, top], weights fp32 [T, top])."""
     z = h.float() @ router.float().T
+    if bias is not None:
+        z = z + bias
     s = torch.sigmoid(z) if spec.score == "sigmoid" else torch.softmax(z, -1)
     c = z if corr is None else s + corr
     if spec.groups > 1:
@@ -219,6 +222,7 @@ def route(h, router, spec, corr=None):
 def experts(h, ids, wts, up, down, spec):
     """[T, top, d]: the chosen experts' weighted outputs (clamped GLUs take the weight on
     their input)."""
+    clamped = spec.expert == "clamped_glu"
     T, d = h.shape
     out = torch.zeros(T, spec.top, d, dtype=h.dtype)
     for e in ids.unique().tolist():
@@ -226,7 +230,10 @@ def experts(h, ids, wts, up, down, spec):
             continue
         t, j = (ids == e).nonzero(as_tuple=True)
         v, wt = h[t].float() @ up[e].float().T, wts[t, j, None]
-        if spec.gated:
+        if spec.expert == "glu":
+            g, u = v.chunk(2, -1)
+            a = F.silu(g) * u
+        elif clamped:
             g, u = (v * wt).chunk(2, -1)
             g, u = g.clamp(max=spec.limit), u.clamp(-spec.limit, spec.limit)
             a, wt = g * torch.sigmoid(spec.alpha * g) * (u + 1.0), 1.0
@@ -245,20 +252,24 @@ def _rotate_pairs(v, positions, cos_sin):
     return torch.stack([a * c - b * s, b * c + a * s], -1).flatten(-2)
 
 
-def gqa_prep(x, w, spec, k, v, positions, slots, cos_sin, dtype, eps):
+def gqa_prep(x, w, spec, k, v, positions, slots, cos_sin, dtype, eps, temp=None, gate=None):
     T, H, D, Dp = positions.numel(), spec.heads, spec.dim, spec.dim_pad
     R = 0 if cos_sin is None else cos_sin.shape[1]
     x = slab_sum(x)
+    if gate is not None:
+        gate.copy_(torch.sigmoid(x[:, spec.qkv_cols:spec.in_cols]))
     if w.get("in_b") is not None:
         x = x[:, :w["in_b"].numel()] + w["in_b"]
 
-    def turned(z, wn, heads):
+    def turned(z, wn, heads, factor=None):
         z = z.reshape(T, heads, Dp)
         if wn is not None:
             z = z / torch.sqrt(z.pow(2).sum(-1, keepdim=True) / D + eps) * wn
         if R:
             turn = _rotate_pairs if spec.rotary.interleaved else _rotate
             z = torch.cat([turn(z[..., :R], positions, cos_sin), z[..., R:]], -1)
+        if factor is not None:
+            z = z * factor[positions.long()][:, None, None]
         return z.to(dtype)
 
     if k is not None:
@@ -268,7 +279,7 @@ def gqa_prep(x, w, spec, k, v, positions, slots, cos_sin, dtype, eps):
         keep = slots >= 0
         b, o = slots[keep] // page, slots[keep] % page
         k[b, :, o], v[b, :, o] = kk[keep], vv[keep]
-    return turned(x[:, :H * Dp], w.get("q_norm"), H).reshape(T, H * Dp)
+    return turned(x[:, :H * Dp], w.get("q_norm"), H, temp).reshape(T, H * Dp)
 
 
 def _visible(pos, mask):
@@ -279,7 +290,8 @@ def _visible(pos, mask):
     return torch.cat([torch.arange(0, min(first, lo)), torch.arange(lo, pos + 1)])
 
 
-def gqa_attend(out, q, k, v, block_tables, q_start, positions, H, mask, scale, sinks):
+def gqa_attend(out, q, k, v, block_tables, q_start, positions, H, mask, scale, sinks, cap=0.0,
+               dist=None, gate=None):
     T, G, page = positions.numel(), k.shape[1], k.shape[2]
     qv = q.view(T, G, H // G, -1).float()
     ov = out.view(T, H, -1)
@@ -289,7 +301,13 @@ def gqa_attend(out, q, k, v, block_tables, q_start, positions, H, mask, scale, s
             b = block_tables[s, key // page].long()
             kr, vr = k[b, :, key % page].float(), v[b, :, key % page].float()  # [n, G, w]
             sc = torch.matmul(qv[t], kr.permute(1, 2, 0)).reshape(H, -1) * scale
+            if cap:
+                sc = cap * torch.tanh(sc / cap)
+            if dist is not None:
+                far = (int(positions[t]) - key).float()
+                sc = sc - dist[0][:, None] * torch.log(1.0 + dist[1][:, None] * far)
             if sinks is not None:
                 sc = torch.cat([sc, sinks[:, None]], 1)
             p = torch.softmax(sc, -1)[:, :key.numel()].view(G, H // G, -1)
-            ov[t] = torch.matmul(p, vr.permute(1, 0, 2)).reshape(H, -1).to(q.dtype)
+            o = torch.matmul(p, vr.permute(1, 0, 2)).reshape(H, -1)
+            ov[t] = (o if gate is None else o * gate[t][:, None]).to(q.dtype)
