@@ -97,7 +97,8 @@ def parse(argv=None):
                     help="multi-GPU first-contact check in a fresh child per rank before any "
                          "pod starts (parallel/preflight.py): peer access, RCCL init + "
                          "all-reduce, IPC all-reduce checked against it; auto = on with GPUs")
-    ap.add_argument("--compare", choices=["sivadra", "sekazen", "bisuzen"], default=None,
+    ap.add_argument("--compare", choices=["sivadra", "sekazen", "bisuzen", "tarunex"],
+                    default=None,
                     help="prefill / decode throughput of a model design beside the closest "
                          "model at equal size (one GPU, engine API; no serving path)")
     ap.add_argument("--compare-only", default=None, metavar="MODEL[,MODEL]",

@@ -15,7 +15,8 @@ import torch
 
 PAIRS = {"sivadra": [("sivadra-1b", "llama-1b-shape"), ("sivadra-8b", "llama-3-8b")],
          "sekazen": [("sekazen-3b", "mixtral-3b-shape"), ("sekazen-8x7b", "mixtral-8x7b")],
-         "bisuzen": [("bisuzen-3b", "sekazen-3b"), ("bisuzen-8b", "sivadra-8b")]}
+         "bisuzen": [("bisuzen-3b", "sekazen-3b"), ("bisuzen-8b", "sivadra-8b")],
+         "tarunex": [("tarunex-3b", "sekazen-3b"), ("tarunex-8b", "sivadra-8b")]}
 PREFILL = [(1, 8192), (8, 2048), (32, 512)]
 DECODE = [(1, 2048), (32, 1024), (128, 1024), (256, 512)]
 

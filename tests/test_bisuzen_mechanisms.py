@@ -140,8 +140,9 @@ def test_projection_to_queries_and_pages(kind, shape, run):
     H, G, D, V, R = shape
     rot = {"dims": R, "base": 500.0}
     spec = AttentionSpec(H, G, D, V, 1.0, RotarySpec(R, 500.0, interleaved=True)
-                         if kind == "rotated" else None, sink=False,
-                         qk_norm="unit" if kind == "unit" else None, bias=kind == "rotated")
+                         if kind == "rotated" else None, sink=None,
+                         qk_norm="unit" if kind == "unit" else None,
+                         bias="qkvo" if kind == "rotated" else "")
     eps, d, T, page = 1e-2, 40, 21, 16
     mod = GroupedQueryAttention(spec, Stub(dev, dt, eps))
     W = {"q": rnd(H * D, d, g=g), "k": rnd(G * D, d, g=g), "v": rnd(G * V, d, g=g),
@@ -199,8 +200,8 @@ def masked(kind, size, keep, n):
 def attn_spec(kind, size, keep, shape, scale=None, sink=True):
     H, G, D, V = shape
     mask = {"chunk": size} if kind == "chunk" else {"window": size, "keep_first": keep}
-    return AttentionSpec(H, G, D, V, scale or 1.5 * D ** -0.5, None, sink=sink, qk_norm=None,
-                         **mask)
+    return AttentionSpec(H, G, D, V, scale or 1.5 * D ** -0.5, None,
+                         sink="learned" if sink else None, qk_norm=None, **mask)
 
 
 def attended(q, k, v, seen, scale, sinks):

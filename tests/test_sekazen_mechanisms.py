@@ -164,7 +164,8 @@ SHAPES = {  # heads, kv heads, dim, vdim, rotated dims
 
 def spec_of(shape, window=0, scale=None, sink=True):
     H, G, D, V, R = SHAPES[shape]
-    return AttentionSpec(H, G, D, V, scale or D ** -0.5, RotarySpec(R, 1e4), window, sink)
+    return AttentionSpec(H, G, D, V, scale or D ** -0.5, RotarySpec(R, 1e4), window,
+                         "learned" if sink else None)
 
 
 @pytest.mark.parametrize("run", RUNS)
