@@ -24,6 +24,7 @@ softmax, a router or a recurrence in fp32; fp32 models run every kernel and GEMM
 from __future__ import annotations
 
 import math
+import os
 from dataclasses import dataclass
 
 import torch
@@ -32,11 +33,18 @@ import torch.nn.functional as F
 from .. import ops
 from ..ops import mixers as mops
 from ..parallel import state as pstate
+from ..parallel.overlap import side_stream
 from .config import ModelConfig
 from .feedforward import MLPS
 from .layers import tensor_shapes
 from .mixers import MIXERS, rotary_table
 from .projection import Parts, Projections
+
+
+# rows of a decode step, and of any other, that run a joined layer's sublayers on two
+# streams: below, an eager step waits for its launches; above, either one fills the chip
+FORK_DECODE = int(os.environ.get("OMNIA_FORK_DECODE", "256"))
+FORK_PREFILL = 1024, int(os.environ.get("OMNIA_FORK_PREFILL", "8192"))
 
 
 @dataclass
@@ -119,7 +127,8 @@ class HybridModel(Projections):
                                      getattr(l.mlp, "bias", False) for l in cfg.layers):
             raise ValueError(f"{cfg.name}: joined sublayers have no output biases")
         self.w = self._pack(weights if weights is not None else self._random())
-        ops.dgemm_prepare(self.device)
+        for branch in range(2 if cfg.design.joined else 1):
+            ops.dgemm_prepare(self.device, branch)
 
     # ------------------------------------------------------------ weights
     def rotary(self, rot) -> torch.Tensor:
@@ -242,11 +251,25 @@ class HybridModel(Projections):
                 return [self.w["final_norm"]]
             return [ws[i]["pre1"]] + ([ws[i]["pre2"]] if self.mlps[i] else [])
 
+        rows = x.shape[0]
+        fork = x.is_cuda and (rows <= FORK_DECODE if dec else
+                              FORK_PREFILL[0] <= rows <= FORK_PREFILL[1])
         h = mops.joined_residual(x, [], norms(0), dt, self._pass_input(fb, 0), fresh=True)
         for i, (w, mixer, mlp) in enumerate(zip(ws, self.mixers, self.mlps)):
-            parts = [(mixer.sublayer(w["mix"], h[0], fb, kv.layers[i])["m"], False)]
+            if fork and mlp:
+                # the sublayers do not need each other: the feed-forward on a stream of its
+                # own.  Tensors of either stream live until the streams have met
+                main, side = torch.cuda.current_stream(), side_stream(self.device)
+                side.wait_stream(main)
+                with ops.on_branch(1, side):
+                    f = mlp.forward(w["mlp"], h[1], dec)
+                y = mixer.sublayer(w["mix"], h[0], fb, kv.layers[i])["m"]
+                main.wait_stream(side)
+            else:
+                y = mixer.sublayer(w["mix"], h[0], fb, kv.layers[i])["m"]
+                f = mlp.forward(w["mlp"], h[1], dec) if mlp else None
+            parts = [(y, False)]
             if mlp:
-                f = mlp.forward(w["mlp"], h[1], dec)
                 parts.append((f["m"], f.get("slots", False)))
                 if "shared" in f:
                     parts.append((f["shared"], False))

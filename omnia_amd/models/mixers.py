@@ -295,6 +295,7 @@ class GroupedQueryAttention(Mixer):
              torch.zeros(s.heads, device=self.model.device) if s.sink else None}
         if s.distance_bias:
             w["dist"] = torch.stack([get("r1").float(), get("r2").float()]).contiguous()
+            w["bounded"] = mops.scores_bounded(s, w["dist"])
         if s.qk_norm:
             w["q_norm"] = norm("q.norm")
             if own:
@@ -337,7 +338,8 @@ class GroupedQueryAttention(Mixer):
     def _prefill(self, w, q, pages, fb, positions, out, gate=None):
         page, more = pages[0].shape[2], dict(out=out, dist=w.get("dist"), gate=gate)
         if self.mfma and page & (page - 1) == 0:
-            return mops.gqa_prefill(q, pages, fb, self.spec, w["sink"], **more)
+            return mops.gqa_prefill(q, pages, fb, self.spec, w["sink"],
+                                    bounded=w.get("bounded", False), **more)
         return mops.gqa_attend(q, pages, fb.block_tables, fb.q_start_loc, positions, self.spec,
                                w["sink"], **more)
 

@@ -8,6 +8,7 @@ the mock/CPU engine path).
 """
 from __future__ import annotations
 
+import contextlib
 import importlib
 import os
 import threading
@@ -110,14 +111,36 @@ _dgemm_on = os.environ.get("OMNIA_DGEMM", "1") != "0"
 _dgemm_force = os.environ.get("OMNIA_DGEMM", "") == "force"
 
 
-def dgemm_prepare(device) -> None:
-    """Allocate the split-K workspace + zeroed tile counters for ``device``.
+_dgemm_branch = 0  # which of a step's concurrent streams calls (see on_branch)
+
+
+def _dgemm_key(dev: torch.device, branch: int):
+    i = dev.index if dev.index is not None else torch.cuda.current_device()
+    return (i, branch) if branch else i
+
+
+@contextlib.contextmanager
+def on_branch(n: int, stream):
+    """Run on ``stream`` beside the main one, as branch ``n`` > 0 of a step: kernels with a
+    workspace take that branch's (``dgemm_prepare(device, n)``)."""
+    global _dgemm_branch
+    was, _dgemm_branch = _dgemm_branch, n
+    try:
+        with torch.cuda.stream(stream):
+            yield
+    finally:
+        _dgemm_branch = was
+
+
+def dgemm_prepare(device, branch: int = 0) -> None:
+    """Allocate the split-K workspace + zeroed tile counters for ``device``, for each of the
+    streams that work at the same time its own.
 
     Call eagerly (model init) so nothing is allocated while a hipGraph captures."""
     dev = torch.device(device)
     if dev.type != "cuda":
         return
-    key = dev.index if dev.index is not None else torch.cuda.current_device()
+    key = _dgemm_key(dev, branch)
     if key not in _dgemm_ws:
         _dgemm_ws[key] = (torch.empty(_DGEMM_WS_FLOATS, dtype=torch.float32, device=dev),
                           torch.zeros(_DGEMM_CNT, dtype=torch.int32, device=dev))
@@ -190,9 +213,9 @@ def _dgemm(mode: int, x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None
     cfg = dgemm_config(M, N, K, mode)
     if cfg is None:
         return None
-    key = x.device.index if x.device.index is not None else torch.cuda.current_device()
+    key = _dgemm_key(x.device, _dgemm_branch)
     if key not in _dgemm_ws:
-        dgemm_prepare(x.device)
+        dgemm_prepare(x.device, _dgemm_branch)
     ws, cnt = _dgemm_ws[key]
     x = x.contiguous()
     out = x.new_empty(M, N) if out is None else out

@@ -200,7 +200,7 @@ int omnia_gqa_prefill(void* out, const void* q, const void* kc, const void* vc,
                       const int* block_tables, int bt_stride, const int* q_start,
                       const int* seq_lens, const int* tile_seq, const int* tile_q0, int n_tiles,
                       int page, int H, int G, int Dp, int Vp, Mask mask, Score score,
-                      const float* sinks, const float* gate, hipStream_t s);
+                      const float* sinks, const float* gate, int bounded, hipStream_t s);
 int omnia_joined_residual(void* h1, void* h2, int f32, float* x, int fresh, int rows, int d,
                           const void* am, int at, int aS, int64_t arow, int64_t apart,
                           const void* bm, int bS, int64_t brow, int64_t bpart, const void* cm,
@@ -1885,7 +1885,7 @@ void gqa_decode(at::Tensor out, OptT part_o, OptT part_ml, at::Tensor q, at::Ten
 void gqa_prefill(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor block_tables,
                  at::Tensor q_start, at::Tensor seq_lens, at::Tensor tile_seq, at::Tensor tile_q0,
                  int64_t H, MaskT mask, double scale, OptT sinks, double cap, OptT dist,
-                 OptT gate) {
+                 OptT gate, bool bounded) {
   CHECK_GPU(q); CHECK_BF16(q);
   TORCH_CHECK(q.dim() == 2, "q [T, H*Dp]");
   const KV s = kv_sizes(out, q, k, v, q.size(0), H, sinks);
@@ -1896,7 +1896,7 @@ void gqa_prefill(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::T
                              veci(tile_seq, nt, "tile_seq"), veci(tile_q0, nt, "tile_q0"), nt,
                              s.page, H, s.G, s.Dp, s.Vp, mask_of(mask),
                              score_of(scale, cap, dist, H), opt_ptr<float>(sinks),
-                             opt_vecf(gate, q.size(0) * H, "gate"), cur_stream()),
+                             opt_vecf(gate, q.size(0) * H, "gate"), bounded, cur_stream()),
            "gqa_prefill");
 }
 

@@ -13,7 +13,10 @@
 // of which a wave sees nothing are not computed.  The
 // sink is the initial term of the online softmax (maximum = sink, sum = 1).  Caps and
 // distance biases (score.h) are applied to the score tile in registers; the head's gate joins
-// the last division.
+// the last division.  Capped scores that only lose by their distance are bounded: exp(s) fits
+// fp32 as it is, and neither a running maximum nor a rescaling is needed.  A tile is then
+// worked on in halves of 32 keys, its biases are a table of distances in LDS, and the
+// denominator sums the same rounded P as the output.
 #include <type_traits>
 
 #include "mask.h"
@@ -62,15 +65,17 @@ struct Args {
   Score2 score;
 };
 
-// KEEP: windows hold the sequence's first p.mask.keep keys as well.  SHAPED: scores are
-// capped or lose a distance bias
-template <int DK, int DV, bool KEEP, bool SHAPED>
+// KEEP: windows hold the sequence's first p.mask.keep keys as well.  SHAPE: scores are plain
+// (0), capped or biased (1), capped and biased within bounds (2)
+template <int DK, int DV, bool KEEP, int SHAPE>
 __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Args p) {
   // two K | V stages as separate objects: reads of one cannot alias the DMA into the other
   __shared__ __attribute__((aligned(16))) char st0[128 * (DK + DV)];
   __shared__ __attribute__((aligned(16))) char st1[128 * (DK + DV)];
   constexpr int kMaxPages = 1024;  // pages of the visible range staged in LDS
   __shared__ int pg_lds[kMaxPages];
+  // SHAPE 2: per wave, cap - bias of the 95 distances between its rows and a tile's keys
+  __shared__ float dist_lds[SHAPE == 2 ? 4 : 1][96];
 
   const int HB = 1 << p.hb_lg, group = p.H / p.G;
   // blocks of one key/value head are neighbours: (head block, tile, sub-tile)
@@ -140,11 +145,12 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
     dma1(t, std::integral_constant<int, DV>{}, p.vc, st + 128 * DK);
   };
 
-  const float r1 = SHAPED && p.score.r1 ? p.score.r1[h] : 0.f;
-  const float r2 = SHAPED && p.score.r1 ? p.score.r2[h] : 0.f;
-  const float to2 = SHAPED ? 1.f : p.score.mul;  // the tile's scores to base 2
-  float m_run = p.sinks ? p.sinks[h] * 1.4426950408889634f : -1e30f;
-  float l_run = p.sinks ? 1.f : 0.f;
+  const float r1 = SHAPE && p.score.r1 ? p.score.r1[h] : 0.f;
+  const float r2 = SHAPE && p.score.r1 ? p.score.r2[h] : 0.f;
+  const float to2 = SHAPE ? 1.f : p.score.mul;  // the tile's scores to base 2
+  const float sink = p.sinks ? p.sinks[h] * 1.4426950408889634f : -1e30f;
+  float m_run = sink;
+  float l_run = p.sinks && SHAPE != 2 ? 1.f : 0.f;
   float16v o[DV / 32];
 #pragma unroll
   for (int d = 0; d < DV / 32; ++d)
@@ -165,7 +171,78 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
     const char* Kl = buf ? st1 : st0;
     const char* Vl = Kl + 128 * DK;
     const int k0 = t * 64;
-    if (k0 <= wmax && (k0 + 63 >= lo_min || (KEEP && k0 < keep))) {  // wave-uniform: some row sees some key
+    // S^T of 32 keys
+    auto scores = [&](int half) {
+      float16v a;
+#pragma unroll
+      for (int r = 0; r < 16; ++r) a[r] = 0.f;
+#pragma unroll
+      for (int ks = 0; ks < DK / 16; ++ks)
+        a = mfma32(*reinterpret_cast<const short8*>(Kl + img<DK>(half * 32 + ql, 2 * ks + hi)),
+                   qf[ks], a);
+      return a;
+    };
+    // O^T += V^T P^T over the 16 keys of a k-step
+    auto add = [&](int st, short8 pb) {
+      typedef short v4s __attribute__((ext_vector_type(4)));
+      typedef __attribute__((address_space(3))) v4s* lds_v4s;
+      const int kb = (st >> 1) * 32 + 16 * (st & 1) + 4 * (g >> 1) + qg;
+#pragma unroll
+      for (int d = 0; d < DV / 32; ++d) {
+        const int ch = d * 4 + 2 * (g & 1) + (pp >> 1);
+        const v4s lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+            (lds_v4s)(Vl + img<DV>(kb, ch) + 8 * (pp & 1)));
+        const v4s hv = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+            (lds_v4s)(Vl + img<DV>(kb + 8, ch) + 8 * (pp & 1)));
+        o[d] = mfma32(__builtin_shufflevector(lo, hv, 0, 1, 2, 3, 4, 5, 6, 7), pb, o[d]);
+      }
+    };
+    // wave-uniform: some row sees some key
+    const bool seen = k0 <= wmax && (k0 + 63 >= lo_min || (KEEP && k0 < keep));
+    if (SHAPE == 2 && seen) {
+      // entry t: distance (first row + 31) - (first key) - t; keys ahead of a row are masked
+      float* dist = dist_lds[w];
+      const int far = off + q0 + 31 - k0;
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const int t = lane + 64 * i;
+        if (t < 95)
+          dist[t] = p.score.cap - r1 * log2_(__builtin_fmaf(r2, (float)max(far - t, 0), 1.f));
+      }
+      __builtin_amdgcn_wave_barrier();
+      const float* mine = dist + 31 - ql + 4 * hi;
+#pragma unroll
+      for (int half = 0; half < 2; ++half) {
+        if (k0 + 32 * half > wmax) break;
+        float16v sa = scores(half);
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+          const float e = __builtin_amdgcn_exp2f(sa[r] * p.score.mul) + 1.f;
+          sa[r] = __builtin_fmaf(-2.f * p.score.cap, __builtin_amdgcn_rcpf(e),
+                                 mine[half * 32 + (r & 3) + 8 * (r >> 2)]);
+        }
+        if (k0 + 63 > wmin || k0 < lo_max) {  // an edge crosses the tile
+          const int top = qpos - k0 - 4 * hi, bot = qlo - k0 - 4 * hi;
+#pragma unroll
+          for (int r = 0; r < 16; ++r) {
+            const int kk = half * 32 + (r & 3) + 8 * (r >> 2);
+            sa[r] = kk > top || kk < bot ? -INFINITY : sa[r];
+          }
+        }
+#pragma unroll
+        for (int st = 0; st < 2; ++st) {
+          short8 pb;
+#pragma unroll
+          for (int j = 0; j < 8; ++j)
+            pb[j] = __builtin_bit_cast(short, (__bf16)__builtin_amdgcn_exp2f(sa[8 * st + j]));
+          const uint4v pairs = __builtin_bit_cast(uint4v, pb);
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            l_run += __uint_as_float(pairs[j] << 16) + __uint_as_float(pairs[j] & 0xffff0000u);
+          add(2 * half + st, pb);
+        }
+      }
+    } else if (seen) {
       float16v sa[2];
 #pragma unroll
       for (int half = 0; half < 2; ++half) {
@@ -176,14 +253,13 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
           sa[half] = mfma32(*reinterpret_cast<const short8*>(Kl + img<DK>(half * 32 + ql, 2 * ks + hi)),
                             qf[ks], sa[half]);
       }
-      if constexpr (SHAPED) {
-        const bool capped = p.score.cap > 0.f;
+      if constexpr (SHAPE == 1) {
         const float one = __builtin_fmaf(r2, (float)(qpos - k0 - 4 * hi), 1.f);
 #pragma unroll
         for (int half = 0; half < 2; ++half)
 #pragma unroll
           for (int r = 0; r < 16; ++r) sa[half][r] *= p.score.mul;
-        if (capped) {
+        if (p.score.cap > 0.f) {
 #pragma unroll
           for (int half = 0; half < 2; ++half)
 #pragma unroll
@@ -234,29 +310,18 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
           const float e = __builtin_amdgcn_exp2f(
-              SHAPED ? sa[half][r] - m_run : __builtin_fmaf(sa[half][r], to2, -m_run));
+              SHAPE ? sa[half][r] - m_run : __builtin_fmaf(sa[half][r], to2, -m_run));
           sa[half][r] = e;
           lsum += e;
         }
       l_run += lsum + __shfl_xor(lsum, 32, 64);
-      typedef short v4s __attribute__((ext_vector_type(4)));
-      typedef __attribute__((address_space(3))) v4s* lds_v4s;
 #pragma unroll
       for (int st = 0; st < 4; ++st) {
         short8 pb;
 #pragma unroll
         for (int j = 0; j < 8; ++j)
           pb[j] = __builtin_bit_cast(short, (__bf16)sa[st >> 1][8 * (st & 1) + j]);
-        const int kb = (st >> 1) * 32 + 16 * (st & 1) + 4 * (g >> 1) + qg;
-#pragma unroll
-        for (int d = 0; d < DV / 32; ++d) {
-          const int ch = d * 4 + 2 * (g & 1) + (pp >> 1);
-          const v4s lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-              (lds_v4s)(Vl + img<DV>(kb, ch) + 8 * (pp & 1)));
-          const v4s hv = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-              (lds_v4s)(Vl + img<DV>(kb + 8, ch) + 8 * (pp & 1)));
-          o[d] = mfma32(__builtin_shufflevector(lo, hv, 0, 1, 2, 3, 4, 5, 6, 7), pb, o[d]);
-        }
+        add(st, pb);
       }
     }
     __syncthreads();  // the next tile landed and this one is read by all waves
@@ -265,6 +330,8 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
     body(j, B0{});
     if (j + 1 < nt) body(j + 1, B1{});
   }
+  if constexpr (SHAPE == 2)
+    l_run += __shfl_xor(l_run, 32, 64) + (p.sinks ? __builtin_amdgcn_exp2f(sink) : 0.f);
   if (row_ok) {
     const float inv = (p.gate ? p.gate[(int64_t)(qs + qr) * p.H + h] : 1.f) / l_run;
     bf16_t* orow = p.out + ((int64_t)(qs + qr) * p.H + h) * DV;
@@ -284,12 +351,14 @@ __global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void prefill_kernel(Ar
 
 extern "C" {
 
+// bounded: r1, r2 >= 0 in all heads, the cap at most 40 and sinks of ordinary size
 int omnia_gqa_prefill(void* out, const void* q, const void* kc, const void* vc,
                       const int* block_tables, int bt_stride, const int* q_start,
                       const int* seq_lens, const int* tile_seq, const int* tile_q0, int n_tiles,
                       int page, int H, int G, int Dp, int Vp, Mask mask, Score score,
-                      const float* sinks, const float* gate, hipStream_t s) {
+                      const float* sinks, const float* gate, int bounded, hipStream_t s) {
   if (G < 1 || H % G || !mask.ok() || !score.ok()) return -1;
+  if (bounded && (!(score.cap > 0.f && score.cap <= 40.f) || !score.r1)) return -5;
   int page_lg = 0;
   while (page_lg < 30 && (1 << page_lg) < page) ++page_lg;
   if ((1 << page_lg) != page) return -2;
@@ -303,13 +372,15 @@ int omnia_gqa_prefill(void* out, const void* q, const void* kc, const void* vc,
 #define OMNIA_GQ(K, V)                                                  \
   if (Dp == K && Vp == V) {                                             \
     if (!score.plain() && keep)                                         \
-      prefill_kernel<K, V, true, true><<<n_tiles * H, 256, 0, s>>>(a);  \
+      prefill_kernel<K, V, true, 1><<<n_tiles * H, 256, 0, s>>>(a);     \
+    else if (bounded)                                                   \
+      prefill_kernel<K, V, false, 2><<<n_tiles * H, 256, 0, s>>>(a);    \
     else if (!score.plain())                                            \
-      prefill_kernel<K, V, false, true><<<n_tiles * H, 256, 0, s>>>(a); \
+      prefill_kernel<K, V, false, 1><<<n_tiles * H, 256, 0, s>>>(a);    \
     else if (keep)                                                      \
-      prefill_kernel<K, V, true, false><<<n_tiles * H, 256, 0, s>>>(a); \
+      prefill_kernel<K, V, true, 0><<<n_tiles * H, 256, 0, s>>>(a);     \
     else                                                                \
-      prefill_kernel<K, V, false, false><<<n_tiles * H, 256, 0, s>>>(a);\
+      prefill_kernel<K, V, false, 0><<<n_tiles * H, 256, 0, s>>>(a);    \
     return (int)hipGetLastError();                                      \
   }
 #define OMNIA_GQV(K) \

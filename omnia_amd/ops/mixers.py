@@ -459,13 +459,21 @@ def gqa_decode(q, pages, block_tables, positions, spec, sinks, splits: int, out=
     return out
 
 
-def gqa_prefill(q, pages, fb, spec, sinks, out=None, dist=None, gate=None):
-    """bf16 prefill portions (``fb``'s query tiles of 128 rows)."""
+def scores_bounded(spec, dist) -> bool:
+    """Capped scores that distance only lowers, with no learned sink: their exponentials need
+    no maximum taken off (fp32 holds exp(40) times any context)."""
+    return (0.0 < spec.softcap <= 40.0 and spec.sink != "learned" and dist is not None
+            and bool((dist >= 0).all()))
+
+
+def gqa_prefill(q, pages, fb, spec, sinks, out=None, dist=None, gate=None, bounded=False):
+    """bf16 prefill portions (``fb``'s query tiles of 128 rows).  ``bounded``:
+    :func:`scores_bounded`."""
     if out is None:
         out = torch.empty(q.shape[0], spec.heads * spec.v_pad, dtype=q.dtype, device=q.device)
     if checks.active(q):
         checks.paged("gqa_prefill", fb.block_tables, fb.seq_lens, pages[0])
     kernels().gqa_prefill(out, q, *pages, fb.block_tables, fb.q_start_loc, fb.seq_lens,
                           fb.tile_seq, fb.tile_q0, spec.heads, spec.mask, spec.scale, sinks,
-                          spec.softcap, dist, gate)
+                          spec.softcap, dist, gate, bounded)
     return out
