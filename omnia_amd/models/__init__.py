@@ -1,5 +1,5 @@
 """Model families served by the in-node engine (Llama-3 dense, Mixtral MoE, and the
-layer lists Sivadra, Sekazen and Bisuzen)."""
+layer lists Sivadra, Sekazen, Bisuzen and Tarunex)."""
 from .config import REGISTRY, ModelConfig, resolve  # noqa: F401
 
 

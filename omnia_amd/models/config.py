@@ -325,15 +325,15 @@ TINY_TARUNEX = ModelConfig(
 # model named beside each
 TARUNEX_3B = ModelConfig(  # sekazen-3b
     name="tarunex-3b", arch="tarunex", vocab_size=32768, hidden_size=2048, num_layers=16,
-    intermediate_size=3072, max_position=131072, embed_scale=8.0, logit_scale=0.25,
-    logit_softcap=30.0, bos_token_id=256, eos_token_ids=(257,),
+    intermediate_size=3072, max_position=131072, embed_scale=8.0, logit_scale=0.5,
+    logit_softcap=40.0, bos_token_id=256, eos_token_ids=(257,),
     layers=looped(((LayerSpec(_biased(16, 8, 128, 8192), _shared(3072, 8, 2, 2048)),) * 3
                    + (LayerSpec(_latent(16, 1024, 500000.0), _shared(3072, 8, 2, 2048)),)) * 3,
                   4, 8, 2))
 TARUNEX_8B = ModelConfig(  # sivadra-8b
     name="tarunex-8b", arch="tarunex", vocab_size=128256, hidden_size=4096, num_layers=32,
-    intermediate_size=7168, max_position=131072, embed_scale=8.0, logit_scale=0.25,
-    logit_softcap=30.0, bos_token_id=256, eos_token_ids=(257,),
+    intermediate_size=7168, max_position=131072, embed_scale=8.0, logit_scale=0.5,
+    logit_softcap=40.0, bos_token_id=256, eos_token_ids=(257,),
     layers=looped(((LayerSpec(_biased(32, 8, 128, 8192), _shared(7168, 3, 1, 7168)),)
                    + (LayerSpec(_latent(32, 1536, 500000.0), _shared(7168, 3, 1, 7168)),)) * 10,
                   4, 16, 2))

@@ -146,6 +146,29 @@ def test_long_prompt(models, run):
           max_tokens=4608)
 
 
+@pytest.mark.gpu
+@pytest.mark.parametrize("run", RUNS[1:])
+def test_two_streams(models, run, monkeypatch):
+    """Sublayers side by side give what they give one after another: a long prompt, then
+    replays of decode graphs with eager steps between."""
+    from omnia_amd.models import hybrid
+
+    cfg = sc.CASES["tile"]
+    t, u = sc.tokens(cfg, 1130, 30), sc.tokens(cfg, 40, 31)
+    sched = [[("a", t[:1100])]]
+    for k, x in enumerate(t[1100:]):
+        sched.append([("a", [x])] + ([("b", u[k:k + 2])] if k % 7 == 0 else []))
+    got = []
+    for rows, span in ((256, (1024, 8192)), (0, (1, 0))):
+        monkeypatch.setattr(hybrid, "FORK_DECODE", rows)
+        monkeypatch.setattr(hybrid, "FORK_PREFILL", span)
+        z, rp = sc.replay(models("tile")[2], sched, run[1], run[0], max_tokens=1280)
+        assert rp.engine.runner.stats["graph_replays"] >= 20
+        got.append(z)
+    for i in "ab":
+        assert sc.error(got[0][i], got[1][i].double()) < 1e-6
+
+
 @pytest.mark.parametrize("run", RUNS)
 def test_rows_do_not_depend_on_their_batch(models, run):
     """The same prompt and decoded tokens, alone and in a full batch of strangers."""

@@ -315,6 +315,28 @@ def test_shaped_scores(shape, page, cap, dist, window, keep, run):
 
 
 @pytest.mark.parametrize("run", RUNS)
+def test_distance_that_raises_scores(run):
+    """Negative biases, and caps past what fp32 exponentials hold, keep the running maximum."""
+    g = gen(14)
+    r = torch.tensor([[-3.0, 0.5, -0.7, 0.0], [2.0, 0.1, 5.0, 1.0]], dtype=torch.float64)
+    for cap, low in ((8.0, False), (300.0, True), (41.0, True), (40.0, True)):
+        spec = spec_of((4, 2, 64, 64), cap=cap, scale=2.0, temp=None)
+        rr = r.abs() if low else r
+        assert mops.scores_bounded(spec, rr) == (low and cap == 40.0)
+        P = make_paged(run, spec, g, r=rr)
+        n, gates = 200, torch.ones(200, 4, dtype=torch.float64)
+        q, k, v = rnd(n, 4, 64, g=g), rnd(n, 2, 64, g=g), rnd(n, 2, 64, g=g)
+        if P.dt == torch.bfloat16 and cap > 100:  # sharp scores of rounded products
+            q = 0.25 * q
+        bt, sinks = P.put(k, v), torch.zeros(4, device=P.dev)
+        want = dense(q, k, v, spec, rr, gates)
+        lim = {torch.float32: 2e-4, torch.bfloat16: 0.03}[P.dt]
+        assert rel(P.prefill_gated([q], [bt], [n], sinks, gates), want) < lim, cap
+        d = P.decode_gated(q[-1:], [bt], [n], sinks, gates[:1], 3)
+        assert rel(d[0], want[-1]) < lim, cap
+
+
+@pytest.mark.parametrize("run", RUNS)
 @pytest.mark.parametrize("n", [140, 700])
 def test_one_key_that_stands_out(n, run):
     """One key far above all others, near and far away, at page borders and ends of tiles: its
